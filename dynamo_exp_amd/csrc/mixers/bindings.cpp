@@ -21,8 +21,13 @@ int dxm_embed_streams(float*, const void*, const int64_t*, int, int, int, int64_
 int dxm_section_norm(void*, const void*, int64_t, const float*, int, int, float, int, hipStream_t);
 int dxm_depth_mix(float*, float*, int64_t, int, const float*, const int64_t*, int, float, const float*, void*,
                   const void*, int64_t, const float*, int, int, hipStream_t);
-int dxm_retention(float*, float*, int, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*,
-                  float, const int64_t*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
+int dxm_linear_scan(int, float*, float*, int, const void*, int64_t, const void*, int64_t, const void*, int64_t, float,
+                    float, int, const float*, const void*, int64_t, const float*, const float*, const float*, float,
+                    const int64_t*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
+int dxm_norm_rope_cache(void*, int64_t, const int64_t*, const int64_t*, int, int, int, int, int, const float*,
+                        const float*, float, const float*, int, void*, void*, int, hipStream_t);
+int dxm_gate_group_norm(void*, int64_t, const float*, const void*, int64_t, const float*, int, int, int, float, int,
+                        hipStream_t);
 int dxm_latent_rope(void*, const void*, const void*, int64_t, int, int, const void*, int64_t, const float*, float,
                     const float*, int, float, const int64_t*, const int64_t*, void*, int, int, int, int, int,
                     hipStream_t);
@@ -30,12 +35,12 @@ int dxm_gather_rows(void*, const void*, const int64_t*, int, int, int64_t, int, 
 int dxm_residual_step(float*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*,
                       const void*, int64_t, const float*, float, int, const float*, const float*, void*, void*, int, int,
                       int, hipStream_t);
-int dxm_act_mul(void*, const void*, int64_t, const void*, int64_t, int, int, int64_t, int, float, float, int,
+int dxm_act_mul(void*, const void*, int64_t, const void*, int64_t, int, int, int64_t, int, float, float, float, int,
                 hipStream_t);
 int dxm_delta_rule(float*, float*, int, float*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
                    int64_t, const void*, int64_t, const float*, const float*, float, float, const int64_t*, const int*,
                    const int*, int, int, int, int, int, int, hipStream_t);
-int dxm_conv_rope_cache(void*, const void*, int64_t, const float*, int, const void*, int, const int64_t*,
+int dxm_conv_rope_cache(void*, const void*, int64_t, const float*, const float*, int, int, const void*, int, const int64_t*,
                         const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, const float*,
                         int, void*, void*, int, hipStream_t);
 int dxm_conv_state_update(void*, int, const void*, int64_t, const int64_t*, const int*, const int*, int, int, int, int,
@@ -98,13 +103,26 @@ PYBIND11_MODULE(_C_mixers, m) {
                         P(out), P(c), cs, F(cw), W, f32, S(st)),
           "depth_mix");
   });
-  m.def("retention", [](u out, u state, int n_slots, u q, int64_t qs, u k, int64_t ks, u v, int64_t vs, u decay,
-                        float k_scale, u pos, u seq_rows, u slots, int n_seq, int T, int H, int dk, int dv, int f32,
-                        u st) {
-    check(dxm_retention(F(out), F(state), n_slots, P(q), qs, P(k), ks, P(v), vs, F(decay), k_scale,
-                        reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int*>(seq_rows),
-                        reinterpret_cast<const int*>(slots), n_seq, T, H, dk, dv, f32, S(st)),
-          "retention");
+  m.def("linear_scan", [](int mode, u out, u state, int n_slots, u q, int64_t qs, u k, int64_t ks, u v, int64_t vs,
+                          float q_scale, float k_scale, int qk_rep, u decay, u gate, int64_t gs, u g_bias, u rate,
+                          u skip, float inv_tau, u pos, u seq_rows, u slots, int n_seq, int T, int H, int dk, int dv,
+                          int f32, u st) {
+    check(dxm_linear_scan(mode, F(out), F(state), n_slots, P(q), qs, P(k), ks, P(v), vs, q_scale, k_scale, qk_rep,
+                          F(decay), P(gate), gs, F(g_bias), F(rate), F(skip), inv_tau,
+                          reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int*>(seq_rows),
+                          reinterpret_cast<const int*>(slots), n_seq, T, H, dk, dv, f32, S(st)),
+          "linear_scan");
+  });
+  m.def("norm_rope_cache", [](u x, int64_t xs, u pos, u slots, int rows, int n_q, int n_k, int d, int v_w, u qw, u kw,
+                              float eps, u inv_freq, int half, u kc, u vc, int f32, u st) {
+    check(dxm_norm_rope_cache(P(x), xs, reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int64_t*>(slots),
+                              rows, n_q, n_k, d, v_w, F(qw), F(kw), eps, F(inv_freq), half, P(kc), P(vc), f32, S(st)),
+          "norm_rope_cache");
+  });
+  m.def("gate_group_norm", [](u out, int64_t os, u y, u z, int64_t zs, u w, int rows, int n_groups, int n, float eps,
+                              int f32, u st) {
+    check(dxm_gate_group_norm(P(out), os, F(y), P(z), zs, F(w), rows, n_groups, n, eps, f32, S(st)),
+          "gate_group_norm");
   });
   m.def("latent_rope", [](u q_out, u qa, u q, int64_t qs, int q_head, int q_off, u kv, int64_t kvs, u cn, float eps,
                           u inv_freq, int half, float mag, u pos, u slots, u cache, int T, int H, int r, int dr,
@@ -125,8 +143,8 @@ PYBIND11_MODULE(_C_mixers, m) {
           "residual_step");
   });
   m.def("act_mul", [](u out, u gate, int64_t gs, u up, int64_t us, int rows, int Fw, int64_t os, int act, float limit,
-                      float alpha, int f32, u st) {
-    check(dxm_act_mul(P(out), P(gate), gs, P(up), us, rows, Fw, os, act, limit, alpha, f32, S(st)), "act_mul");
+                      float alpha, float post, int f32, u st) {
+    check(dxm_act_mul(P(out), P(gate), gs, P(up), us, rows, Fw, os, act, limit, alpha, post, f32, S(st)), "act_mul");
   });
   m.def("moe_route", [](u idx, u w, u z, u corr, int T, int E, int top, int n_groups, int keep, int score,
                         int group_max, u st) {
@@ -143,10 +161,10 @@ PYBIND11_MODULE(_C_mixers, m) {
                          dv, f32, S(st)),
           "delta_rule");
   });
-  m.def("conv_rope_cache", [](u q, u x, int64_t xs, u cw, int taps, u tail, int n_slots, u pos, u kv_slots, u row_seq,
+  m.def("conv_rope_cache", [](u q, u x, int64_t xs, u cw, u cb, int silu, int taps, u tail, int n_slots, u pos, u kv_slots, u row_seq,
                               u seq_rows, u slots, int n_seq, int T, int n_q, int n_k, int d, int dv, u inv_freq,
                               int half, u kc, u vc, int f32, u st) {
-    check(dxm_conv_rope_cache(P(q), P(x), xs, F(cw), taps, P(tail), n_slots, reinterpret_cast<const int64_t*>(pos),
+    check(dxm_conv_rope_cache(P(q), P(x), xs, F(cw), F(cb), silu, taps, P(tail), n_slots, reinterpret_cast<const int64_t*>(pos),
                               reinterpret_cast<const int64_t*>(kv_slots), reinterpret_cast<const int*>(row_seq),
                               reinterpret_cast<const int*>(seq_rows), reinterpret_cast<const int*>(slots), n_seq, T,
                               n_q, n_k, d, dv, F(inv_freq), half, P(kc), P(vc), f32, S(st)),

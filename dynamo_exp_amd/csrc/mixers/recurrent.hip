@@ -1,7 +1,8 @@
 // Kernels with per-sequence state for gfx950: the generalized delta rule (a
-// running matrix per head), retention (a fixed decay per head), short causal convolutions over time fused with
-// rotary positions and the paged cache write, the convolution tail update, and
-// the per-head unit-RMS + gate that follows a recurrent mixer.
+// running matrix per head), short causal convolutions over time (bias and
+// activation optional) fused with rotary positions and the paged cache write,
+// the convolution tail update, and the norms + gates that follow a recurrent
+// mixer.  (Linear recurrences without a removal term: linear_scan.hip.)
 //
 // State lives in slots ([slots, ...] tensors); a step names the slot of each of
 // its sequences (state_slots [n_seq], -1: a padding row that touches nothing)
@@ -12,18 +13,9 @@
 // Every kernel is a template over the activation element (bf16 bits or float);
 // decays, removal rates, unit keys, the running matrix, angles and all sums are
 // fp32 whatever the element is.  Sizes are run-time arguments.
-#include "../kernels/common.h"
+#include "recurrent.h"
 
 namespace {
-
-template <typename T> __device__ __forceinline__ float ldf(const T* p, int64_t i);
-template <> __device__ __forceinline__ float ldf<bf16_t>(const bf16_t* p, int64_t i) { return bf16_to_f32(p[i]); }
-template <> __device__ __forceinline__ float ldf<float>(const float* p, int64_t i) { return p[i]; }
-template <typename T> __device__ __forceinline__ void stf(T* p, int64_t i, float v);
-template <> __device__ __forceinline__ void stf<bf16_t>(bf16_t* p, int64_t i, float v) { p[i] = f32_to_bf16(v); }
-template <> __device__ __forceinline__ void stf<float>(float* p, int64_t i, float v) { p[i] = v; }
-
-__device__ __forceinline__ float sigmoidf_(float z) { return 1.f / (1.f + expf(-z)); }
 
 // ---------------------------------------------------------------------------
 // Generalized delta rule.  Per (sequence, head) a matrix S [dk, dv]:
@@ -45,8 +37,6 @@ __device__ __forceinline__ float sigmoidf_(float z) { return 1.f / (1.f + expf(-
 // 3, dk]): it is elementwise work and would otherwise sit in the sequential
 // chain.  Tokens are staged through LDS kTok at a time, fetched into registers
 // one block ahead (the latency hides behind the current block's recurrence).
-constexpr int kRows = 16;  // state rows per thread
-constexpr int kTok = 8;    // tokens per staged block
 
 struct DeltaArgs {
   float* out;    // [T, H * dv]
@@ -59,20 +49,6 @@ struct DeltaArgs {
   const int* slots;
   int n_slots, T, H, dk, dv;
 };
-
-template <int CTRL> __device__ __forceinline__ float dpp_f(float v) {
-  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, false));
-}
-// sum over the R lanes of an aligned lane group (R <= 16), the result in every lane of the group:
-// neighbours within a quad, the other pair of the quad, the other quad of a half row (half-row
-// mirror: the quads already hold one value each), the other half of a row of 16 (row mirror)
-template <int R> __device__ __forceinline__ float group_sum(float v) {
-  if constexpr (R >= 2) v += dpp_f<0xB1>(v);
-  if constexpr (R >= 4) v += dpp_f<0x4E>(v);
-  if constexpr (R >= 8) v += dpp_f<0x141>(v);
-  if constexpr (R >= 16) v += dpp_f<0x140>(v);
-  return v;
-}
 
 // one wave per (row, head): u = k / sqrt(sum k^2 + key_eps), w = exp(-decay_scale sigmoid(wl + w_bias)),
 // a u with a = sigmoid(al + a_bias)
@@ -319,247 +295,8 @@ void launch_delta(const DeltaArgs& g, int n_seq, hipStream_t st) {
 }
 
 // ---------------------------------------------------------------------------
-// Retention: linear attention with one fixed decay per head, no softmax and no
-// denominator.  Per (sequence, head) a matrix S [dk, dv]:
-//     S_t = decay_h S_(t-1) + (k_scale k_t) v_t^T,   o_t = S_t^T q_t.
-// Columns of S are independent: R neighbouring lanes share a column (lane r of
-// the group owns rows r, r + R, ..., up to kRows of them, in registers) and join
-// their partial q^T S by DPP lane exchanges; a workgroup owns blockDim / R
-// columns of one (sequence, head).  Tokens are staged through LDS kTok at a
-// time (q, scaled k: [kTok][dk]; v: [kTok][columns]).  State layout as for the
-// delta rule: [slots, H, dv, dk], a column's rows contiguous.
-struct RetArgs {
-  float* out;    // [T, H * dv]
-  float* state;  // [slots, H, dv, dk]
-  const void *q, *k, *v;
-  int64_t qs, ks, vs;  // row strides (elements)
-  const float* decay;  // [H]
-  float k_scale;
-  const int64_t* pos;
-  const int* seq_rows;  // null: row i is sequence i
-  const int* slots;
-  int n_slots, T, H, dk, dv;
-};
-
-template <typename T, int R>
-__global__ void __launch_bounds__(256) retention_kernel(RetArgs g) {
-  extern __shared__ float ret_lds[];
-  const int s = blockIdx.x, h = blockIdx.y;
-  const int tid = threadIdx.x, cols = blockDim.x / R;
-  const int cl = tid / R, r = tid % R;
-  const int col0 = blockIdx.z * cols, j = col0 + cl;
-  const int r0 = g.seq_rows ? g.seq_rows[s] : s, r1 = g.seq_rows ? g.seq_rows[s + 1] : s + 1;
-  if (r1 <= r0 || r0 < 0 || r1 > g.T) return;
-  const bool colok = j < g.dv;
-  const int slot = g.slots[s];
-  const int64_t ow = (int64_t)g.H * g.dv;
-  if (slot < 0 || slot >= g.n_slots) {  // a padding row: zeros out, no state touched
-    for (int t = r0; t < r1; ++t)
-      if (r == 0 && colok) g.out[(int64_t)t * ow + h * g.dv + j] = 0.f;
-    return;
-  }
-  float* qs_ = ret_lds;
-  float* ks_ = qs_ + kTok * g.dk;
-  float* vs_ = ks_ + kTok * g.dk;
-  float* sp = g.state + (((int64_t)slot * g.H + h) * g.dv + (colok ? j : 0)) * g.dk;
-  const bool fresh = g.pos[r0] == 0;
-  float S[kRows];
-#pragma unroll
-  for (int ii = 0; ii < kRows; ++ii) {
-    const int i = r + R * ii;
-    S[ii] = (!fresh && colok && i < g.dk) ? sp[i] : 0.f;
-  }
-  const float dec = g.decay[h];
-  const T* q = (const T*)g.q;
-  const T* k = (const T*)g.k;
-  const T* v = (const T*)g.v;
-  for (int t0 = r0; t0 < r1; t0 += kTok) {
-    const int nt = r1 - t0 < kTok ? r1 - t0 : kTok;
-    __syncthreads();  // the previous block's reads are done
-    for (int e = tid; e < nt * g.dk; e += blockDim.x) {
-      const int tt = e / g.dk, i = e - tt * g.dk;
-      qs_[e] = ldf<T>(q, (int64_t)(t0 + tt) * g.qs + h * g.dk + i);
-      ks_[e] = ldf<T>(k, (int64_t)(t0 + tt) * g.ks + h * g.dk + i) * g.k_scale;
-    }
-    for (int e = tid; e < nt * cols; e += blockDim.x) {
-      const int tt = e / cols, c = e - tt * cols;
-      vs_[e] = col0 + c < g.dv ? ldf<T>(v, (int64_t)(t0 + tt) * g.vs + h * g.dv + col0 + c) : 0.f;
-    }
-    __syncthreads();
-    for (int tt = 0; tt < nt; ++tt) {
-      const float vj = vs_[tt * cols + cl];
-      const float* qt = qs_ + tt * g.dk;
-      const float* kt = ks_ + tt * g.dk;
-      float acc = 0.f;
-#pragma unroll
-      for (int ii = 0; ii < kRows; ++ii) {
-        const int i = r + R * ii;
-        if (i < g.dk) {
-          S[ii] = dec * S[ii] + kt[i] * vj;
-          acc += qt[i] * S[ii];
-        }
-      }
-      acc = group_sum<R>(acc);
-      if (r == 0 && colok) g.out[(int64_t)(t0 + tt) * ow + h * g.dv + j] = acc;
-    }
-  }
-  if (colok) {
-#pragma unroll
-    for (int ii = 0; ii < kRows; ++ii) {
-      const int i = r + R * ii;
-      if (i < g.dk) sp[i] = S[ii];
-    }
-  }
-}
-
-// The same for key widths dk = 16 R and 16-byte aligned operands: nothing in the token loop is
-// conditional.  Lane r of a column's group owns the four row quads 4 (r + R qd) .. + 3, qd < 4, so
-// a group's 128-bit LDS reads of a q or k row are neighbouring chunks and the state is read and
-// written as 16-byte runs.  The next block's eight tokens (q, k of the head, v of the workgroup's
-// columns) are fetched into registers as 16-byte chunks while the current block's chain runs.
-typedef uint32_t ret_u32x4 __attribute__((ext_vector_type(4)));
-
-template <typename T> __device__ __forceinline__ void chunk_to_f32(const ret_u32x4& c, float* o);
-template <> __device__ __forceinline__ void chunk_to_f32<bf16_t>(const ret_u32x4& c, float* o) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) o[2 * i] = bf16lo(c[i]), o[2 * i + 1] = bf16hi(c[i]);
-}
-template <> __device__ __forceinline__ void chunk_to_f32<float>(const ret_u32x4& c, float* o) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) o[i] = __uint_as_float(c[i]);
-}
-
-template <typename T, int R>
-__global__ void __launch_bounds__(256) retention_fast_kernel(RetArgs g) {
-  constexpr int dk = 16 * R, cols = 256 / R, VEC = 16 / (int)sizeof(T);
-  constexpr int QC = dk / VEC, VC = cols / VEC;          // chunks per token row
-  constexpr int QK_CH = kTok * QC, V_CH = kTok * VC, N_CH = 2 * QK_CH + V_CH;
-  constexpr int PER = (N_CH + 255) / 256;
-  __shared__ __attribute__((aligned(16))) float qs_[kTok * dk];
-  __shared__ __attribute__((aligned(16))) float ks_[kTok * dk];
-  __shared__ __attribute__((aligned(16))) float vs_[kTok * cols];
-  const int s = blockIdx.x, h = blockIdx.y;
-  const int tid = threadIdx.x, cl = tid / R, r = tid % R;
-  const int col0 = blockIdx.z * cols, j = col0 + cl;
-  const int r0 = g.seq_rows ? g.seq_rows[s] : s, r1 = g.seq_rows ? g.seq_rows[s + 1] : s + 1;
-  if (r1 <= r0 || r0 < 0 || r1 > g.T) return;
-  const int slot = g.slots[s];
-  const int64_t ow = (int64_t)g.H * g.dv;
-  if (slot < 0 || slot >= g.n_slots) {  // a padding row: zeros out, no state touched
-    for (int t = r0; t < r1; ++t)
-      if (r == 0) g.out[(int64_t)t * ow + h * g.dv + j] = 0.f;
-    return;
-  }
-  float* sp = g.state + (((int64_t)slot * g.H + h) * g.dv + j) * dk;
-  const bool fresh = g.pos[r0] == 0;
-  float S[16];
-#pragma unroll
-  for (int qd = 0; qd < 4; ++qd) {
-    const f32x4 v4 = fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 4 * (r + R * qd));
-#pragma unroll
-    for (int e = 0; e < 4; ++e) S[4 * qd + e] = v4[e];
-  }
-  const float dec = g.decay[h];
-  const T* q = (const T*)g.q + (int64_t)h * dk;
-  const T* k = (const T*)g.k + (int64_t)h * dk;
-  const T* v = (const T*)g.v + (int64_t)h * g.dv + col0;
-  ret_u32x4 pf[PER];
-  auto fetch = [&](int t0) {
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int c = tid + i * 256;
-      const T* src = nullptr;
-      if (c < QK_CH) {
-        const int tt = c / QC;
-        if (t0 + tt < r1) src = q + (int64_t)(t0 + tt) * g.qs + (c % QC) * VEC;
-      } else if (c < 2 * QK_CH) {
-        const int c2 = c - QK_CH, tt = c2 / QC;
-        if (t0 + tt < r1) src = k + (int64_t)(t0 + tt) * g.ks + (c2 % QC) * VEC;
-      } else if (c < N_CH) {
-        const int c2 = c - 2 * QK_CH, tt = c2 / VC;
-        if (t0 + tt < r1) src = v + (int64_t)(t0 + tt) * g.vs + (c2 % VC) * VEC;
-      }
-      pf[i] = src ? *reinterpret_cast<const ret_u32x4*>(src) : ret_u32x4{0u, 0u, 0u, 0u};
-    }
-  };
-  auto commit = [&]() {
-#pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int c = tid + i * 256;
-      float f[VEC];
-      chunk_to_f32<T>(pf[i], f);
-      float* dst = nullptr;
-      if (c < QK_CH) {
-        dst = qs_ + c * VEC;
-      } else if (c < 2 * QK_CH) {
-        dst = ks_ + (c - QK_CH) * VEC;
-#pragma unroll
-        for (int e = 0; e < VEC; ++e) f[e] *= g.k_scale;
-      } else if (c < N_CH) {
-        dst = vs_ + (c - 2 * QK_CH) * VEC;
-      }
-      if (dst) {
-#pragma unroll
-        for (int e = 0; e < VEC; e += 4) *reinterpret_cast<f32x4*>(dst + e) = f32x4{f[e], f[e + 1], f[e + 2], f[e + 3]};
-      }
-    }
-  };
-  fetch(r0);
-  for (int t0 = r0; t0 < r1; t0 += kTok) {
-    const int nt = r1 - t0 < kTok ? r1 - t0 : kTok;
-    __syncthreads();  // the previous block's reads are done
-    commit();
-    __syncthreads();
-    if (t0 + kTok < r1) fetch(t0 + kTok);
-    for (int tt = 0; tt < nt; ++tt) {
-      const float vj = vs_[tt * cols + cl];
-      float acc = 0.f;
-#pragma unroll
-      for (int qd = 0; qd < 4; ++qd) {
-        const f32x4 kk = *reinterpret_cast<const f32x4*>(ks_ + tt * dk + 4 * (r + R * qd));
-        const f32x4 qq = *reinterpret_cast<const f32x4*>(qs_ + tt * dk + 4 * (r + R * qd));
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          S[4 * qd + e] = dec * S[4 * qd + e] + kk[e] * vj;
-          acc += qq[e] * S[4 * qd + e];
-        }
-      }
-      acc = group_sum<R>(acc);
-      if (r == 0) g.out[(int64_t)(t0 + tt) * ow + h * g.dv + j] = acc;
-    }
-  }
-#pragma unroll
-  for (int qd = 0; qd < 4; ++qd)
-    *reinterpret_cast<f32x4*>(sp + 4 * (r + R * qd)) = f32x4{S[4 * qd], S[4 * qd + 1], S[4 * qd + 2], S[4 * qd + 3]};
-}
-
-// whether the unconditional kernel serves the launch: dk = 16 R exactly, whole column blocks,
-// 16-byte aligned rows and sections
-template <typename T, int R>
-bool retention_fast_ok(const RetArgs& g) {
-  constexpr int VEC = 16 / (int)sizeof(T), cols = 256 / R;
-  auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-  return g.dk == 16 * R && g.dv % cols == 0 && cols % VEC == 0 && g.qs % VEC == 0 && g.ks % VEC == 0 &&
-         g.vs % VEC == 0 && al(g.q) && al(g.k) && al(g.v) && al(g.state);
-}
-
-template <typename T, int R>
-void launch_retention(const RetArgs& g, int n_seq, hipStream_t st) {
-  if (retention_fast_ok<T, R>(g)) {
-    hipLaunchKernelGGL((retention_fast_kernel<T, R>), dim3(n_seq, g.H, g.dv / (256 / R)), dim3(256), 0, st, g);
-    return;
-  }
-
-  int nt = (R * g.dv + 63) / 64 * 64;
-  nt = nt > 256 ? 256 : nt;
-  const int cols = nt / R;
-  const size_t lds = (size_t)(2 * kTok * g.dk + kTok * cols) * sizeof(float);
-  hipLaunchKernelGGL((retention_kernel<T, R>), dim3(n_seq, g.H, (g.dv + cols - 1) / cols), dim3(nt), lds, st, g);
-}
-
-// ---------------------------------------------------------------------------
 // Short causal convolution over time on the leading C = n_q d + n_k (d + dv)
-// columns of a fused projection, then rotary positions on the first 2 * half
+// columns of a fused projection (plus a bias and silu where given), then rotary positions on the first 2 * half
 // columns of every q and k head (column i paired with i + half), q to its own
 // tensor, k and v into the paged caches.  y_t = sum_j cw[j][c] u_(t - taps + 1 + j);
 // u at positions before the step's first row of the sequence comes from the
@@ -569,6 +306,8 @@ struct ConvArgs {
   const void* x;
   int64_t xs;
   const float* cw;  // [taps, C] (tap-major: a run of channels shares a load)
+  const float* cb;  // [C] bias or null
+  int silu;         // silu after the convolution (in front of the rotation)
   int taps;
   const void* tail;  // [slots, taps - 1, C]
   int n_slots;
@@ -599,7 +338,7 @@ __global__ void __launch_bounds__(256) conv_rope_cache_kernel(ConvArgs g) {
   const T* x = (const T*)g.x;
   const T* tail = (const T*)g.tail + (int64_t)(live ? slot : 0) * m * C;
   auto conv = [&](int c) -> float {
-    float y = 0.f;
+    float y = g.cb ? g.cb[c] : 0.f;
     for (int jj = 0; jj < g.taps; ++jj) {
       const int64_t qp = p - m + jj;
       float u = 0.f;
@@ -607,7 +346,7 @@ __global__ void __launch_bounds__(256) conv_rope_cache_kernel(ConvArgs g) {
       else if (qp >= 0) u = ldf<T>(tail, (qp - p0 + m) * C + c);
       y += g.cw[(int64_t)jj * C + c] * u;
     }
-    return y;
+    return g.silu ? y * sigmoidf_(y) : y;
   };
   // the row's angles: one cosine and sine per rotated pair, shared by all heads
   extern __shared__ float cs_sn[];  // [half] cosines, [half] sines
@@ -637,30 +376,6 @@ __global__ void __launch_bounds__(256) conv_rope_cache_kernel(ConvArgs g) {
 // 4 fp32): a thread takes a run of the low rotary half together with its partner run of the
 // high half, so every channel is convolved once and every angle evaluated once.  Needs d, dv,
 // half, the row stride and the cache widths to be multiples of V, and 16-byte aligned bases.
-template <typename T, int V> struct VecIO;
-template <> struct VecIO<bf16_t, 8> {
-  __device__ static __forceinline__ void ld(const bf16_t* p, float* o) {
-    const u16x8 a = *reinterpret_cast<const u16x8*>(p);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) o[2 * i] = bf16lo(a.w[i]), o[2 * i + 1] = bf16hi(a.w[i]);
-  }
-  __device__ static __forceinline__ void st(bf16_t* p, const float* v) {
-    u16x8 a;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) a.w[i] = pack_bf16x2(v[2 * i], v[2 * i + 1]);
-    *reinterpret_cast<u16x8*>(p) = a;
-  }
-};
-template <> struct VecIO<float, 4> {
-  __device__ static __forceinline__ void ld(const float* p, float* o) {
-    const f32x4 a = *reinterpret_cast<const f32x4*>(p);
-    o[0] = a[0], o[1] = a[1], o[2] = a[2], o[3] = a[3];
-  }
-  __device__ static __forceinline__ void st(float* p, const float* v) {
-    *reinterpret_cast<f32x4*>(p) = f32x4{v[0], v[1], v[2], v[3]};
-  }
-};
-
 // A workgroup takes kConvRows consecutive rows of the step (they may belong to different
 // sequences); the taps loop is outermost, so a thread loads a tap's weights once for all its rows.
 constexpr int kConvRows = 4;
@@ -720,9 +435,11 @@ __global__ void __launch_bounds__(128) conv_rope_cache_vec_kernel(ConvArgs g) {
     }
     float y[kConvRows][V], z[kConvRows][V];
 #pragma unroll
-    for (int r = 0; r < kConvRows; ++r)
+    for (int i = 0; i < V; ++i) {
+      const float b = g.cb ? g.cb[c + i] : 0.f, b2 = g.cb && pair ? g.cb[c + g.half + i] : 0.f;
 #pragma unroll
-      for (int i = 0; i < V; ++i) y[r][i] = z[r][i] = 0.f;
+      for (int r = 0; r < kConvRows; ++r) y[r][i] = live[r] ? b : 0.f, z[r][i] = live[r] ? b2 : 0.f;
+    }
     for (int jj = 0; jj < g.taps; ++jj) {
       float w[V], w2[V];
       const float* wp = g.cw + (int64_t)jj * C + c;
@@ -751,6 +468,13 @@ __global__ void __launch_bounds__(128) conv_rope_cache_vec_kernel(ConvArgs g) {
     }
 #pragma unroll
     for (int r = 0; r < kConvRows; ++r) {
+      if (g.silu) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) {
+          y[r][i] *= sigmoidf_(y[r][i]);
+          if (pair) z[r][i] *= sigmoidf_(z[r][i]);
+        }
+      }
       if (pair) {
         float lo[V], hi[V];
         const float* cs = cs_sn + 2 * r * g.half + e;
@@ -865,16 +589,80 @@ __global__ void __launch_bounds__(256) head_norm_gate_kernel(T* __restrict__ out
   }
 }
 
-}  // namespace
-
-#define DISPATCH_T(f32, ...)          \
-  if (f32) {                          \
-    using T = float;                  \
-    __VA_ARGS__;                      \
-  } else {                            \
-    using T = bf16_t;                 \
-    __VA_ARGS__;                      \
+// out = y silu(z), divided by the root mean square of its group (n equal groups of the row, eps inside the
+// root), times w: the gate enters in front of the norm.  One workgroup per (row, group); a thread keeps its
+// elements (V neighbours at a time, up to kGnKeep times) in registers between the mean square and the result.
+constexpr int kGnKeep = 4;
+template <typename T, int V, int NT>
+__global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out, int64_t os,
+                                                             const float* __restrict__ y, const T* __restrict__ z,
+                                                             int64_t zs, const float* __restrict__ w, int n_groups,
+                                                             int n, float eps) {
+  __shared__ float red[16];
+  const int64_t row = blockIdx.x / n_groups;
+  const int c0 = (int)(blockIdx.x - row * n_groups) * n;
+  const float* yp = y + row * (int64_t)n_groups * n + c0;
+  const T* zp = z + row * zs + c0;
+  auto load = [&](int e, float* x) {
+    float a[V], b[V];
+    if constexpr (V == 1) {
+      a[0] = yp[e];
+      b[0] = ldf<T>(zp, e);
+    } else {
+#pragma unroll
+      for (int i = 0; i < V; i += 4) VecIO<float, 4>::ld(yp + e + i, a + i);
+      VecIO<T, V>::ld(zp + e, b);
+    }
+#pragma unroll
+    for (int i = 0; i < V; ++i) x[i] = a[i] * b[i] * sigmoidf_(b[i]);
+  };
+  float x[kGnKeep][V], ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < kGnKeep; ++k) {
+    const int e = (threadIdx.x + NT * k) * V;
+#pragma unroll
+    for (int i = 0; i < V; ++i) x[k][i] = 0.f;
+    if (e < n) load(e, x[k]);
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss += x[k][i] * x[k][i];
   }
+  for (int e = (threadIdx.x + NT * kGnKeep) * V; e < n; e += NT * V) {
+    float t[V];
+    load(e, t);
+#pragma unroll
+    for (int i = 0; i < V; ++i) ss += t[i] * t[i];
+  }
+  const float inv = rsqrtf(block_reduce_sum(ss, red) / (float)n + eps);
+  auto put = [&](int e, const float* xv) {
+    float o[V];
+#pragma unroll
+    for (int i = 0; i < V; ++i) o[i] = xv[i] * inv * w[c0 + e + i];
+    if constexpr (V == 1) stf<T>(out, row * os + c0 + e, o[0]);
+    else VecIO<T, V>::st(out + row * os + c0 + e, o);
+  };
+#pragma unroll
+  for (int k = 0; k < kGnKeep; ++k)
+    if ((int)(threadIdx.x + NT * k) * V < n) put((threadIdx.x + NT * k) * V, x[k]);
+  for (int e = (threadIdx.x + NT * kGnKeep) * V; e < n; e += NT * V) {
+    float t[V];
+    load(e, t);
+    put(e, t);
+  }
+}
+
+template <typename T, int V>
+void launch_gate_group_norm(void* out, int64_t os, const float* y, const void* z, int64_t zs, const float* w, int rows,
+                            int n_groups, int n, float eps, hipStream_t st) {
+  const dim3 grid((unsigned)((int64_t)rows * n_groups));
+  if (n > 64 * V)
+    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 256>), grid, dim3(256), 0, st, (T*)out, os, y, (const T*)z, zs, w,
+                       n_groups, n, eps);
+  else
+    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 64>), grid, dim3(64), 0, st, (T*)out, os, y, (const T*)z, zs, w,
+                       n_groups, n, eps);
+}
+
+}  // namespace
 
 extern "C" {
 
@@ -900,27 +688,8 @@ int dxm_delta_rule(float* out, float* state, int n_slots, float* prep, const voi
   return 0;
 }
 
-int dxm_retention(float* out, float* state, int n_slots, const void* q, int64_t qs, const void* k, int64_t ks,
-                  const void* v, int64_t vs, const float* decay, float k_scale, const int64_t* pos,
-                  const int* seq_rows, const int* slots, int n_seq, int T_, int H, int dk, int dv, int f32,
-                  hipStream_t st) {
-  if (n_seq <= 0 || T_ <= 0) return 0;
-  if (H < 1 || dk < 1 || dv < 1 || n_slots < 1 || H > 65535 || (int64_t)T_ * H * dv > 0x7fffffffffffLL) return 1;
-  if (dk > kRows * 16) return 2;  // wider keys need more lanes per column than instantiated
-  if (!out || !state || !pos || !slots || !decay || !q || !k || !v) return 3;
-  if (!seq_rows && n_seq != T_) return 4;
-  RetArgs g{out, state, q, k, v, qs, ks, vs, decay, k_scale, pos, seq_rows, slots, n_slots, T_, H, dk, dv};
-  const int need = (dk + kRows - 1) / kRows;
-  if (need <= 1) { DISPATCH_T(f32, (launch_retention<T, 1>(g, n_seq, st))); }
-  else if (need <= 2) { DISPATCH_T(f32, (launch_retention<T, 2>(g, n_seq, st))); }
-  else if (need <= 4) { DISPATCH_T(f32, (launch_retention<T, 4>(g, n_seq, st))); }
-  else if (need <= 8) { DISPATCH_T(f32, (launch_retention<T, 8>(g, n_seq, st))); }
-  else { DISPATCH_T(f32, (launch_retention<T, 16>(g, n_seq, st))); }
-  DX_CHECK_LAUNCH();
-  return 0;
-}
-
-int dxm_conv_rope_cache(void* q_out, const void* x, int64_t xs, const float* cw, int taps, const void* tail,
+int dxm_conv_rope_cache(void* q_out, const void* x, int64_t xs, const float* cw, const float* cb, int silu, int taps,
+                        const void* tail,
                         int n_slots, const int64_t* pos, const int64_t* kv_slots, const int* row_seq,
                         const int* seq_rows, const int* slots, int n_seq, int T_, int n_q, int n_k, int d, int dv,
                         const float* inv_freq, int half, void* kc, void* vc, int f32, hipStream_t st) {
@@ -929,7 +698,7 @@ int dxm_conv_rope_cache(void* q_out, const void* x, int64_t xs, const float* cw,
   if ((half && !inv_freq) || (n_k && (!kc || !vc)) || (taps > 1 && !tail) || !cw || !pos || !kv_slots || !slots)
     return 2;
   if ((row_seq == nullptr) != (seq_rows == nullptr) || (!row_seq && n_seq != T_)) return 3;
-  ConvArgs g{q_out, x, xs, cw, taps, tail, n_slots, pos, kv_slots, row_seq, seq_rows, slots, n_seq, T_,
+  ConvArgs g{q_out, x, xs, cw, cb, silu, taps, tail, n_slots, pos, kv_slots, row_seq, seq_rows, slots, n_seq, T_,
              n_q, n_k, d, dv, inv_freq, half, kc, vc};
   const int V = f32 ? 4 : 8, esz = f32 ? 4 : 2;
   auto al = [&](const void* ptr) { return (uintptr_t)ptr % 16 == 0; };
@@ -969,6 +738,22 @@ int dxm_head_norm_gate(void* out, const float* o, const float* w, const void* ga
     DISPATCH_T(f32, hipLaunchKernelGGL((head_norm_gate_kernel<T, 1>), grid, dim3(256), 0, st, (T*)out, o, w,
                                        (const T*)gate, gs, n_vec, H, dv, eps, gate_act));
   }
+  DX_CHECK_LAUNCH();
+  return 0;
+}
+
+int dxm_gate_group_norm(void* out, int64_t os, const float* y, const void* z, int64_t zs, const float* w, int rows,
+                        int n_groups, int n, float eps, int f32, hipStream_t st) {
+  if (rows <= 0) return 0;
+  if (n_groups < 1 || n < 1 || (int64_t)rows * n_groups > 0x7fffffff) return 1;
+  if (!out || !y || !z || !w) return 2;
+  const int V = f32 ? 4 : 8;
+  auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  const bool vec = n % V == 0 && os % V == 0 && zs % V == 0 && al(out) && al(y) && al(z);
+  if (vec && f32) launch_gate_group_norm<float, 4>(out, os, y, z, zs, w, rows, n_groups, n, eps, st);
+  else if (vec) launch_gate_group_norm<bf16_t, 8>(out, os, y, z, zs, w, rows, n_groups, n, eps, st);
+  else if (f32) launch_gate_group_norm<float, 1>(out, os, y, z, zs, w, rows, n_groups, n, eps, st);
+  else launch_gate_group_norm<bf16_t, 1>(out, os, y, z, zs, w, rows, n_groups, n, eps, st);
   DX_CHECK_LAUNCH();
   return 0;
 }

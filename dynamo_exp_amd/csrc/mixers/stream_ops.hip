@@ -469,7 +469,7 @@ template <typename T, int V>
 __global__ void __launch_bounds__(kThreads) act_mul_kernel(T* __restrict__ out, const T* __restrict__ gate,
                                                            int64_t g_stride, const T* __restrict__ up,
                                                            int64_t u_stride, int F, int64_t out_stride, int act,
-                                                           float limit, float alpha) {
+                                                           float limit, float alpha, float post) {
   const int64_t r = blockIdx.y;
   for (int c = (blockIdx.x * kThreads + threadIdx.x) * V; c < F; c += gridDim.x * kThreads * V) {
     float g[V], u[V], o[V];
@@ -483,6 +483,7 @@ __global__ void __launch_bounds__(kThreads) act_mul_kernel(T* __restrict__ out, 
       } else {
         o[e] = act_fn(g[e], act) * (up ? u[e] : 1.f);
       }
+      o[e] *= post;
     }
     stv<T, V>(out + r * out_stride + c, o);
   }
@@ -674,7 +675,7 @@ int dxm_residual_step(float* X, const void* a, int64_t a_stride, const void* b, 
 }
 
 int dxm_act_mul(void* out, const void* gate, int64_t g_stride, const void* up, int64_t u_stride, int rows, int F,
-                int64_t out_stride, int act, float limit, float alpha, int f32, hipStream_t st) {
+                int64_t out_stride, int act, float limit, float alpha, float post, int f32, hipStream_t st) {
   if (rows <= 0 || F <= 0) return 0;
   if (act < 0 || act > 6 || (act == 6 && (!up || !(limit > 0.f)))) return 1;
   const int esz = f32 ? 4 : 2;
@@ -689,12 +690,12 @@ int dxm_act_mul(void* out, const void* gate, int64_t g_stride, const void* up, i
       DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, 4>), dim3(gx, nr), dim3(kThreads), 0, st,
                                          (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,
                                          up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act,
-                                         limit, alpha));
+                                         limit, alpha, post));
     } else {
       DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, 1>), dim3(gx, nr), dim3(kThreads), 0, st,
                                          (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,
                                          up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act,
-                                         limit, alpha));
+                                         limit, alpha, post));
     }
   }
   DX_CHECK_LAUNCH();

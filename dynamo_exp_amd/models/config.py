@@ -137,7 +137,8 @@ class LayeredConfig:
     each naming its mixer type, the mixer's sizes and constants, and its
     feed-forward (or none), with an optional `loop` that repeats a span of
     layers with shared weights and per-pass caches, and optional parallel
-    residual streams.  Every size and constant comes from the file; the
+    residual streams.  A layer entry may name another layer whose weights it
+    runs (`weights_of`).  Every size and constant comes from the file; the
     engine-facing fields below mirror ModelConfig's."""
 
     name: str = "layered"
@@ -171,6 +172,20 @@ class LayeredConfig:
             raise ValueError(f"bad loop {lp!r} for {n} layers")
         return list(range(a)) + list(range(a, b)) * times + list(range(b, n))
 
+    def weight_layers(self) -> list[int]:
+        """Per layer, the layer whose tensors it runs: itself, or the one its
+        `weights_of` names."""
+        out = []
+        for i in range(len(self.layers)):
+            j, seen = i, set()
+            while self.layers[j].get("weights_of") is not None:
+                seen.add(j)
+                j = int(self.layers[j]["weights_of"])
+                if not 0 <= j < len(self.layers) or j in seen:
+                    raise ValueError(f"layer {i}: weights_of leads to no layer with weights of its own")
+            out.append(j)
+        return out
+
     @property
     def num_hidden_layers(self) -> int:
         return len(self.layer_runs())
@@ -184,6 +199,8 @@ class LayeredConfig:
             return n + self._nefivik_params()
         if self.architecture == "Sobivik":
             return n - W + 1 + self._sobivik_params()
+        if self.architecture == "Povurax":
+            return n + self._povurax_params()
         for L in self.layers:
             m, t = L["mixer"], L["type"]
             H, d, dv = m["heads"], m["dim"], m["vdim"]
@@ -262,6 +279,28 @@ class LayeredConfig:
                 n += 3 * W * L["mlp"]["ff"]
         return n
 
+    def _povurax_params(self) -> int:
+        W, n = self.hidden_size, 0
+        for i, L in enumerate(self.layers):
+            m, mlp = L["mixer"], L.get("mlp")
+            if L.get("weights_of") is not None:
+                continue
+            n += W
+            if L["type"] == "parallel":
+                a, b = m["left"], m["right"]
+                H, G, d, dv = a["heads"], a["kv_heads"], a["dim"], a["vdim"]
+                n += (H + G) * d * (W + 1) + G * dv * W + 2 * H * dv * W
+                inner, bc = b["heads"] * b["vdim"], 2 * b["groups"] * b["state"]
+                n += (2 * inner + bc + b["heads"]) * W + (inner + bc) * (int(b["conv"]) + 1) + 3 * b["heads"]
+                n += inner + W * inner
+            else:
+                H, d, dv = m["heads"], m["dim"], m["vdim"]
+                lo = int(m.get("decay_rank") or min(16, W))
+                n += (2 * H * d + 3 * H * dv) * W + dv + lo * (W + H * d) + H * d
+            if mlp:
+                n += W + 3 * W * mlp["ff"]
+        return n
+
     def to_dict(self) -> dict:
         return dataclasses.asdict(self)
 
@@ -301,7 +340,7 @@ class LayeredConfig:
 
 
 # config.json `architecture` values served by LayeredConfig
-LAYERED_ARCHITECTURES = ("Bekulix", "Bolinex", "Nefivik", "Sobivik")
+LAYERED_ARCHITECTURES = ("Bekulix", "Bolinex", "Nefivik", "Sobivik", "Povurax")
 
 
 def _bekulix_preset(name, W, ff, n_layers, heads, kv_heads, d, rank, window, chunk, vocab=32000, streams=4):
@@ -391,6 +430,30 @@ def _sobivik_preset(name, W, ff, n_layers, heads, kv_heads, d, rank, q_rank, rot
                          rms_norm_eps=1e-5, embedding_scale=float(W) ** 0.5, logit_scale=0.25, canon={"taps": taps})
 
 
+def _povurax_preset(name, W, ff, n_layers, heads, kv_heads, d, ssm_heads, ssm_dim, state, groups, vocab=32000, conv=4,
+                    rot_dims=None, share=True):
+    """A Povurax stack at a real model's layer sizes: layers with attention
+    and a state-space mixer side by side and a clamped gated feed-forward, each
+    followed by a gated linear attention layer without one; with `share`, every
+    parallel layer after the first runs the first one's weights."""
+    par = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5,
+                    "rot": {"base": 500000.0, "dims": rot_dims or d}}, "left_scale": 0.5,
+           "right": {"heads": ssm_heads, "vdim": ssm_dim, "state": state, "groups": groups, "norm_groups": groups,
+                     "conv": conv}, "right_scale": 0.75}
+    gla = {"heads": heads, "dim": d, "vdim": d, "tau": 16.0}
+    layers = []
+    for i in range(n_layers):
+        if i % 2:
+            layers.append({"type": "gla", "mixer": dict(gla), "mlp": None})
+            continue
+        layers.append({"type": "parallel", "mixer": {**par, "left": dict(par["left"]), "right": dict(par["right"])},
+                       "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
+        if share and i:
+            layers[-1]["weights_of"] = 0
+    return LayeredConfig(name=name, architecture="Povurax", vocab_size=vocab, hidden_size=W, layers=layers,
+                         rms_norm_eps=1e-5, embedding_scale=float(W) ** 0.5)
+
+
 # CLIP ViT-L/14 at 336 px, the LLaVA-1.5 vision tower; features from the
 # second-to-last layer, CLS dropped, projected by a 2-layer GELU MLP
 CLIP_L_336 = {
@@ -469,6 +532,14 @@ PRESETS["sobivik-tiny"] = _sobivik_preset("sobivik-tiny", 192, 384, 6, 4, 2, 32,
 # Llama-3-8B's layer sizes (width 4096, ff 14336, 32 x 128 heads, 8 KV heads), 9 layers; latent rank 192 + 64 rotated
 PRESETS["sobivik-8b-shapes"] = _sobivik_preset("sobivik-8b-shapes", 4096, 14336, 9, 32, 8, 128, 192, 1536, 64, 1024,
                                                64, vocab=128256)
+
+
+PRESETS["povurax-tiny"] = _povurax_preset("povurax-tiny", 192, 320, 5, 4, 2, 32, 5, 24, 16, 1, vocab=512, conv=3,
+                                          rot_dims=16)
+# Llama-3-8B's layer sizes (width 4096, ff 14336, 32 x 128 heads, 8 KV heads), 8 layers; state-space half of
+# 128 heads x 64 channels with 128 states
+PRESETS["povurax-8b-shapes"] = _povurax_preset("povurax-8b-shapes", 4096, 14336, 8, 32, 8, 128, 128, 64, 128, 8,
+                                               vocab=128256, share=False)
 
 
 def get_config(name_or_path: str) -> ModelConfig:

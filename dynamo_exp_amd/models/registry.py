@@ -42,6 +42,12 @@ def _sobivik():
     return SobivikForCausalLM
 
 
+def _povurax():
+    from .povurax import PovuraxForCausalLM
+
+    return PovuraxForCausalLM
+
+
 # architecture -> (class loader, activation dtypes the class has kernels for)
 MODEL_REGISTRY = {
     "LlamaForCausalLM": (_llama, ("bfloat16",)),
@@ -50,6 +56,7 @@ MODEL_REGISTRY = {
     "Bolinex": (_bolinex, ("bfloat16", "float32")),
     "Nefivik": (_nefivik, ("bfloat16", "float32")),
     "Sobivik": (_sobivik, ("bfloat16", "float32")),
+    "Povurax": (_povurax, ("bfloat16", "float32")),
 }
 
 

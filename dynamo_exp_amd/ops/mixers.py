@@ -293,10 +293,11 @@ def glu_act(gu: torch.Tensor, act: str = "relu", limit: float = 0.0, alpha: floa
 
 
 def act_mul(gate: torch.Tensor, up: torch.Tensor | None = None, act: str = "silu", limit: float = 0.0,
-            alpha: float = 1.0) -> torch.Tensor:
-    """act(gate) * up, [T, F] (up None: the activation alone).  gate and up may
+            alpha: float = 1.0, out: torch.Tensor | None = None, scale: float = 1.0) -> torch.Tensor:
+    """act(gate) * up * scale, [T, F] (up None: the activation alone).  gate and up may
     be column sections of wider tensors (contiguous rows, any row stride), e.g.
-    a gate that is part of a fused projection's output.
+    a gate that is part of a fused projection's output; so may `out`, the place
+    of the result (e.g. one part of the next projection's input).
     'swiglu_clamp' is the clamped gated unit: with g = min(gate, limit) and
     u = clamp(up, -limit, limit) the result is g * sigmoid(alpha * g) * (u + 1)."""
     T, F = gate.shape
@@ -307,15 +308,21 @@ def act_mul(gate: torch.Tensor, up: torch.Tensor | None = None, act: str = "silu
         raise ValueError("act_mul: [T, F] sections with contiguous rows and one dtype")
     if act == "swiglu_clamp" and (up is None or not limit > 0):
         raise ValueError("act_mul: the clamped gated unit needs `up` and a positive limit")
+    if out is not None and (out.shape != gate.shape or out.stride(1) != 1 or out.dtype != gate.dtype):
+        raise ValueError("act_mul: out is [T, F] of gate's dtype with contiguous rows")
     if not gate.is_cuda:
         if act == "swiglu_clamp":
             g, u = gate.float().clamp(max=limit), up.float().clamp(-limit, limit)
-            return (g * torch.sigmoid(alpha * g) * (u + 1.0)).to(gate.dtype)
-        o = _act(gate.float(), act)
-        return (o * up.float() if up is not None else o).to(gate.dtype)
-    out = torch.empty((T, F), dtype=gate.dtype, device=gate.device)
+            o = g * torch.sigmoid(alpha * g) * (u + 1.0)
+        else:
+            o = _act(gate.float(), act)
+            o = o * up.float() if up is not None else o
+        o = (o * scale).to(gate.dtype)
+        return o if out is None else out.copy_(o)
+    if out is None:
+        out = torch.empty((T, F), dtype=gate.dtype, device=gate.device)
     _m().act_mul(out.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(up), up.stride(0) if up is not None else 0, T, F,
-                 F, ACTS[act], float(limit), float(alpha), _f32(gate), _stream())
+                 out.stride(0), ACTS[act], float(limit), float(alpha), float(scale), _f32(gate), _stream())
     return out
 
 
@@ -378,6 +385,54 @@ def headprep_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor
                         _ptr(q_w), _ptr(k_w), float(eps), coef, every, kc.data_ptr(), _ptr(vc) if v_mode else 0,
                         v_mode, v_off, v_w, _ptr(v_first), v_first.stride(0) if v_first is not None else 0,
                         float(v_lambda), _f32(x), _stream())
+
+
+def norm_rope_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n_q: int, n_k: int, d: int, v_w: int,
+                    q_w: torch.Tensor | None, k_w: torch.Tensor | None, eps: float, inv_freq: torch.Tensor | None,
+                    kc: torch.Tensor, vc: torch.Tensor) -> None:
+    """Per row of a fused projection output x = [q (n_q d) | k (n_k d) | v (v_w) | ...]:
+    q and k are each divided by the root mean square of their whole section
+    (all heads together), times q_w [n_q d] / k_w [n_k d] (None: no norm); then
+    in every q and k head columns (2i, 2i + 1), i < len(inv_freq), are rotated by
+    the angle position * inv_freq[i], the rest pass unchanged.  q in place, k and
+    v into the paged caches kc [slots, n_k d], vc [slots, v_w] (rows with slot < 0
+    cache nothing)."""
+    T = x.shape[0]
+    nq, nk = n_q * d, n_k * d
+    half = 0 if inv_freq is None else inv_freq.numel()
+    for t, n in ((q_w, "q_w"), (k_w, "k_w"), (inv_freq, "inv_freq")):
+        _fp32_param(t, n)
+    if x.stride(-1) != 1 or x.shape[1] < nq + nk + v_w or 2 * half > d or (q_w is not None and q_w.numel() != nq) or \
+            (k_w is not None and k_w.numel() != nk):
+        raise ValueError("norm_rope_cache: sections or weights do not fit the row")
+    if kc.shape[-1] != nk or vc.shape[-1] != v_w or kc.dtype != x.dtype or vc.dtype != x.dtype or \
+            not kc.is_contiguous() or not vc.is_contiguous():
+        raise ValueError("norm_rope_cache: cache row widths / dtype do not match the sections")
+    if not x.is_cuda:
+        ok = slots >= 0
+        ang = positions.to(torch.float32)[:, None] * inv_freq[None, :] if half else None
+
+        def prep(sec, w, n):
+            y = sec.to(torch.float32, copy=True)
+            if w is not None:
+                y = y * torch.rsqrt((y * y).mean(-1, keepdim=True) + eps) * w
+            y = y.reshape(T, n, d)
+            if half:
+                c, s = torch.cos(ang)[:, None, :], torch.sin(ang)[:, None, :]
+                u, v = y[..., 0:2 * half:2].clone(), y[..., 1:2 * half:2].clone()
+                y[..., 0:2 * half:2] = u * c - v * s
+                y[..., 1:2 * half:2] = v * c + u * s
+            return y.reshape(T, n * d).to(x.dtype)
+
+        kc[slots[ok]] = prep(x[:, nq:nq + nk], k_w, n_k)[ok]
+        vc[slots[ok]] = x[ok, nq + nk:nq + nk + v_w]
+        x[:, :nq] = prep(x[:, :nq], q_w, n_q)
+        return
+    if positions.dtype != torch.int64 or slots.dtype != torch.int64:
+        raise TypeError("positions and slots must be int64")
+    _m().norm_rope_cache(x.data_ptr(), x.stride(0), positions.data_ptr(), slots.data_ptr(), T, n_q, n_k, d, v_w,
+                         _ptr(q_w), _ptr(k_w), float(eps), _ptr(inv_freq), half, kc.data_ptr(), vc.data_ptr(), _f32(x),
+                         _stream())
 
 
 # ----------------------------------------------------------------- attention

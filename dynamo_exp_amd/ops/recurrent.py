@@ -1,8 +1,10 @@
 """Ops with per-sequence state: the generalized delta rule (a running matrix
-per head), retention (a running matrix with a fixed decay per head), short
-causal convolutions over time fused with rotary positions and the paged cache
-write, the query / key preparation of latent attention with a rotated key
-part, and the per-head unit-RMS + gate that follows a recurrent mixer.
+per head), linear recurrences (a running matrix whose decay is fixed per head:
+retention; a function of the token's step size: state-space duality; or one per
+key channel and token: gated linear attention), short causal convolutions over
+time fused with rotary positions and the paged cache write, the query / key
+preparation of latent attention with a rotated key part, and the norms + gates
+that follow a recurrent mixer.
 
 State lives in slots: state tensors are [slots, ...], the engine's KV manager
 hands a slot to every live request, and a step names the slot of each of its
@@ -13,7 +15,8 @@ step); within a sequence rows are consecutive positions.  A sequence whose
 first row of the step is at position 0 starts from zero state, whatever its
 slot held before, so slots need no clearing when they change hands.
 
-GPU tensors run the gfx950 kernels of ``_C_mixers`` (csrc/mixers/recurrent.hip);
+GPU tensors run the gfx950 kernels of ``_C_mixers`` (csrc/mixers/recurrent.hip,
+linear_scan.hip);
 CPU tensors run the PyTorch forms below.  Decays, removal rates, unit keys and
 the state are fp32 in every dtype.
 """
@@ -139,14 +142,16 @@ def latent_rope(qa: torch.Tensor, q: torch.Tensor, q_head: int, q_off: int, kv: 
 def conv_rope_cache(x: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor, positions: torch.Tensor,
                     kv_slots: torch.Tensor, row_seq: torch.Tensor | None, seq_rows: torch.Tensor | None,
                     state_slots: torch.Tensor, n_q: int, n_k: int, d: int, dv: int, inv_freq: torch.Tensor | None,
-                    kc: torch.Tensor | None, vc: torch.Tensor | None) -> torch.Tensor:
+                    kc: torch.Tensor | None, vc: torch.Tensor | None, bias: torch.Tensor | None = None,
+                    act: str | None = None) -> torch.Tensor:
     """Per row of a fused projection x = [q (n_q d) | k (n_k d) | v (n_k dv) | ...]:
     every channel c of the C = n_q d + n_k (d + dv) leading columns is
     convolved over time, y_t = sum_j conv_w[j, c] u_(t - taps + 1 + j) (conv_w
     [taps, C] fp32, tap-major: the transpose of a checkpoint's [C, taps]), where u
     at a position before the step's first row of the sequence comes from
     conv_state [slots, taps - 1, C] (the last taps - 1 projected rows the
-    sequence had before this step) and is zero before position 0.  Then the
+    sequence had before this step) and is zero before position 0; with bias
+    [C] (fp32) y_t += bias, and with act 'silu' y_t <- y_t sigmoid(y_t).  Then the
     first 2 len(inv_freq) columns of every q and k head are rotated by the
     angles position * inv_freq, column i paired with column i + len(inv_freq).
     Returns q [T, n_q d]; k and v go to the paged caches kc [slots, n_k d],
@@ -157,7 +162,10 @@ def conv_rope_cache(x: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Ten
     taps, C = conv_w.shape
     n_seq = state_slots.numel()
     _fp32_param(conv_w, "conv_w")
+    _fp32_param(bias, "bias")
     _fp32_param(inv_freq, "inv_freq")
+    if act not in (None, "silu") or (bias is not None and bias.numel() != C):
+        raise ValueError("conv_rope_cache: act is None or 'silu', bias one number per channel")
     _check_step(positions, seq_rows, state_slots)
     half = 0 if inv_freq is None else inv_freq.numel()
     if C != n_q * d + n_k * (d + dv) or x.shape[1] < C or x.stride(1) != 1 or 2 * half > d or taps < 1:
@@ -181,8 +189,12 @@ def conv_rope_cache(x: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Ten
                 if p0 - (taps - 1) + m < 0:
                     hist[m] = 0.0
             u = torch.cat([hist, x[r0:r1, :C].float()], 0)
+            if bias is not None:
+                y[r0:r1] += bias
             for j in range(taps):
                 y[r0:r1] += u[j:j + r1 - r0] * conv_w[j]
+        if act == "silu":
+            y = y * torch.sigmoid(y)
         qk = y[:, : (n_q + n_k) * d].reshape(T, n_q + n_k, d)
         if half:
             ang = positions.to(torch.float32)[:, None] * inv_freq[None, :]
@@ -200,7 +212,8 @@ def conv_rope_cache(x: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Ten
             ((row_seq is None) != (seq_rows is None)):
         raise TypeError("conv_rope_cache: int64 kv_slots, int32 row_seq together with seq_rows")
     q = torch.empty((T, n_q * d), dtype=x.dtype, device=x.device)
-    _m().conv_rope_cache(q.data_ptr(), x.data_ptr(), x.stride(0), conv_w.data_ptr(), taps, conv_state.data_ptr(),
+    _m().conv_rope_cache(q.data_ptr(), x.data_ptr(), x.stride(0), conv_w.data_ptr(), _ptr(bias),
+                         int(act == "silu"), taps, conv_state.data_ptr(),
                          conv_state.shape[0], positions.data_ptr(), kv_slots.data_ptr(), _ptr(row_seq), _ptr(seq_rows),
                          state_slots.data_ptr(), n_seq, T, n_q, n_k, d, dv, _ptr(inv_freq), half, _ptr(kc), _ptr(vc),
                          _f32(x), _stream())
@@ -302,6 +315,69 @@ def delta_rule(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, a: torch.Tenso
     return out
 
 
+SCAN_MODES = {"fixed": 0, "step": 1, "channel": 2}
+
+
+def _linear_scan(mode: str, q, k, v, state, positions, seq_rows, state_slots, n_heads: int, dk: int, dv: int,
+                 q_scale: float = 1.0, k_scale: float = 1.0, qk_heads: int | None = None, decay=None, gate=None,
+                 g_bias=None, rate=None, skip=None, tau: float = 1.0) -> torch.Tensor:
+    """S_t = D_t S_(t-1) + (k_scale k_t) (u_t v_t)^T,  o_t = S_t^T (q_scale q_t) + skip[h] v_t, with D_t and
+    u_t by mode (csrc/mixers/linear_scan.hip); head h reads q / k head h // (n_heads / qk_heads)."""
+    T, H, n_seq = q.shape[0], n_heads, state_slots.numel()
+    G = qk_heads or H
+    for t, n in ((decay, "decay"), (g_bias, "bias"), (rate, "rate"), (skip, "skip")):
+        _fp32_param(t, n)
+    _check_step(positions, seq_rows, state_slots)
+    if H % G:
+        raise ValueError(f"linear scan: {H} heads over {G} query / key heads")
+    gw = {"fixed": None, "step": H, "channel": H * dk}[mode]
+    for t, wd in ((q, G * dk), (k, G * dk), (v, H * dv)) + (((gate, gw),) if gw else ()):
+        if t.shape != (T, wd) or t.stride(1) != 1 or t.dtype != q.dtype:
+            raise ValueError("linear scan: q, k [T, heads dk], v [T, H dv] and the decay / step logits with contiguous "
+                             "rows, one dtype")
+    if state.shape[1:] != (H, dv, dk) or state.dtype != torch.float32 or not state.is_contiguous():
+        raise ValueError("linear scan: state is contiguous float32 [slots, H, dv, dk]")
+    for t, wd in ((decay, H), (rate, H), (skip, H), (g_bias, gw)):
+        if t is not None and t.numel() != wd:
+            raise ValueError("linear scan: one decay / rate / skip per head, one bias per logit")
+    if not q.is_cuda:
+        out = torch.zeros((T, H, dv), dtype=torch.float32)
+        qf = (q.float() * q_scale).view(T, G, dk).repeat_interleave(H // G, 1)
+        kf = (k.float() * k_scale).view(T, G, dk).repeat_interleave(H // G, 1)
+        vf = v.float().reshape(T, H, dv)
+        z = gate.float() + (g_bias if g_bias is not None else 0.0) if gw else None
+        uv = vf
+        if mode == "fixed":
+            D = decay[None, :, None].expand(T, H, 1)
+        elif mode == "step":
+            u = torch.nn.functional.softplus(z, threshold=1e4)
+            D, uv = torch.exp(-rate * u)[:, :, None], vf * u[:, :, None]
+        else:
+            D = torch.exp(torch.nn.functional.logsigmoid(z) / tau).view(T, H, dk)
+        b = _seq_bounds(seq_rows, n_seq)
+        for s in range(n_seq):
+            r0, r1 = b[s], b[s + 1]
+            sl = int(state_slots[s])
+            if sl < 0 or r1 <= r0:
+                continue
+            S = state[sl].transpose(1, 2).clone() if int(positions[r0]) > 0 else \
+                torch.zeros((H, dk, dv), dtype=torch.float32)
+            for t in range(r0, r1):
+                S = D[t][:, :, None] * S + kf[t][:, :, None] * uv[t][:, None, :]
+                out[t] = torch.einsum("hi,hij->hj", qf[t], S)
+                if skip is not None:
+                    out[t] += skip[:, None] * vf[t]
+            state[sl] = S.transpose(1, 2)
+        return out.view(T, H * dv)
+    out = torch.empty((T, H * dv), dtype=torch.float32, device=q.device)
+    _m().linear_scan(SCAN_MODES[mode], out.data_ptr(), state.data_ptr(), state.shape[0], q.data_ptr(), q.stride(0),
+                     k.data_ptr(), k.stride(0), v.data_ptr(), v.stride(0), float(q_scale), float(k_scale), H // G,
+                     _ptr(decay), _ptr(gate), gate.stride(0) if gate is not None else 0, _ptr(g_bias), _ptr(rate),
+                     _ptr(skip), 1.0 / float(tau), positions.data_ptr(), _ptr(seq_rows), state_slots.data_ptr(), n_seq, T,
+                     H, dk, dv, _f32(q), _stream())
+    return out
+
+
 def retention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, k_scale: float,
               state: torch.Tensor, positions: torch.Tensor, seq_rows: torch.Tensor | None, state_slots: torch.Tensor,
               n_heads: int, dk: int, dv: int) -> torch.Tensor:
@@ -313,38 +389,37 @@ def retention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Te
     q, k [T, H dk] and v [T, H dv] are column sections (contiguous rows, any
     row stride) of projection outputs; decay fp32 [H].  Returns o [T, H dv]
     fp32.  Everything but reading the inputs is fp32."""
-    T = q.shape[0]
-    n_seq = state_slots.numel()
-    _fp32_param(decay, "decay")
-    _check_step(positions, seq_rows, state_slots)
-    for t, wd in ((q, dk), (k, dk), (v, dv)):
-        if t.shape != (T, n_heads * wd) or t.stride(1) != 1 or t.dtype != q.dtype:
-            raise ValueError("retention: q, k [T, H dk] and v [T, H dv] with contiguous rows, one dtype")
-    if state.shape[1:] != (n_heads, dv, dk) or state.dtype != torch.float32 or not state.is_contiguous() or \
-            decay.numel() != n_heads:
-        raise ValueError("retention: state is contiguous float32 [slots, H, dv, dk], decay [H]")
-    if not q.is_cuda:
-        H = n_heads
-        out = torch.zeros((T, H, dv), dtype=torch.float32)
-        qf, kf, vf = q.float().view(T, H, dk), k.float().view(T, H, dk) * k_scale, v.float().view(T, H, dv)
-        b = _seq_bounds(seq_rows, n_seq)
-        for s in range(n_seq):
-            r0, r1 = b[s], b[s + 1]
-            sl = int(state_slots[s])
-            if sl < 0 or r1 <= r0:
-                continue
-            S = state[sl].transpose(1, 2).clone() if int(positions[r0]) > 0 else \
-                torch.zeros((H, dk, dv), dtype=torch.float32)
-            for t in range(r0, r1):
-                S = decay[:, None, None] * S + kf[t][:, :, None] * vf[t][:, None, :]
-                out[t] = torch.einsum("hi,hij->hj", qf[t], S)
-            state[sl] = S.transpose(1, 2)
-        return out.view(T, H * dv)
-    out = torch.empty((T, n_heads * dv), dtype=torch.float32, device=q.device)
-    _m().retention(out.data_ptr(), state.data_ptr(), state.shape[0], q.data_ptr(), q.stride(0), k.data_ptr(),
-                   k.stride(0), v.data_ptr(), v.stride(0), decay.data_ptr(), float(k_scale), positions.data_ptr(),
-                   _ptr(seq_rows), state_slots.data_ptr(), n_seq, T, n_heads, dk, dv, _f32(q), _stream())
-    return out
+    return _linear_scan("fixed", q, k, v, state, positions, seq_rows, state_slots, n_heads, dk, dv, k_scale=k_scale,
+                        decay=decay)
+
+
+def ssd(x: torch.Tensor, B: torch.Tensor, C: torch.Tensor, dt: torch.Tensor, dt_bias: torch.Tensor | None,
+        rate: torch.Tensor, skip: torch.Tensor | None, state: torch.Tensor, positions: torch.Tensor,
+        seq_rows: torch.Tensor | None, state_slots: torch.Tensor, n_heads: int, n_groups: int, N: int,
+        P: int) -> torch.Tensor:
+    """State-space duality (Mamba-2's recurrence) over the rows of a step, per
+    sequence and head from the sequence's state S [N, P] (fp32, stored as for
+    retention: [slots, H, P, N]; updated in place), with the step size
+    u_t = softplus(dt_t + dt_bias[h]):
+        S_t = exp(-rate[h] u_t) S_(t-1) + u_t B_t x_t^T,     y_t = S_t^T C_t + skip[h] x_t.
+    x [T, H P]; B, C [T, n_groups N] shared by H / n_groups heads each; dt [T, H]
+    -- column sections, any row stride.  Returns y [T, H P] fp32."""
+    return _linear_scan("step", C, B, x, state, positions, seq_rows, state_slots, n_heads, N, P, qk_heads=n_groups,
+                        gate=dt, g_bias=dt_bias, rate=rate, skip=skip)
+
+
+def gated_linear_attention(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, z: torch.Tensor,
+                           z_bias: torch.Tensor | None, tau: float, q_scale: float, state: torch.Tensor,
+                           positions: torch.Tensor, seq_rows: torch.Tensor | None, state_slots: torch.Tensor,
+                           n_heads: int, dk: int, dv: int) -> torch.Tensor:
+    """Gated linear attention over the rows of a step, per sequence and head
+    from the sequence's state S [dk, dv] (fp32, stored as for retention; updated
+    in place), with a decay per key channel and token, alpha_t =
+    sigmoid(z_t + z_bias)^(1 / tau):
+        S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,     o_t = S_t^T (q_scale q_t).
+    q, k, z [T, H dk] and v [T, H dv] are column sections.  Returns o [T, H dv] fp32."""
+    return _linear_scan("channel", q, k, v, state, positions, seq_rows, state_slots, n_heads, dk, dv, q_scale=q_scale,
+                        gate=z, g_bias=z_bias, tau=tau)
 
 
 GATE_ACTS = {"sigmoid": 0, "silu": 1}
@@ -377,4 +452,31 @@ def head_norm_gate(o: torch.Tensor, n_heads: int, weight: torch.Tensor | None, g
     _m().head_norm_gate(out.data_ptr(), o.data_ptr(), _ptr(weight), _ptr(gate), gate.stride(0) if gate is not None else 0,
                         T, n_heads, W // n_heads, float(eps), GATE_ACTS[gate_act], int(out_dtype == torch.float32),
                         _stream())
+    return out
+
+
+def gate_group_norm(y: torch.Tensor, z: torch.Tensor, weight: torch.Tensor, n_groups: int, eps: float,
+                    out_dtype: torch.dtype, out: torch.Tensor | None = None) -> torch.Tensor:
+    """y [T, W] fp32 times silu(z) (z [T, W], a column section of the
+    activation dtype), then every one of n_groups equal parts of the row divided
+    by its own root mean square (sqrt(mean + eps)), times weight [W] (fp32), in
+    out_dtype: the gate enters in front of the norm.  out: where the result
+    goes, e.g. a column section of the next projection's input."""
+    T, W = y.shape
+    _fp32_param(weight, "weight")
+    if y.dtype != torch.float32 or not y.is_contiguous() or W % n_groups or weight.numel() != W:
+        raise ValueError("gate_group_norm: y is contiguous float32 [T, W], one weight per column, equal parts")
+    if z.shape != y.shape or z.stride(1) != 1 or z.dtype != out_dtype:
+        raise ValueError("gate_group_norm: gate [T, W] of the output dtype with contiguous rows")
+    if out is None:
+        out = torch.empty((T, W), dtype=out_dtype, device=y.device)
+    elif out.shape != y.shape or out.stride(1) != 1 or out.dtype != out_dtype:
+        raise ValueError("gate_group_norm: out is [T, W] of the output dtype with contiguous rows")
+    if not y.is_cuda:
+        zf = z.float()
+        o = (y * zf * torch.sigmoid(zf)).view(T, n_groups, W // n_groups)
+        o = (o * torch.rsqrt((o * o).mean(-1, keepdim=True) + eps)).reshape(T, W) * weight
+        return out.copy_(o.to(out_dtype))
+    _m().gate_group_norm(out.data_ptr(), out.stride(0), y.data_ptr(), z.data_ptr(), z.stride(0), weight.data_ptr(), T,
+                         n_groups, W // n_groups, float(eps), int(out_dtype == torch.float32), _stream())
     return out
