@@ -1,6 +1,7 @@
-"""`bench.py --layered`: the layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik)
-beside the closest existing model (Llama; for Nefivik also Bolinex, for Sobivik
-also Bekulix, the closest layer-listed ones) at equal layer sizes, random weights.
+"""`bench.py --layered`: the layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik,
+Povurax) beside the closest existing model (Llama; for Nefivik also Bolinex, for
+Sobivik also Bekulix, for Povurax also Sobivik, the closest layer-listed ones) at
+equal layer sizes, random weights.
 `--layered-family` picks which family runs (default: Bekulix and Bolinex).
 
 Two parts, both on one GPU:
@@ -24,7 +25,8 @@ import torch
 from .. import ops
 from ..engine.engine import EngineConfig, LLMEngine
 from ..engine.request import SamplingParams
-from ..models.config import ModelConfig, _bekulix_preset, _bolinex_preset, _nefivik_preset, _sobivik_preset
+from ..models.config import (ModelConfig, _bekulix_preset, _bolinex_preset, _nefivik_preset, _povurax_preset,
+                             _sobivik_preset)
 from ..ops import mixers as mx
 from ..ops import moe
 from ..ops import recurrent as rc
@@ -69,6 +71,14 @@ def _sobivik_config(s: dict):
     feed-forwards, the depth average after every layer."""
     return _sobivik_preset(f"sobivik {s['W']}", s["W"], s["ff"], s["layers"], s["H"], s["G"], s["d"], 192,
                            s["W"] // 4, 64, 1024, 64, vocab=s["vocab"])
+
+
+def _povurax_config(s: dict):
+    """Povurax at the size's layer shapes: causal attention beside a state-space half of twice the
+    width (64 channels and 128 states a head, 8 groups) and gated linear attention in turn, all with
+    dense feed-forwards, no layer sharing another's weights."""
+    return _povurax_preset(f"povurax {s['W']}", s["W"], s["ff"], s["layers"], s["H"], s["G"], s["d"], 2 * s["W"] // 64, 64,
+                           128, 8, vocab=s["vocab"], share=False, gla_ff=True)
 
 
 def _timed(fn, iters=10, warm=2) -> float:
@@ -558,6 +568,107 @@ def sobivik_kernels(s: dict, L: int, B: int, T: int) -> dict:
     return res
 
 
+def povurax_kernels(s: dict, L: int, B: int, T: int) -> dict:
+    """Povurax's kernels alone, each beside its counterpart: the two scans beside retention of the
+    same matrix sizes (4 prompts of L / 2 tokens; B decode rows); the norm + rotation + cache write
+    beside the per-head norm + cache write and Nefivik's convolution + rotation + cache write; the
+    convolution with bias and silu beside Sobivik's input convolution; the gated group norm beside the
+    per-head norm + gate; the output gate and the clamped unit beside silu_and_mul; the residual step
+    with a cast beside the one with a norm.  (Causal attention: attention_kernels.)"""
+    H, G, d, W, ff, bs = s["H"], s["G"], s["d"], s["W"], s["ff"], 64
+    dev, dt = "cuda", torch.bfloat16
+    res = {}
+
+    def put(name, us, byts=None, flops=None, **kw):
+        res[name] = {"us": round(us, 1), **kw}
+        if byts:
+            res[name]["TB/s"] = round(byts / us / 1e6, 2)
+        if flops:
+            res[name]["TFLOPs"] = round(flops / us / 1e6, 1)
+
+    print(f"[layered] povurax kernels {W}", file=sys.stderr, flush=True)
+    # ---- scans: prompts, then decode rows.  (heads, dk, dv, q / k heads)
+    P, N, Gs = 64, 128, 8
+    Hs = 2 * W // P
+    inner, C = Hs * P, Hs * P + 2 * Gs * N
+    for tag, n_seq, rows in (("prefill", 4, L // 2), ("decode", B, 1)):
+        Tn = n_seq * rows
+        pos = (torch.arange(rows, device=dev) + 1).repeat(n_seq)
+        seq_rows = torch.arange(0, Tn + 1, rows, dtype=torch.int32, device=dev) if rows > 1 else None
+        slots = torch.arange(n_seq, dtype=torch.int32, device=dev)
+        step = (pos, seq_rows, slots)
+
+        def scan(name, fn, heads, dk, dv, io):
+            st = n_seq * heads * dk * dv * 4 * 2  # state read and written
+            us = _timed(fn)
+            put(f"{name}_{tag}", us, io + st, 2.0 * 2 * Tn * heads * dk * dv, tok_per_s=round(Tn / us * 1e6),
+                state_TBs=round(st / us / 1e6, 2))
+
+        x = torch.randn(Tn, C, device=dev, dtype=dt) * 0.5
+        u = torch.randn(Tn, Hs, device=dev, dtype=dt) - 2
+        rate, D, ub = torch.ones(Hs, device=dev), torch.ones(Hs, device=dev), torch.zeros(Hs, device=dev)
+        state = torch.zeros(n_seq, Hs, P, N, device=dev)
+        scan("ssd", lambda: rc.ssd(x[:, :inner], x[:, inner:inner + Gs * N], x[:, inner + Gs * N:], u, ub, rate, D, state,
+                                   *step, Hs, Gs, N, P), Hs, N, P, Tn * (C * 2 + Hs * 2 + inner * 4))
+        q = torch.randn(Tn, 2 * Hs * N, device=dev, dtype=dt)
+        dec = torch.full((Hs,), 0.97, device=dev)
+        scan("retention_ssd_shape", lambda: rc.retention(q[:, :Hs * N], q[:, Hs * N:], x[:, :inner], dec, 1.0, state, *step, Hs,
+                                                         N, P), Hs, N, P, Tn * (2 * Hs * N * 2 + inner * 6))
+        del q
+        n = H * d
+        p = torch.randn(Tn, 4 * n, device=dev, dtype=dt)
+        z, zb = torch.randn(Tn, n, device=dev, dtype=dt), torch.zeros(n, device=dev)
+        state = torch.zeros(n_seq, H, d, d, device=dev)
+        scan("gla", lambda: rc.gated_linear_attention(p[:, :n], p[:, n:2 * n], p[:, 2 * n:3 * n], z, zb, 16.0, d ** -0.5, state,
+                                                      *step, H, d, d), H, d, d, Tn * n * (4 * 2 + 4))
+        dec = torch.full((H,), 0.97, device=dev)
+        scan("retention", lambda: rc.retention(p[:, :n], p[:, n:2 * n], p[:, 2 * n:3 * n], dec, d ** -0.5, state, *step, H, d,
+                                               d), H, d, d, Tn * n * (3 * 2 + 4))
+        y, gw = torch.randn(Tn, inner, device=dev), torch.ones(inner, device=dev)
+        zg = torch.randn(Tn, inner, device=dev, dtype=dt)
+        put(f"gate_group_norm_{tag}", _timed(lambda: rc.gate_group_norm(y, zg, gw, Gs, 1e-5, dt)), Tn * inner * (4 + 2 + 2))
+        put(f"head_norm_gate_{tag}", _timed(lambda: rc.head_norm_gate(y, Hs, gw, zg, 1e-5, dt, gate_act="silu")),
+            Tn * inner * (4 + 2 + 2))
+        del x, y, zg, p, z, state
+    # ---- convolution with bias and silu beside the plain one
+    taps = 4
+    x, cw, cb = torch.randn(T, C, device=dev, dtype=dt), torch.randn(taps, C, device=dev), torch.randn(C, device=dev)
+    tail = torch.zeros(1, taps - 1, C, device=dev, dtype=dt)
+    posT = torch.arange(T, device=dev)
+    rs = torch.zeros(T, dtype=torch.int32, device=dev)
+    sr = torch.tensor([0, T], dtype=torch.int32, device=dev)
+    s0 = torch.zeros(1, dtype=torch.int32, device=dev)
+    for name, kw in (("conv_bias_silu", dict(bias=cb, act="silu")), ("sobivik_input_conv", {})):
+        put(name, _timed(lambda: rc.conv_rope_cache(x, cw, tail, posT, posT, rs, sr, s0, 1, 0, C, 0, None, None, None, **kw)),
+            T * C * 2 * 2)
+    # ---- norm over all heads + rotation + cache write
+    nbt = T // bs + 1
+    kc, vc = (torch.zeros(nbt * bs, G * d, device=dev, dtype=dt) for _ in range(2))
+    qkv = torch.randn(T, (H + 2 * G) * d, device=dev, dtype=dt)
+    qn, kn = torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    inv = rc.rotary_frequencies(d, 500000.0).to(dev)
+    byts = T * d * 2 * (2 * H + 4 * G)
+    put("norm_rope_cache", _timed(lambda: mx.norm_rope_cache(qkv, posT, posT, H, G, d, G * d, qn, kn, 1e-5, inv, kc, vc)), byts)
+    put("headprep_cache", _timed(lambda: mx.headprep_cache(qkv, posT, posT, H, G, d, H * d, qn[:d], kn[:d], 1e-5, None, kc, vc,
+                                                           2, (H + G) * d, G * d)), byts)
+    cwq, tq = torch.randn(taps, (H + 2 * G) * d, device=dev), torch.zeros(1, taps - 1, (H + 2 * G) * d, device=dev, dtype=dt)
+    put("nefivik_conv_rope_cache", _timed(lambda: rc.conv_rope_cache(qkv, cwq, tq, posT, posT, rs, sr, s0, H, G, d, d,
+                                                                     inv[:d // 4].contiguous(), kc, vc)), byts)
+    # ---- gates, feed-forward unit, residual step
+    a, g = torch.randn(T, H * d, device=dev, dtype=dt), torch.randn(T, H * d, device=dev, dtype=dt)
+    o = torch.empty(T, H * d + inner, device=dev, dtype=dt)
+    put("output_gate_into_section", _timed(lambda: mx.act_mul(g, a, "sigmoid", out=o[:, :H * d], scale=0.5)), T * H * d * 6)
+    gu = torch.randn(T, 2 * ff, device=dev, dtype=dt)
+    put("glu_act_swiglu_clamp", _timed(lambda: mx.glu_act(gu, "swiglu_clamp", 7.0, 1.702)), T * ff * 2 * 3)
+    put("llama_silu_and_mul", _timed(lambda: ops.silu_and_mul(gu)), T * ff * 2 * 3)
+    X, c, nw = torch.randn(T, W, device=dev), torch.randn(T, W, device=dev, dtype=dt), torch.ones(W, device=dev)
+    put("residual_step_addend_cast", _timed(lambda: mx.residual_step(X, c=c, c_w=nw, eps=1e-5, want_cast=True, out_dtype=dt)),
+        T * W * (4 + 4 + 2 + 2))
+    put("residual_step_addend_rmsnorm", _timed(lambda: mx.residual_step(X, c=c, c_w=nw, eps=1e-5, norm="rms", norm_w=nw,
+                                                                        out_dtype=dt)), T * W * (4 + 4 + 2 + 2))
+    return res
+
+
 def run_layered_compare(args, dev) -> dict:
     isl, osl = min(args.isl, 2048), min(args.osl, 64)
     fam = getattr(args, "layered_family", "all")
@@ -574,6 +685,11 @@ def run_layered_compare(args, dev) -> dict:
             row["sobivik"] = engine_throughput(_sobivik_config(s), dev, isl, osl, 4, 64, args.seed)
             row["sobivik_kernels"] = sobivik_kernels(s, 4096, 64, 8192)
             row["bekulix"] = engine_throughput(bek, dev, isl, osl, 4, 64, args.seed)
+        if fam == "povurax":
+            row["povurax"] = engine_throughput(_povurax_config(s), dev, isl, osl, 4, 64, args.seed)
+            row["povurax_kernels"] = povurax_kernels(s, 4096, 64, 8192)
+            row["sobivik"] = engine_throughput(_sobivik_config(s), dev, isl, osl, 4, 64, args.seed)
+            row["params"] = {c.name: c.num_params() for c in (_povurax_config(s), _sobivik_config(s))}
         if fam == "nefivik":
             row["nefivik"] = engine_throughput(_nefivik_config(s), dev, isl, osl, 4, 64, args.seed)
             row["nefivik_kernels"] = nefivik_kernels(s, 4096, 64, 8192)
@@ -586,6 +702,6 @@ def run_layered_compare(args, dev) -> dict:
         if fam in ("all", "bekulix"):
             row["rowwise_kernels"] = rowwise_kernels(s, 8192)
         sizes[name] = row
-    return {"metric": "layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik) beside Llama at equal layer sizes: engine prefill / "
-                      "decode tokens/s and kernels alone", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
+    return {"metric": "layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik, Povurax) beside Llama at equal layer sizes: "
+                      "engine prefill / decode tokens/s and kernels alone", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
             "family": fam, "data": "synthetic (random-token prompts, random-init weights)", "sizes": sizes}

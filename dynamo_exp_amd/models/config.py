@@ -431,11 +431,12 @@ def _sobivik_preset(name, W, ff, n_layers, heads, kv_heads, d, rank, q_rank, rot
 
 
 def _povurax_preset(name, W, ff, n_layers, heads, kv_heads, d, ssm_heads, ssm_dim, state, groups, vocab=32000, conv=4,
-                    rot_dims=None, share=True):
+                    rot_dims=None, share=True, gla_ff=False):
     """A Povurax stack at a real model's layer sizes: layers with attention
     and a state-space mixer side by side and a clamped gated feed-forward, each
-    followed by a gated linear attention layer without one; with `share`, every
-    parallel layer after the first runs the first one's weights."""
+    followed by a gated linear attention layer, without a feed-forward unless
+    `gla_ff`; with `share`, every parallel layer after the first runs the first
+    one's weights."""
     par = {"left": {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5,
                     "rot": {"base": 500000.0, "dims": rot_dims or d}}, "left_scale": 0.5,
            "right": {"heads": ssm_heads, "vdim": ssm_dim, "state": state, "groups": groups, "norm_groups": groups,
@@ -444,7 +445,8 @@ def _povurax_preset(name, W, ff, n_layers, heads, kv_heads, d, ssm_heads, ssm_di
     layers = []
     for i in range(n_layers):
         if i % 2:
-            layers.append({"type": "gla", "mixer": dict(gla), "mlp": None})
+            layers.append({"type": "gla", "mixer": dict(gla),
+                           "mlp": {"kind": "dense", "ff": ff, "limit": 7.0} if gla_ff else None})
             continue
         layers.append({"type": "parallel", "mixer": {**par, "left": dict(par["left"]), "right": dict(par["right"])},
                        "mlp": {"kind": "dense", "ff": ff, "limit": 7.0}})
