@@ -1,0 +1,498 @@
+// Chunked, matrix-core form of the linear recurrences for prompt portions in
+// bf16 (the token-by-token form and the definitions: linear_scan.hip).  One
+// workgroup of four waves walks a sequence's rows of one (head, 64 columns)
+// chunk by chunk; wave w owns 16 columns p of the running matrix, which stays in
+// fp32 accumulators for the whole walk.  With E(a, b) the decay from token a to
+// token b, a chunk is three products,
+//     o_t = E(start, t) S^T q_t + sum_(s <= t) (q_t . E(s, t) k_s) u_s v_s,
+//     S  <- E(start, end) S + sum_s (E(s, end) u_s k_s) v_s^T.
+// q, k, v are bf16 as projected; whatever carries a decay, a step size or the
+// state enters its product as the sum of two bf16 numbers (hi + lo, 16 bits of
+// mantissa), and all sums are fp32.
+//
+// v_mfma_f32_16x16x32_bf16: lane l = 16 g + c holds row (column) c of A (B) at
+// eight k-slots of its group g, and of the result column c, rows 4 g .. 4 g + 3.
+// Which k a slot stands for is free as long as A and B agree: with slots {4 g +
+// 0..3, 16 + 4 g + 0..3} a pair of result tiles of S is an A operand as it lies in
+// the registers.
+#include "linear_scan.h"
+
+namespace {
+
+__device__ __forceinline__ bf16x8_t as_bf16x8(const raw_u32x4& v) { return __builtin_bit_cast(bf16x8_t, v); }
+
+// eight k-slots from one 16-byte run / from two 8-byte runs 16 elements apart
+__device__ __forceinline__ bf16x8_t frag8(const bf16_t* p) { return as_bf16x8(*reinterpret_cast<const raw_u32x4*>(p)); }
+__device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p) {
+  const uint2 a = *reinterpret_cast<const uint2*>(p), b = *reinterpret_cast<const uint2*>(p + 16);
+  return as_bf16x8(raw_u32x4{a.x, a.y, b.x, b.y});
+}
+
+// hi + lo bf16 parts of four floats
+__device__ __forceinline__ void split4(const float* v, uint2& hi, uint2& lo) {
+  hi.x = pack_bf16x2(v[0], v[1]);
+  hi.y = pack_bf16x2(v[2], v[3]);
+  lo.x = pack_bf16x2(v[0] - bf16lo(hi.x), v[1] - bf16hi(hi.x));
+  lo.y = pack_bf16x2(v[2] - bf16lo(hi.y), v[3] - bf16hi(hi.y));
+}
+__device__ __forceinline__ void split8(const float* v, raw_u32x4& hi, raw_u32x4& lo) {
+  uint2 h0, l0, h1, l1;
+  split4(v, h0, l0);
+  split4(v + 4, h1, l1);
+  hi = raw_u32x4{h0.x, h0.y, h1.x, h1.y};
+  lo = raw_u32x4{l0.x, l0.y, l1.x, l1.y};
+}
+
+// four rows of eight elements each -> element e of all four rows, 8 bytes
+__device__ __forceinline__ uint2 column4(const raw_u32x4* r, int e) {
+  const int w = e >> 1;
+  if (e & 1)
+    return uint2{(r[0][w] >> 16) | (r[1][w] & 0xffff0000u), (r[2][w] >> 16) | (r[3][w] & 0xffff0000u)};
+  return uint2{(r[0][w] & 0xffffu) | (r[1][w] << 16), (r[2][w] & 0xffffu) | (r[3][w] << 16)};
+}
+
+__device__ __forceinline__ f32x4 mfma32(bf16x8_t a, bf16x8_t b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+__device__ __forceinline__ f32x4 mfma16(uint2 a, uint2 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(i16x4, a), __builtin_bit_cast(i16x4, b), c, 0, 0, 0);
+}
+
+constexpr float kLog2e = 1.4426950408889634f;
+constexpr int kPB = 64;  // columns of a workgroup
+
+// the workgroup's sequence: its rows and slot; false: nothing to do
+struct Walk {
+  int r0, n, h, hq, col0, slot;
+  bool fresh;
+};
+__device__ __forceinline__ bool open_walk(const ScanArgs& g, Walk& w) {
+  const int s = blockIdx.z;
+  w.h = blockIdx.y;
+  w.hq = w.h / g.qk_rep;
+  w.col0 = blockIdx.x * kPB;
+  w.r0 = g.seq_rows[s];
+  w.n = g.seq_rows[s + 1] - w.r0;
+  if (w.n < g.min_rows || w.r0 < 0 || w.r0 + w.n > g.T) return false;
+  w.slot = g.slots[s];
+  if (w.slot < 0 || w.slot >= g.n_slots) {  // padding: zeros out, no state touched
+    for (int i = threadIdx.x; i < w.n * kPB; i += blockDim.x)
+      g.out[(int64_t)(w.r0 + i / kPB) * g.H * g.dv + (int64_t)w.h * g.dv + w.col0 + i % kPB] = 0.f;
+    return false;
+  }
+  w.fresh = g.pos[w.r0] == 0;
+  return true;
+}
+
+// ---------------------------------------------------------------------------
+// One decay per token and head (kFixed, kStep): chunks of 64 tokens.  The decays
+// between the chunk's tokens form a [64, 64] matrix of their own, which
+// multiplies the q k^T products element by element: each wave forms 16 token
+// rows of it (only the tiles on and below the diagonal) and shares them through LDS.
+template <int DK, int MODE>
+__global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
+  constexpr int Q = 64, KP = DK + 8, SP = Q + 8;  // tokens per chunk; padded LDS rows
+  constexpr int NO = DK / 8, NI = 16 * NO;        // staged items of q / k: 4 tokens x 8 channels
+  constexpr int NM = DK / 16, NK = DK / 32;
+  static_assert(NI <= 256 && DK % 32 == 0, "one staged item per thread");
+  __shared__ __attribute__((aligned(16))) bf16_t Cs[Q * KP];   // q [t][n]
+  __shared__ __attribute__((aligned(16))) bf16_t Bs[Q * KP];   // k [s][n]
+  __shared__ __attribute__((aligned(16))) bf16_t BT[DK * SP];  // k [n][s]
+  __shared__ __attribute__((aligned(16))) bf16_t xT[kPB * SP];  // v [p][s]
+  __shared__ __attribute__((aligned(16))) bf16_t Mh[Q * SP], Ml[Q * SP];  // weights [t][s]
+  __shared__ __attribute__((aligned(16))) float Ls[Q], us[Q], ws[Q];  // log2 decay since the start, step, step x decay to the end
+  Walk w;
+  if (!open_walk(g, w)) return;
+  const int tid = threadIdx.x, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
+  const int sq = tid & 15, oc = tid >> 4;  // staging: token quad, channel octet
+  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
+  f32x4 S[NM];
+#pragma unroll
+  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  const bf16_t* q = (const bf16_t*)g.q + (int64_t)w.r0 * g.qs + (int64_t)w.hq * DK + 8 * oc;
+  const bf16_t* k = (const bf16_t*)g.k + (int64_t)w.r0 * g.ks + (int64_t)w.hq * DK + 8 * oc;
+  const bf16_t* v = (const bf16_t*)g.v + (int64_t)w.r0 * g.vs + (int64_t)w.h * g.dv + w.col0 + 8 * oc;
+  const float skip = g.skip ? g.skip[w.h] : 0.f, qsc = g.q_scale;
+  const float fixed_l2 = MODE == kFixed ? fmaxf(log2f(g.decay[w.h]), -1e6f) : 0.f;
+  raw_u32x4 rq[4], rk[4], rv[4];
+  float ru = 0.f, rl = 0.f;  // step and log2 decay of token tid (first wave)
+  auto fetch = [&](int t0) {
+    const raw_u32x4 zero{0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = t0 + 4 * sq + i;
+      const bool ok = t < w.n;
+      rq[i] = NI == 256 || tid < NI ? (ok ? *reinterpret_cast<const raw_u32x4*>(q + (int64_t)t * g.qs) : zero) : zero;
+      rk[i] = NI == 256 || tid < NI ? (ok ? *reinterpret_cast<const raw_u32x4*>(k + (int64_t)t * g.ks) : zero) : zero;
+      rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + (int64_t)t * g.vs) : zero;
+    }
+    if (tid < Q) {
+      ru = rl = 0.f;
+      if (t0 + tid < w.n) {
+        if constexpr (MODE == kFixed) {
+          ru = 1.f;
+          rl = fixed_l2;
+        } else {
+          ru = step_size<bf16_t>(g, w.r0 + t0 + tid, w.h);
+          rl = -g.rate[w.h] * ru * kLog2e;
+        }
+      }
+    }
+  };
+  fetch(0);
+  for (int t0 = 0; t0 < w.n; t0 += Q) {
+    __syncthreads();  // the previous chunk is consumed
+    if (NI == 256 || tid < NI) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        *reinterpret_cast<raw_u32x4*>(Cs + (4 * sq + i) * KP + 8 * oc) = rq[i];
+        *reinterpret_cast<raw_u32x4*>(Bs + (4 * sq + i) * KP + 8 * oc) = rk[i];
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(BT + (8 * oc + e) * SP + 4 * sq) = column4(rk, e);
+    }
+    if (tid < 128) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(xT + (8 * oc + e) * SP + 4 * sq) = column4(rv, e);
+    }
+    if (tid < Q) {  // one wave: log decays since the chunk's start (inclusive scan)
+      float L = rl;
+#pragma unroll
+      for (int o = 1; o < 64; o <<= 1) {
+        const float y = __shfl_up(L, o, 64);
+        if (tid >= o) L += y;
+      }
+      const float u = ru * g.k_scale;
+      Ls[tid] = L;
+      us[tid] = u;
+      ws[tid] = u * fast_exp2(__shfl(L, 63, 64) - L);
+    }
+    __syncthreads();
+    if (t0 + Q < w.n) fetch(t0 + Q);
+    {  // weights of 16 query tokens: (q_t . k_s) E(s, t) u_s
+      const int t = 16 * wave + c16;
+      bf16x8_t cq[NK];
+#pragma unroll
+      for (int kk = 0; kk < NK; ++kk) cq[kk] = frag8(Cs + t * KP + 32 * kk + 8 * g4);
+      const float Lt = Ls[t];
+      for (int j = 0; j <= (wave | 1); ++j) {
+        float m4[4] = {0.f, 0.f, 0.f, 0.f};
+        const int s0 = 16 * j + 4 * g4;
+        if (j <= wave) {
+          f32x4 a{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int kk = 0; kk < NK; ++kk) a = mfma32(frag8(Bs + (16 * j + c16) * KP + 32 * kk + 8 * g4), cq[kk], a);
+          const f32x4 L4 = *reinterpret_cast<const f32x4*>(Ls + s0), u4 = *reinterpret_cast<const f32x4*>(us + s0);
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            if (s0 + r <= t) m4[r] = a[r] * fast_exp2(Lt - L4[r]) * u4[r] * qsc;
+            if (s0 + r == t) m4[r] += skip;
+          }
+        }
+        uint2 hi, lo;
+        split4(m4, hi, lo);
+        *reinterpret_cast<uint2*>(Mh + t * SP + s0) = hi;
+        *reinterpret_cast<uint2*>(Ml + t * SP + s0) = lo;
+      }
+    }
+    __syncthreads();
+    const int p = 16 * wave + c16;
+    bf16x8_t xf[2], Sh[NK], Sl[NK];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) xf[kk] = frag8(xT + p * SP + 32 * kk + 8 * g4);
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) {
+      float s8[8];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s8[e] = S[2 * kk][e], s8[4 + e] = S[2 * kk + 1][e];
+      raw_u32x4 hi, lo;
+      split8(s8, hi, lo);
+      Sh[kk] = as_bf16x8(hi);
+      Sl[kk] = as_bf16x8(lo);
+    }
+#pragma unroll
+    for (int tt = 0; tt < Q / 16; ++tt) {
+      if (t0 + 16 * tt >= w.n) break;
+      const int t = 16 * tt + c16;
+      f32x4 a{0.f, 0.f, 0.f, 0.f}, b{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kk = 0; kk < NK; ++kk) {
+        const bf16x8_t cf = frag4_4(Cs + t * KP + 32 * kk + 4 * g4);
+        a = mfma32(Sh[kk], cf, a);
+        b = mfma32(Sl[kk], cf, b);
+      }
+      const float e = fast_exp2(Ls[t]) * qsc;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) a[r] = (a[r] + b[r]) * e, b[r] = 0.f;
+#pragma unroll
+      for (int kk = 0; kk <= tt / 2; ++kk) {
+        a = mfma32(xf[kk], frag8(Mh + t * SP + 32 * kk + 8 * g4), a);
+        b = mfma32(xf[kk], frag8(Ml + t * SP + 32 * kk + 8 * g4), b);
+      }
+      if (t0 + t < w.n)
+        *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + t) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) =
+            f32x4{a[0] + b[0], a[1] + b[1], a[2] + b[2], a[3] + b[3]};
+    }
+    const float eq = fast_exp2(Ls[Q - 1]);
+    bf16x8_t xh[2], xl[2];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      const raw_u32x4 x4 = __builtin_bit_cast(raw_u32x4, xf[kk]);
+      float x8[8];
+#pragma unroll
+      for (int e = 0; e < 8; e += 4) {
+        const f32x4 w4 = *reinterpret_cast<const f32x4*>(ws + 32 * kk + 8 * g4 + e);
+        x8[e] = bf16lo(x4[e / 2]) * w4[0];
+        x8[e + 1] = bf16hi(x4[e / 2]) * w4[1];
+        x8[e + 2] = bf16lo(x4[e / 2 + 1]) * w4[2];
+        x8[e + 3] = bf16hi(x4[e / 2 + 1]) * w4[3];
+      }
+      raw_u32x4 hi, lo;
+      split8(x8, hi, lo);
+      xh[kk] = as_bf16x8(hi);
+      xl[kk] = as_bf16x8(lo);
+    }
+#pragma unroll
+    for (int m = 0; m < NM; ++m) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[m][r] *= eq;
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        const bf16x8_t bf = frag8(BT + (16 * m + c16) * SP + 32 * kk + 8 * g4);
+        S[m] = mfma32(bf, xh[kk], S[m]);
+        S[m] = mfma32(bf, xl[kk], S[m]);
+      }
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < NM; ++m) *reinterpret_cast<f32x4*>(sp + 16 * m) = S[m];
+}
+
+// ---------------------------------------------------------------------------
+// A decay per token and key channel (kChannel): chunks of 16 tokens, so that the
+// products between a chunk's tokens are one tile.  There the decay of a pair
+// factors through the chunk's middle token m per channel, q_t E(m, t) and k_s E(s, m)
+// (one of the two may exceed 1); their product is the pair's decay exactly, unless a
+// channel decays so far inside a half chunk that a factor would leave the
+// number range: then the tile is summed pair by pair with exponent differences.
+// A chunk's operands are formed one chunk ahead into the other half of the
+// double-buffered LDS, so their exponentials run beside the matrix products.
+// Lanes of one DPP row of 16 hold the 16 tokens of the same eight channels:
+// the running log decays are row scans.
+template <int DK> struct ChannelBuf {
+  static constexpr int KP = DK + 8, SP = 20;
+  bf16_t qi[2][16 * KP];  // hi, lo of q E(start, t) [t][n]
+  bf16_t qm[2][16 * KP];  //           q E(m, t)     [t][n]
+  bf16_t km[2][16 * KP];  //           k E(s, m)     [s][n]
+  bf16_t ke[2][DK * SP];  //           k E(s, end)   [n][s]
+  bf16_t vT[kPB * SP];    // v [p][s]
+  float eq[DK];           // E(start, end)
+  int far[4];             // per wave: a factor would leave the number range
+};
+
+constexpr float kFarLog2 = 96.f;  // a half chunk that decays by more than 2^-96 in some channel is summed pair by pair
+
+// log2 of sigmoid(z)^(1 / tau)
+__device__ __forceinline__ float channel_log2(float z, float inv_tau) {
+  const float y = z * kLog2e;
+  return -(fmaxf(-y, 0.f) + __builtin_amdgcn_logf(1.f + fast_exp2(-fabsf(y)))) * inv_tau;
+}
+
+template <int DK>
+__global__ void __launch_bounds__(256, 2) channel_chunk_kernel(ScanArgs g) {
+  using Buf = ChannelBuf<DK>;
+  constexpr int Q = 16, KP = Buf::KP, SP = Buf::SP, NM = DK / 16, NK = DK / 32;
+  static_assert(DK % 32 == 0 && DK <= 128, "one staged item per thread");
+  __shared__ __attribute__((aligned(16))) Buf bufs[2];
+  Walk w;
+  if (!open_walk(g, w)) return;
+  const int tid = threadIdx.x, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
+  const int oc = tid >> 4;                 // staging: token c16, channel octet (q, k, decays)
+  const bool has_k = oc < DK / 8;
+  const int ov = oc - (16 - kPB / 8);      // ... column octet (v, the upper threads)
+  const bool has_v = ov >= 0;
+  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
+  f32x4 S[NM];
+#pragma unroll
+  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  const bf16_t* q = (const bf16_t*)g.q + (int64_t)w.r0 * g.qs + (int64_t)w.hq * DK;
+  const bf16_t* k = (const bf16_t*)g.k + (int64_t)w.r0 * g.ks + (int64_t)w.hq * DK;
+  const bf16_t* z = (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + (int64_t)w.h * DK;
+  const bf16_t* v = (const bf16_t*)g.v + (int64_t)w.r0 * g.vs + (int64_t)w.h * g.dv + w.col0;
+  const float* zb = g.g_bias ? g.g_bias + w.h * DK : nullptr;
+  float bias[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) bias[e] = zb && has_k ? zb[8 * oc + e] : 0.f;
+  raw_u32x4 rq, rk, rz, rv;
+  bool live = false;
+  auto fetch = [&](int t0) {
+    const raw_u32x4 zero{0u, 0u, 0u, 0u};
+    const int64_t t = t0 + c16;
+    live = t < w.n;
+    rq = live && has_k ? *reinterpret_cast<const raw_u32x4*>(q + t * g.qs + 8 * oc) : zero;
+    rk = live && has_k ? *reinterpret_cast<const raw_u32x4*>(k + t * g.ks + 8 * oc) : zero;
+    rz = live && has_k ? *reinterpret_cast<const raw_u32x4*>(z + t * g.gs + 8 * oc) : zero;
+    rv = live && has_v ? *reinterpret_cast<const raw_u32x4*>(v + t * g.vs + 8 * ov) : zero;
+  };
+  auto stage = [&](Buf& b) {
+    bool far = false;
+    if (has_k) {
+      float qi[8], qm[8], km[8], ke[8], eq[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const uint32_t zw = rz[e >> 1], qw = rq[e >> 1], kw = rk[e >> 1];
+        float L = live ? channel_log2((e & 1 ? bf16hi(zw) : bf16lo(zw)) + bias[e], g.inv_tau) : 0.f;
+        L += dpp_f<0x111>(L);  // inclusive scan over the row's 16 tokens
+        L += dpp_f<0x112>(L);
+        L += dpp_f<0x114>(L);
+        L += dpp_f<0x118>(L);
+        const float Lm = dpp_f<0x157>(L), Le = dpp_f<0x15F>(L);  // token 7 (the middle), token 15 (the end)
+        const float d = L - Lm;
+        far |= fabsf(d) > kFarLog2;
+        const float qv = (e & 1 ? bf16hi(qw) : bf16lo(qw)) * g.q_scale, kv = (e & 1 ? bf16hi(kw) : bf16lo(kw)) * g.k_scale;
+        const float dc = fminf(fmaxf(d, -kFarLog2), kFarLog2);  // (finite whatever the decays)
+        qi[e] = qv * fast_exp2(L);
+        qm[e] = qv * fast_exp2(dc);
+        km[e] = kv * fast_exp2(-dc);
+        ke[e] = kv * fast_exp2(Le - L);
+        eq[e] = fast_exp2(Le);
+      }
+      raw_u32x4 hi, lo;
+      bf16_t* at = b.qi[0] + c16 * KP + 8 * oc;
+      split8(qi, hi, lo);
+      *reinterpret_cast<raw_u32x4*>(at) = hi;
+      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+      at = b.qm[0] + c16 * KP + 8 * oc;
+      split8(qm, hi, lo);
+      *reinterpret_cast<raw_u32x4*>(at) = hi;
+      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+      at = b.km[0] + c16 * KP + 8 * oc;
+      split8(km, hi, lo);
+      *reinterpret_cast<raw_u32x4*>(at) = hi;
+      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+      split8(ke, hi, lo);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int i = (8 * oc + e) * SP + c16;
+        b.ke[0][i] = (bf16_t)(e & 1 ? hi[e >> 1] >> 16 : hi[e >> 1] & 0xffffu);
+        b.ke[1][i] = (bf16_t)(e & 1 ? lo[e >> 1] >> 16 : lo[e >> 1] & 0xffffu);
+      }
+      if (c16 == 15) {
+#pragma unroll
+        for (int e = 0; e < 8; e += 4) *reinterpret_cast<f32x4*>(b.eq + 8 * oc + e) = f32x4{eq[e], eq[e + 1], eq[e + 2], eq[e + 3]};
+      }
+    }
+    if (has_v) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) b.vT[(8 * ov + e) * SP + c16] = (bf16_t)(e & 1 ? rv[e >> 1] >> 16 : rv[e >> 1] & 0xffffu);
+    }
+    const int any = __any(far);
+    if ((tid & 63) == 0) b.far[wave] = any;
+  };
+  auto pair_by_pair = [&](int t0, f32x4& a) {  // a[r] = sum_n q_t k_s E(s, t), s = 4 g4 + r, t = c16
+    a = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (t0 + c16 >= w.n) return;
+    const int64_t t = t0 + c16;
+    for (int n = 0; n < DK; ++n) {
+      const float qv = bf16_to_f32(q[t * g.qs + n]) * g.q_scale, zbn = zb ? zb[n] : 0.f;
+      float E = 0.f;  // log2 decay from s to t, s walking down from t
+      for (int s = c16; s >= 4 * g4; --s) {
+        if (s < 4 * g4 + 4) {
+          const float x = qv * bf16_to_f32(k[(int64_t)(t0 + s) * g.ks + n]) * g.k_scale * fast_exp2(E);
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            if (s == 4 * g4 + r) a[r] += x;
+        }
+        E += channel_log2(bf16_to_f32(z[(int64_t)(t0 + s) * g.gs + n]) + zbn, g.inv_tau);
+      }
+    }
+  };
+  fetch(0);
+  stage(bufs[0]);
+  if (Q < w.n) fetch(Q);
+  for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
+    __syncthreads();  // this chunk is staged; the other half is consumed
+    const Buf& b = bufs[cur];
+    if (t0 + Q < w.n) {
+      stage(bufs[cur ^ 1]);
+      if (t0 + 2 * Q < w.n) fetch(t0 + 2 * Q);
+    }
+    // weights of the chunk's pairs, [s][t] (every wave forms the tile it needs itself)
+    f32x4 a{0.f, 0.f, 0.f, 0.f}, a1 = a, a2 = a;
+    if (b.far[0] | b.far[1] | b.far[2] | b.far[3]) {
+      pair_by_pair(t0, a);
+    } else {
+#pragma unroll
+      for (int kk = 0; kk < NK; ++kk) {
+        const int o = c16 * KP + 32 * kk + 8 * g4;
+        const bf16x8_t kh = frag8(b.km[0] + o), qh = frag8(b.qm[0] + o);
+        a = mfma32(kh, qh, a);
+        a1 = mfma32(kh, frag8(b.qm[1] + o), a1);
+        a2 = mfma32(frag8(b.km[1] + o), qh, a2);
+      }
+    }
+    float m4[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) m4[r] = 4 * g4 + r <= c16 ? a[r] + (a1[r] + a2[r]) : 0.f;
+    uint2 Ah, Al;
+    split4(m4, Ah, Al);
+    const uint2 vf = *reinterpret_cast<const uint2*>(b.vT + (16 * wave + c16) * SP + 4 * g4);
+    f32x4 y{0.f, 0.f, 0.f, 0.f}, y1 = y, y2 = y;
+#pragma unroll
+    for (int kk = 0; kk < NK; ++kk) {
+      float s8[8];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) s8[e] = S[2 * kk][e], s8[4 + e] = S[2 * kk + 1][e];
+      raw_u32x4 hi, lo;
+      split8(s8, hi, lo);
+      const int o = c16 * KP + 32 * kk + 4 * g4;
+      const bf16x8_t qh = frag4_4(b.qi[0] + o), Sh = as_bf16x8(hi);
+      y = mfma32(Sh, qh, y);
+      y1 = mfma32(as_bf16x8(lo), qh, y1);
+      y2 = mfma32(Sh, frag4_4(b.qi[1] + o), y2);
+    }
+    y = mfma16(vf, Ah, y);
+    y1 = mfma16(vf, Al, y1);
+    if (t0 + c16 < w.n) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) y[r] += y1[r] + y2[r];
+      *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + c16) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) = y;
+    }
+#pragma unroll
+    for (int m = 0; m < NM; ++m) {
+      const f32x4 e4 = *reinterpret_cast<const f32x4*>(b.eq + 16 * m + 4 * g4);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
+      const int o = (16 * m + c16) * SP + 4 * g4;
+      S[m] = mfma16(*reinterpret_cast<const uint2*>(b.ke[0] + o), vf, S[m]);
+      S[m] = mfma16(*reinterpret_cast<const uint2*>(b.ke[1] + o), vf, S[m]);
+    }
+  }
+#pragma unroll
+  for (int m = 0; m < NM; ++m) *reinterpret_cast<f32x4*>(sp + 16 * m) = S[m];
+}
+
+}  // namespace
+
+// sizes and alignment the chunked kernels take (bf16 rows as 16-byte runs, whole column blocks)
+bool chunk_scan_ok(int mode, const ScanArgs& g) {
+  auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  return (g.dk == 32 || g.dk == 64 || g.dk == 128) && g.dv % kPB == 0 && g.qs % 8 == 0 && g.ks % 8 == 0 &&
+         g.vs % 8 == 0 && al(g.q) && al(g.k) && al(g.v) && al(g.state) && al(g.out) &&
+         (mode != kChannel || (g.gs % 8 == 0 && al(g.g) && !g.skip));
+}
+
+#define CHUNK_DK(KERNEL)                                                                                           \
+  if (g.dk == 32) hipLaunchKernelGGL((KERNEL(32)), grid, dim3(256), 0, st, g);                                     \
+  else if (g.dk == 64) hipLaunchKernelGGL((KERNEL(64)), grid, dim3(256), 0, st, g);                                \
+  else hipLaunchKernelGGL((KERNEL(128)), grid, dim3(256), 0, st, g);
+
+void launch_chunk_scan(int mode, const ScanArgs& g, int n_seq, hipStream_t st) {
+  const dim3 grid(g.dv / kPB, g.H, n_seq);
+#define FIXED_K(D) chunk_scan_kernel<D, kFixed>
+#define STEP_K(D) chunk_scan_kernel<D, kStep>
+#define CHANNEL_K(D) channel_chunk_kernel<D>
+  if (mode == kFixed) { CHUNK_DK(FIXED_K) }
+  else if (mode == kStep) { CHUNK_DK(STEP_K) }
+  else { CHUNK_DK(CHANNEL_K) }
+}

@@ -11,47 +11,18 @@
 // kRows rows each, in registers) and join their partial q^T S by DPP lane
 // exchanges; a workgroup owns blockDim / R columns of one (sequence, head).
 // Tokens are staged through LDS kTok at a time.  State layout [slots, H, dv,
-// dk]: a column's rows are contiguous.  Slots, seq_rows and the reset at
-// position 0 as in recurrent.hip.  Decays, step sizes, the state and all sums
+// dk]: a column's rows are contiguous.  This file scans token by token (any
+// sizes, decode steps, fp32); chunk_scan.hip has the matrix-core form for prompt
+// portions in bf16.  Slots, seq_rows and the reset at position 0 as in
+// recurrent.hip.  Decays, step sizes, the state and all sums
 // are fp32 whatever the activation element is.
-#include "recurrent.h"
+#include "linear_scan.h"
 
 namespace {
 
-enum ScanMode { kFixed = 0, kStep = 1, kChannel = 2 };
-
-struct ScanArgs {
-  float* out;    // [T, H * dv]
-  float* state;  // [slots, H, dv, dk]
-  const void *q, *k, *v;
-  int64_t qs, ks, vs;  // row strides (elements)
-  float q_scale, k_scale;
-  int qk_rep;          // heads that share a q / k head
-  const float* decay;  // kFixed: [H]
-  const void* g;       // kStep: step logits [T, H]; kChannel: decay logits [T, H * dk]
-  int64_t gs;
-  const float* g_bias;  // [H] / [H * dk] or null
-  const float* rate;    // kStep: [H]
-  const float* skip;    // [H] or null
-  float inv_tau;        // kChannel
-  const int64_t* pos;
-  const int* seq_rows;  // null: row i is sequence i
-  const int* slots;
-  int n_slots, T, H, dk, dv;
-};
-
-__device__ __forceinline__ float softplusf_(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-
-// sigmoid(z)^(1 / tau) = exp(-softplus(-z) / tau).  Only the exponent's absolute error matters, so the
-// plain log of 1 + e serves (its error is below 1e-7 where log1p would return e itself).
-__device__ __forceinline__ float channel_decay(float z, float inv_tau) {
-  const float sp = fmaxf(-z, 0.f) + __logf(1.f + __expf(-fabsf(z)));
-  return __expf(-sp * inv_tau);
-}
-
 // step size and decay of one (row, head)
 template <typename T> __device__ __forceinline__ float2 step_terms(const ScanArgs& g, int64_t row, int h) {
-  const float u = softplusf_(ldf<T>((const T*)g.g, row * g.gs + h) + (g.g_bias ? g.g_bias[h] : 0.f));
+  const float u = step_size<T>(g, row, h);
   return float2{u, expf(-g.rate[h] * u)};
 }
 
@@ -65,7 +36,7 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
   const int cl = tid / R, r = tid % R;
   const int col0 = blockIdx.z * cols, j = col0 + cl;
   const int r0 = g.seq_rows ? g.seq_rows[s] : s, r1 = g.seq_rows ? g.seq_rows[s + 1] : s + 1;
-  if (r1 <= r0 || r0 < 0 || r1 > g.T) return;
+  if (r1 <= r0 || r0 < 0 || r1 > g.T || r1 - r0 > g.max_rows) return;
   const bool colok = j < g.dv;
   const int slot = g.slots[s];
   const int64_t ow = (int64_t)g.H * g.dv;
@@ -147,8 +118,6 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
 // a group's 128-bit LDS reads of a row vector are neighbouring chunks and the state is read and
 // written as 16-byte runs.  The next block's eight tokens (q, k, decay logits of the head, v of the
 // workgroup's columns) are fetched into registers as 16-byte chunks while the current block's chain runs.
-typedef uint32_t raw_u32x4 __attribute__((ext_vector_type(4)));
-
 template <typename T> __device__ __forceinline__ void chunk_to_f32(const raw_u32x4& c, float* o);
 template <> __device__ __forceinline__ void chunk_to_f32<bf16_t>(const raw_u32x4& c, float* o) {
 #pragma unroll
@@ -176,7 +145,7 @@ __global__ void __launch_bounds__(256) scan_fast_kernel(ScanArgs g) {
   const int tid = threadIdx.x, cl = tid / R, r = tid % R;
   const int col0 = blockIdx.z * cols, j = col0 + cl;
   const int r0 = g.seq_rows ? g.seq_rows[s] : s, r1 = g.seq_rows ? g.seq_rows[s + 1] : s + 1;
-  if (r1 <= r0 || r0 < 0 || r1 > g.T) return;
+  if (r1 <= r0 || r0 < 0 || r1 > g.T || r1 - r0 > g.max_rows) return;
   const int slot = g.slots[s];
   const int64_t ow = (int64_t)g.H * g.dv;
   if (slot < 0 || slot >= g.n_slots) {  // a padding row: zeros out, no state touched
@@ -341,7 +310,19 @@ extern "C" int dxm_linear_scan(int mode, float* out, float* state, int n_slots, 
   if (!seq_rows && n_seq != T_) return 4;
   if (qk_rep < 1 || H % qk_rep) return 5;
   ScanArgs g{out, state, q, k, v, qs, ks, vs, q_scale, k_scale, qk_rep, decay, gate, gs, g_bias, rate, skip, inv_tau,
-             pos, seq_rows, slots, n_slots, T_, H, dk, dv};
+             pos, seq_rows, slots, n_slots, T_, H, dk, dv, 1, 0x7fffffff};
+  // prompt portions in bf16: matrix-core chunks where the sizes fit; shorter runs of a sequence
+  // (decode tokens among them) stay with the token scan
+  if (!f32 && seq_rows && n_seq <= 65535 && T_ >= kChunkMinRows + n_seq - 1 && chunk_scan_ok(mode, g)) {
+    if ((mode == kFixed && !decay) || (mode == kStep && (!gate || !rate)) || (mode == kChannel && !gate)) return 6;
+    g.min_rows = kChunkMinRows;
+    launch_chunk_scan(mode, g, n_seq, st);
+    if (n_seq == 1) {
+      DX_CHECK_LAUNCH();
+      return 0;
+    }
+    g.max_rows = kChunkMinRows - 1;
+  }
   if (mode == kFixed) {
     if (!decay) return 6;
     DISPATCH_T(f32, (dispatch_rows<T, kFixed>(g, n_seq, st)));

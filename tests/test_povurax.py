@@ -158,7 +158,8 @@ def section(t, extra, device):
 
 
 # ----------------------------------------------------------------- mechanisms alone
-SCAN_PORTIONS = [[(41,), (41,)], [(19, 2, 1, 1, 9, 8, 1), (3, 30, 7, 1)]]
+SCAN_T = 150
+SCAN_PORTIONS = [[(150,), (150,)], [(19, 2, 1, 1, 9, 8, 1, 64, 45), (3, 30, 7, 1, 65, 16, 17, 11)]]
 
 
 def check_scan(device, run, want, state):
@@ -171,7 +172,7 @@ def check_scan(device, run, want, state):
                 got[s].append(o[int(meta[2][i]):int(meta[2][i + 1])].cpu())
         for s in range(2):
             w, S = want[s]
-            assert torch.allclose(torch.cat(got[s]).double(), w.reshape(41, -1), atol=3e-4, rtol=1e-4)
+            assert torch.allclose(torch.cat(got[s]).double(), w.reshape(SCAN_T, -1), atol=3e-4, rtol=1e-4)
             assert torch.allclose(state[3 if s == 0 else 1].cpu().double().transpose(1, 2), S, atol=3e-4, rtol=1e-4)
 
 
@@ -182,7 +183,7 @@ def test_ssd_scan_alone(device, dtype, H, G, N, P):
     """The state-space recurrence with its step sizes, shared B / C groups and skip, then a decode step
     with a padding row; x, B, C, dt are sections of wider rows."""
     torch.manual_seed(N)
-    T, dt_ = 41, DT[dtype]
+    T, dt_ = SCAN_T, DT[dtype]
     x, B, C = torch.randn(2, T, H * P).to(dt_), torch.randn(2, T, G * N).to(dt_), torch.randn(2, T, G * N).to(dt_)
     dt = (torch.randn(2, T, H) * 2).to(dt_)
     bias, A_log, D = torch.randn(H) - 1, torch.rand(H) * 2, torch.randn(H)
@@ -208,12 +209,13 @@ def test_ssd_scan_alone(device, dtype, H, G, N, P):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("H,dk,dv,tau", [(3, 10, 14, 8.0), (1, 1, 1, 1.0), (2, 64, 64, 16.0), (2, 128, 32, 4.0), (1, 34, 3, 2.0),
-                                         (1, 16, 256, 16.0), (2, 256, 32, 16.0), (1, 48, 40, 0.5), (2, 32, 128, 16.0)])
+                                         (1, 16, 256, 16.0), (2, 256, 32, 16.0), (1, 48, 40, 0.5), (2, 32, 128, 16.0),
+                                         (1, 64, 64, 0.25), (1, 128, 64, 0.5)])
 def test_gla_scan_alone(device, dtype, H, dk, dv, tau):
     """Gated linear attention: a decay per key channel, from hardly any to nearly total (logits far below
     zero, where the decay is a power of e / tau, and far above), then a decode step with a padding row."""
     torch.manual_seed(dk)
-    T, dt_ = 41, DT[dtype]
+    T, dt_ = SCAN_T, DT[dtype]
     q, k, z = (torch.randn(2, T, H * dk).to(dt_) for _ in range(3))
     z = z * 3
     z[:, ::7] -= 40.0
