@@ -58,6 +58,24 @@ __device__ __forceinline__ f32x4 mfma16(uint2 a, uint2 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(i16x4, a), __builtin_bit_cast(i16x4, b), c, 0, 0, 0);
 }
 
+// inclusive sums over the 64 lanes: within rows of 16, then the last lane of a row (of a half) into the next
+template <int CTRL, int ROWS> __device__ __forceinline__ float dpp_rows(float v) {
+  return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, ROWS, 0xf, false));
+}
+__device__ __forceinline__ float row_scan_sum(float v) {
+  v += dpp_f<0x111>(v);
+  v += dpp_f<0x112>(v);
+  v += dpp_f<0x114>(v);
+  v += dpp_f<0x118>(v);
+  return v;
+}
+__device__ __forceinline__ float wave_scan_sum(float v) {
+  v = row_scan_sum(v);
+  v += dpp_rows<0x142, 0xa>(v);
+  v += dpp_rows<0x143, 0xc>(v);
+  return v;
+}
+
 constexpr float kLog2e = 1.4426950408889634f;
 constexpr int kPB = 64;  // columns of a workgroup
 
@@ -115,7 +133,10 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
   const float skip = g.skip ? g.skip[w.h] : 0.f, qsc = g.q_scale;
   const float fixed_l2 = MODE == kFixed ? fmaxf(log2f(g.decay[w.h]), -1e6f) : 0.f;
   raw_u32x4 rq[4], rk[4], rv[4];
-  float ru = 0.f, rl = 0.f;  // step and log2 decay of token tid (first wave)
+  bf16_t rg = 0;  // step logit of token tid (first wave)
+  const bf16_t* gl = MODE == kStep ? (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + w.h : nullptr;
+  const float g_bias = MODE == kStep && g.g_bias ? g.g_bias[w.h] : 0.f;
+  const float rate_l2 = MODE == kStep ? -g.rate[w.h] * kLog2e : 0.f;
   auto fetch = [&](int t0) {
     const raw_u32x4 zero{0u, 0u, 0u, 0u};
 #pragma unroll
@@ -126,18 +147,7 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       rk[i] = NI == 256 || tid < NI ? (ok ? *reinterpret_cast<const raw_u32x4*>(k + (int64_t)t * g.ks) : zero) : zero;
       rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + (int64_t)t * g.vs) : zero;
     }
-    if (tid < Q) {
-      ru = rl = 0.f;
-      if (t0 + tid < w.n) {
-        if constexpr (MODE == kFixed) {
-          ru = 1.f;
-          rl = fixed_l2;
-        } else {
-          ru = step_size<bf16_t>(g, w.r0 + t0 + tid, w.h);
-          rl = -g.rate[w.h] * ru * kLog2e;
-        }
-      }
-    }
+    if (MODE == kStep && tid < Q && t0 + tid < w.n) rg = gl[(int64_t)(t0 + tid) * g.gs];
   };
   fetch(0);
   for (int t0 = 0; t0 < w.n; t0 += Q) {
@@ -156,16 +166,18 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(xT + (8 * oc + e) * SP + 4 * sq) = column4(rv, e);
     }
     if (tid < Q) {  // one wave: log decays since the chunk's start (inclusive scan)
-      float L = rl;
-#pragma unroll
-      for (int o = 1; o < 64; o <<= 1) {
-        const float y = __shfl_up(L, o, 64);
-        if (tid >= o) L += y;
+      const bool ok = t0 + tid < w.n;
+      float u = ok ? 1.f : 0.f, L = ok ? fixed_l2 : 0.f;
+      if (MODE == kStep && ok) {
+        u = softplusf_(bf16_to_f32(rg) + g_bias);
+        L = rate_l2 * u;
       }
-      const float u = ru * g.k_scale;
+      L = wave_scan_sum(L);
+      u *= g.k_scale;
       Ls[tid] = L;
       us[tid] = u;
-      ws[tid] = u * fast_exp2(__shfl(L, 63, 64) - L);
+      const float Lend = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, L), 63));
+      ws[tid] = u * fast_exp2(Lend - L);
     }
     __syncthreads();
     if (t0 + Q < w.n) fetch(t0 + Q);
@@ -270,27 +282,29 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
 
 // ---------------------------------------------------------------------------
 // A decay per token and key channel (kChannel): chunks of 16 tokens, so that the
-// products between a chunk's tokens are one tile.  There the decay of a pair
-// factors through the chunk's middle token m per channel, q_t E(m, t) and k_s E(s, m)
-// (one of the two may exceed 1); their product is the pair's decay exactly, unless a
-// channel decays so far inside a half chunk that a factor would leave the
-// number range: then the tile is summed pair by pair with exponent differences.
-// A chunk's operands are formed one chunk ahead into the other half of the
-// double-buffered LDS, so their exponentials run beside the matrix products.
-// Lanes of one DPP row of 16 hold the 16 tokens of the same eight channels:
-// the running log decays are row scans.
+// products between a chunk's tokens are one tile.  With L the log decays summed
+// from the chunk's start, the decay of a pair factors per channel into e^L of the
+// query token and e^-L of the key token, and
+//     S <- e^L(end) (S + sum_s (k_s e^-L(s)) v_s^T)
+// takes the same scaled keys.  Where a channel decays so far inside a chunk that
+// e^-L would leave the number range, the pairs are summed one by one with
+// exponent differences, and the scaled keys carry e^(L(end) - L(s)) instead, with
+// e^L(end) on S alone.
+// Four waves (the upper ones) form a chunk's operands, one chunk ahead, in the
+// other half of the double-buffered LDS; the lower four run the matrix products.
+// In an upper wave the lanes of one DPP row of 16 hold the 16 tokens of the same
+// eight channels, so the running log decays are row scans.
 template <int DK> struct ChannelBuf {
   static constexpr int KP = DK + 8, SP = 20;
-  bf16_t qi[2][16 * KP];  // hi, lo of q E(start, t) [t][n]
-  bf16_t qm[2][16 * KP];  //           q E(m, t)     [t][n]
-  bf16_t km[2][16 * KP];  //           k E(s, m)     [s][n]
-  bf16_t ke[2][DK * SP];  //           k E(s, end)   [n][s]
+  bf16_t qi[2][16 * KP];  // hi, lo of q e^L                  [t][n]
+  bf16_t km[2][16 * KP];  //           k e^-L                 [s][n]
+  bf16_t ke[2][DK * SP];  //           the same, transposed   [n][s]
   bf16_t vT[kPB * SP];    // v [p][s]
-  float eq[DK];           // E(start, end)
-  int far[4];             // per wave: a factor would leave the number range
+  float eq[DK];           // e^L(end)
+  int far[4];             // per forming wave: e^-L would leave the number range
 };
 
-constexpr float kFarLog2 = 96.f;  // a half chunk that decays by more than 2^-96 in some channel is summed pair by pair
+constexpr float kFarLog2 = 96.f;  // log2 of the largest e^-L used as a factor
 
 // log2 of sigmoid(z)^(1 / tau)
 __device__ __forceinline__ float channel_log2(float z, float inv_tau) {
@@ -299,96 +313,110 @@ __device__ __forceinline__ float channel_log2(float z, float inv_tau) {
 }
 
 template <int DK>
-__global__ void __launch_bounds__(256, 2) channel_chunk_kernel(ScanArgs g) {
+__global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
   using Buf = ChannelBuf<DK>;
   constexpr int Q = 16, KP = Buf::KP, SP = Buf::SP, NM = DK / 16, NK = DK / 32;
   static_assert(DK % 32 == 0 && DK <= 128, "one staged item per thread");
   __shared__ __attribute__((aligned(16))) Buf bufs[2];
   Walk w;
   if (!open_walk(g, w)) return;
-  const int tid = threadIdx.x, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
-  const int oc = tid >> 4;                 // staging: token c16, channel octet (q, k, decays)
-  const bool has_k = oc < DK / 8;
-  const int ov = oc - (16 - kPB / 8);      // ... column octet (v, the upper threads)
-  const bool has_v = ov >= 0;
-  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
-  f32x4 S[NM];
-#pragma unroll
-  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  const bool former = threadIdx.x >= 256;
+  const int tid = threadIdx.x & 255, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
   const bf16_t* q = (const bf16_t*)g.q + (int64_t)w.r0 * g.qs + (int64_t)w.hq * DK;
   const bf16_t* k = (const bf16_t*)g.k + (int64_t)w.r0 * g.ks + (int64_t)w.hq * DK;
   const bf16_t* z = (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + (int64_t)w.h * DK;
   const bf16_t* v = (const bf16_t*)g.v + (int64_t)w.r0 * g.vs + (int64_t)w.h * g.dv + w.col0;
   const float* zb = g.g_bias ? g.g_bias + w.h * DK : nullptr;
-  float bias[8];
+
+  if (former) {  // ---- operands of the chunks
+    const int oc = tid >> 4;  // token c16, channel octet (q, k, decays)
+    const bool has_k = oc < DK / 8;
+    const int ov = oc - (16 - kPB / 8);  // ... column octet (v, the upper threads)
+    const bool has_v = ov >= 0;
+    float bias[8];
 #pragma unroll
-  for (int e = 0; e < 8; ++e) bias[e] = zb && has_k ? zb[8 * oc + e] : 0.f;
-  raw_u32x4 rq, rk, rz, rv;
-  bool live = false;
-  auto fetch = [&](int t0) {
-    const raw_u32x4 zero{0u, 0u, 0u, 0u};
-    const int64_t t = t0 + c16;
-    live = t < w.n;
-    rq = live && has_k ? *reinterpret_cast<const raw_u32x4*>(q + t * g.qs + 8 * oc) : zero;
-    rk = live && has_k ? *reinterpret_cast<const raw_u32x4*>(k + t * g.ks + 8 * oc) : zero;
-    rz = live && has_k ? *reinterpret_cast<const raw_u32x4*>(z + t * g.gs + 8 * oc) : zero;
-    rv = live && has_v ? *reinterpret_cast<const raw_u32x4*>(v + t * g.vs + 8 * ov) : zero;
-  };
-  auto stage = [&](Buf& b) {
-    bool far = false;
-    if (has_k) {
-      float qi[8], qm[8], km[8], ke[8], eq[8];
+    for (int e = 0; e < 8; ++e) bias[e] = zb && has_k ? zb[8 * oc + e] : 0.f;
+    raw_u32x4 rq, rk, rz, rv;
+    bool live = false;
+    auto fetch = [&](int t0) {
+      const raw_u32x4 zero{0u, 0u, 0u, 0u};
+      const int64_t t = t0 + c16;
+      live = t < w.n;
+      rz = live && has_k ? *reinterpret_cast<const raw_u32x4*>(z + t * g.gs + 8 * oc) : zero;
+      rq = live && has_k ? *reinterpret_cast<const raw_u32x4*>(q + t * g.qs + 8 * oc) : zero;
+      rk = live && has_k ? *reinterpret_cast<const raw_u32x4*>(k + t * g.ks + 8 * oc) : zero;
+      rv = live && has_v ? *reinterpret_cast<const raw_u32x4*>(v + t * g.vs + 8 * ov) : zero;
+    };
+    auto form = [&](Buf& b) {
+      bool far = false;
+      float L[8];
+      if (has_k) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const uint32_t zw = rz[e >> 1], qw = rq[e >> 1], kw = rk[e >> 1];
-        float L = live ? channel_log2((e & 1 ? bf16hi(zw) : bf16lo(zw)) + bias[e], g.inv_tau) : 0.f;
-        L += dpp_f<0x111>(L);  // inclusive scan over the row's 16 tokens
-        L += dpp_f<0x112>(L);
-        L += dpp_f<0x114>(L);
-        L += dpp_f<0x118>(L);
-        const float Lm = dpp_f<0x157>(L), Le = dpp_f<0x15F>(L);  // token 7 (the middle), token 15 (the end)
-        const float d = L - Lm;
-        far |= fabsf(d) > kFarLog2;
-        const float qv = (e & 1 ? bf16hi(qw) : bf16lo(qw)) * g.q_scale, kv = (e & 1 ? bf16hi(kw) : bf16lo(kw)) * g.k_scale;
-        const float dc = fminf(fmaxf(d, -kFarLog2), kFarLog2);  // (finite whatever the decays)
-        qi[e] = qv * fast_exp2(L);
-        qm[e] = qv * fast_exp2(dc);
-        km[e] = kv * fast_exp2(-dc);
-        ke[e] = kv * fast_exp2(Le - L);
-        eq[e] = fast_exp2(Le);
+        for (int e = 0; e < 8; ++e) {
+          const uint32_t zw = rz[e >> 1];
+          L[e] = row_scan_sum(live ? channel_log2((e & 1 ? bf16hi(zw) : bf16lo(zw)) + bias[e], g.inv_tau) : 0.f);
+          far |= L[e] < -kFarLog2;
+        }
       }
-      raw_u32x4 hi, lo;
-      bf16_t* at = b.qi[0] + c16 * KP + 8 * oc;
-      split8(qi, hi, lo);
-      *reinterpret_cast<raw_u32x4*>(at) = hi;
-      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
-      at = b.qm[0] + c16 * KP + 8 * oc;
-      split8(qm, hi, lo);
-      *reinterpret_cast<raw_u32x4*>(at) = hi;
-      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
-      at = b.km[0] + c16 * KP + 8 * oc;
-      split8(km, hi, lo);
-      *reinterpret_cast<raw_u32x4*>(at) = hi;
-      *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
-      split8(ke, hi, lo);
+      const bool any = __any(far);
+      if ((tid & 63) == 0) b.far[wave] = any;
+      if (has_k) {
+        float x[8], y[8];
+        raw_u32x4 hi, lo;
+        bf16_t* at = b.qi[0] + c16 * KP + 8 * oc;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int i = (8 * oc + e) * SP + c16;
-        b.ke[0][i] = (bf16_t)(e & 1 ? hi[e >> 1] >> 16 : hi[e >> 1] & 0xffffu);
-        b.ke[1][i] = (bf16_t)(e & 1 ? lo[e >> 1] >> 16 : lo[e >> 1] & 0xffffu);
+        for (int e = 0; e < 8; ++e) {
+          const uint32_t qw = rq[e >> 1];
+          y[e] = fast_exp2(L[e]);
+          x[e] = (e & 1 ? bf16hi(qw) : bf16lo(qw)) * g.q_scale * y[e];
+        }
+        if (c16 == 15) {
+          *reinterpret_cast<f32x4*>(b.eq + 8 * oc) = f32x4{y[0], y[1], y[2], y[3]};
+          *reinterpret_cast<f32x4*>(b.eq + 8 * oc + 4) = f32x4{y[4], y[5], y[6], y[7]};
+        }
+        split8(x, hi, lo);
+        *reinterpret_cast<raw_u32x4*>(at) = hi;
+        *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const uint32_t kw = rk[e >> 1];
+          // (a wave with a far channel: relative to the chunk's end, for S; its pairs are summed one by one)
+          x[e] = (e & 1 ? bf16hi(kw) : bf16lo(kw)) * g.k_scale * fast_exp2((any ? dpp_f<0x15F>(L[e]) : 0.f) - L[e]);
+        }
+        at = b.km[0] + c16 * KP + 8 * oc;
+        split8(x, hi, lo);
+        *reinterpret_cast<raw_u32x4*>(at) = hi;
+        *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int i = (8 * oc + e) * SP + c16;
+          b.ke[0][i] = (bf16_t)(e & 1 ? hi[e >> 1] >> 16 : hi[e >> 1] & 0xffffu);
+          b.ke[1][i] = (bf16_t)(e & 1 ? lo[e >> 1] >> 16 : lo[e >> 1] & 0xffffu);
+        }
       }
-      if (c16 == 15) {
+      if (has_v) {
 #pragma unroll
-        for (int e = 0; e < 8; e += 4) *reinterpret_cast<f32x4*>(b.eq + 8 * oc + e) = f32x4{eq[e], eq[e + 1], eq[e + 2], eq[e + 3]};
+        for (int e = 0; e < 8; ++e) b.vT[(8 * ov + e) * SP + c16] = (bf16_t)(e & 1 ? rv[e >> 1] >> 16 : rv[e >> 1] & 0xffffu);
+      }
+    };
+    fetch(0);
+    form(bufs[0]);
+    if (Q < w.n) fetch(Q);
+    for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
+      __syncthreads();  // chunk t0 is formed; the other half is consumed
+      if (t0 + Q < w.n) {
+        form(bufs[cur ^ 1]);
+        if (t0 + 2 * Q < w.n) fetch(t0 + 2 * Q);
       }
     }
-    if (has_v) {
+    return;
+  }
+
+  // ---- products.  (The barriers of the two loops pair up: one per chunk in each.)
+  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
+  f32x4 S[NM];
 #pragma unroll
-      for (int e = 0; e < 8; ++e) b.vT[(8 * ov + e) * SP + c16] = (bf16_t)(e & 1 ? rv[e >> 1] >> 16 : rv[e >> 1] & 0xffffu);
-    }
-    const int any = __any(far);
-    if ((tid & 63) == 0) b.far[wave] = any;
-  };
+  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
   auto pair_by_pair = [&](int t0, f32x4& a) {  // a[r] = sum_n q_t k_s E(s, t), s = 4 g4 + r, t = c16
     a = f32x4{0.f, 0.f, 0.f, 0.f};
     if (t0 + c16 >= w.n) return;
@@ -407,36 +435,26 @@ __global__ void __launch_bounds__(256, 2) channel_chunk_kernel(ScanArgs g) {
       }
     }
   };
-  fetch(0);
-  stage(bufs[0]);
-  if (Q < w.n) fetch(Q);
   for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
-    __syncthreads();  // this chunk is staged; the other half is consumed
+    __syncthreads();  // this chunk is formed
     const Buf& b = bufs[cur];
-    if (t0 + Q < w.n) {
-      stage(bufs[cur ^ 1]);
-      if (t0 + 2 * Q < w.n) fetch(t0 + 2 * Q);
-    }
+    const int far[4] = {b.far[0], b.far[1], b.far[2], b.far[3]};
+    const uint2 vf = *reinterpret_cast<const uint2*>(b.vT + (16 * wave + c16) * SP + 4 * g4);
     // weights of the chunk's pairs, [s][t] (every wave forms the tile it needs itself)
     f32x4 a{0.f, 0.f, 0.f, 0.f}, a1 = a, a2 = a;
-    if (b.far[0] | b.far[1] | b.far[2] | b.far[3]) {
+    const bool any_far = far[0] | far[1] | far[2] | far[3];
+    if (any_far) {
       pair_by_pair(t0, a);
     } else {
 #pragma unroll
       for (int kk = 0; kk < NK; ++kk) {
-        const int o = c16 * KP + 32 * kk + 8 * g4;
-        const bf16x8_t kh = frag8(b.km[0] + o), qh = frag8(b.qm[0] + o);
+        const int o = c16 * KP + 32 * kk + 4 * g4;
+        const bf16x8_t kh = frag4_4(b.km[0] + o), qh = frag4_4(b.qi[0] + o);
         a = mfma32(kh, qh, a);
-        a1 = mfma32(kh, frag8(b.qm[1] + o), a1);
-        a2 = mfma32(frag8(b.km[1] + o), qh, a2);
+        a1 = mfma32(kh, frag4_4(b.qi[1] + o), a1);
+        a2 = mfma32(frag4_4(b.km[1] + o), qh, a2);
       }
     }
-    float m4[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) m4[r] = 4 * g4 + r <= c16 ? a[r] + (a1[r] + a2[r]) : 0.f;
-    uint2 Ah, Al;
-    split4(m4, Ah, Al);
-    const uint2 vf = *reinterpret_cast<const uint2*>(b.vT + (16 * wave + c16) * SP + 4 * g4);
     f32x4 y{0.f, 0.f, 0.f, 0.f}, y1 = y, y2 = y;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
@@ -451,21 +469,35 @@ __global__ void __launch_bounds__(256, 2) channel_chunk_kernel(ScanArgs g) {
       y1 = mfma32(as_bf16x8(lo), qh, y1);
       y2 = mfma32(Sh, frag4_4(b.qi[1] + o), y2);
     }
+#pragma unroll
+    for (int m = 0; m < NM; ++m) {
+      // a forming wave covers 32 channels: its keys are relative to the chunk's start, or (far) to its end
+      const f32x4 e4 = *reinterpret_cast<const f32x4*>(b.eq + 16 * m + 4 * g4);
+      const bool late = far[m / 2];
+      const int o = (16 * m + c16) * SP + 4 * g4;
+      const uint2 kh = *reinterpret_cast<const uint2*>(b.ke[0] + o), kl = *reinterpret_cast<const uint2*>(b.ke[1] + o);
+      if (late) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
+      }
+      S[m] = mfma16(kh, vf, S[m]);
+      S[m] = mfma16(kl, vf, S[m]);
+      if (!late) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
+      }
+    }
+    float m4[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) m4[r] = 4 * g4 + r <= c16 ? a[r] + (a1[r] + a2[r]) : 0.f;
+    uint2 Ah, Al;
+    split4(m4, Ah, Al);
     y = mfma16(vf, Ah, y);
     y1 = mfma16(vf, Al, y1);
     if (t0 + c16 < w.n) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) y[r] += y1[r] + y2[r];
       *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + c16) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) = y;
-    }
-#pragma unroll
-    for (int m = 0; m < NM; ++m) {
-      const f32x4 e4 = *reinterpret_cast<const f32x4*>(b.eq + 16 * m + 4 * g4);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
-      const int o = (16 * m + c16) * SP + 4 * g4;
-      S[m] = mfma16(*reinterpret_cast<const uint2*>(b.ke[0] + o), vf, S[m]);
-      S[m] = mfma16(*reinterpret_cast<const uint2*>(b.ke[1] + o), vf, S[m]);
     }
   }
 #pragma unroll
@@ -482,17 +514,17 @@ bool chunk_scan_ok(int mode, const ScanArgs& g) {
          (mode != kChannel || (g.gs % 8 == 0 && al(g.g) && !g.skip));
 }
 
-#define CHUNK_DK(KERNEL)                                                                                           \
-  if (g.dk == 32) hipLaunchKernelGGL((KERNEL(32)), grid, dim3(256), 0, st, g);                                     \
-  else if (g.dk == 64) hipLaunchKernelGGL((KERNEL(64)), grid, dim3(256), 0, st, g);                                \
-  else hipLaunchKernelGGL((KERNEL(128)), grid, dim3(256), 0, st, g);
+#define CHUNK_DK(KERNEL, NT)                                                  \
+  if (g.dk == 32) hipLaunchKernelGGL((KERNEL(32)), grid, NT, 0, st, g);       \
+  else if (g.dk == 64) hipLaunchKernelGGL((KERNEL(64)), grid, NT, 0, st, g);  \
+  else hipLaunchKernelGGL((KERNEL(128)), grid, NT, 0, st, g);
 
 void launch_chunk_scan(int mode, const ScanArgs& g, int n_seq, hipStream_t st) {
   const dim3 grid(g.dv / kPB, g.H, n_seq);
 #define FIXED_K(D) chunk_scan_kernel<D, kFixed>
 #define STEP_K(D) chunk_scan_kernel<D, kStep>
 #define CHANNEL_K(D) channel_chunk_kernel<D>
-  if (mode == kFixed) { CHUNK_DK(FIXED_K) }
-  else if (mode == kStep) { CHUNK_DK(STEP_K) }
-  else { CHUNK_DK(CHANNEL_K) }
+  if (mode == kFixed) { CHUNK_DK(FIXED_K, dim3(256)) }
+  else if (mode == kStep) { CHUNK_DK(STEP_K, dim3(256)) }
+  else { CHUNK_DK(CHANNEL_K, dim3(512)) }
 }
