@@ -540,8 +540,7 @@ def sobivik_kernels(s: dict, L: int, B: int, T: int) -> dict:
     rs = torch.zeros(T, dtype=torch.int32, device=dev)
     sr = torch.tensor([0, T], dtype=torch.int32, device=dev)
     s0 = torch.zeros(1, dtype=torch.int32, device=dev)
-    put("input_conv", _timed(lambda: rc.conv_rope_cache(x, cw, tail, posT, posT, rs, sr, s0, 1, 0, W, 0, None, None, None)),
-        T * W * 2 * 2)
+    put("input_conv", _timed(lambda: rc.causal_conv(x, cw, tail, posT, rs, sr, s0)), T * W * 2 * 2)
     C = (H + 2 * G) * d
     xq = torch.randn(T, C, device=dev, dtype=dt)
     cwq = torch.randn(taps, C, device=dev)
@@ -639,8 +638,7 @@ def povurax_kernels(s: dict, L: int, B: int, T: int) -> dict:
     sr = torch.tensor([0, T], dtype=torch.int32, device=dev)
     s0 = torch.zeros(1, dtype=torch.int32, device=dev)
     for name, kw in (("conv_bias_silu", dict(bias=cb, act="silu")), ("sobivik_input_conv", {})):
-        put(name, _timed(lambda: rc.conv_rope_cache(x, cw, tail, posT, posT, rs, sr, s0, 1, 0, C, 0, None, None, None, **kw)),
-            T * C * 2 * 2)
+        put(name, _timed(lambda: rc.causal_conv(x, cw, tail, posT, rs, sr, s0, **kw)), T * C * 2 * 2)
     # ---- norm over all heads + rotation + cache write
     nbt = T // bs + 1
     kc, vc = (torch.zeros(nbt * bs, G * d, device=dev, dtype=dt) for _ in range(2))

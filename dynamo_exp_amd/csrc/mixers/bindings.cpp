@@ -43,6 +43,9 @@ int dxm_delta_rule(float*, float*, int, float*, const void*, int64_t, const void
 int dxm_conv_rope_cache(void*, const void*, int64_t, const float*, const float*, int, int, const void*, int, const int64_t*,
                         const int64_t*, const int*, const int*, const int*, int, int, int, int, int, int, const float*,
                         int, void*, void*, int, hipStream_t);
+int dxm_conv_run_ok(int64_t, int, int, int, uint64_t, int);
+int dxm_conv_run(void*, const void*, int64_t, const float*, const float*, int, int, void*, int, const int64_t*,
+                 const int*, const int*, const int*, int, int, int, int, hipStream_t);
 int dxm_conv_state_update(void*, int, const void*, int64_t, const int64_t*, const int*, const int*, int, int, int, int,
                           int, hipStream_t);
 int dxm_head_norm_gate(void*, const float*, const float*, const void*, int64_t, int, int, int, float, int, int,
@@ -169,6 +172,15 @@ PYBIND11_MODULE(_C_mixers, m) {
                               reinterpret_cast<const int*>(seq_rows), reinterpret_cast<const int*>(slots), n_seq, T,
                               n_q, n_k, d, dv, F(inv_freq), half, P(kc), P(vc), f32, S(st)),
           "conv_rope_cache");
+  });
+  m.def("conv_run_ok", &dxm_conv_run_ok);
+  m.def("conv_run", [](u out, u x, int64_t xs, u cw, u cb, int silu, int taps, u tail, int n_slots, u pos, u row_seq,
+                       u seq_rows, u slots, int n_seq, int T, int C, int f32, u st) {
+    check(dxm_conv_run(P(out), P(x), xs, F(cw), F(cb), silu, taps, P(tail), n_slots,
+                       reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int*>(row_seq),
+                       reinterpret_cast<const int*>(seq_rows), reinterpret_cast<const int*>(slots), n_seq, T, C, f32,
+                       S(st)),
+          "conv_run");
   });
   m.def("conv_state_update", [](u tail, int n_slots, u x, int64_t xs, u pos, u seq_rows, u slots, int n_seq, int T,
                                 int C, int taps, int f32, u st) {

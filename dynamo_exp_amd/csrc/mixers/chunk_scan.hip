@@ -23,10 +23,11 @@ __device__ __forceinline__ bf16x8_t as_bf16x8(const raw_u32x4& v) { return __bui
 
 // eight k-slots from one 16-byte run / from two 8-byte runs 16 elements apart
 __device__ __forceinline__ bf16x8_t frag8(const bf16_t* p) { return as_bf16x8(*reinterpret_cast<const raw_u32x4*>(p)); }
-__device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p) {
-  const uint2 a = *reinterpret_cast<const uint2*>(p), b = *reinterpret_cast<const uint2*>(p + 16);
+__device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p, const bf16_t* p16) {
+  const uint2 a = *reinterpret_cast<const uint2*>(p), b = *reinterpret_cast<const uint2*>(p16);
   return as_bf16x8(raw_u32x4{a.x, a.y, b.x, b.y});
 }
+__device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p) { return frag4_4(p, p + 16); }
 
 // hi + lo bf16 parts of four floats
 __device__ __forceinline__ void split4(const float* v, uint2& hi, uint2& lo) {
@@ -107,17 +108,26 @@ __device__ __forceinline__ bool open_walk(const ScanArgs& g, Walk& w) {
 // between the chunk's tokens form a [64, 64] matrix of their own, which
 // multiplies the q k^T products element by element: each wave forms 16 token
 // rows of it (only the tiles on and below the diagonal) and shares them through LDS.
+// LDS rows are cut into 16-byte pieces that an XOR with row bits moves around, so that the 16 rows a fragment
+// read touches (whichever lane groups the hardware serves together) and the staging writes (rows 4 apart) lie on
+// different banks: element offset of piece pc of row r in a [..][DK] and in a [..][64] image.
+template <int DK> __device__ __forceinline__ int koff(int r, int pc) {
+  if constexpr (DK == 128) return r * 128 + ((pc ^ ((r & 12) | ((r & 3) ^ (r >> 4)))) << 3);
+  return r * (DK + 8) + (pc << 3);  // (narrow rows: padding)
+}
+__device__ __forceinline__ int soff(int r, int pc) { return r * 64 + ((pc ^ ((r >> 1) & 7)) << 3); }
+
 template <int DK, int MODE>
 __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
-  constexpr int Q = 64, KP = DK + 8, SP = Q + 8;  // tokens per chunk; padded LDS rows
+  constexpr int Q = 64, KP = DK == 128 ? DK : DK + 8;  // tokens per chunk; LDS row of q and k
   constexpr int NO = DK / 8, NI = 16 * NO;        // staged items of q / k: 4 tokens x 8 channels
   constexpr int NM = DK / 16, NK = DK / 32;
   static_assert(NI <= 256 && DK % 32 == 0, "one staged item per thread");
   __shared__ __attribute__((aligned(16))) bf16_t Cs[Q * KP];   // q [t][n]
   __shared__ __attribute__((aligned(16))) bf16_t Bs[Q * KP];   // k [s][n]
-  __shared__ __attribute__((aligned(16))) bf16_t BT[DK * SP];  // k [n][s]
-  __shared__ __attribute__((aligned(16))) bf16_t xT[kPB * SP];  // v [p][s]
-  __shared__ __attribute__((aligned(16))) bf16_t Mh[Q * SP], Ml[Q * SP];  // weights [t][s]
+  __shared__ __attribute__((aligned(16))) bf16_t BT[DK * Q];  // k [n][s]
+  __shared__ __attribute__((aligned(16))) bf16_t xT[kPB * Q];  // v [p][s]
+  __shared__ __attribute__((aligned(16))) bf16_t Mh[Q * Q], Ml[Q * Q];  // weights [t][s]
   __shared__ __attribute__((aligned(16))) float Ls[Q], us[Q], ws[Q];  // log2 decay since the start, step, step x decay to the end
   Walk w;
   if (!open_walk(g, w)) return;
@@ -127,9 +137,10 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
   f32x4 S[NM];
 #pragma unroll
   for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
-  const bf16_t* q = (const bf16_t*)g.q + (int64_t)w.r0 * g.qs + (int64_t)w.hq * DK + 8 * oc;
-  const bf16_t* k = (const bf16_t*)g.k + (int64_t)w.r0 * g.ks + (int64_t)w.hq * DK + 8 * oc;
-  const bf16_t* v = (const bf16_t*)g.v + (int64_t)w.r0 * g.vs + (int64_t)w.h * g.dv + w.col0 + 8 * oc;
+  // the thread's first row of the chunk being fetched
+  const bf16_t* q = (const bf16_t*)g.q + (int64_t)(w.r0 + 4 * sq) * g.qs + (int64_t)w.hq * DK + 8 * oc;
+  const bf16_t* k = (const bf16_t*)g.k + (int64_t)(w.r0 + 4 * sq) * g.ks + (int64_t)w.hq * DK + 8 * oc;
+  const bf16_t* v = (const bf16_t*)g.v + (int64_t)(w.r0 + 4 * sq) * g.vs + (int64_t)w.h * g.dv + w.col0 + 8 * oc;
   const float skip = g.skip ? g.skip[w.h] : 0.f, qsc = g.q_scale;
   const float fixed_l2 = MODE == kFixed ? fmaxf(log2f(g.decay[w.h]), -1e6f) : 0.f;
   raw_u32x4 rq[4], rk[4], rv[4];
@@ -141,12 +152,14 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
     const raw_u32x4 zero{0u, 0u, 0u, 0u};
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int t = t0 + 4 * sq + i;
-      const bool ok = t < w.n;
-      rq[i] = NI == 256 || tid < NI ? (ok ? *reinterpret_cast<const raw_u32x4*>(q + (int64_t)t * g.qs) : zero) : zero;
-      rk[i] = NI == 256 || tid < NI ? (ok ? *reinterpret_cast<const raw_u32x4*>(k + (int64_t)t * g.ks) : zero) : zero;
-      rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + (int64_t)t * g.vs) : zero;
+      const bool ok = t0 + 4 * sq + i < w.n;
+      rq[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(q + i * g.qs) : zero;
+      rk[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(k + i * g.ks) : zero;
+      rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + i * g.vs) : zero;
     }
+    q += Q * g.qs;
+    k += Q * g.ks;
+    v += Q * g.vs;
     if (MODE == kStep && tid < Q && t0 + tid < w.n) rg = gl[(int64_t)(t0 + tid) * g.gs];
   };
   fetch(0);
@@ -155,15 +168,15 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
     if (NI == 256 || tid < NI) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        *reinterpret_cast<raw_u32x4*>(Cs + (4 * sq + i) * KP + 8 * oc) = rq[i];
-        *reinterpret_cast<raw_u32x4*>(Bs + (4 * sq + i) * KP + 8 * oc) = rk[i];
+        *reinterpret_cast<raw_u32x4*>(Cs + koff<DK>(4 * sq + i, oc)) = rq[i];
+        *reinterpret_cast<raw_u32x4*>(Bs + koff<DK>(4 * sq + i, oc)) = rk[i];
       }
 #pragma unroll
-      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(BT + (8 * oc + e) * SP + 4 * sq) = column4(rk, e);
+      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(BT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rk, e);
     }
     if (tid < 128) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(xT + (8 * oc + e) * SP + 4 * sq) = column4(rv, e);
+      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(xT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rv, e);
     }
     if (tid < Q) {  // one wave: log decays since the chunk's start (inclusive scan)
       const bool ok = t0 + tid < w.n;
@@ -185,7 +198,7 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       const int t = 16 * wave + c16;
       bf16x8_t cq[NK];
 #pragma unroll
-      for (int kk = 0; kk < NK; ++kk) cq[kk] = frag8(Cs + t * KP + 32 * kk + 8 * g4);
+      for (int kk = 0; kk < NK; ++kk) cq[kk] = frag8(Cs + koff<DK>(t, 4 * kk + g4));
       const float Lt = Ls[t];
       for (int j = 0; j <= (wave | 1); ++j) {
         float m4[4] = {0.f, 0.f, 0.f, 0.f};
@@ -193,7 +206,7 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
         if (j <= wave) {
           f32x4 a{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int kk = 0; kk < NK; ++kk) a = mfma32(frag8(Bs + (16 * j + c16) * KP + 32 * kk + 8 * g4), cq[kk], a);
+          for (int kk = 0; kk < NK; ++kk) a = mfma32(frag8(Bs + koff<DK>(16 * j + c16, 4 * kk + g4)), cq[kk], a);
           const f32x4 L4 = *reinterpret_cast<const f32x4*>(Ls + s0), u4 = *reinterpret_cast<const f32x4*>(us + s0);
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
@@ -203,15 +216,15 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
         }
         uint2 hi, lo;
         split4(m4, hi, lo);
-        *reinterpret_cast<uint2*>(Mh + t * SP + s0) = hi;
-        *reinterpret_cast<uint2*>(Ml + t * SP + s0) = lo;
+        *reinterpret_cast<uint2*>(Mh + soff(t, s0 >> 3) + (s0 & 7)) = hi;
+        *reinterpret_cast<uint2*>(Ml + soff(t, s0 >> 3) + (s0 & 7)) = lo;
       }
     }
     __syncthreads();
     const int p = 16 * wave + c16;
     bf16x8_t xf[2], Sh[NK], Sl[NK];
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) xf[kk] = frag8(xT + p * SP + 32 * kk + 8 * g4);
+    for (int kk = 0; kk < 2; ++kk) xf[kk] = frag8(xT + soff(p, 4 * kk + g4));
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
       float s8[8];
@@ -229,7 +242,7 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       f32x4 a{0.f, 0.f, 0.f, 0.f}, b{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < NK; ++kk) {
-        const bf16x8_t cf = frag4_4(Cs + t * KP + 32 * kk + 4 * g4);
+        const bf16x8_t cf = frag4_4(Cs + koff<DK>(t, 4 * kk + (g4 >> 1)) + 4 * (g4 & 1), Cs + koff<DK>(t, 4 * kk + 2 + (g4 >> 1)) + 4 * (g4 & 1));
         a = mfma32(Sh[kk], cf, a);
         b = mfma32(Sl[kk], cf, b);
       }
@@ -238,8 +251,8 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       for (int r = 0; r < 4; ++r) a[r] = (a[r] + b[r]) * e, b[r] = 0.f;
 #pragma unroll
       for (int kk = 0; kk <= tt / 2; ++kk) {
-        a = mfma32(xf[kk], frag8(Mh + t * SP + 32 * kk + 8 * g4), a);
-        b = mfma32(xf[kk], frag8(Ml + t * SP + 32 * kk + 8 * g4), b);
+        a = mfma32(xf[kk], frag8(Mh + soff(t, 4 * kk + g4)), a);
+        b = mfma32(xf[kk], frag8(Ml + soff(t, 4 * kk + g4)), b);
       }
       if (t0 + t < w.n)
         *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + t) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) =
@@ -270,7 +283,7 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       for (int r = 0; r < 4; ++r) S[m][r] *= eq;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
-        const bf16x8_t bf = frag8(BT + (16 * m + c16) * SP + 32 * kk + 8 * g4);
+        const bf16x8_t bf = frag8(BT + soff(16 * m + c16, 4 * kk + g4));
         S[m] = mfma32(bf, xh[kk], S[m]);
         S[m] = mfma32(bf, xl[kk], S[m]);
       }

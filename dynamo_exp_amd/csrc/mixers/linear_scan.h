@@ -40,8 +40,6 @@ template <typename T> __device__ __forceinline__ float step_size(const ScanArgs&
   return softplusf_(ldf<T>((const T*)g.g, row * g.gs + h) + (g.g_bias ? g.g_bias[h] : 0.f));
 }
 
-typedef uint32_t raw_u32x4 __attribute__((ext_vector_type(4)));
-
 // a sequence with at least this many rows in the step goes through the chunked kernels
 constexpr int kChunkMinRows = 8;
 

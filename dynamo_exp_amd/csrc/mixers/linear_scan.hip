@@ -118,16 +118,6 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
 // a group's 128-bit LDS reads of a row vector are neighbouring chunks and the state is read and
 // written as 16-byte runs.  The next block's eight tokens (q, k, decay logits of the head, v of the
 // workgroup's columns) are fetched into registers as 16-byte chunks while the current block's chain runs.
-template <typename T> __device__ __forceinline__ void chunk_to_f32(const raw_u32x4& c, float* o);
-template <> __device__ __forceinline__ void chunk_to_f32<bf16_t>(const raw_u32x4& c, float* o) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) o[2 * i] = bf16lo(c[i]), o[2 * i + 1] = bf16hi(c[i]);
-}
-template <> __device__ __forceinline__ void chunk_to_f32<float>(const raw_u32x4& c, float* o) {
-#pragma unroll
-  for (int i = 0; i < 4; ++i) o[i] = __uint_as_float(c[i]);
-}
-
 template <typename T, int R, int MODE>
 __global__ void __launch_bounds__(256) scan_fast_kernel(ScanArgs g) {
   constexpr int dk = 16 * R, cols = 256 / R, VEC = 16 / (int)sizeof(T);

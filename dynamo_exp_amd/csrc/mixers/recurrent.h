@@ -18,6 +18,11 @@ template <> __device__ __forceinline__ void stf<float>(float* p, int64_t i, floa
 
 __device__ __forceinline__ float sigmoidf_(float z) { return 1.f / (1.f + expf(-z)); }
 
+// the same from the hardware's exp2 and reciprocal (relative error a few 1e-7): per-element gates of wide rows
+__device__ __forceinline__ float fast_sigmoid(float z) {
+  return __builtin_amdgcn_rcpf(1.f + fast_exp2(z * -1.4426950408889634f));
+}
+
 template <int CTRL> __device__ __forceinline__ float dpp_f(float v) {
   return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, false));
 }
@@ -46,6 +51,17 @@ template <> struct VecIO<bf16_t, 8> {
     *reinterpret_cast<u16x8*>(p) = a;
   }
 };
+// 16 raw bytes as floats
+typedef uint32_t raw_u32x4 __attribute__((ext_vector_type(4)));
+template <typename T> __device__ __forceinline__ void chunk_to_f32(const raw_u32x4& c, float* o);
+template <> __device__ __forceinline__ void chunk_to_f32<bf16_t>(const raw_u32x4& c, float* o) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o[2 * i] = bf16lo(c[i]), o[2 * i + 1] = bf16hi(c[i]);
+}
+template <> __device__ __forceinline__ void chunk_to_f32<float>(const raw_u32x4& c, float* o) {
+#pragma unroll
+  for (int i = 0; i < 4; ++i) o[i] = __uint_as_float(c[i]);
+}
 template <> struct VecIO<float, 4> {
   __device__ static __forceinline__ void ld(const float* p, float* o) {
     const f32x4 a = *reinterpret_cast<const f32x4*>(p);

@@ -493,6 +493,95 @@ __global__ void __launch_bounds__(128) conv_rope_cache_vec_kernel(ConvArgs g) {
   }
 }
 
+// The convolution alone (no heads, no rotation, no cache) with the taps known at compile time: a thread
+// walks V neighbouring channels down R consecutive rows of the step with the last TAPS - 1 inputs in
+// registers, so an input row is read once (and its TAPS - 1 predecessors at the start of a run).  The inputs
+// before a run's or a sequence's first row come from the step's earlier rows or from the tail state.
+// R = 1 with one row per sequence (a decode step) also writes the new tail: the thread holds all of it.
+template <typename T, int V, int TAPS, int R>
+__global__ void __launch_bounds__(128) conv_run_kernel(ConvArgs g, T* __restrict__ new_tail) {
+  constexpr int M = TAPS - 1;
+  const int C = g.d, c = (blockIdx.x * 128 + threadIdx.x) * V, t0 = blockIdx.y * R;
+  if (c >= C) return;
+  const T* x = (const T*)g.x + c;
+  raw_u32x4 in[R];
+  float h[M > 0 ? M : 1][V], w[TAPS][V], b[V];
+#pragma unroll
+  for (int i = 0; i < R; ++i)
+    if (t0 + i < g.T) in[i] = *reinterpret_cast<const raw_u32x4*>(x + (int64_t)(t0 + i) * g.xs);
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+    for (int e = 0; e < V; e += 4) VecIO<float, 4>::ld(g.cw + (int64_t)j * C + c + e, w[j] + e);
+#pragma unroll
+  for (int e = 0; e < V; ++e) b[e] = g.cb ? g.cb[c + e] : 0.f;
+  auto seq_of = [&](int t) { return g.row_seq ? g.row_seq[t] : t; };
+  int s = seq_of(t0), slot = -1;
+  const bool one = R == 1 || (t0 + R <= g.T && seq_of(t0 + R - 1) == s);  // the run lies in one sequence
+  bool live = false;
+  auto enter = [&](int t) {  // row t begins a run of sequence s: its slot, and the inputs in front of it
+    const bool seq_ok = s >= 0 && s < g.n_seq;
+    slot = seq_ok ? g.slots[s] : -1;
+    const int r0 = seq_ok ? (g.seq_rows ? g.seq_rows[s] : t) : t;
+    live = slot >= 0 && slot < g.n_slots && r0 >= 0 && r0 <= t;
+    if (M == 0 || !live) return;
+    const T* tl = (const T*)g.tail + (int64_t)slot * M * C + c;
+    const int64_t p = g.pos[t];
+#pragma unroll
+    for (int m = 0; m < M; ++m) {  // h[m]: the input at position p - M + m
+      const int back = M - m, rel = t - r0 - back;  // its row in this step's run of the sequence
+#pragma unroll
+      for (int e = 0; e < V; ++e) h[m][e] = 0.f;
+      if (p >= back) VecIO<T, V>::ld(rel >= 0 ? x + (int64_t)(r0 + rel) * g.xs : tl + (int64_t)(rel + M) * C, h[m]);
+    }
+  };
+  enter(t0);
+#pragma unroll
+  for (int i = 0; i < R; ++i) {
+    const int t = t0 + i;
+    if (t >= g.T) break;
+    if (i > 0 && !one) {
+      const int s2 = seq_of(t);
+      if (s2 != s) {
+        s = s2;
+        enter(t);
+      }
+    }
+    float xi[V], y[V];
+    chunk_to_f32<T>(in[i], xi);
+#pragma unroll
+    for (int e = 0; e < V; ++e) {
+      float a = b[e];
+#pragma unroll
+      for (int m = 0; m < M; ++m) a += w[m][e] * h[m][e];
+      a += w[M][e] * xi[e];
+      if (g.silu) a *= fast_sigmoid(a);
+      y[e] = live ? a : 0.f;
+    }
+    VecIO<T, V>::st((T*)g.q_out + (int64_t)t * C + c, y);
+    if constexpr (M > 0) {
+#pragma unroll
+      for (int m = 0; m + 1 < M; ++m)
+#pragma unroll
+        for (int e = 0; e < V; ++e) h[m][e] = h[m + 1][e];
+#pragma unroll
+      for (int e = 0; e < V; ++e) h[M - 1][e] = xi[e];
+      if (R == 1 && new_tail && live) {
+#pragma unroll
+        for (int m = 0; m < M; ++m) VecIO<T, V>::st(new_tail + ((int64_t)slot * M + m) * C + c, h[m]);
+      }
+    }
+  }
+}
+
+template <typename T, int V, int TAPS> void launch_conv_run(const ConvArgs& g, hipStream_t st) {
+  const int gx = (g.d / V + 127) / 128;
+  if (!g.row_seq)
+    hipLaunchKernelGGL((conv_run_kernel<T, V, TAPS, 1>), dim3(gx, g.T), dim3(128), 0, st, g, (T*)g.tail);
+  else
+    hipLaunchKernelGGL((conv_run_kernel<T, V, TAPS, 8>), dim3(gx, (g.T + 7) / 8), dim3(128), 0, st, g, (T*)nullptr);
+}
+
 // tail [slots, m, C] <- the last m projected rows of every sequence of the step
 template <typename T>
 __global__ void __launch_bounds__(256) conv_state_update_kernel(T* __restrict__ tail, int n_slots,
@@ -569,7 +658,7 @@ __global__ void __launch_bounds__(256) head_norm_gate_kernel(T* __restrict__ out
       if (w) y[i] *= w[h * dv + e + i];
       if (gate) {  // gate_act 0: sigmoid(z); 1: silu, z sigmoid(z)
         const float z = ldf<T>(gate, row * gs + h * dv + e + i);
-        y[i] *= gate_act ? z * sigmoidf_(z) : sigmoidf_(z);
+        y[i] *= gate_act ? z * fast_sigmoid(z) : fast_sigmoid(z);
       }
     }
     if constexpr (V == 2 && sizeof(T) == 2) {
@@ -614,7 +703,7 @@ __global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out
       VecIO<T, V>::ld(zp + e, b);
     }
 #pragma unroll
-    for (int i = 0; i < V; ++i) x[i] = a[i] * b[i] * sigmoidf_(b[i]);
+    for (int i = 0; i < V; ++i) x[i] = a[i] * b[i] * fast_sigmoid(b[i]);
   };
   float x[kGnKeep][V], ss = 0.f;
 #pragma unroll
@@ -709,6 +798,36 @@ int dxm_conv_rope_cache(void* q_out, const void* x, int64_t xs, const float* cw,
   if (vec && f32) hipLaunchKernelGGL((conv_rope_cache_vec_kernel<float, 4>), vgrid, dim3(128), kConvRows * lds, st, g);
   else if (vec) hipLaunchKernelGGL((conv_rope_cache_vec_kernel<bf16_t, 8>), vgrid, dim3(128), kConvRows * lds, st, g);
   else { DISPATCH_T(f32, hipLaunchKernelGGL(conv_rope_cache_kernel<T>, dim3(T_), dim3(256), lds, st, g)); }
+  DX_CHECK_LAUNCH();
+  return 0;
+}
+
+// The convolution alone, for 1 to 4 taps and channels in whole 16-byte runs (any other: returns 1 and does
+// nothing; dxm_conv_rope_cache takes every size).  A step of one row per sequence (row_seq null) also leaves the
+// new tail in `tail`; a step of longer runs leaves it to dxm_conv_state_update.
+int dxm_conv_run_ok(int64_t xs, int C, int taps, int T_, uint64_t ptrs, int f32) {
+  const int V = f32 ? 4 : 8;
+  return taps >= 1 && taps <= 4 && C > 0 && C % V == 0 && xs % V == 0 && ptrs % 16 == 0 && T_ < 65535;
+}
+
+int dxm_conv_run(void* out, const void* x, int64_t xs, const float* cw, const float* cb, int silu, int taps, void* tail,
+                 int n_slots, const int64_t* pos, const int* row_seq, const int* seq_rows, const int* slots, int n_seq,
+                 int T_, int C, int f32, hipStream_t st) {
+  if (T_ <= 0) return 0;
+  const uint64_t ptrs = (uint64_t)out | (uint64_t)x | (uint64_t)cw | (uint64_t)tail;
+  if (!dxm_conv_run_ok(xs, C, taps, T_, ptrs, f32)) return 1;
+  if (!out || !x || !cw || !pos || !slots || (taps > 1 && !tail)) return 2;
+  if ((row_seq == nullptr) != (seq_rows == nullptr) || (!row_seq && n_seq != T_)) return 3;
+  ConvArgs g{out, x, xs, cw, cb, silu, taps, tail, n_slots, pos, nullptr, row_seq, seq_rows, slots, n_seq, T_,
+             1, 0, C, 0, nullptr, 0, nullptr, nullptr};
+#define CONV_RUN(TAPS) \
+  if (f32) launch_conv_run<float, 4, TAPS>(g, st); \
+  else launch_conv_run<bf16_t, 8, TAPS>(g, st);
+  if (taps == 1) { CONV_RUN(1) }
+  else if (taps == 2) { CONV_RUN(2) }
+  else if (taps == 3) { CONV_RUN(3) }
+  else { CONV_RUN(4) }
+#undef CONV_RUN
   DX_CHECK_LAUNCH();
   return 0;
 }

@@ -15,7 +15,7 @@ in the activation dtype:
          norm_rope_cache(p_q, p_k, p_v)                 HIP  one RMS norm over all heads of q (of k), rotary
                                                              (interleaved pairs), K / V into the paged caches
     a  = attention(q, K, V)                             HIP  tile kernel (prompt chunks) / grouped decode / row kernel
-    c  = conv_rope_cache(p_x|B|C, bias, silu)           HIP  short causal convolution over time, tail state per slot
+    c  = causal_conv(p_x|B|C, bias, silu)               HIP  short causal convolution over time, tail state per slot
     s  = ssd(c_x, c_B, c_C, p_dt; S)                    HIP  S <- exp(-rate u) S + u B x^T, y = S^T C + D x, fp32
     o  = [left_scale a sigmoid(p_g) |                   HIP  act_mul, gate_group_norm: both write their part of
           right_scale groupnorm(s silu(p_z)) w]              the one row that the output projection reads
@@ -355,11 +355,8 @@ class PovuraxForCausalLM:
                          self._parts(T, H, H // G, meta), False, *tl)
         mx.act_mul(p[:, g0:z0], y.view(T, nv), "sigmoid", out=o[:, :nv], scale=L["left_scale"])
         # right: state-space mixer
-        u = p[:, c0:c0 + C]
-        xbc = rc.conv_rope_cache(u, L["conv_w"], tail, meta.positions, meta.slot_mapping,
-                                 meta.row_seq if meta.is_prefill else None, meta.seq_rows, meta.state_slots, 1, 0, C, 0,
-                                 None, None, None, bias=L["conv_b"], act="silu")
-        rc.conv_state_update(u, tail, meta.positions, meta.seq_rows, meta.state_slots)
+        xbc = rc.causal_conv(p[:, c0:c0 + C], L["conv_w"], tail, meta.positions, meta.row_seq if meta.is_prefill else None,
+                             meta.seq_rows, meta.state_slots, bias=L["conv_b"], act="silu")
         y = rc.ssd(xbc[:, :inner], xbc[:, inner:inner + Gs * N], xbc[:, inner + Gs * N:], p[:, c0 + C:c0 + C + Hs],
                    L["dt_bias"], L["rate"], L["skip"], state, meta.positions, meta.seq_rows, meta.state_slots, Hs, Gs, N, P)
         rc.gate_group_norm(y, p[:, z0:c0], L["gn"], b["norm_groups"], eps, self.dtype, out=o[:, nv:])

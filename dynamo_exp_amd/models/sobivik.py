@@ -13,7 +13,7 @@ is the embedding output and plane i + 1 starts as layer i's input (the depth
 average of planes 0 .. i) and is updated in place into layer i's result:
 
   x, h = depth_mix(planes 0..i, dwa of layer i-1)          HIP  weighted sum over depth + rms(x) g1: one pass
-  h    = h + conv(h)                                       HIP  conv_rope_cache (taps over time; tail state per slot)
+  h    = h + conv(h)                                       HIP  causal_conv (taps over time; tail state per slot)
   attention (differential)
     p  = h @ [Wq | Wk | Wv | Wg]^T                         hipBLASLt, one fused projection
          headprep_cache: K (two maps per head), V -> pages HIP
@@ -444,12 +444,8 @@ class SobivikForCausalLM:
         for i, L in enumerate(self.layers):
             ci, ri = self._state_index[i]
             if ci is not None:
-                cstate = meta.state[ci]
-                hc = rc.conv_rope_cache(h, L["canon_w"], cstate, meta.positions, meta.slot_mapping,
-                                        meta.row_seq if meta.is_prefill else None, meta.seq_rows, meta.state_slots,
-                                        1, 0, W, 0, None, None, None)
-                rc.conv_state_update(h, cstate, meta.positions, meta.seq_rows, meta.state_slots)
-                h = hc
+                h = rc.causal_conv(h, L["canon_w"], meta.state[ci], meta.positions,
+                                   meta.row_seq if meta.is_prefill else None, meta.seq_rows, meta.state_slots)
             kc, vc = kv_caches[i]
             if L["type"] == "attention":
                 y = self._diff_attention(L, h, meta, kc, vc, seq, tables, bs)

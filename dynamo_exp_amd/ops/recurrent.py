@@ -252,6 +252,39 @@ def conv_state_update(x: torch.Tensor, conv_state: torch.Tensor, positions: torc
                            _f32(x), _stream())
 
 
+def causal_conv(x: torch.Tensor, conv_w: torch.Tensor, conv_state: torch.Tensor, positions: torch.Tensor,
+                row_seq: torch.Tensor | None, seq_rows: torch.Tensor | None, state_slots: torch.Tensor,
+                bias: torch.Tensor | None = None, act: str | None = None) -> torch.Tensor:
+    """The short convolution of conv_rope_cache alone -- on x [T, C], a column
+    section, with optional bias and act 'silu' -- together with the update of its
+    state: conv_state [slots, taps - 1, C] then holds the last taps - 1 rows of x of
+    every sequence of the step.  Returns [T, C]."""
+    T, C = x.shape
+    taps = conv_w.shape[0]
+    if x.is_cuda and _m().conv_run_ok(x.stride(0), C, taps, T, x.data_ptr() | conv_w.data_ptr() | conv_state.data_ptr(),
+                                      _f32(x)):
+        _fp32_param(conv_w, "conv_w")
+        _fp32_param(bias, "bias")
+        _check_step(positions, seq_rows, state_slots)
+        if act not in (None, "silu") or conv_w.shape[1] != C or (bias is not None and bias.numel() != C) or \
+                x.stride(1) != 1 or conv_state.shape[1:] != (taps - 1, C) or conv_state.dtype != x.dtype or \
+                not conv_state.is_contiguous():
+            raise ValueError("causal_conv: one weight column, bias and state column per channel of x, in its dtype")
+        if (row_seq is None) != (seq_rows is None) or (row_seq is not None and row_seq.dtype != torch.int32):
+            raise TypeError("causal_conv: int32 row_seq together with seq_rows")
+        out = torch.empty((T, C), dtype=x.dtype, device=x.device)
+        _m().conv_run(out.data_ptr(), x.data_ptr(), x.stride(0), conv_w.data_ptr(), _ptr(bias), int(act == "silu"), taps,
+                      conv_state.data_ptr(), conv_state.shape[0], positions.data_ptr(), _ptr(row_seq), _ptr(seq_rows),
+                      state_slots.data_ptr(), state_slots.numel(), T, C, _f32(x), _stream())
+        if row_seq is not None:  # (a decode step's kernel has written the new state)
+            conv_state_update(x, conv_state, positions, seq_rows, state_slots)
+        return out
+    out = conv_rope_cache(x, conv_w, conv_state, positions, torch.full_like(positions, -1), row_seq, seq_rows, state_slots,
+                          1, 0, C, 0, None, None, None, bias=bias, act=act)
+    conv_state_update(x, conv_state, positions, seq_rows, state_slots)
+    return out
+
+
 # ----------------------------------------------------------------- generalized delta rule
 DELTA_DECAY_SCALE = math.exp(-0.5)
 

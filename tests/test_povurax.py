@@ -318,7 +318,7 @@ def test_norm_rope_cache_alone(device, dtype, H, G, d, dv, dims):
 
 
 @pytest.mark.parametrize("device", DEVICES)
-@pytest.mark.parametrize("taps,C", [(4, 72), (1, 32), (5, 102), (2, 1), (8, 64)])
+@pytest.mark.parametrize("taps,C", [(4, 72), (1, 32), (5, 102), (2, 1), (8, 64), (2, 1040), (3, 24), (4, 30)])
 def test_convolution_bias_silu_alone(device, taps, C):
     """The short convolution with bias and silu, two sequences in portions down to one row (shorter than the
     taps), slots reused with garbage in them, channels that are a section of wider rows."""
@@ -328,11 +328,12 @@ def test_convolution_bias_silu_alone(device, taps, C):
     want = [O.silu(O.channel_conv(x[s].double(), w.double(), b.double())) for s in range(2)]
     tail = torch.randn(4, taps - 1, C, device=device)
     got = [[], []]
-    for live, cuts, (pos, row_seq, seq_rows, slots) in interleave([[1, 1, 2, 9, 1, 9], [23]], [2, 0], device):
+    for live, cuts, (pos, row_seq, seq_rows, slots) in interleave([[1, 1, 2, 8, 1, 9, 1], [1, 1, 19, 1, 1]], [2, 0], device):
         xs = section(torch.cat([x[s, p:p + n] for s, (p, n) in zip(live, cuts)]), 8, device)
-        y = rc.conv_rope_cache(xs, w.t().contiguous().to(device), tail, pos, torch.zeros_like(pos), row_seq, seq_rows, slots,
-                               1, 0, C, 0, None, None, None, bias=b.to(device), act="silu")
-        rc.conv_state_update(xs, tail, pos, seq_rows, slots)
+        if all(n == 1 for _, n in cuts):  # a decode step: row i is sequence i
+            row_seq = seq_rows = None
+        y = rc.causal_conv(xs, w.t().contiguous().to(device), tail, pos, row_seq, seq_rows, slots, bias=b.to(device), act="silu")
+        seq_rows = torch.tensor([0] + [n for _, n in cuts]).cumsum(0)
         for i, s in enumerate(live):
             got[s].append(y[int(seq_rows[i]):int(seq_rows[i + 1])].cpu())
     for s in range(2):
