@@ -71,6 +71,9 @@ int dxm_tile_attention(void*, const void*, int64_t, const void*, const void*, co
 int dxm_group_decode(float*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
                      int, int, int, int, int, int, int, int, int, float, int, int, float, const float*, const float*, int,
                      const float*, int, int, hipStream_t);
+int dxm_stream_decode_ok(int, int, int, int, int);
+int dxm_stream_decode(float*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
+                      int, int, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
 int dxm_merge_parts(void*, const float*, int64_t, int, int, int, const void*, int64_t, int, int, const float*, int,
                     hipStream_t);
 }
@@ -235,7 +238,15 @@ PYBIND11_MODULE(_C_mixers, m) {
                            int n_qh, int maps, int group, int d, int dv, int Wk, int Wv, float scale, int mask,
                            int size, float cap, u r1, u r2, int wfn, u hbias, u gate, int64_t gs, int keep, u sink,
                            int parts, int out_f32, u st) {
-    check(dxm_group_decode(F(ws), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
+    // plain heads over pages of whole tiles take the streaming kernel (same workspace)
+    if (cap == 0.f && !r1 && !wfn && !hbias && !keep && qs % 8 == 0 && (q | kc | vc) % 16 == 0 &&
+        dxm_stream_decode_ok(d, dv, group, bs, mask))
+      check(dxm_stream_decode(F(ws), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
+                              reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs, rows, n_qh,
+                              maps, group, d, dv, Wk, Wv, scale, mask, size, parts, S(st)),
+            "stream_decode");
+    else
+      check(dxm_group_decode(F(ws), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
                            reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs, rows, n_qh,
                            maps, group, d, dv, Wk, Wv, scale, mask, size, cap, F(r1), F(r2), wfn, F(hbias), keep,
                            parts, S(st)),

@@ -376,7 +376,7 @@ def test_gates_and_clamp_alone(device, F):
 
 # ----------------------------------------------------------------- crafted: one key stands out
 @pytest.mark.parametrize("device,dtype", CASES)
-@pytest.mark.parametrize("d,dv,bs", [(32, 32, 16), (12, 20, 8), (64, 128, 8)])
+@pytest.mark.parametrize("d,dv,bs", [(32, 32, 16), (12, 20, 8), (64, 128, 8), (128, 128, 64), (64, 64, 128)])
 def test_far_keys(device, dtype, d, dv, bs):
     """A cache of empty keys in which one matches the query strongly and carries a marked value: the first
     token, page borders, among hundreds, the query's own token; a key just behind the query is not seen.
@@ -408,6 +408,38 @@ def test_far_keys(device, dtype, d, dv, bs):
                 got = mx.attention(q, kc, vc, pos, seq, table, bs, H, 1, H // G, d, dv, 0.25, "causal", 0, parts, False, *tl)
                 err = float((got.float() - want).abs().max())
                 assert err < (1e-4 if dtype == "float32" else 2e-2), (p, mark, seq is None, parts, err)
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("d,n_qh,G,maps,bs", [(128, 8, 2, 1, 64), (64, 3, 1, 1, 128), (128, 16, 1, 1, 64), (64, 4, 2, 2, 64)])
+@pytest.mark.parametrize("size", [0, 1, 64, 65, 100])
+def test_decode_rows_over_whole_tile_pages(d, n_qh, G, maps, bs, size):
+    """bf16 decode rows over pages of whole 64-key tiles (the streaming kernel): rows at tile and page edges
+    and at position 0, keys in parts, windows that start inside a tile, pages whose unused rows hold NaN."""
+    torch.manual_seed(d + size)
+    ps = [0, 1, 63, 64, 127, 128, 299]
+    n_kh, group, B = G * maps, n_qh // maps // G, len(ps)
+    T, per = 300, -(-300 // bs)
+    k, v = torch.randn(B, T, n_kh, d).bfloat16(), torch.randn(B, T, G, d).bfloat16()
+    q = torch.randn(B, n_qh, d).bfloat16()
+    table = torch.randperm(B * per, generator=torch.Generator().manual_seed(1)).to(torch.int32).view(B, per)
+    kc = torch.full((B * per * bs, n_kh * d), float("nan"), dtype=torch.bfloat16)
+    vc = torch.full((B * per * bs, G * d), float("nan"), dtype=torch.bfloat16)
+    want = torch.zeros(B, n_qh, d, dtype=torch.float64)
+    for b, p in enumerate(ps):
+        j = torch.arange(p + 1)
+        sl = table[b].long()[j // bs] * bs + j % bs
+        kc[sl], vc[sl] = k[b, :p + 1].reshape(p + 1, -1), v[b, :p + 1].reshape(p + 1, -1)
+        near = j[max(0, p - size + 1) if size else 0:]
+        for h in range(n_qh):
+            head, mp = h // maps, h % maps
+            w = torch.softmax((k[b, near, head // group * maps + mp].double() @ q[b, h].double()) * 0.3, 0)
+            want[b, h] = w @ v[b, near, head // group].double()
+    pos = torch.tensor(ps).cuda()
+    for parts in (1, 3):
+        got = mx.attention(q.reshape(B, -1).cuda(), kc.cuda(), vc.cuda(), pos, None, table.cuda(), bs, n_qh, maps, group, d, d,
+                           0.3, "window" if size else "causal", size, parts, True)
+        assert float((got.cpu().double() - want).abs().max()) < 1e-3 * max(1.0, float(want.abs().max()))
 
 
 # ----------------------------------------------------------------- whole model
