@@ -26,9 +26,11 @@ template <typename T> __device__ __forceinline__ float2 step_terms(const ScanArg
   return float2{u, expf(-g.rate[h] * u)};
 }
 
+constexpr int kMaxKey = 512;
+
 // Any sizes: rows and columns beyond dk / dv are guarded one by one.  Lane r of a column's group owns
 // rows r, r + R, ...
-template <typename T, int R, int MODE>
+template <typename T, int R, int MODE, int ROWS = kRows>
 __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
   extern __shared__ float scan_lds[];
   const int s = blockIdx.x, h = blockIdx.y, hq = h / g.qk_rep;
@@ -51,9 +53,9 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
   float* gs_ = vs_ + kTok * cols;  // kStep: (step, decay) per token; kChannel: [kTok][dk] decays
   float* sp = g.state + (((int64_t)slot * g.H + h) * g.dv + (colok ? j : 0)) * g.dk;
   const bool fresh = g.pos[r0] == 0;
-  float S[kRows];
+  float S[ROWS];
 #pragma unroll
-  for (int ii = 0; ii < kRows; ++ii) {
+  for (int ii = 0; ii < ROWS; ++ii) {
     const int i = r + R * ii;
     S[ii] = (!fresh && colok && i < g.dk) ? sp[i] : 0.f;
   }
@@ -93,7 +95,7 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
       const float* gt = gs_ + tt * g.dk;
       float acc = 0.f;
 #pragma unroll
-      for (int ii = 0; ii < kRows; ++ii) {
+      for (int ii = 0; ii < ROWS; ++ii) {
         const int i = r + R * ii;
         if (i < g.dk) {
           S[ii] = (MODE == kChannel ? gt[i] : dec) * S[ii] + kt[i] * uv;
@@ -106,7 +108,7 @@ __global__ void __launch_bounds__(256) scan_kernel(ScanArgs g) {
   }
   if (colok) {
 #pragma unroll
-    for (int ii = 0; ii < kRows; ++ii) {
+    for (int ii = 0; ii < ROWS; ++ii) {
       const int i = r + R * ii;
       if (i < g.dk) sp[i] = S[ii];
     }
@@ -263,17 +265,19 @@ bool scan_fast_ok(const ScanArgs& g) {
          (MODE != kChannel || (g.gs % VEC == 0 && al(g.g)));
 }
 
-template <typename T, int R, int MODE>
+template <typename T, int R, int MODE, int ROWS = kRows>
 void launch_scan(const ScanArgs& g, int n_seq, hipStream_t st) {
-  if (scan_fast_ok<T, R, MODE>(g)) {
-    hipLaunchKernelGGL((scan_fast_kernel<T, R, MODE>), dim3(n_seq, g.H, g.dv / (256 / R)), dim3(256), 0, st, g);
-    return;
+  if constexpr (ROWS == kRows) {
+    if (scan_fast_ok<T, R, MODE>(g)) {
+      hipLaunchKernelGGL((scan_fast_kernel<T, R, MODE>), dim3(n_seq, g.H, g.dv / (256 / R)), dim3(256), 0, st, g);
+      return;
+    }
   }
   int nt = (R * g.dv + 63) / 64 * 64;
   nt = nt > 256 ? 256 : nt;
   const int cols = nt / R;
   const size_t lds = (size_t)((MODE == kChannel ? 3 : 2) * kTok * g.dk + kTok * cols + 2 * kTok) * sizeof(float);
-  hipLaunchKernelGGL((scan_kernel<T, R, MODE>), dim3(n_seq, g.H, (g.dv + cols - 1) / cols), dim3(nt), lds, st, g);
+  hipLaunchKernelGGL((scan_kernel<T, R, MODE, ROWS>), dim3(n_seq, g.H, (g.dv + cols - 1) / cols), dim3(nt), lds, st, g);
 }
 
 template <typename T, int MODE>
@@ -283,7 +287,8 @@ void dispatch_rows(const ScanArgs& g, int n_seq, hipStream_t st) {
   else if (need <= 2) launch_scan<T, 2, MODE>(g, n_seq, st);
   else if (need <= 4) launch_scan<T, 4, MODE>(g, n_seq, st);
   else if (need <= 8) launch_scan<T, 8, MODE>(g, n_seq, st);
-  else launch_scan<T, 16, MODE>(g, n_seq, st);
+  else if (need <= 16) launch_scan<T, 16, MODE>(g, n_seq, st);
+  else launch_scan<T, 16, MODE, kMaxKey / 16>(g, n_seq, st);
 }
 
 }  // namespace
@@ -295,7 +300,7 @@ extern "C" int dxm_linear_scan(int mode, float* out, float* state, int n_slots, 
                                const int* slots, int n_seq, int T_, int H, int dk, int dv, int f32, hipStream_t st) {
   if (n_seq <= 0 || T_ <= 0) return 0;
   if (H < 1 || dk < 1 || dv < 1 || n_slots < 1 || H > 65535 || (int64_t)T_ * H * dv > 0x7fffffffffffLL) return 1;
-  if (dk > kRows * 16) return 2;  // wider keys need more lanes per column than instantiated
+  if (dk > kMaxKey) return 2;  // wider keys need more rows per lane than instantiated
   if (!out || !state || !pos || !slots || !q || !k || !v) return 3;
   if (!seq_rows && n_seq != T_) return 4;
   if (qk_rep < 1 || H % qk_rep) return 5;

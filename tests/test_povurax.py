@@ -114,7 +114,7 @@ def close(got, want, dtype, what=""):
     if dtype == "float32":
         assert float(err.max()) < 3e-4, f"{what}: error {float(err.max()):.3g} at row {int(err.argmax())}"
     else:
-        assert float(err.median()) < 4e-2 and float((err > 8e-2).float().mean()) <= 0.2, \
+        assert float(err.median()) < 2e-2 and float((err > 6e-2).float().mean()) <= 0.05, \
             f"{what}: median error {float(err.median()):.3g}, max {float(err.max()):.3g}"
 
 
@@ -178,7 +178,7 @@ def check_scan(device, run, want, state):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("H,G,N,P", [(4, 2, 14, 10), (1, 1, 1, 1), (2, 1, 128, 64), (4, 4, 16, 256), (3, 1, 33, 7),
-                                     (8, 2, 64, 64), (2, 2, 256, 16), (6, 3, 32, 48), (2, 1, 200, 3)])
+                                     (8, 2, 64, 64), (2, 2, 256, 16), (6, 3, 32, 48), (2, 1, 200, 3), (2, 1, 300, 5)])
 def test_ssd_scan_alone(device, dtype, H, G, N, P):
     """The state-space recurrence with its step sizes, shared B / C groups and skip, then a decode step
     with a padding row; x, B, C, dt are sections of wider rows."""
@@ -210,7 +210,7 @@ def test_ssd_scan_alone(device, dtype, H, G, N, P):
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("H,dk,dv,tau", [(3, 10, 14, 8.0), (1, 1, 1, 1.0), (2, 64, 64, 16.0), (2, 128, 32, 4.0), (1, 34, 3, 2.0),
                                          (1, 16, 256, 16.0), (2, 256, 32, 16.0), (1, 48, 40, 0.5), (2, 32, 128, 16.0),
-                                         (1, 64, 64, 0.25), (1, 128, 64, 0.5)])
+                                         (1, 64, 64, 0.25), (1, 128, 64, 0.5), (1, 512, 2, 16.0)])
 def test_gla_scan_alone(device, dtype, H, dk, dv, tau):
     """Gated linear attention: a decay per key channel, from hardly any to nearly total (logits far below
     zero, where the decay is a power of e / tau, and far above), then a decode step with a padding row."""
@@ -392,7 +392,8 @@ def test_far_keys(device, dtype, d, dv, bs):
     q = e0.repeat(H)[None].to(device, dt)
     kc = torch.zeros(48 * bs, G * d, device=device, dtype=dt)
     vc = torch.zeros(48 * bs, G * dv, device=device, dtype=dt)
-    for p in (T - 1, 150, bs * 9, bs * 9 - 1, 1, 0):
+    for p in {T - 1, 150, T // bs * bs, T // bs * bs - 1, bs, 1, 0}:
+        assert p < T
         for mark in {0, 1, p, p + 1, p - 1, bs - 1, bs, p // bs * bs, p // bs * bs - 1}:
             if not 0 <= mark < T:
                 continue
