@@ -27,7 +27,6 @@ __device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p, const bf16_t* p16) 
   const uint2 a = *reinterpret_cast<const uint2*>(p), b = *reinterpret_cast<const uint2*>(p16);
   return as_bf16x8(raw_u32x4{a.x, a.y, b.x, b.y});
 }
-__device__ __forceinline__ bf16x8_t frag4_4(const bf16_t* p) { return frag4_4(p, p + 16); }
 
 // hi + lo bf16 parts of four floats
 __device__ __forceinline__ void split4(const float* v, uint2& hi, uint2& lo) {
@@ -54,9 +53,6 @@ __device__ __forceinline__ uint2 column4(const raw_u32x4* r, int e) {
 
 __device__ __forceinline__ f32x4 mfma32(bf16x8_t a, bf16x8_t b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
-}
-__device__ __forceinline__ f32x4 mfma16(uint2 a, uint2 b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x16bf16_1k(__builtin_bit_cast(i16x4, a), __builtin_bit_cast(i16x4, b), c, 0, 0, 0);
 }
 
 // inclusive sums over the 64 lanes: within rows of 16, then the last lane of a row (of a half) into the next
@@ -294,30 +290,34 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
 }
 
 // ---------------------------------------------------------------------------
-// A decay per token and key channel (kChannel): chunks of 16 tokens, so that the
-// products between a chunk's tokens are one tile.  With L the log decays summed
-// from the chunk's start, the decay of a pair factors per channel into e^L of the
-// query token and e^-L of the key token, and
+// A decay per token and key channel (kChannel): chunks of 32 tokens.  With L the
+// log decays summed from the chunk's start, the decay of a pair factors per channel
+// into e^L of the query token and e^-L of the key token, and
 //     S <- e^L(end) (S + sum_s (k_s e^-L(s)) v_s^T)
 // takes the same scaled keys.  Where a channel decays so far inside a chunk that
 // e^-L would leave the number range, the pairs are summed one by one with
 // exponent differences, and the scaled keys carry e^(L(end) - L(s)) instead, with
 // e^L(end) on S alone.
-// Four waves (the upper ones) form a chunk's operands, one chunk ahead, in the
+// Eight waves (the upper ones) form a chunk's operands, one chunk ahead, in the
 // other half of the double-buffered LDS; the lower four run the matrix products.
-// In an upper wave the lanes of one DPP row of 16 hold the 16 tokens of the same
-// eight channels, so the running log decays are row scans.
+// The lanes of half an upper wave hold the 32 tokens of the same eight channels,
+// so the running log decays are DPP scans.  Channels and tokens are stored in the
+// order of the k-slots (slot_of32), so that every fragment is one 16-byte read.
 template <int DK> struct ChannelBuf {
-  static constexpr int KP = DK + 8, SP = 20;
-  bf16_t qi[2][16 * KP];  // hi, lo of q e^L                  [t][n]
-  bf16_t km[2][16 * KP];  //           k e^-L                 [s][n]
+  static constexpr int KP = DK + 8, SP = 40;
+  bf16_t qi[2][32 * KP];  // hi, lo of q e^L                  [t][n]
+  bf16_t km[2][32 * KP];  //           k e^-L                 [s][n]
   bf16_t ke[2][DK * SP];  //           the same, transposed   [n][s]
   bf16_t vT[kPB * SP];    // v [p][s]
   float eq[DK];           // e^L(end)
-  int far[4];             // per forming wave: e^-L would leave the number range
+  int far[8];             // per forming wave (16 channels): e^-L would leave the number range
 };
 
 constexpr float kFarLog2 = 96.f;  // log2 of the largest e^-L used as a factor
+constexpr int kFormThreads = 512, kProdThreads = 256;
+
+// place of element i of a run of 32: group g's slots are {4 g .. + 3, 16 + 4 g .. + 3}
+__device__ __forceinline__ int slot_of32(int i) { return 8 * ((i >> 2) & 3) + 4 * (i >> 4) + (i & 3); }
 
 // log2 of sigmoid(z)^(1 / tau)
 __device__ __forceinline__ float channel_log2(float z, float inv_tau) {
@@ -326,15 +326,16 @@ __device__ __forceinline__ float channel_log2(float z, float inv_tau) {
 }
 
 template <int DK>
-__global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
+__global__ void __launch_bounds__(kFormThreads + kProdThreads, 3) channel_chunk_kernel(ScanArgs g) {
   using Buf = ChannelBuf<DK>;
-  constexpr int Q = 16, KP = Buf::KP, SP = Buf::SP, NM = DK / 16, NK = DK / 32;
+  constexpr int Q = 32, KP = Buf::KP, SP = Buf::SP, NM = DK / 16, NK = DK / 32;
   static_assert(DK % 32 == 0 && DK <= 128, "one staged item per thread");
   __shared__ __attribute__((aligned(16))) Buf bufs[2];
   Walk w;
   if (!open_walk(g, w)) return;
-  const bool former = threadIdx.x >= 256;
-  const int tid = threadIdx.x & 255, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
+  const bool former = threadIdx.x >= kProdThreads;
+  const int tid = former ? threadIdx.x - kProdThreads : threadIdx.x;
+  const int wave = tid >> 6, lane = tid & 63;
   const bf16_t* q = (const bf16_t*)g.q + (int64_t)w.r0 * g.qs + (int64_t)w.hq * DK;
   const bf16_t* k = (const bf16_t*)g.k + (int64_t)w.r0 * g.ks + (int64_t)w.hq * DK;
   const bf16_t* z = (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + (int64_t)w.h * DK;
@@ -342,10 +343,12 @@ __global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
   const float* zb = g.g_bias ? g.g_bias + w.h * DK : nullptr;
 
   if (former) {  // ---- operands of the chunks
-    const int oc = tid >> 4;  // token c16, channel octet (q, k, decays)
+    const int tok = lane & 31, oc = 2 * wave + (lane >> 5);  // token, channels 8 oc .. + 7 (q, k, decays)
     const bool has_k = oc < DK / 8;
-    const int ov = oc - (16 - kPB / 8);  // ... column octet (v, the upper threads)
+    const int ov = oc - (16 - kPB / 8);  // ... columns 8 ov .. + 7 (v, the last waves)
     const bool has_v = ov >= 0;
+    const int ts = slot_of32(tok);
+    const int n0 = (8 * oc & ~31) + slot_of32(8 * oc & 31), n1 = (8 * oc & ~31) + slot_of32((8 * oc & 31) + 4);
     float bias[8];
 #pragma unroll
     for (int e = 0; e < 8; ++e) bias[e] = zb && has_k ? zb[8 * oc + e] : 0.f;
@@ -353,7 +356,7 @@ __global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
     bool live = false;
     auto fetch = [&](int t0) {
       const raw_u32x4 zero{0u, 0u, 0u, 0u};
-      const int64_t t = t0 + c16;
+      const int64_t t = t0 + tok;
       live = t < w.n;
       rz = live && has_k ? *reinterpret_cast<const raw_u32x4*>(z + t * g.gs + 8 * oc) : zero;
       rq = live && has_k ? *reinterpret_cast<const raw_u32x4*>(q + t * g.qs + 8 * oc) : zero;
@@ -362,87 +365,92 @@ __global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
     };
     auto form = [&](Buf& b) {
       bool far = false;
-      float L[8];
+      float L[8], x[8];
       if (has_k) {
+        chunk_to_f32<bf16_t>(rz, x);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          const uint32_t zw = rz[e >> 1];
-          L[e] = row_scan_sum(live ? channel_log2((e & 1 ? bf16hi(zw) : bf16lo(zw)) + bias[e], g.inv_tau) : 0.f);
+          const float l = row_scan_sum(live ? channel_log2(x[e] + bias[e], g.inv_tau) : 0.f);
+          L[e] = l + dpp_rows<0x142, 0xa>(l);  // the second row of 16 goes on from the first one's end
           far |= L[e] < -kFarLog2;
         }
       }
       const bool any = __any(far);
-      if ((tid & 63) == 0) b.far[wave] = any;
+      if (lane == 0) b.far[wave] = any;
       if (has_k) {
-        float x[8], y[8];
+        float y[8];
         raw_u32x4 hi, lo;
-        bf16_t* at = b.qi[0] + c16 * KP + 8 * oc;
+        chunk_to_f32<bf16_t>(rq, x);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          const uint32_t qw = rq[e >> 1];
           y[e] = fast_exp2(L[e]);
-          x[e] = (e & 1 ? bf16hi(qw) : bf16lo(qw)) * g.q_scale * y[e];
+          x[e] *= y[e];
         }
-        if (c16 == 15) {
+        if (tok == 31) {
           *reinterpret_cast<f32x4*>(b.eq + 8 * oc) = f32x4{y[0], y[1], y[2], y[3]};
           *reinterpret_cast<f32x4*>(b.eq + 8 * oc + 4) = f32x4{y[4], y[5], y[6], y[7]};
         }
-        split8(x, hi, lo);
-        *reinterpret_cast<raw_u32x4*>(at) = hi;
-        *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+        auto put = [&](bf16_t(*dst)[32 * KP]) {
+          split8(x, hi, lo);
+          *reinterpret_cast<uint2*>(dst[0] + tok * KP + n0) = uint2{hi[0], hi[1]};
+          *reinterpret_cast<uint2*>(dst[0] + tok * KP + n1) = uint2{hi[2], hi[3]};
+          *reinterpret_cast<uint2*>(dst[1] + tok * KP + n0) = uint2{lo[0], lo[1]};
+          *reinterpret_cast<uint2*>(dst[1] + tok * KP + n1) = uint2{lo[2], lo[3]};
+        };
+        put(b.qi);
+        chunk_to_f32<bf16_t>(rk, x);
+        if (any) {  // (a wave with a far channel: relative to the chunk's end, for S; its pairs are summed one by one)
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const uint32_t kw = rk[e >> 1];
-          // (a wave with a far channel: relative to the chunk's end, for S; its pairs are summed one by one)
-          x[e] = (e & 1 ? bf16hi(kw) : bf16lo(kw)) * g.k_scale * fast_exp2((any ? dpp_f<0x15F>(L[e]) : 0.f) - L[e]);
+          for (int e = 0; e < 8; ++e) L[e] -= __shfl(L[e], lane | 31, 64);
         }
-        at = b.km[0] + c16 * KP + 8 * oc;
-        split8(x, hi, lo);
-        *reinterpret_cast<raw_u32x4*>(at) = hi;
-        *reinterpret_cast<raw_u32x4*>(at + 16 * KP) = lo;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) x[e] *= g.k_scale * fast_exp2(-L[e]);
+        put(b.km);
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
-          const int i = (8 * oc + e) * SP + c16;
+          const int i = (8 * oc + e) * SP + ts;
           b.ke[0][i] = (bf16_t)(e & 1 ? hi[e >> 1] >> 16 : hi[e >> 1] & 0xffffu);
           b.ke[1][i] = (bf16_t)(e & 1 ? lo[e >> 1] >> 16 : lo[e >> 1] & 0xffffu);
         }
       }
       if (has_v) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) b.vT[(8 * ov + e) * SP + c16] = (bf16_t)(e & 1 ? rv[e >> 1] >> 16 : rv[e >> 1] & 0xffffu);
+        for (int e = 0; e < 8; ++e) b.vT[(8 * ov + e) * SP + ts] = (bf16_t)(e & 1 ? rv[e >> 1] >> 16 : rv[e >> 1] & 0xffffu);
       }
     };
     fetch(0);
     form(bufs[0]);
-    if (Q < w.n) fetch(Q);
+    fetch(Q);
     for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
       __syncthreads();  // chunk t0 is formed; the other half is consumed
       if (t0 + Q < w.n) {
         form(bufs[cur ^ 1]);
-        if (t0 + 2 * Q < w.n) fetch(t0 + 2 * Q);
+        fetch(t0 + 2 * Q);
       }
     }
     return;
   }
 
   // ---- products.  (The barriers of the two loops pair up: one per chunk in each.)
+  const int c16 = lane & 15, g4 = lane >> 4;
   float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
   f32x4 S[NM];
 #pragma unroll
   for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
-  auto pair_by_pair = [&](int t0, f32x4& a) {  // a[r] = sum_n q_t k_s E(s, t), s = 4 g4 + r, t = c16
+  auto pair_by_pair = [&](int t0, int st, int tt, f32x4& a) {  // a[r] = sum_n q_t k_s E(s, t), s = 16 st + 4 g4 + r, t = 16 tt + c16
     a = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (t0 + c16 >= w.n) return;
-    const int64_t t = t0 + c16;
+    const int tl = 16 * tt + c16, s_lo = 16 * st + 4 * g4;
+    const int64_t t = t0 + tl;
+    if (t >= w.n) return;
     for (int n = 0; n < DK; ++n) {
-      const float qv = bf16_to_f32(q[t * g.qs + n]) * g.q_scale, zbn = zb ? zb[n] : 0.f;
+      const float qv = bf16_to_f32(q[t * g.qs + n]), zbn = zb ? zb[n] : 0.f;
       float E = 0.f;  // log2 decay from s to t, s walking down from t
-      for (int s = c16; s >= 4 * g4; --s) {
-        if (s < 4 * g4 + 4) {
+      for (int s = tl; s >= s_lo; --s) {
+        if (s < s_lo + 4) {
           const float x = qv * bf16_to_f32(k[(int64_t)(t0 + s) * g.ks + n]) * g.k_scale * fast_exp2(E);
 #pragma unroll
           for (int r = 0; r < 4; ++r)
-            if (s == 4 * g4 + r) a[r] += x;
+            if (s == s_lo + r) a[r] += x;
         }
         E += channel_log2(bf16_to_f32(z[(int64_t)(t0 + s) * g.gs + n]) + zbn, g.inv_tau);
       }
@@ -451,67 +459,85 @@ __global__ void __launch_bounds__(512, 2) channel_chunk_kernel(ScanArgs g) {
   for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
     __syncthreads();  // this chunk is formed
     const Buf& b = bufs[cur];
-    const int far[4] = {b.far[0], b.far[1], b.far[2], b.far[3]};
-    const uint2 vf = *reinterpret_cast<const uint2*>(b.vT + (16 * wave + c16) * SP + 4 * g4);
-    // weights of the chunk's pairs, [s][t] (every wave forms the tile it needs itself)
-    f32x4 a{0.f, 0.f, 0.f, 0.f}, a1 = a, a2 = a;
-    const bool any_far = far[0] | far[1] | far[2] | far[3];
-    if (any_far) {
-      pair_by_pair(t0, a);
-    } else {
+    int far[8], any_far = 0;
 #pragma unroll
-      for (int kk = 0; kk < NK; ++kk) {
-        const int o = c16 * KP + 32 * kk + 4 * g4;
-        const bf16x8_t kh = frag4_4(b.km[0] + o), qh = frag4_4(b.qi[0] + o);
-        a = mfma32(kh, qh, a);
-        a1 = mfma32(kh, frag4_4(b.qi[1] + o), a1);
-        a2 = mfma32(frag4_4(b.km[1] + o), qh, a2);
-      }
-    }
-    f32x4 y{0.f, 0.f, 0.f, 0.f}, y1 = y, y2 = y;
+    for (int i = 0; i < 8; ++i) far[i] = b.far[i], any_far |= far[i];
+    const bf16x8_t vf = frag8(b.vT + (16 * wave + c16) * SP + 8 * g4);
+    // the chunk's pair weights [s][t] as three 16 x 16 tiles (every wave forms what it needs itself), and S^T q:
+    // five sums, taken in turn so that dependent instructions are far apart
+    const f32x4 zero{0.f, 0.f, 0.f, 0.f};
+    f32x4 a00 = zero, a01 = zero, a11 = zero, y0 = zero, y1 = zero;
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
+      const int o0 = c16 * KP + 32 * kk + 8 * g4, o1 = o0 + 16 * KP;
+      const bf16x8_t k0 = frag8(b.km[0] + o0), k1 = frag8(b.km[0] + o1), q0 = frag8(b.qi[0] + o0), q1 = frag8(b.qi[0] + o1);
+      const bf16x8_t k0l = frag8(b.km[1] + o0), k1l = frag8(b.km[1] + o1), q0l = frag8(b.qi[1] + o0),
+                     q1l = frag8(b.qi[1] + o1);
       float s8[8];
 #pragma unroll
       for (int e = 0; e < 4; ++e) s8[e] = S[2 * kk][e], s8[4 + e] = S[2 * kk + 1][e];
       raw_u32x4 hi, lo;
       split8(s8, hi, lo);
-      const int o = c16 * KP + 32 * kk + 4 * g4;
-      const bf16x8_t qh = frag4_4(b.qi[0] + o), Sh = as_bf16x8(hi);
-      y = mfma32(Sh, qh, y);
-      y1 = mfma32(as_bf16x8(lo), qh, y1);
-      y2 = mfma32(Sh, frag4_4(b.qi[1] + o), y2);
+      const bf16x8_t Sh = as_bf16x8(hi), Sl = as_bf16x8(lo);
+      a00 = mfma32(k0, q0, a00);
+      a01 = mfma32(k0, q1, a01);
+      a11 = mfma32(k1, q1, a11);
+      y0 = mfma32(Sh, q0, y0);
+      y1 = mfma32(Sh, q1, y1);
+      a00 = mfma32(k0, q0l, a00);
+      a01 = mfma32(k0, q1l, a01);
+      a11 = mfma32(k1, q1l, a11);
+      y0 = mfma32(Sl, q0, y0);
+      y1 = mfma32(Sl, q1, y1);
+      a00 = mfma32(k0l, q0, a00);
+      a01 = mfma32(k0l, q1, a01);
+      a11 = mfma32(k1l, q1, a11);
+      y0 = mfma32(Sh, q0l, y0);
+      y1 = mfma32(Sh, q1l, y1);
     }
 #pragma unroll
     for (int m = 0; m < NM; ++m) {
-      // a forming wave covers 32 channels: its keys are relative to the chunk's start, or (far) to its end
+      // a forming wave's 16 channels: their keys are relative to the chunk's start, or (far) to its end
       const f32x4 e4 = *reinterpret_cast<const f32x4*>(b.eq + 16 * m + 4 * g4);
-      const bool late = far[m / 2];
-      const int o = (16 * m + c16) * SP + 4 * g4;
-      const uint2 kh = *reinterpret_cast<const uint2*>(b.ke[0] + o), kl = *reinterpret_cast<const uint2*>(b.ke[1] + o);
-      if (late) {
+      const int o = (16 * m + c16) * SP + 8 * g4;
+      const bf16x8_t kh = frag8(b.ke[0] + o), kl = frag8(b.ke[1] + o);
+      if (far[m]) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
       }
-      S[m] = mfma16(kh, vf, S[m]);
-      S[m] = mfma16(kl, vf, S[m]);
-      if (!late) {
+      S[m] = mfma32(kh, vf, S[m]);
+      S[m] = mfma32(kl, vf, S[m]);
+      if (!far[m]) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) S[m][r] *= e4[r];
       }
     }
-    float m4[4];
-#pragma unroll
-    for (int r = 0; r < 4; ++r) m4[r] = 4 * g4 + r <= c16 ? a[r] + (a1[r] + a2[r]) : 0.f;
-    uint2 Ah, Al;
-    split4(m4, Ah, Al);
-    y = mfma16(vf, Ah, y);
-    y1 = mfma16(vf, Al, y1);
-    if (t0 + c16 < w.n) {
-#pragma unroll
-      for (int r = 0; r < 4; ++r) y[r] += y1[r] + y2[r];
-      *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + c16) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) = y;
+    if (any_far) {
+      pair_by_pair(t0, 0, 0, a00);
+      pair_by_pair(t0, 0, 1, a01);
+      pair_by_pair(t0, 1, 1, a11);
     }
+    float w0[8], w1[8];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const bool seen = 4 * g4 + r <= c16;
+      w0[r] = seen ? a00[r] : 0.f;
+      w0[4 + r] = 0.f;
+      w1[r] = a01[r];
+      w1[4 + r] = seen ? a11[r] : 0.f;
+    }
+    raw_u32x4 h0, l0, h1, l1;
+    split8(w0, h0, l0);
+    split8(w1, h1, l1);
+    y0 = mfma32(vf, as_bf16x8(h0), y0);
+    y1 = mfma32(vf, as_bf16x8(h1), y1);
+    y0 = mfma32(vf, as_bf16x8(l0), y0);
+    y1 = mfma32(vf, as_bf16x8(l1), y1);
+    float* o = g.out + ((int64_t)(w.r0 + t0 + c16) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) y0[r] *= g.q_scale, y1[r] *= g.q_scale;
+    if (t0 + c16 < w.n) *reinterpret_cast<f32x4*>(o) = y0;
+    if (t0 + 16 + c16 < w.n) *reinterpret_cast<f32x4*>(o + (int64_t)16 * g.H * g.dv) = y1;
   }
 #pragma unroll
   for (int m = 0; m < NM; ++m) *reinterpret_cast<f32x4*>(sp + 16 * m) = S[m];
@@ -539,5 +565,5 @@ void launch_chunk_scan(int mode, const ScanArgs& g, int n_seq, hipStream_t st) {
 #define CHANNEL_K(D) channel_chunk_kernel<D>
   if (mode == kFixed) { CHUNK_DK(FIXED_K, dim3(256)) }
   else if (mode == kStep) { CHUNK_DK(STEP_K, dim3(256)) }
-  else { CHUNK_DK(CHANNEL_K, dim3(512)) }
+  else { CHUNK_DK(CHANNEL_K, dim3(kFormThreads + kProdThreads)) }
 }
