@@ -1,8 +1,8 @@
 // Chunked, matrix-core form of the linear recurrences for prompt portions in
 // bf16 (the token-by-token form and the definitions: linear_scan.hip).  One
-// workgroup of four waves walks a sequence's rows of one (head, 64 columns)
-// chunk by chunk; wave w owns 16 columns p of the running matrix, which stays in
-// fp32 accumulators for the whole walk.  With E(a, b) the decay from token a to
+// workgroup walks a sequence's rows of one (head, 64 columns) chunk by chunk;
+// each of its four product waves owns 16 columns p of the running matrix, which
+// stays in fp32 accumulators for the whole walk.  With E(a, b) the decay from token a to
 // token b, a chunk is three products,
 //     o_t = E(start, t) S^T q_t + sum_(s <= t) (q_t . E(s, t) k_s) u_s v_s,
 //     S  <- E(start, end) S + sum_s (E(s, end) u_s k_s) v_s^T.
@@ -102,8 +102,10 @@ __device__ __forceinline__ bool open_walk(const ScanArgs& g, Walk& w) {
 // ---------------------------------------------------------------------------
 // One decay per token and head (kFixed, kStep): chunks of 64 tokens.  The decays
 // between the chunk's tokens form a [64, 64] matrix of their own, which
-// multiplies the q k^T products element by element: each wave forms 16 token
-// rows of it (only the tiles on and below the diagonal) and shares them through LDS.
+// multiplies the q k^T products element by element.  Four waves (the upper ones)
+// stage a chunk's rows and form these weights, 16 token rows each (only the tiles
+// on and below the diagonal), one chunk ahead, in the other half of the
+// double-buffered LDS; the lower four form the outputs and walk the state.
 // LDS rows are cut into 16-byte pieces that an XOR with row bits moves around, so that the 16 rows a fragment
 // read touches (whichever lane groups the hardware serves together) and the staging writes (rows 4 apart) lie on
 // different banks: element offset of piece pc of row r in a [..][DK] and in a [..][64] image.
@@ -113,97 +115,99 @@ template <int DK> __device__ __forceinline__ int koff(int r, int pc) {
 }
 __device__ __forceinline__ int soff(int r, int pc) { return r * 64 + ((pc ^ ((r >> 1) & 7)) << 3); }
 
+template <int DK> struct ChunkBuf {
+  bf16_t q[64 * (DK == 128 ? DK : DK + 8)];  // [t][n]
+  bf16_t kT[DK * 64];                        // k [n][s]
+  bf16_t vT[kPB * 64];                       // v [p][s]
+  bf16_t m[2][64 * 64];                      // hi, lo of the pair weights [t][s]
+  float L[64], u[64], w[64];  // log2 decay since the start, step, step x decay to the end
+};
+
 template <int DK, int MODE>
-__global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
-  constexpr int Q = 64, KP = DK == 128 ? DK : DK + 8;  // tokens per chunk; LDS row of q and k
-  constexpr int NO = DK / 8, NI = 16 * NO;        // staged items of q / k: 4 tokens x 8 channels
+__global__ void __launch_bounds__(512, 2) chunk_scan_kernel(ScanArgs g) {
+  constexpr int Q = 64;                       // tokens per chunk
+  constexpr int NO = DK / 8, NI = 16 * NO;    // staged items of q / k: 4 tokens x 8 channels
   constexpr int NM = DK / 16, NK = DK / 32;
   static_assert(NI <= 256 && DK % 32 == 0, "one staged item per thread");
-  __shared__ __attribute__((aligned(16))) bf16_t Cs[Q * KP];   // q [t][n]
-  __shared__ __attribute__((aligned(16))) bf16_t Bs[Q * KP];   // k [s][n]
-  __shared__ __attribute__((aligned(16))) bf16_t BT[DK * Q];  // k [n][s]
-  __shared__ __attribute__((aligned(16))) bf16_t xT[kPB * Q];  // v [p][s]
-  __shared__ __attribute__((aligned(16))) bf16_t Mh[Q * Q], Ml[Q * Q];  // weights [t][s]
-  __shared__ __attribute__((aligned(16))) float Ls[Q], us[Q], ws[Q];  // log2 decay since the start, step, step x decay to the end
+  __shared__ __attribute__((aligned(16))) ChunkBuf<DK> bufs[2];
+  __shared__ __attribute__((aligned(16))) bf16_t ks[sizeof(bufs[0].q) / sizeof(bf16_t)];  // k [s][n]
   Walk w;
   if (!open_walk(g, w)) return;
-  const int tid = threadIdx.x, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
-  const int sq = tid & 15, oc = tid >> 4;  // staging: token quad, channel octet
-  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
-  f32x4 S[NM];
-#pragma unroll
-  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
-  // the thread's first row of the chunk being fetched
-  const bf16_t* q = (const bf16_t*)g.q + (int64_t)(w.r0 + 4 * sq) * g.qs + (int64_t)w.hq * DK + 8 * oc;
-  const bf16_t* k = (const bf16_t*)g.k + (int64_t)(w.r0 + 4 * sq) * g.ks + (int64_t)w.hq * DK + 8 * oc;
-  const bf16_t* v = (const bf16_t*)g.v + (int64_t)(w.r0 + 4 * sq) * g.vs + (int64_t)w.h * g.dv + w.col0 + 8 * oc;
-  const float skip = g.skip ? g.skip[w.h] : 0.f, qsc = g.q_scale;
-  const float fixed_l2 = MODE == kFixed ? fmaxf(log2f(g.decay[w.h]), -1e6f) : 0.f;
-  raw_u32x4 rq[4], rk[4], rv[4];
-  bf16_t rg = 0;  // step logit of token tid (first wave)
-  const bf16_t* gl = MODE == kStep ? (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + w.h : nullptr;
-  const float g_bias = MODE == kStep && g.g_bias ? g.g_bias[w.h] : 0.f;
-  const float rate_l2 = MODE == kStep ? -g.rate[w.h] * kLog2e : 0.f;
-  auto fetch = [&](int t0) {
-    const raw_u32x4 zero{0u, 0u, 0u, 0u};
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const bool ok = t0 + 4 * sq + i < w.n;
-      rq[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(q + i * g.qs) : zero;
-      rk[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(k + i * g.ks) : zero;
-      rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + i * g.vs) : zero;
-    }
-    q += Q * g.qs;
-    k += Q * g.ks;
-    v += Q * g.vs;
-    if (MODE == kStep && tid < Q && t0 + tid < w.n) rg = gl[(int64_t)(t0 + tid) * g.gs];
-  };
-  fetch(0);
-  for (int t0 = 0; t0 < w.n; t0 += Q) {
-    __syncthreads();  // the previous chunk is consumed
-    if (NI == 256 || tid < NI) {
+  const bool former = threadIdx.x >= 256;
+  const int tid = threadIdx.x & 255, wave = tid >> 6, c16 = tid & 15, g4 = (tid & 63) >> 4;
+
+  if (former) {  // ---- stage the chunks' rows; form the pair weights
+    const int sq = tid & 15, oc = tid >> 4;  // token quad, channel octet
+    // the thread's first row of the chunk being fetched
+    const bf16_t* q = (const bf16_t*)g.q + (int64_t)(w.r0 + 4 * sq) * g.qs + (int64_t)w.hq * DK + 8 * oc;
+    const bf16_t* k = (const bf16_t*)g.k + (int64_t)(w.r0 + 4 * sq) * g.ks + (int64_t)w.hq * DK + 8 * oc;
+    const bf16_t* v = (const bf16_t*)g.v + (int64_t)(w.r0 + 4 * sq) * g.vs + (int64_t)w.h * g.dv + w.col0 + 8 * oc;
+    const float skip = g.skip ? g.skip[w.h] : 0.f, qsc = g.q_scale;
+    const float fixed_l2 = MODE == kFixed ? fmaxf(log2f(g.decay[w.h]), -1e6f) : 0.f;
+    bf16_t rg = 0;  // step logit of token tid (first wave)
+    const bf16_t* gl = MODE == kStep ? (const bf16_t*)g.g + (int64_t)w.r0 * g.gs + w.h : nullptr;
+    const float g_bias = MODE == kStep && g.g_bias ? g.g_bias[w.h] : 0.f;
+    const float rate_l2 = MODE == kStep ? -g.rate[w.h] * kLog2e : 0.f;
+    raw_u32x4 rq[4], rk[4], rv[4];
+    auto fetch = [&](int t0) {
+      const raw_u32x4 zero{0u, 0u, 0u, 0u};
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        *reinterpret_cast<raw_u32x4*>(Cs + koff<DK>(4 * sq + i, oc)) = rq[i];
-        *reinterpret_cast<raw_u32x4*>(Bs + koff<DK>(4 * sq + i, oc)) = rk[i];
+        const bool ok = t0 + 4 * sq + i < w.n;
+        rq[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(q + i * g.qs) : zero;
+        rk[i] = (NI == 256 || tid < NI) && ok ? *reinterpret_cast<const raw_u32x4*>(k + i * g.ks) : zero;
+        rv[i] = tid < 128 && ok ? *reinterpret_cast<const raw_u32x4*>(v + i * g.vs) : zero;
       }
+      q += Q * g.qs;
+      k += Q * g.ks;
+      v += Q * g.vs;
+      if (MODE == kStep && tid < Q && t0 + tid < w.n) rg = gl[(int64_t)(t0 + tid) * g.gs];
+    };
+    auto stage = [&](ChunkBuf<DK>& b, int t0) {
+      if (NI == 256 || tid < NI) {
 #pragma unroll
-      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(BT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rk, e);
-    }
-    if (tid < 128) {
+        for (int i = 0; i < 4; ++i) {
+          *reinterpret_cast<raw_u32x4*>(b.q + koff<DK>(4 * sq + i, oc)) = rq[i];
+          *reinterpret_cast<raw_u32x4*>(ks + koff<DK>(4 * sq + i, oc)) = rk[i];
+        }
 #pragma unroll
-      for (int e = 0; e < 8; ++e) *reinterpret_cast<uint2*>(xT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rv, e);
-    }
-    if (tid < Q) {  // one wave: log decays since the chunk's start (inclusive scan)
-      const bool ok = t0 + tid < w.n;
-      float u = ok ? 1.f : 0.f, L = ok ? fixed_l2 : 0.f;
-      if (MODE == kStep && ok) {
-        u = softplusf_(bf16_to_f32(rg) + g_bias);
-        L = rate_l2 * u;
+        for (int e = 0; e < 8; ++e)
+          *reinterpret_cast<uint2*>(b.kT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rk, e);
       }
-      L = wave_scan_sum(L);
-      u *= g.k_scale;
-      Ls[tid] = L;
-      us[tid] = u;
-      const float Lend = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, L), 63));
-      ws[tid] = u * fast_exp2(Lend - L);
-    }
-    __syncthreads();
-    if (t0 + Q < w.n) fetch(t0 + Q);
-    {  // weights of 16 query tokens: (q_t . k_s) E(s, t) u_s
+      if (tid < 128) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          *reinterpret_cast<uint2*>(b.vT + soff(8 * oc + e, sq >> 1) + 4 * (sq & 1)) = column4(rv, e);
+      }
+      if (tid < Q) {  // one wave: log decays since the chunk's start (inclusive scan)
+        const bool ok = t0 + tid < w.n;
+        float u = ok ? 1.f : 0.f, L = ok ? fixed_l2 : 0.f;
+        if (MODE == kStep && ok) {
+          u = softplusf_(bf16_to_f32(rg) + g_bias);
+          L = rate_l2 * u;
+        }
+        L = wave_scan_sum(L);
+        u *= g.k_scale;
+        b.L[tid] = L;
+        b.u[tid] = u;
+        const float Lend = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, L), 63));
+        b.w[tid] = u * fast_exp2(Lend - L);
+      }
+    };
+    auto weigh = [&](ChunkBuf<DK>& b) {  // 16 query tokens per wave: (q_t . k_s) E(s, t) u_s
       const int t = 16 * wave + c16;
       bf16x8_t cq[NK];
 #pragma unroll
-      for (int kk = 0; kk < NK; ++kk) cq[kk] = frag8(Cs + koff<DK>(t, 4 * kk + g4));
-      const float Lt = Ls[t];
-      for (int j = 0; j <= (wave | 1); ++j) {
+      for (int kk = 0; kk < NK; ++kk) cq[kk] = frag8(b.q + koff<DK>(t, 4 * kk + g4));
+      const float Lt = b.L[t];
+      for (int j = 0; j <= (wave | 1); ++j) {  // (an even wave's last half fragment is zero)
         float m4[4] = {0.f, 0.f, 0.f, 0.f};
         const int s0 = 16 * j + 4 * g4;
         if (j <= wave) {
           f32x4 a{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int kk = 0; kk < NK; ++kk) a = mfma32(frag8(Bs + koff<DK>(16 * j + c16, 4 * kk + g4)), cq[kk], a);
-          const f32x4 L4 = *reinterpret_cast<const f32x4*>(Ls + s0), u4 = *reinterpret_cast<const f32x4*>(us + s0);
+          for (int kk = 0; kk < NK; ++kk) a = mfma32(frag8(ks + koff<DK>(16 * j + c16, 4 * kk + g4)), cq[kk], a);
+          const f32x4 L4 = *reinterpret_cast<const f32x4*>(b.L + s0), u4 = *reinterpret_cast<const f32x4*>(b.u + s0);
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
             if (s0 + r <= t) m4[r] = a[r] * fast_exp2(Lt - L4[r]) * u4[r] * qsc;
@@ -212,15 +216,42 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
         }
         uint2 hi, lo;
         split4(m4, hi, lo);
-        *reinterpret_cast<uint2*>(Mh + soff(t, s0 >> 3) + (s0 & 7)) = hi;
-        *reinterpret_cast<uint2*>(Ml + soff(t, s0 >> 3) + (s0 & 7)) = lo;
+        *reinterpret_cast<uint2*>(b.m[0] + soff(t, s0 >> 3) + (s0 & 7)) = hi;
+        *reinterpret_cast<uint2*>(b.m[1] + soff(t, s0 >> 3) + (s0 & 7)) = lo;
+      }
+    };
+    fetch(0);
+    stage(bufs[0], 0);
+    __syncthreads();  // chunk 0 is staged
+    fetch(Q);
+    weigh(bufs[0]);
+    for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
+      const bool more = t0 + Q < w.n;
+      __syncthreads();  // chunk t0 is weighed; the other half is consumed
+      if (more) stage(bufs[cur ^ 1], t0 + Q);
+      __syncthreads();  // chunk t0 + Q is staged
+      if (more) {
+        fetch(t0 + 2 * Q);
+        weigh(bufs[cur ^ 1]);
       }
     }
+    return;
+  }
+
+  // ---- outputs and state.  (The barriers of the two roles pair up: one in front, two per chunk.)
+  float* sp = g.state + (((int64_t)w.slot * g.H + w.h) * g.dv + w.col0 + 16 * wave + c16) * DK + 4 * g4;
+  f32x4 S[NM];
+#pragma unroll
+  for (int m = 0; m < NM; ++m) S[m] = w.fresh ? f32x4{0.f, 0.f, 0.f, 0.f} : *reinterpret_cast<const f32x4*>(sp + 16 * m);
+  const float qsc = g.q_scale;
+  const int p = 16 * wave + c16;
+  __syncthreads();
+  for (int t0 = 0, cur = 0; t0 < w.n; t0 += Q, cur ^= 1) {
     __syncthreads();
-    const int p = 16 * wave + c16;
+    const ChunkBuf<DK>& b = bufs[cur];
     bf16x8_t xf[2], Sh[NK], Sl[NK];
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) xf[kk] = frag8(xT + soff(p, 4 * kk + g4));
+    for (int kk = 0; kk < 2; ++kk) xf[kk] = frag8(b.vT + soff(p, 4 * kk + g4));
 #pragma unroll
     for (int kk = 0; kk < NK; ++kk) {
       float s8[8];
@@ -231,43 +262,42 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       Sh[kk] = as_bf16x8(hi);
       Sl[kk] = as_bf16x8(lo);
     }
-#pragma unroll
-    for (int tt = 0; tt < Q / 16; ++tt) {
-      if (t0 + 16 * tt >= w.n) break;
+    auto output = [&](int tt) {  // 16 tokens x the wave's 16 columns
+      if (t0 + 16 * tt >= w.n) return;
       const int t = 16 * tt + c16;
-      f32x4 a{0.f, 0.f, 0.f, 0.f}, b{0.f, 0.f, 0.f, 0.f};
+      f32x4 a{0.f, 0.f, 0.f, 0.f}, a1{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kk = 0; kk < NK; ++kk) {
-        const bf16x8_t cf = frag4_4(Cs + koff<DK>(t, 4 * kk + (g4 >> 1)) + 4 * (g4 & 1), Cs + koff<DK>(t, 4 * kk + 2 + (g4 >> 1)) + 4 * (g4 & 1));
+        const bf16x8_t cf = frag4_4(b.q + koff<DK>(t, 4 * kk + (g4 >> 1)) + 4 * (g4 & 1),
+                                    b.q + koff<DK>(t, 4 * kk + 2 + (g4 >> 1)) + 4 * (g4 & 1));
         a = mfma32(Sh[kk], cf, a);
-        b = mfma32(Sl[kk], cf, b);
+        a1 = mfma32(Sl[kk], cf, a1);
       }
-      const float e = fast_exp2(Ls[t]) * qsc;
+      const float e = fast_exp2(b.L[t]) * qsc;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) a[r] = (a[r] + b[r]) * e, b[r] = 0.f;
+      for (int r = 0; r < 4; ++r) a[r] = (a[r] + a1[r]) * e, a1[r] = 0.f;
 #pragma unroll
       for (int kk = 0; kk <= tt / 2; ++kk) {
-        a = mfma32(xf[kk], frag8(Mh + soff(t, 4 * kk + g4)), a);
-        b = mfma32(xf[kk], frag8(Ml + soff(t, 4 * kk + g4)), b);
+        a = mfma32(xf[kk], frag8(b.m[0] + soff(t, 4 * kk + g4)), a);
+        a1 = mfma32(xf[kk], frag8(b.m[1] + soff(t, 4 * kk + g4)), a1);
       }
       if (t0 + t < w.n)
         *reinterpret_cast<f32x4*>(g.out + ((int64_t)(w.r0 + t0 + t) * g.H + w.h) * g.dv + w.col0 + 16 * wave + 4 * g4) =
-            f32x4{a[0] + b[0], a[1] + b[1], a[2] + b[2], a[3] + b[3]};
-    }
-    const float eq = fast_exp2(Ls[Q - 1]);
+            f32x4{a[0] + a1[0], a[1] + a1[1], a[2] + a1[2], a[3] + a1[3]};
+    };
+    output(0);
+    output(1);
+    __syncthreads();
+    output(2);
+    output(3);
+    const float eq = fast_exp2(b.L[Q - 1]);
     bf16x8_t xh[2], xl[2];
 #pragma unroll
     for (int kk = 0; kk < 2; ++kk) {
-      const raw_u32x4 x4 = __builtin_bit_cast(raw_u32x4, xf[kk]);
       float x8[8];
+      chunk_to_f32<bf16_t>(__builtin_bit_cast(raw_u32x4, xf[kk]), x8);
 #pragma unroll
-      for (int e = 0; e < 8; e += 4) {
-        const f32x4 w4 = *reinterpret_cast<const f32x4*>(ws + 32 * kk + 8 * g4 + e);
-        x8[e] = bf16lo(x4[e / 2]) * w4[0];
-        x8[e + 1] = bf16hi(x4[e / 2]) * w4[1];
-        x8[e + 2] = bf16lo(x4[e / 2 + 1]) * w4[2];
-        x8[e + 3] = bf16hi(x4[e / 2 + 1]) * w4[3];
-      }
+      for (int e = 0; e < 8; ++e) x8[e] *= b.w[32 * kk + 8 * g4 + e];
       raw_u32x4 hi, lo;
       split8(x8, hi, lo);
       xh[kk] = as_bf16x8(hi);
@@ -279,9 +309,9 @@ __global__ void __launch_bounds__(256, 2) chunk_scan_kernel(ScanArgs g) {
       for (int r = 0; r < 4; ++r) S[m][r] *= eq;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
-        const bf16x8_t bf = frag8(BT + soff(16 * m + c16, 4 * kk + g4));
-        S[m] = mfma32(bf, xh[kk], S[m]);
-        S[m] = mfma32(bf, xl[kk], S[m]);
+        const bf16x8_t kf = frag8(b.kT + soff(16 * m + c16, 4 * kk + g4));
+        S[m] = mfma32(kf, xh[kk], S[m]);
+        S[m] = mfma32(kf, xl[kk], S[m]);
       }
     }
   }
@@ -563,7 +593,7 @@ void launch_chunk_scan(int mode, const ScanArgs& g, int n_seq, hipStream_t st) {
 #define FIXED_K(D) chunk_scan_kernel<D, kFixed>
 #define STEP_K(D) chunk_scan_kernel<D, kStep>
 #define CHANNEL_K(D) channel_chunk_kernel<D>
-  if (mode == kFixed) { CHUNK_DK(FIXED_K, dim3(256)) }
-  else if (mode == kStep) { CHUNK_DK(STEP_K, dim3(256)) }
+  if (mode == kFixed) { CHUNK_DK(FIXED_K, dim3(512)) }
+  else if (mode == kStep) { CHUNK_DK(STEP_K, dim3(512)) }
   else { CHUNK_DK(CHANNEL_K, dim3(kFormThreads + kProdThreads)) }
 }
