@@ -678,6 +678,58 @@ __global__ void __launch_bounds__(256) head_norm_gate_kernel(T* __restrict__ out
   }
 }
 
+// The same for heads of up to 256 elements in whole runs of four: LPH neighbouring lanes (a power of two)
+// share a head, four elements each, so a wave works on 64 / LPH heads with 16-byte accesses.
+template <typename T, int LPH>
+__global__ void __launch_bounds__(256) head_norm_gate_vec_kernel(T* __restrict__ out, const float* __restrict__ o,
+                                                                 const float* __restrict__ w, const T* __restrict__ gate,
+                                                                 int64_t gs, int64_t n_vec, int H, int dv, float eps,
+                                                                 int gate_act) {
+  const int64_t v = (int64_t)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
+  const int e = (threadIdx.x % LPH) * 4;
+  if (v >= n_vec) return;  // (whole lane groups)
+  const bool on = e < dv;
+  const int64_t row = v / H;
+  const int c = (int)(v - row * H) * dv + e;  // column of the row
+  f32x4 x{0.f, 0.f, 0.f, 0.f};
+  float z[4] = {0.f, 0.f, 0.f, 0.f};
+  if (on) {
+    x = *reinterpret_cast<const f32x4*>(o + v * dv + e);
+    if (gate) {
+      if constexpr (sizeof(T) == 2) {
+        const uint2 t = *reinterpret_cast<const uint2*>((const bf16_t*)gate + row * gs + c);
+        z[0] = bf16lo(t.x), z[1] = bf16hi(t.x), z[2] = bf16lo(t.y), z[3] = bf16hi(t.y);
+      } else {
+        VecIO<float, 4>::ld((const float*)gate + row * gs + c, z);
+      }
+    }
+  }
+  float ss = x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+#pragma unroll
+  for (int m = LPH / 2; m > 0; m >>= 1) ss += __shfl_xor(ss, m, 64);
+  const float inv = rsqrtf(ss / (float)dv + eps);
+  if (!on) return;
+  float y[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    y[i] = x[i] * inv;
+    if (w) y[i] *= w[c + i];
+    if (gate) y[i] *= gate_act ? z[i] * fast_sigmoid(z[i]) : fast_sigmoid(z[i]);
+  }
+  if constexpr (sizeof(T) == 2)
+    *reinterpret_cast<uint2*>((bf16_t*)out + v * dv + e) = uint2{pack_bf16x2(y[0], y[1]), pack_bf16x2(y[2], y[3])};
+  else
+    VecIO<float, 4>::st((float*)out + v * dv + e, y);
+}
+
+template <typename T, int LPH>
+void launch_head_norm_vec(void* out, const float* o, const float* w, const void* gate, int64_t gs, int64_t n_vec, int H,
+                          int dv, float eps, int gate_act, hipStream_t st) {
+  const int per = 256 / LPH;
+  hipLaunchKernelGGL((head_norm_gate_vec_kernel<T, LPH>), dim3((unsigned)((n_vec + per - 1) / per)), dim3(256), 0, st,
+                     (T*)out, o, w, (const T*)gate, gs, n_vec, H, dv, eps, gate_act);
+}
+
 // out = y silu(z), divided by the root mean square of its group (n equal groups of the row, eps inside the
 // root), times w: the gate enters in front of the norm.  One workgroup per (row, group); a thread keeps its
 // elements (V neighbours at a time, up to kGnKeep times) in registers between the mean square and the result.
@@ -849,6 +901,18 @@ int dxm_head_norm_gate(void* out, const float* o, const float* w, const void* ga
   if (H < 1 || dv < 1 || (int64_t)rows * H > 0x7fffffff || gate_act < 0 || gate_act > 1) return 1;
   const int64_t n_vec = (int64_t)rows * H;
   const dim3 grid((unsigned)((n_vec + 3) / 4));
+  const int esz = f32 ? 4 : 2;
+  if (dv % 4 == 0 && dv <= 256 && gs % 4 == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)out % (4 * esz) == 0 &&
+      (uintptr_t)gate % (4 * esz) == 0) {
+    DISPATCH_T(f32, {
+      if (dv <= 32) launch_head_norm_vec<T, 8>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
+      else if (dv <= 64) launch_head_norm_vec<T, 16>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
+      else if (dv <= 128) launch_head_norm_vec<T, 32>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
+      else launch_head_norm_vec<T, 64>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
+    });
+    DX_CHECK_LAUNCH();
+    return 0;
+  }
   const bool v2 = dv % 2 == 0 && gs % 2 == 0 && (uintptr_t)o % 8 == 0 && (uintptr_t)out % 4 == 0;
   if (v2) {
     DISPATCH_T(f32, hipLaunchKernelGGL((head_norm_gate_kernel<T, 2>), grid, dim3(256), 0, st, (T*)out, o, w,

@@ -356,6 +356,19 @@ def test_gate_group_norm_alone(device, dtype, W, groups):
     assert bool((out[:, :8] == 9.0).all()) and bool((out[:, 8 + W:] == 9.0).all())
 
 
+@pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("H,dv", [(3, 14), (2, 32), (5, 64), (3, 128), (2, 200), (7, 12), (1, 300), (3, 5)])
+def test_head_norm_silu_gate_alone(device, dtype, H, dv):
+    """The per-head unit norm with a weight shared by the heads, then the silu gate (behind the norm)."""
+    torch.manual_seed(dv)
+    T, eps, dt = 5, 1e-5, DT[dtype]
+    o, z, w = torch.randn(T, H * dv) * 3, (torch.randn(T, H * dv + 8) * 2).to(dt), torch.randn(dv)
+    got = rc.head_norm_gate(o.to(device), H, w.repeat(H).to(device), z.to(device)[:, 8:], eps, dt, gate_act="silu")
+    want = (O.unit_rms(o.double().view(T, H, dv), eps) * w.double()).reshape(T, -1) * O.silu(z[:, 8:].double())
+    tol = dict(atol=1e-4, rtol=1e-4) if dtype == "float32" else dict(atol=1e-2, rtol=1e-2)
+    assert torch.allclose(got.cpu().double(), want, **tol)
+
+
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("F", [24, 21])
 def test_gates_and_clamp_alone(device, F):
