@@ -456,6 +456,42 @@ def test_decode_rows_over_whole_tile_pages(d, n_qh, G, maps, bs, size):
         assert float((got.cpu().double() - want).abs().max()) < 1e-3 * max(1.0, float(want.abs().max()))
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("d,n_qh,G,bs", [(128, 8, 2, 64), (64, 4, 2, 128), (128, 12, 2, 64), (64, 16, 2, 64), (128, 3, 1, 64)])
+@pytest.mark.parametrize("size", [0, 1, 64, 65, 100])
+def test_prompt_rows_over_whole_tile_pages(d, n_qh, G, bs, size):
+    """bf16 prompt rows over pages of whole 64-key tiles (the streaming kernel where heads pair up): portions
+    that start at position 0, inside a cached prefix and at a tile's edge, one of two rows, beside a decode row;
+    windows that start inside a tile, pages whose unused rows hold NaN."""
+    torch.manual_seed(d + size)
+    chunks = [(0, 150), (37, 263), (64, 2), (190, 130), (5, 1)]  # (first position, rows); the last a decode row
+    group, B, T = n_qh // G, len(chunks), 330
+    per = -(-T // bs)
+    k, v = torch.randn(B, T, G, d).bfloat16(), torch.randn(B, T, G, d).bfloat16()
+    table = torch.randperm(B * per, generator=torch.Generator().manual_seed(1)).to(torch.int32).view(B, per)
+    kc = torch.full((B * per * bs, G * d), float("nan"), dtype=torch.bfloat16)
+    vc = torch.full((B * per * bs, G * d), float("nan"), dtype=torch.bfloat16)
+    q = torch.randn(sum(n for _, n in chunks), n_qh, d).bfloat16()
+    want, tiles, r0 = torch.zeros(q.shape, dtype=torch.float64), [], 0
+    for b, (p, n) in enumerate(chunks):
+        j = torch.arange(p + n)
+        sl = table[b].long()[j // bs] * bs + j % bs
+        kc[sl], vc[sl] = k[b, :p + n].reshape(p + n, -1), v[b, :p + n].reshape(p + n, -1)
+        dist = torch.arange(p, p + n)[:, None] - j[None, :]
+        vis = (dist >= 0) & ((dist < size) if size else torch.ones_like(dist, dtype=torch.bool))
+        for h in range(n_qh):
+            sc = (q[r0:r0 + n, h].double() @ k[b, :p + n, h // group].double().T) * 0.2
+            want[r0:r0 + n, h] = torch.softmax(sc.masked_fill(~vis, float("-inf")), -1) @ v[b, :p + n, h // group].double()
+        if b < B - 1:
+            tiles += mx.tile_list(r0, n)
+        r0 += n
+    pos, row_seq, _, _ = step_meta("cuda", chunks, [0] * B)
+    got = mx.attention(q.reshape(r0, -1).cuda(), kc.cuda(), vc.cuda(), pos, row_seq, table.cuda(), bs, n_qh, 1, group, d, d, 0.2,
+                       "window" if size else "causal", size, 1, False, torch.tensor(tiles, dtype=torch.int32, device="cuda"),
+                       r0 - 1)
+    assert float((got.cpu().double() - want).abs().max()) < 2e-2 * max(1.0, float(want.abs().max()))
+
+
 # ----------------------------------------------------------------- whole model
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("name", list(CONFIGS))
@@ -531,15 +567,16 @@ def test_long_decode_and_first_tokens(device, dtype):
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
-def test_long_prompt_portions(device, dtype):
+@pytest.mark.parametrize("bs", [8, 64])
+def test_long_prompt_portions(device, dtype, bs):
     """A prompt of several hundred tokens in portions that end inside and at the edges of the kernels' token
     blocks and tiles (63, 64, 65, 128 + 1, ...), beside a second sequence."""
-    cfg = config([layer(par(H=2, G=1, d=32, dv=32, dims=32, base=1e4, Hs=2, P=64, N=64, groups=1, norm_groups=1, conv=4), 32),
+    cfg = config([layer(par(H=4, G=2, d=64, dv=64, dims=32, base=1e4, Hs=2, P=64, N=64, groups=1, norm_groups=1, conv=4), 32),
                   layer(gla(H=1, d=64, dv=64, tau=16.0), 0)], width=32)
     sd = weights(cfg, 16)
     a, b = tokens(330, cfg.vocab_size, 17), tokens(200, cfg.vocab_size, 18)
     wa, wb = O.forward(cfg_dict(cfg), sd, a)[0], O.forward(cfg_dict(cfg), sd, b)[0]
-    eng = engine(cfg, sd, device, dtype, blocks=80)
+    eng = engine(cfg, sd, device, dtype, blocks=640 // bs, bs=bs)
     ga, gb, pa, pb = [], [], 0, 0
     for na, nb in ((63, 64), (65, 1), (129, 127), (1, 2), (64, 6), (8, 0)):
         ent = [("a", a[pa:pa + na], list(range(na)))] + ([("b", b[pb:pb + nb], list(range(nb)))] if nb else [])
