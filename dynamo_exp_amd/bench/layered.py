@@ -652,6 +652,16 @@ def povurax_kernels(s: dict, L: int, B: int, T: int) -> dict:
     cwq, tq = torch.randn(taps, (H + 2 * G) * d, device=dev), torch.zeros(1, taps - 1, (H + 2 * G) * d, device=dev, dtype=dt)
     put("nefivik_conv_rope_cache", _timed(lambda: rc.conv_rope_cache(qkv, cwq, tq, posT, posT, rs, sr, s0, H, G, d, d,
                                                                      inv[:d // 4].contiguous(), kc, vc)), byts)
+    # ---- causal prompt attention with fine weights (attention_kernels has it without)
+    nbl = L // bs
+    q = torch.randn(L, H * d, device=dev, dtype=dt)
+    kl, vl = (torch.randn(nbl * bs, G * d, device=dev, dtype=dt) for _ in range(2))
+    bt = torch.arange(nbl, dtype=torch.int32, device=dev).view(1, nbl)
+    tiles = torch.tensor(mx.tile_list(0, L), dtype=torch.int32, device=dev)
+    seq = torch.zeros(L, dtype=torch.int32, device=dev)
+    put("prefill_causal_fine_weights", _timed(lambda: mx.attention(
+        q, kl, vl, posT[:L], seq, bt, bs, H, 1, H // G, d, d, d ** -0.5, "causal", 0, 1, False, tiles, L, fine_weights=True)),
+        None, 4 * d * H * L * (L + 1) / 2)
     # ---- gates, feed-forward unit, residual step
     a, g = torch.randn(T, H * d, device=dev, dtype=dt), torch.randn(T, H * d, device=dev, dtype=dt)
     o = torch.empty(T, H * d + inner, device=dev, dtype=dt)

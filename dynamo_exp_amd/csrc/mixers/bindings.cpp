@@ -67,13 +67,13 @@ int dxm_row_attention(void*, float*, const void*, int64_t, const void*, const vo
 int dxm_tile_attention_ok(int, int);
 int dxm_tile_attention(void*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*,
                        int, int, const int*, int, int, int, int, int, int, int, int, float, int, int, float, const float*,
-                       const float*, int, const float*, const void*, int64_t, int, const float*, int, hipStream_t);
+                       const float*, int, const float*, const void*, int64_t, int, const float*, int, int, hipStream_t);
 int dxm_group_decode(float*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
                      int, int, int, int, int, int, int, int, int, float, int, int, float, const float*, const float*, int,
                      const float*, int, int, hipStream_t);
 int dxm_stream_prefill_ok(int, int, int, int, int, int);
 int dxm_stream_prefill(void*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
-                       int, const int*, int, int, int, int, int, int, int, float, int, int, hipStream_t);
+                       int, const int*, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
 int dxm_stream_decode_ok(int, int, int, int, int);
 int dxm_stream_decode(float*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
                       int, int, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
@@ -230,20 +230,20 @@ PYBIND11_MODULE(_C_mixers, m) {
   m.def("tile_attention", [](u out, u q, int64_t qs, u kc, u vc, u pos, u seq, u bt, int bts, int bs, u tiles,
                              int n_tiles, int n_qh, int maps, int group, int d, int dv, int Wk, int Wv, float scale,
                              int mask, int size, float cap, u r1, u r2, int wfn, u hbias, u gate, int64_t gs,
-                             int keep, u sink, int out_f32, u st) {
+                             int keep, u sink, int out_f32, int fine, u st) {
     // plain heads over pages of whole tiles take the streaming kernel
     if (cap == 0.f && !r1 && !wfn && !hbias && !gate && !keep && !sink && !out_f32 && qs % 8 == 0 &&
         (q | kc | vc) % 16 == 0 && dxm_stream_prefill_ok(d, dv, maps, group, bs, mask))
       check(dxm_stream_prefill(P(out), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
                                reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs,
                                reinterpret_cast<const int*>(tiles), n_tiles, n_qh, group, d, dv, Wk, Wv, scale, mask, size,
-                               S(st)),
+                               fine, S(st)),
             "stream_prefill");
     else
       check(dxm_tile_attention(P(out), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
                              reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs,
                              reinterpret_cast<const int*>(tiles), n_tiles, n_qh, maps, group, d, dv, Wk, Wv, scale,
-                             mask, size, cap, F(r1), F(r2), wfn, F(hbias), P(gate), gs, keep, F(sink), out_f32, S(st)),
+                             mask, size, cap, F(r1), F(r2), wfn, F(hbias), P(gate), gs, keep, F(sink), out_f32, fine, S(st)),
           "tile_attention");
   });
   m.def("group_decode", [](u out, u ws, u q, int64_t qs, u kc, u vc, u pos, u seq, u bt, int bts, int bs, int rows,

@@ -13,7 +13,8 @@
 // free.  Weights enter the value product as the sum of two bf16 numbers.
 // stream_prefill: eight waves per (64 or 128 prompt rows, 4 or 2 heads of a
 // group), 32 rows of one head each, sharing every key tile; tiles are
-// double-buffered in LDS.  Weights enter the value product as bf16.
+// double-buffered in LDS.  Weights enter the value product as bf16, or (FINE) as
+// the sum of two.
 #include "recurrent.h"
 
 namespace {
@@ -244,7 +245,7 @@ template <int D> __device__ __forceinline__ int kimg(int r, int pc) {
   return r * D + ((pc ^ (D == 128 ? r & 15 : (r >> 1) & 7)) << 3);
 }
 
-template <int D, int DV, int HPW>
+template <int D, int DV, int HPW, bool FINE>
 __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a) {
   constexpr int NK = D / 32, NC = DV / 16, RT = 8 / HPW, ROWS = 32 * RT;  // waves along the rows, rows per workgroup
   constexpr int KCH = D / 8, KI = 64 * KCH / 256;  // K items (16 bytes) per thread of the upper waves
@@ -349,7 +350,7 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
             if (dist < 0 || (a.size && dist >= a.size)) S[qb][kb][r] = -INFINITY;
           }
     }
-    bf16x8_t P[2][2];
+    bf16x8_t P[2][2], Pl[2][2];  // weights (FINE: hi and lo)
 #pragma unroll
     for (int qb = 0; qb < 2; ++qb) {
       float m = S[qb][0][0];
@@ -373,15 +374,17 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
       float add = 0.f;
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk) {
-        raw_u32x4 pk;
+        raw_u32x4 pk, pl;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           const float w0 = fast_exp2(fmaf(S[qb][2 * kk + e / 2][2 * (e % 2)], a.scale_log2, -mu));
           const float w1 = fast_exp2(fmaf(S[qb][2 * kk + e / 2][2 * (e % 2) + 1], a.scale_log2, -mu));
           add += w0 + w1;
           pk[e] = pack_bf16x2(w0, w1);
+          if constexpr (FINE) pl[e] = pack_bf16x2(w0 - bf16lo(pk[e]), w1 - bf16hi(pk[e]));
         }
         P[qb][kk] = __builtin_bit_cast(bf16x8_t, pk);
+        if constexpr (FINE) Pl[qb][kk] = __builtin_bit_cast(bf16x8_t, pl);
       }
       lsum[qb] += add;
     }
@@ -392,6 +395,10 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
         const bf16x8_t vf = frag16(V + voff(16 * cb + c16, 4 * kk + g4));
         O[0][cb] = mma(vf, P[0][kk], O[0][cb]);
         O[1][cb] = mma(vf, P[1][kk], O[1][cb]);
+        if constexpr (FINE) {
+          O[0][cb] = mma(vf, Pl[0][kk], O[0][cb]);
+          O[1][cb] = mma(vf, Pl[1][kk], O[1][cb]);
+        }
       }
   }
 #pragma unroll
@@ -410,14 +417,14 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
   }
 }
 
-template <int D, int HPW> void launch_stream_prefill(const StreamTileArgs& a0, int n_tiles, hipStream_t st) {
+template <int D, int HPW, bool FINE> void launch_stream_prefill(const StreamTileArgs& a0, int n_tiles, hipStream_t st) {
   StreamTileArgs a = a0;
   a.subs = 128 / (32 * (8 / HPW));
   const int step = 65535 / a.subs;
   for (int t0 = 0; t0 < n_tiles; t0 += step) {
     a.tiles = a0.tiles + 2 * t0;
     const int nt = n_tiles - t0 < step ? n_tiles - t0 : step;
-    hipLaunchKernelGGL((stream_prefill_kernel<D, D, HPW>), dim3(a.n_qh / HPW, nt * a.subs), dim3(512), 0, st, a);
+    hipLaunchKernelGGL((stream_prefill_kernel<D, D, HPW, FINE>), dim3(a.n_qh / HPW, nt * a.subs), dim3(512), 0, st, a);
   }
 }
 
@@ -433,7 +440,8 @@ int dxm_stream_prefill_ok(int d, int dv, int maps, int group, int bs, int mask) 
 
 int dxm_stream_prefill(void* out, const void* q, int64_t q_stride, const void* kc, const void* vc, const int64_t* pos,
                        const int* seq, const int* bt, int bt_stride, int bs, const int* tiles, int n_tiles, int n_qh,
-                       int group, int d, int dv, int Wk, int Wv, float scale, int mask, int size, hipStream_t st) {
+                       int group, int d, int dv, int Wk, int Wv, float scale, int mask, int size, int fine,
+                       hipStream_t st) {
   if (n_tiles <= 0) return 0;
   if (!dxm_stream_prefill_ok(d, dv, 1, group, bs, mask)) return 2;
   if (n_qh < 1 || n_qh % group) return 1;
@@ -444,10 +452,14 @@ int dxm_stream_prefill(void* out, const void* q, int64_t q_stride, const void* k
   StreamTileArgs a{(bf16_t*)out, (const bf16_t*)q, q_stride, (const bf16_t*)kc, (const bf16_t*)vc, pos, seq, bt, bt_stride,
                    __builtin_ctz((unsigned)bs), tiles, 1, n_qh, group, Wk, Wv, scale * 1.4426950408889634f,
                    mask ? size : 0};
-  if (d == 128 && group % 4 == 0) launch_stream_prefill<128, 4>(a, n_tiles, st);
-  else if (d == 128) launch_stream_prefill<128, 2>(a, n_tiles, st);
-  else if (group % 4 == 0) launch_stream_prefill<64, 4>(a, n_tiles, st);
-  else launch_stream_prefill<64, 2>(a, n_tiles, st);
+#define STREAM_PREFILL(D, HPW)                                  \
+  if (fine) launch_stream_prefill<D, HPW, true>(a, n_tiles, st); \
+  else launch_stream_prefill<D, HPW, false>(a, n_tiles, st);
+  if (d == 128 && group % 4 == 0) { STREAM_PREFILL(128, 4) }
+  else if (d == 128) { STREAM_PREFILL(128, 2) }
+  else if (group % 4 == 0) { STREAM_PREFILL(64, 4) }
+  else { STREAM_PREFILL(64, 2) }
+#undef STREAM_PREFILL
   DX_CHECK_LAUNCH();
   return 0;
 }

@@ -182,12 +182,13 @@ template <> __device__ __forceinline__ void store4<bf16_t>(bf16_t* o, f32x4 v) {
   *reinterpret_cast<uint2*>(o) = w;
 }
 
-template <int DB, int DVB, typename OutT>
+template <int DB, int DVB, typename OutT, bool FINE>
 __global__ void __launch_bounds__(256, (DB + DVB <= 16 ? 2 : 1)) tile_attention_kernel(TileArgs a) {
   constexpr int d = DB * 16, dv = DVB * 16, ks_stride = d + 8;
   // fp32 output (the two-map layers, whose a1 - lambda a2 amplifies errors): the weights enter
-  // the second product as hi + lo; bf16 output: as one bf16, like every other bf16 activation
-  constexpr bool kHiLo = sizeof(OutT) == 4;
+  // the second product as hi + lo; bf16 output: as one bf16, like every other bf16 activation, unless
+  // the caller asks for fine weights
+  constexpr bool kHiLo = FINE || sizeof(OutT) == 4;
   constexpr bool X32 = DB % 2 == 0;  // d a multiple of 32: the K = 32 MFMA for the scores too
   constexpr int DB2 = X32 ? DB / 2 : 1;
   extern __shared__ __attribute__((aligned(16))) bf16_t smem[];
@@ -622,10 +623,10 @@ int launch_group(const GroupArgs& a0, int rows, hipStream_t st) {
   return 0;
 }
 
-template <int DB, int DVB, typename OutT>
+template <int DB, int DVB, typename OutT, bool FINE>
 int launch_tiles(const TileArgs& a, int n_tiles, hipStream_t st) {
   const size_t lds = (size_t)(kKeys * (DB * 16 + 8) + DVB * 16 * kVtStride) * sizeof(bf16_t);
-  auto kern = tile_attention_kernel<DB, DVB, OutT>;
+  auto kern = tile_attention_kernel<DB, DVB, OutT, FINE>;
   if (lds > 48 * 1024) {
     static bool raised = false;  // per instantiation
     if (!raised) {
@@ -648,7 +649,9 @@ int launch_tiles(const TileArgs& a, int n_tiles, hipStream_t st) {
 
 #define TILE_CASE(DB_, DVB_)                                                               \
   if (d == DB_ * 16 && dv == DVB_ * 16)                                                    \
-    return out_f32 ? launch_tiles<DB_, DVB_, float>(a, n_tiles, st) : launch_tiles<DB_, DVB_, bf16_t>(a, n_tiles, st);
+    return out_f32 ? launch_tiles<DB_, DVB_, float, false>(a, n_tiles, st)                 \
+           : fine  ? launch_tiles<DB_, DVB_, bf16_t, true>(a, n_tiles, st)                 \
+                   : launch_tiles<DB_, DVB_, bf16_t, false>(a, n_tiles, st);
 
 extern "C" {
 
@@ -664,7 +667,8 @@ int dxm_tile_attention(void* out, const void* q, int64_t q_stride, const void* k
                        const int* seq, const int* bt, int bt_stride, int bs, const int* tiles, int n_tiles, int n_qh,
                        int maps, int group, int d, int dv, int Wk, int Wv, float scale, int mask, int size,
                        float softcap, const float* r1, const float* r2, int wfn, const float* hbias, const void* gate,
-                       int64_t gate_stride, int keep, const float* sink, int out_f32, hipStream_t st) {
+                       int64_t gate_stride, int keep, const float* sink, int out_f32, int fine,
+                       hipStream_t st) {
   if (n_tiles <= 0) return 0;
   if (softcap < 0.f || (r1 && !r2) || wfn < 0 || wfn > 1 || keep < 0 || (keep && mask != 1)) return 6;
   if (n_qh < 1 || maps < 1 || group < 1 || n_qh % maps || (n_qh / maps) % group || n_qh > 65535) return 1;

@@ -352,7 +352,7 @@ class PovuraxForCausalLM:
                            kc, vc)
         tl = (meta.row_tiles, meta.num_prefill_tokens) if meta.is_prefill else (None, 0)
         y = mx.attention(p, kc, vc, meta.positions, seq, tables, bs, H, 1, H // G, d, dv, a["scale"], "causal", 0,
-                         self._parts(T, H, H // G, meta), False, *tl)
+                         self._parts(T, H, H // G, meta), False, *tl, fine_weights=True)
         mx.act_mul(p[:, g0:z0], y.view(T, nv), "sigmoid", out=o[:, :nv], scale=L["left_scale"])
         # right: state-space mixer
         xbc = rc.causal_conv(p[:, c0:c0 + C], L["conv_w"], tail, meta.positions, meta.row_seq if meta.is_prefill else None,

@@ -474,12 +474,14 @@ def attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, positions: to
               out_f32: bool = False, tiles: torch.Tensor | None = None, n_tile_rows: int = 0, softcap: float = 0.0,
               dist_bias: tuple[torch.Tensor, torch.Tensor] | None = None, weights: str = "softmax",
               head_bias: torch.Tensor | None = None, head_gate: torch.Tensor | None = None, keep_first: int = 0,
-              sink: torch.Tensor | None = None) -> torch.Tensor:
+              sink: torch.Tensor | None = None, fine_weights: bool = False) -> torch.Tensor:
     """Attention of one step's rows: the first n_tile_rows rows (prompt chunks,
     cut into `tiles` [n, 2] = first row, row count) on the matrix-core prefill
     kernel where it applies, all other rows (decode tokens; every row when it
     does not apply) on the row kernel.  Same arguments and result as
-    row_attention."""
+    row_attention.  fine_weights: prompt rows' softmax weights enter the product with the
+    values as the sum of two bf16 numbers also where the result is bf16 (decode rows'
+    always do)."""
     T = q.shape[0]
     if not tile_attention_ok(q, d, dv) or not scale > 0:  # the matrix-core kernels fold a positive scale
         return row_attention(q, kc, vc, positions, seq, block_tables, block_size, n_qh, maps, group, d, dv, scale,
@@ -512,7 +514,7 @@ def attention(q: torch.Tensor, kc: torch.Tensor, vc: torch.Tensor, positions: to
             raise TypeError("attention: prompt-chunk rows need seq and int32 tiles")
         _m().tile_attention(out.data_ptr(), q.data_ptr(), q.stride(0), kc.data_ptr(), vc.data_ptr(),
                             positions.data_ptr(), seq.data_ptr(), *common, tiles.data_ptr(), tiles.shape[0], *heads,
-                            _ptr(head_gate), gs, int(keep_first), _ptr(sink), int(out_f32), _stream())
+                            _ptr(head_gate), gs, int(keep_first), _ptr(sink), int(out_f32), int(fine_weights), _stream())
     n_dec = T - n_tile_rows
     if n_dec:  # decode rows: the heads of a K/V group share one wave's key tiles
         r0 = n_tile_rows
