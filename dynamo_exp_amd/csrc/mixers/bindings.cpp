@@ -17,7 +17,7 @@ extern "C" {
 int dxm_stream_step(float*, const void*, int64_t, const float*, const float*, const float*, const float*, float, void*,
                     int64_t, int, int, int, int, hipStream_t);
 int dxm_embed_streams(float*, const void*, const int64_t*, int, int, int, int64_t, const void*, const int64_t*,
-                      int64_t, float, int, hipStream_t);
+                      int64_t, float, const float*, float, int, hipStream_t);
 int dxm_section_norm(void*, const void*, int64_t, const float*, int, int, float, int, hipStream_t);
 int dxm_depth_mix(float*, float*, int64_t, int, const float*, const int64_t*, int, float, const float*, void*,
                   const void*, int64_t, const float*, int, int, hipStream_t);
@@ -25,18 +25,19 @@ int dxm_linear_scan(int, float*, float*, int, const void*, int64_t, const void*,
                     float, int, const float*, const void*, int64_t, const float*, const float*, const float*, float,
                     const int64_t*, const int*, const int*, int, int, int, int, int, int, hipStream_t);
 int dxm_norm_rope_cache(void*, int64_t, const int64_t*, const int64_t*, int, int, int, int, int, const float*,
-                        const float*, float, const float*, int, void*, void*, int, hipStream_t);
+                        const float*, float, const float*, int, void*, void*, int, int, int, hipStream_t);
 int dxm_gate_group_norm(void*, int64_t, const float*, const void*, int64_t, const float*, int, int, int, float, int,
                         hipStream_t);
 int dxm_latent_rope(void*, const void*, const void*, int64_t, int, int, const void*, int64_t, const float*, float,
-                    const float*, int, float, const int64_t*, const int64_t*, void*, int, int, int, int, int,
+                    const float*, int, float, const int64_t*, const int64_t*, void*, int, int, int, int, int, int,
                     hipStream_t);
 int dxm_gather_rows(void*, const void*, const int64_t*, int, int, int64_t, int, hipStream_t);
 int dxm_residual_step(float*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const float*,
                       const void*, int64_t, const float*, float, int, const float*, const float*, void*, void*, int, int,
-                      int, hipStream_t);
-int dxm_act_mul(void*, const void*, int64_t, const void*, int64_t, int, int, int64_t, int, float, float, float, int,
-                hipStream_t);
+                      const void*, int64_t, const float*, const float*, const float*, const void*, const float*,
+                      const int*, int, int, const void*, int64_t, const int64_t*, int, hipStream_t);
+int dxm_act_mul(void*, const void*, int64_t, const void*, int64_t, int, int, int64_t, int, float, float, float,
+                const float*, const float*, const float*, int, int64_t, int, hipStream_t);
 int dxm_delta_rule(float*, float*, int, float*, const void*, int64_t, const void*, int64_t, const void*, int64_t, const void*,
                    int64_t, const void*, int64_t, const float*, const float*, float, float, const int64_t*, const int*,
                    const int*, int, int, int, int, int, int, hipStream_t);
@@ -53,7 +54,10 @@ int dxm_head_norm_gate(void*, const float*, const float*, const void*, int64_t, 
 int dxm_headprep_cache(void*, int64_t, const int64_t*, const int64_t*, int, int, int, int, int, const float*,
                        const float*, float, float, double, void*, void*, int, int, int, const void*, int64_t, float,
                        int, hipStream_t);
-int dxm_moe_route(int*, float*, const float*, const float*, int, int, int, int, int, int, int, hipStream_t);
+int dxm_moe_route(int*, float*, const float*, const float*, int, int, int, int, int, int, int, int, float, hipStream_t);
+int dxm_moe_router_ok(int, int, int);
+int dxm_moe_router(int*, float*, float*, const void*, int64_t, const float*, int, int, int, const float*, int, int, int,
+                   int, int, int, int, float, int, hipStream_t);
 int dxm_moe_plan(int*, int*, const int*, int, int, hipStream_t);
 int dxm_grouped_gemm(void*, const void*, int64_t, const void*, const int*, const int*, int, int, int, int, int, int,
                      int, int, hipStream_t);
@@ -98,9 +102,9 @@ PYBIND11_MODULE(_C_mixers, m) {
           "stream_step");
   });
   m.def("embed_streams", [](u X, u table, u ids, int rows, int S_, int W, int64_t vocab, u ptab, u pos, int64_t n_pos,
-                            float scale, int f32, u st) {
+                            float scale, u nw, float eps, int f32, u st) {
     check(dxm_embed_streams(F(X), P(table), reinterpret_cast<const int64_t*>(ids), rows, S_, W, vocab, P(ptab),
-                            reinterpret_cast<const int64_t*>(pos), n_pos, scale, f32, S(st)),
+                            reinterpret_cast<const int64_t*>(pos), n_pos, scale, F(nw), eps, f32, S(st)),
           "embed_streams");
   });
   m.def("section_norm", [](u out, u x, int64_t xs, u w, int rows, int n, float eps, int f32, u st) {
@@ -123,9 +127,10 @@ PYBIND11_MODULE(_C_mixers, m) {
           "linear_scan");
   });
   m.def("norm_rope_cache", [](u x, int64_t xs, u pos, u slots, int rows, int n_q, int n_k, int d, int v_w, u qw, u kw,
-                              float eps, u inv_freq, int half, u kc, u vc, int f32, u st) {
+                              float eps, u inv_freq, int half, u kc, u vc, int act_off, int act_n, int f32, u st) {
     check(dxm_norm_rope_cache(P(x), xs, reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int64_t*>(slots),
-                              rows, n_q, n_k, d, v_w, F(qw), F(kw), eps, F(inv_freq), half, P(kc), P(vc), f32, S(st)),
+                              rows, n_q, n_k, d, v_w, F(qw), F(kw), eps, F(inv_freq), half, P(kc), P(vc), act_off, act_n, f32,
+                              S(st)),
           "norm_rope_cache");
   });
   m.def("gate_group_norm", [](u out, int64_t os, u y, u z, int64_t zs, u w, int rows, int n_groups, int n, float eps,
@@ -135,10 +140,10 @@ PYBIND11_MODULE(_C_mixers, m) {
   });
   m.def("latent_rope", [](u q_out, u qa, u q, int64_t qs, int q_head, int q_off, u kv, int64_t kvs, u cn, float eps,
                           u inv_freq, int half, float mag, u pos, u slots, u cache, int T, int H, int r, int dr,
-                          int f32, u st) {
+                          int interleaved, int f32, u st) {
     check(dxm_latent_rope(P(q_out), P(qa), P(q), qs, q_head, q_off, P(kv), kvs, F(cn), eps, F(inv_freq), half, mag,
                           reinterpret_cast<const int64_t*>(pos), reinterpret_cast<const int64_t*>(slots), P(cache), T,
-                          H, r, dr, f32, S(st)),
+                          H, r, dr, interleaved, f32, S(st)),
           "latent_rope");
   });
   m.def("gather_rows", [](u out, u table, u ids, int rows, int W, int64_t vocab, int f32, u st) {
@@ -146,20 +151,32 @@ PYBIND11_MODULE(_C_mixers, m) {
           "gather_rows");
   });
   m.def("residual_step", [](u X, u a, int64_t as, u b, int64_t bs, u c, int64_t cs, u cw, u cg, int64_t cgs, u cgb,
-                            float eps, int norm, u nw, u nb, u out, u xc, int rows, int W, int f32, u st) {
+                            float eps, int norm, u nw, u nb, u out, u xc, int rows, int W, u d, int64_t ds, u dw, u e,
+                            u bias, u my, u mw, u midx, int experts, int top, u mh, int64_t mhs, u pick, int f32, u st) {
     check(dxm_residual_step(F(X), P(a), as, P(b), bs, P(c), cs, F(cw), P(cg), cgs, F(cgb), eps, norm, F(nw), F(nb),
-                            P(out), P(xc), rows, W, f32, S(st)),
+                            P(out), P(xc), rows, W, P(d), ds, F(dw), F(e), F(bias), P(my), F(mw),
+                            reinterpret_cast<const int*>(midx), experts, top, P(mh), mhs,
+                            reinterpret_cast<const int64_t*>(pick), f32, S(st)),
           "residual_step");
   });
   m.def("act_mul", [](u out, u gate, int64_t gs, u up, int64_t us, int rows, int Fw, int64_t os, int act, float limit,
-                      float alpha, float post, int f32, u st) {
-    check(dxm_act_mul(P(out), P(gate), gs, P(up), us, rows, Fw, os, act, limit, alpha, post, f32, S(st)), "act_mul");
+                      float alpha, float post, u gate_b, u up_b, u row_scale, int u_dv, int64_t u_head, int f32, u st) {
+    check(dxm_act_mul(P(out), P(gate), gs, P(up), us, rows, Fw, os, act, limit, alpha, post, F(gate_b), F(up_b),
+                      F(row_scale), u_dv, u_head, f32, S(st)),
+          "act_mul");
   });
   m.def("moe_route", [](u idx, u w, u z, u corr, int T, int E, int top, int n_groups, int keep, int score,
-                        int group_max, u st) {
+                        int group_max, int renorm, float scale, u st) {
     check(dxm_moe_route(reinterpret_cast<int*>(idx), F(w), F(z), F(corr), T, E, top, n_groups, keep, score, group_max,
-                        S(st)),
+                        renorm, scale, S(st)),
           "moe_route");
+  });
+  m.def("moe_router_ok", &dxm_moe_router_ok);
+  m.def("moe_router", [](u idx, u w, u gates, u h, int64_t hs, u rw, int n_out, int T, int W, u corr, int E, int top,
+                         int n_groups, int keep, int score, int group_max, int renorm, float scale, int f32, u st) {
+    check(dxm_moe_router(reinterpret_cast<int*>(idx), F(w), F(gates), P(h), hs, F(rw), n_out, T, W, F(corr), E, top,
+                         n_groups, keep, score, group_max, renorm, scale, f32, S(st)),
+          "moe_router");
   });
   m.def("delta_rule", [](u out, u state, int n_slots, u prep, u r, int64_t rs, u k, int64_t ks, u v, int64_t vs, u a,
                          int64_t as, u w, int64_t ws, u ab, u wb, float decay_scale, float key_eps, u pos, u seq_rows,

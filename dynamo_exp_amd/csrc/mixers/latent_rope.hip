@@ -11,7 +11,7 @@
 // of one shared head.
 //
 // Rotation: the first 2 * half columns of a dr-wide part, column i paired with
-// i + half, angle = position * inv_freq[i] (fp32, sincosf), cosine and sine
+// i + half or (interleaved) column 2 i with 2 i + 1, angle = position * inv_freq[i] (fp32, sincosf), cosine and sine
 // both multiplied by `mag`; columns from 2 * half on pass unchanged.
 // Norm sums, angles and the rotation are fp32 whatever the element type is.
 #include "../kernels/common.h"
@@ -75,7 +75,7 @@ struct LatentArgs {
 
 // VEC: elements per 16-byte chunk when r, dr, the rotated half, the row strides and the bases allow
 // whole chunks (the query rows, the bulk of the bytes, are then built chunk by chunk), else 1
-template <typename T, int VEC>
+template <typename T, int VEC, bool IL>
 __global__ void __launch_bounds__(256) latent_rope_kernel(LatentArgs g) {
   extern __shared__ float cs_sn[];  // [half] cosines, [half] sines, both times mag
   __shared__ float red[16];
@@ -100,6 +100,10 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatentArgs g) {
   auto rot = [&](const T* src, int e) -> float {
     const float x = ldf<T>(src, e);
     if (e >= 2 * g.half) return x;
+    if constexpr (IL) {
+      const float other = ldf<T>(src, e ^ 1);
+      return x * cs_sn[e >> 1] + (e & 1 ? other : -other) * cs_sn[g.half + (e >> 1)];
+    }
     const int i = e < g.half ? e : e - g.half;
     const float other = ldf<T>(src, e < g.half ? e + g.half : e - g.half);
     return e < g.half ? x * cs_sn[i] - other * cs_sn[g.half + i] : x * cs_sn[i] + other * cs_sn[g.half + i];
@@ -116,7 +120,8 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatentArgs g) {
     // work items of VEC columns per head: copies of qa, rotated pairs of runs (a run of the low half
     // with its partner of the high half, every angle used once), runs that are not rotated
     typedef uint32_t raw4 __attribute__((ext_vector_type(4)));
-    const int n_copy = g.r / VEC, n_pair = g.half / VEC, per = n_copy + n_pair + (g.dr - 2 * g.half) / VEC;
+    const int n_copy = g.r / VEC, n_pair = IL ? g.dr / VEC : g.half / VEC,
+              per = IL ? n_copy + n_pair : n_copy + n_pair + (g.dr - 2 * g.half) / VEC;
     for (int it = tid; it < g.H * per; it += blockDim.x) {
       const int h = it / per, j = it - h * per;
       T* dst = qo + (int64_t)h * Wc;
@@ -124,6 +129,20 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatentArgs g) {
       if (j < n_copy) {
         *reinterpret_cast<raw4*>(dst + j * VEC) =
             *reinterpret_cast<const raw4*>((const T*)g.qa + ((int64_t)h * g.T + t) * g.r + j * VEC);
+      } else if (IL) {  // a run of whole pairs, rotated or not
+        const int e0 = (j - n_copy) * VEC;
+        float x[VEC];
+        VecIO<T, VEC>::ld(src + e0, x);
+#pragma unroll
+        for (int e = 0; e < VEC; e += 2) {
+          const int i = (e0 + e) >> 1;
+          if (i < g.half) {
+            const float cs = cs_sn[i], sn = cs_sn[g.half + i], u = x[e];
+            x[e] = u * cs - x[e + 1] * sn;
+            x[e + 1] = x[e + 1] * cs + u * sn;
+          }
+        }
+        VecIO<T, VEC>::st(dst + g.r + e0, x);
       } else if (j < n_copy + n_pair) {
         const int e0 = (j - n_copy) * VEC;
         float x[VEC], y[VEC], lo[VEC], hi[VEC];
@@ -156,7 +175,7 @@ __global__ void __launch_bounds__(256) latent_rope_kernel(LatentArgs g) {
 extern "C" int dxm_latent_rope(void* q_out, const void* qa, const void* q, int64_t q_stride, int q_head, int q_off,
                                const void* kv, int64_t kv_stride, const float* cn, float eps, const float* inv_freq,
                                int half, float mag, const int64_t* pos, const int64_t* slots, void* cache, int T_, int H,
-                               int r, int dr, int f32, hipStream_t st) {
+                               int r, int dr, int interleaved, int f32, hipStream_t st) {
   if (T_ <= 0) return 0;
   if (H < 1 || r < 1 || dr < 0 || half < 0 || 2 * half > dr || half > 4096) return 1;
   if (!q_out || !qa || !kv || !cn || !pos || !slots || !cache || (dr && !q) || (half && !inv_freq)) return 2;
@@ -165,12 +184,16 @@ extern "C" int dxm_latent_rope(void* q_out, const void* qa, const void* q, int64
                pos, slots, cache, T_, H, r, dr};
   const size_t lds = (size_t)2 * half * sizeof(float);
   const int V = f32 ? 4 : 8;
-  const bool vec = r % V == 0 && dr % V == 0 && half % V == 0 && q_stride % V == 0 && q_head % V == 0 && q_off % V == 0 &&
+  const bool vec = r % V == 0 && dr % V == 0 && (interleaved || half % V == 0) && q_stride % V == 0 && q_head % V == 0 && q_off % V == 0 &&
                    (uintptr_t)q_out % 16 == 0 && (uintptr_t)qa % 16 == 0 && (uintptr_t)q % 16 == 0;
-  if (f32 && vec) hipLaunchKernelGGL((latent_rope_kernel<float, 4>), dim3(T_), dim3(256), lds, st, g);
-  else if (f32) hipLaunchKernelGGL((latent_rope_kernel<float, 1>), dim3(T_), dim3(256), lds, st, g);
-  else if (vec) hipLaunchKernelGGL((latent_rope_kernel<bf16_t, 8>), dim3(T_), dim3(256), lds, st, g);
-  else hipLaunchKernelGGL((latent_rope_kernel<bf16_t, 1>), dim3(T_), dim3(256), lds, st, g);
+#define LATENT_ROPE(T, V)                                                                                      \
+  if (interleaved) hipLaunchKernelGGL((latent_rope_kernel<T, V, true>), dim3(T_), dim3(256), lds, st, g);       \
+  else hipLaunchKernelGGL((latent_rope_kernel<T, V, false>), dim3(T_), dim3(256), lds, st, g);
+  if (f32 && vec) { LATENT_ROPE(float, 4) }
+  else if (f32) { LATENT_ROPE(float, 1) }
+  else if (vec) { LATENT_ROPE(bf16_t, 8) }
+  else { LATENT_ROPE(bf16_t, 1) }
+#undef LATENT_ROPE
   DX_CHECK_LAUNCH();
   return 0;
 }

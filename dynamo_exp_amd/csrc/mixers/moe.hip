@@ -28,27 +28,23 @@ __device__ __forceinline__ void wave_argmax(float& v, int& i) {
   }
 }
 
-// One wave per token.  c[e] = s[e] + corr[e] are the choice scores, s = sigmoid(z)
-// or softmax(z) over all experts; with n_groups > 1 only the experts of the `keep`
-// groups with the largest group score (the sum of their two best choice scores,
-// or with group_max their best) compete; the `top` best are written with weight
-// s (no correction).
-constexpr int kRouteWaves = 4;
-__global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __restrict__ idx, float* __restrict__ w,
-                                                                     const float* __restrict__ z,
-                                                                     const float* __restrict__ corr, int T, int E,
-                                                                     int top, int n_groups, int keep, int score,
-                                                                     int group_max) {
-  extern __shared__ float sm[];
-  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
-  const int64_t t = (int64_t)blockIdx.x * kRouteWaves + wv;
-  const bool on = t < T;
-  float* c = sm + wv * (E + n_groups);
-  float* gs = c + E;
-  const float* zt = z + (on ? t : 0) * E;
+// Expert choice of one token by one wave.  c[e] = s[e] + corr[e] are the choice scores, s = sigmoid(z)
+// or softmax(z) over all experts; with n_groups > 1 only the experts of the `keep` groups with the
+// largest group score (the sum of their two best choice scores, or with group_max their best)
+// compete; the `top` best are written with weight s (no correction), with renorm divided by the sum of
+// the chosen s (+ 1e-20), times scale.  zt [E] (global or LDS), c [E] and gs [n_groups] LDS of the wave.
+// Every wave of the workgroup calls this together (it holds barriers); `on`: the token exists.
+struct RouteArgs {
+  const float* corr;
+  int E, top, n_groups, keep, score, group_max, renorm;
+  float scale;
+};
+__device__ __forceinline__ void route_token(const RouteArgs& g, const float* zt, float* c, float* gs, bool on,
+                                            int* __restrict__ idx, float* __restrict__ w, int lane) {
+  const int E = g.E;
   // score 0: s = sigmoid(z); 1: s = softmax(z) over all experts (zmax, zinv: its maximum and 1 / sum)
   float zmax = 0.f, zinv = 1.f;
-  if (score == 1) {
+  if (g.score == 1) {
     float mxv = -INFINITY;
     for (int e = lane; e < E; e += 64) mxv = fmaxf(mxv, zt[e]);
     zmax = wave_reduce_max(mxv);
@@ -56,14 +52,14 @@ __global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __rest
     for (int e = lane; e < E; e += 64) sm_ += expf(zt[e] - zmax);
     zinv = 1.f / wave_reduce_sum(sm_);
   }
-  for (int e = lane; e < E; e += 64)
-    c[e] = (score == 1 ? expf(zt[e] - zmax) * zinv : 1.f / (1.f + expf(-zt[e]))) + (corr ? corr[e] : 0.f);
+  auto score = [&](int e) { return g.score == 1 ? expf(zt[e] - zmax) * zinv : 1.f / (1.f + expf(-zt[e])); };
+  for (int e = lane; e < E; e += 64) c[e] = score(e) + (g.corr ? g.corr[e] : 0.f);
   __syncthreads();
-  if (n_groups > 1) {
-    const int per = E / n_groups;
-    for (int g = lane; g < n_groups; g += 64) {
+  if (g.n_groups > 1) {
+    const int per = E / g.n_groups;
+    for (int q = lane; q < g.n_groups; q += 64) {
       float a = -INFINITY, b = -INFINITY;  // two largest
-      for (int e = g * per; e < (g + 1) * per; ++e) {
+      for (int e = q * per; e < (q + 1) * per; ++e) {
         const float v = c[e];
         if (v > a) {
           b = a;
@@ -72,29 +68,30 @@ __global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __rest
           b = v;
         }
       }
-      gs[g] = per > 1 && !group_max ? a + b : a;
+      gs[q] = per > 1 && !g.group_max ? a + b : a;
     }
     __syncthreads();
-    for (int k = 0; k < keep; ++k) {  // kept groups are marked +inf
+    for (int k = 0; k < g.keep; ++k) {  // kept groups are marked +inf
       float bv = -INFINITY;
       int bi = 0x7fffffff;
-      for (int g = lane; g < n_groups; g += 64) {
-        const float v = gs[g];
-        if (v != INFINITY && (v > bv || (v == bv && g < bi))) {
+      for (int q = lane; q < g.n_groups; q += 64) {
+        const float v = gs[q];
+        if (v != INFINITY && (v > bv || (v == bv && q < bi))) {
           bv = v;
-          bi = g;
+          bi = q;
         }
       }
       wave_argmax(bv, bi);
       __syncthreads();
-      if (lane == 0 && bi < n_groups) gs[bi] = INFINITY;
+      if (lane == 0 && bi < g.n_groups) gs[bi] = INFINITY;
       __syncthreads();
     }
     for (int e = lane; e < E; e += 64)
       if (gs[e / per] != INFINITY) c[e] = -INFINITY;
     __syncthreads();
   }
-  for (int k = 0; k < top; ++k) {
+  float mine = 0.f, sum = 0.f;  // renorm: lane k's chosen score (top <= 64)
+  for (int k = 0; k < g.top; ++k) {
     float bv = -INFINITY;
     int bi = 0x7fffffff;
     for (int e = lane; e < E; e += 64) {
@@ -107,23 +104,41 @@ __global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __rest
     wave_argmax(bv, bi);
     if (bi >= E) bi = 0;  // nothing left to choose (rejected on the host)
     __syncthreads();
-    if (lane == 0) {
-      c[bi] = -INFINITY;
-      if (on) {
-        idx[t * top + k] = bi;
-        w[t * top + k] = score == 1 ? expf(zt[bi] - zmax) * zinv : 1.f / (1.f + expf(-zt[bi]));
-      }
+    if (lane == 0) c[bi] = -INFINITY;
+    const float s = score(bi);
+    if (g.renorm) {
+      sum += s;
+      if (lane == k) mine = s;
+    }
+    if (lane == 0 && on) {
+      idx[k] = bi;
+      if (!g.renorm) w[k] = s * g.scale;
     }
     __syncthreads();
   }
+  if (g.renorm && on && lane < g.top) w[lane] = mine / (sum + 1e-20f) * g.scale;
+}
+
+// router logits z [T, E] given: one wave per token
+constexpr int kRouteWaves = 4;
+__global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __restrict__ idx, float* __restrict__ w,
+                                                                     const float* __restrict__ z, int T, RouteArgs g) {
+  extern __shared__ float sm[];
+  const int lane = threadIdx.x & 63, wv = threadIdx.x >> 6;
+  const int64_t t = (int64_t)blockIdx.x * kRouteWaves + wv;
+  const bool on = t < T;
+  float* c = sm + wv * (g.E + g.n_groups);
+  const int64_t tc = on ? t : 0;
+  route_token(g, z + tc * g.E, c, c + g.E, on, idx + tc * g.top, w + tc * g.top, lane);
 }
 
 // order [R]: slots sorted by expert, stable; offsets [E + 1].  One workgroup:
 // counts by LDS atomics (the counts do not depend on their order), a serial
 // scan over the experts, then every wave places the slots of its experts in
-// slot order with ballots.  STAGE: the choices are first copied into LDS as
-// bytes (E <= 256, R <= kPlanStage), so the placement passes read no global
-// memory.
+// slot order with ballots.  Choices that are no expert (identity outputs, >= E)
+// get no place: order holds offsets[E] slots.  STAGE: the choices are first
+// copied into LDS as bytes (E <= 255, R <= kPlanStage), so the placement passes
+// read no global memory.
 constexpr int kPlanThreads = 1024;
 constexpr int kPlanStage = 48 * 1024;
 template <bool STAGE>
@@ -140,7 +155,7 @@ __global__ void __launch_bounds__(kPlanThreads) moe_plan_kernel(int* __restrict_
     const int e = idx[r];
     const bool ok = e >= 0 && e < E;
     if (ok) atomicAdd(&cnt[e], 1);
-    if constexpr (STAGE) mine[r] = ok ? (unsigned char)e : 0;  // choices outside the experts are rejected by route
+    if constexpr (STAGE) mine[r] = ok ? (unsigned char)e : 255;
   }
   __syncthreads();
   if (tid == 0) {
@@ -235,6 +250,79 @@ template <typename T> struct Oct {
     if constexpr (sizeof(T) == 4) d[1] = s[1];
   }
 };
+
+// Router in one pass over the normed rows h [T, W]: logits z = h w^T with w [n_out, W] fp32 (the E router rows,
+// then n_out - E rows of gates), true fp32 products of h as it is and w on the fp32 matrix cores
+// (v_mfma_f32_16x16x4_f32), then the choice of every token (route_token); gates[t, j] = sigmoid(z[t, E + j]).
+// A workgroup takes 16 tokens; its NW waves share the width in pieces of 32, 32 outputs per pass, and their partial
+// sums are added in LDS in wave order.
+template <typename T, int NW>
+__global__ void __launch_bounds__(64 * NW) moe_router_kernel(int* __restrict__ idx, float* __restrict__ wgt,
+                                                             float* __restrict__ gates, const T* __restrict__ h,
+                                                             int64_t hs, const float* __restrict__ w, int n_out, int T_,
+                                                             int W, RouteArgs g) {
+  extern __shared__ float rsm[];
+  float* part = rsm;                 // [NW][32 outputs][16 rows + 1]
+  float* z = part + NW * 32 * 17;    // [16 rows][n_out]
+  float* scratch = z + 16 * n_out;   // [NW][E + n_groups]
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6, c16 = lane & 15, g4 = lane >> 4;
+  const int64_t t0 = (int64_t)blockIdx.x * 16;
+  const bool row_on = t0 + c16 < T_;
+  const T* hp = h + (row_on ? t0 + c16 : t0) * hs;
+  auto f = [](T v) -> float {
+    if constexpr (sizeof(T) == 2) return bf16_to_f32(v);
+    else return v;
+  };
+  for (int o0 = 0; o0 < n_out; o0 += 32) {
+    f32x4 C[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+    bool on[2];
+    const float* wp[2];
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+      on[i] = o0 + 16 * i + c16 < n_out;
+      wp[i] = w + (int64_t)(on[i] ? o0 + 16 * i + c16 : 0) * W;
+    }
+    for (int k0 = wv * 32 + 8 * g4; k0 - 8 * g4 < W; k0 += NW * 32) {
+      Oct<T> a;
+      Oct<float> b[2];
+      a.load(hp + k0, W - k0, row_on);
+      b[0].load(wp[0] + k0, W - k0, on[0]);
+      b[1].load(wp[1] + k0, W - k0, on[1]);
+#pragma unroll
+      for (int s = 0; s < 8; ++s) {  // the four lane groups supply k = 8 g4 + s
+        const float x = f(a.v[s]);
+        C[0] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[0].v[s], x, C[0], 0, 0, 0);
+        C[1] = __builtin_amdgcn_mfma_f32_16x16x4f32(b[1].v[s], x, C[1], 0, 0, 0);
+      }
+    }
+    __syncthreads();  // (the previous pass's sums are read)
+    // C[i]: outputs o0 + 16 i + 4 g4 + r of row c16
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) part[(wv * 32 + 16 * i + 4 * g4 + r) * 17 + c16] = C[i][r];
+    __syncthreads();
+    for (int it = tid; it < 32 * 16; it += 64 * NW) {
+      const int o = it >> 4, r = it & 15;
+      float acc = 0.f;
+#pragma unroll
+      for (int k = 0; k < NW; ++k) acc += part[(k * 32 + o) * 17 + r];
+      if (o0 + o < n_out) z[r * n_out + o0 + o] = acc;
+    }
+  }
+  __syncthreads();
+  const int n_gate = n_out - g.E;
+  for (int it = tid; it < 16 * n_gate; it += 64 * NW) {
+    const int r = it / n_gate, j = it - r * n_gate;
+    if (t0 + r < T_) gates[(t0 + r) * n_gate + j] = 1.f / (1.f + expf(-z[r * n_out + g.E + j]));
+  }
+  float* c = scratch + wv * (g.E + g.n_groups);
+  for (int r = wv; r < 16; r += NW) {
+    const bool on = t0 + r < T_;
+    const int64_t t = on ? t0 + r : t0;
+    route_token(g, z + r * n_out, c, c + g.E, on, idx + t * g.top, wgt + t * g.top, lane);
+  }
+}
 
 template <typename T>
 __global__ void __launch_bounds__(256) grouped_gemm_kernel(T* __restrict__ out, const T* __restrict__ a,
@@ -366,17 +454,57 @@ __global__ void __launch_bounds__(256) moe_combine_kernel(T* __restrict__ out, c
 
 extern "C" {
 
-int dxm_moe_route(int* idx, float* w, const float* z, const float* corr, int T, int E, int top, int n_groups,
-                  int keep, int score, int group_max, hipStream_t st) {
-  if (T <= 0) return 0;
-  if (score < 0 || score > 1) return 3;
-  if (E < 1 || n_groups < 1 || E % n_groups || keep < 1 || keep > n_groups || top < 1 ||
-      top > keep * (E / n_groups))
+static int route_args_bad(const RouteArgs& g) {
+  if (g.score < 0 || g.score > 1) return 3;
+  if (g.E < 1 || g.n_groups < 1 || g.E % g.n_groups || g.keep < 1 || g.keep > g.n_groups || g.top < 1 ||
+      g.top > g.keep * (g.E / g.n_groups))
     return 1;
+  if (g.renorm && g.top > 64) return 4;
+  return 0;
+}
+
+int dxm_moe_route(int* idx, float* w, const float* z, const float* corr, int T, int E, int top, int n_groups,
+                  int keep, int score, int group_max, int renorm, float scale, hipStream_t st) {
+  if (T <= 0) return 0;
+  const RouteArgs g{corr, E, top, n_groups, keep, score, group_max, renorm, scale};
+  if (const int bad = route_args_bad(g)) return bad;
   const size_t lds = (size_t)kRouteWaves * (E + n_groups) * sizeof(float);
   if (lds > 48 * 1024) return 2;
   hipLaunchKernelGGL(moe_route_kernel, dim3((T + kRouteWaves - 1) / kRouteWaves), dim3(64 * kRouteWaves), lds, st, idx,
-                     w, z, corr, T, E, top, n_groups, keep, score, group_max);
+                     w, z, T, g);
+  DX_CHECK_LAUNCH();
+  return 0;
+}
+
+// LDS of moe_router with nw waves (bytes); the launcher takes what fits 64 KB
+static size_t router_lds(int nw, int n_out, int E, int n_groups) {
+  return ((size_t)nw * 32 * 17 + 16 * (size_t)n_out + (size_t)nw * (E + n_groups)) * sizeof(float);
+}
+
+// 1 when moe_router takes this many outputs (else: logits by a GEMM, then moe_route)
+int dxm_moe_router_ok(int n_out, int E, int n_groups) {
+  return E >= 1 && n_out >= E && router_lds(8, n_out, E, n_groups) <= 60 * 1024;
+}
+
+int dxm_moe_router(int* idx, float* w, float* gates, const void* h, int64_t h_stride, const float* rw, int n_out, int T,
+                   int W, const float* corr, int E, int top, int n_groups, int keep, int score, int group_max, int renorm,
+                   float scale, int f32, hipStream_t st) {
+  if (T <= 0) return 0;
+  const RouteArgs g{corr, E, top, n_groups, keep, score, group_max, renorm, scale};
+  if (const int bad = route_args_bad(g)) return bad;
+  if (!dxm_moe_router_ok(n_out, E, n_groups) || W < 1) return 2;
+  if (!idx || !w || !h || !rw || (n_out > E && !gates)) return 5;
+  const dim3 grid((unsigned)((T + 15) / 16));
+  // few tokens: more waves share the width
+  const bool many = T <= 1024 && router_lds(16, n_out, E, n_groups) <= 60 * 1024;
+#define ROUTER(TY, NW)                                                                                               \
+  hipLaunchKernelGGL((moe_router_kernel<TY, NW>), grid, dim3(64 * NW), router_lds(NW, n_out, E, n_groups), st, idx, w, \
+                     gates, (const TY*)h, h_stride, rw, n_out, T, W, g);
+  if (f32 && many) { ROUTER(float, 16) }
+  else if (f32) { ROUTER(float, 8) }
+  else if (many) { ROUTER(bf16_t, 16) }
+  else { ROUTER(bf16_t, 8) }
+#undef ROUTER
   DX_CHECK_LAUNCH();
   return 0;
 }
@@ -385,7 +513,7 @@ int dxm_moe_plan(int* order, int* offsets, const int* idx, int R, int E, hipStre
   if (E < 1 || R < 0) return 1;
   const size_t lds = (size_t)(2 * E + 1) * sizeof(int);
   if (lds > 12 * 1024) return 2;
-  if (E <= 256 && R <= kPlanStage)
+  if (E <= 255 && R <= kPlanStage)
     hipLaunchKernelGGL(moe_plan_kernel<true>, dim3(1), dim3(kPlanThreads), lds + R, st, order, offsets, idx, R, E);
   else
     hipLaunchKernelGGL(moe_plan_kernel<false>, dim3(1), dim3(kPlanThreads), lds, st, order, offsets, idx, R, E);

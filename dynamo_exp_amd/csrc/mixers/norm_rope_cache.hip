@@ -5,7 +5,9 @@
 //   * every q and k head is then rotated: columns (2i, 2i + 1), i < half, by the
 //     angle position * inv_freq[i] (interleaved pairs); the rest pass unchanged;
 //   * q is written back in place, k and v go to the paged cache rows of the
-//     token's slot (slot < 0: nothing is cached).
+//     token's slot (slot < 0: nothing is cached);
+//   * another section of the row (the query, key and value of a second, recurrent
+//     mixer that reads the same input) takes silu in place, when one is given.
 // Norm sums, angles and the rotation are fp32 whatever the element type is.
 #include "recurrent.h"
 
@@ -36,6 +38,7 @@ struct NormRopeArgs {
   const float* inv_freq;  // [half]
   int half;
   void *kc, *vc;
+  int act_off, act_n;  // columns act_off .. + act_n of the row: z <- z sigmoid(z) (act_n 0: none)
 };
 
 // V: elements per work item -- 16-byte chunks where the sizes allow, pairs for even head widths, single
@@ -70,11 +73,12 @@ __global__ void __launch_bounds__(256) norm_rope_cache_kernel(NormRopeArgs g) {
       sum(it, a[k]);
     }
   }
-  for (int it = tid + 256 * kKeep; it < items; it += 256) {
-    float v[V];
-    VecIO<T, V>::ld(row + it * V, v);
-    sum(it, v);
-  }
+  if (g.qw || g.kw)
+    for (int it = tid + 256 * kKeep; it < items; it += 256) {
+      float v[V];
+      VecIO<T, V>::ld(row + it * V, v);
+      sum(it, v);
+    }
   sq = wave_reduce_sum(sq);
   sk = wave_reduce_sum(sk);
   if ((tid & 63) == 0) red[tid >> 6] = sq, red[4 + (tid >> 6)] = sk;
@@ -135,6 +139,13 @@ __global__ void __launch_bounds__(256) norm_rope_cache_kernel(NormRopeArgs g) {
       }
     }
   }
+  for (int c = tid * V; c < g.act_n; c += 256 * V) {
+    float z[V];
+    VecIO<T, V>::ld(row + g.act_off + c, z);
+#pragma unroll
+    for (int e = 0; e < V; ++e) z[e] *= fast_sigmoid(z[e]);
+    VecIO<T, V>::st(row + g.act_off + c, z);
+  }
   if (slot >= 0 && g.vc) {
     const T* v = row + nq + nk;
     T* dst = (T*)g.vc + slot * g.v_w;
@@ -155,17 +166,20 @@ template <typename T, int V> void launch_norm_rope(const NormRopeArgs& g, int ro
 
 extern "C" int dxm_norm_rope_cache(void* x, int64_t xs, const int64_t* pos, const int64_t* slots, int rows, int n_q,
                                    int n_k, int d, int v_w, const float* qw, const float* kw, float eps,
-                                   const float* inv_freq, int half, void* kc, void* vc, int f32, hipStream_t st) {
+                                   const float* inv_freq, int half, void* kc, void* vc, int act_off, int act_n,
+                                   int f32, hipStream_t st) {
   if (rows <= 0) return 0;
   if (n_q < 1 || n_k < 1 || d < 1 || v_w < 0 || half < 0 || 2 * half > d || half > 4096) return 1;
   if (!x || !pos || !slots || !kc || (v_w && !vc) || (half && !inv_freq)) return 2;
-  NormRopeArgs g{x, xs, pos, slots, n_q, n_k, d, v_w, qw, kw, eps, inv_freq, half, kc, v_w ? vc : nullptr};
+  if (act_n < 0 || (act_n && act_off < n_q * d + n_k * d + v_w)) return 3;
+  NormRopeArgs g{x, xs, pos, slots, n_q, n_k, d, v_w, qw, kw, eps, inv_freq, half, kc, v_w ? vc : nullptr,
+                 act_off, act_n};
   const int V = f32 ? 4 : 8;
   auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-  const bool vec = d % V == 0 && v_w % V == 0 && xs % V == 0 && al(x) && al(kc) && al(vc);
+  const bool vec = d % V == 0 && v_w % V == 0 && act_off % V == 0 && act_n % V == 0 && xs % V == 0 && al(x) && al(kc) && al(vc);
   if (vec && f32) launch_norm_rope<float, 4>(g, rows, st);
   else if (vec) launch_norm_rope<bf16_t, 8>(g, rows, st);
-  else if (d % 2 == 0) { DISPATCH_T(f32, (launch_norm_rope<T, 2>(g, rows, st))); }
+  else if (d % 2 == 0 && act_n % 2 == 0) { DISPATCH_T(f32, (launch_norm_rope<T, 2>(g, rows, st))); }
   else { DISPATCH_T(f32, (launch_norm_rope<T, 1>(g, rows, st))); }
   DX_CHECK_LAUNCH();
   return 0;

@@ -1,5 +1,5 @@
-// Attention of plain grouped-query heads (softmax weights, causal or window mask,
-// no score terms) over pages of whole 64-key tiles, for gfx950: the general
+// Attention of plain grouped-query heads (softmax weights, causal, window or chunk
+// mask, no score terms) over pages of whole 64-key tiles, for gfx950: the general
 // kernels of tile_attention.hip with the key loop laid out for this case.
 //   * tiles are the 64-key pieces of the pages (pages are multiples of 64 keys),
 //     so a tile's rows are one scalar base plus lane constants;
@@ -32,7 +32,7 @@ struct StreamArgs {
   int n_qh, maps, group;
   int Wk, Wv;
   float scale_log2;
-  int size;  // window (0: causal)
+  int mask, size;
   int parts;
 };
 
@@ -59,6 +59,12 @@ __device__ __forceinline__ void put_v(bf16_t* Vt, const raw_u32x4* r, int kg, in
 __device__ __forceinline__ bf16x8_t frag16(const bf16_t* p) {
   return __builtin_bit_cast(bf16x8_t, *reinterpret_cast<const raw_u32x4*>(p));
 }
+// first key that the query at position p sees (mask 0: causal, 1: window, 2: chunk)
+__device__ __forceinline__ int first_key(int p, int mask, int size) {
+  if (mask == 1) return p - size + 1 > 0 ? p - size + 1 : 0;
+  if (mask == 2) return (int)((unsigned)p / (unsigned)size) * size;
+  return 0;
+}
 __device__ __forceinline__ f32x4 mma(bf16x8_t a, bf16x8_t b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
@@ -77,7 +83,7 @@ __global__ void __launch_bounds__(64, 2) stream_decode_kernel(StreamArgs a) {
   const int gm = blockIdx.x, row = blockIdx.y, part = blockIdx.z;
   const int g = gm / a.maps, m = gm - g * a.maps;
   const int p = __builtin_amdgcn_readfirstlane((int)a.pos[row]);
-  const int lo = a.size && p - a.size + 1 > 0 ? p - a.size + 1 : 0;
+  const int lo = first_key(p, a.mask, a.size);
   const int first = lo >> 6, n_tiles = (p >> 6) - first + 1;
   const int tpp = (n_tiles + a.parts - 1) / a.parts;
   const int t0 = first + part * tpp, t1 = min(t0 + tpp, first + n_tiles);
@@ -237,7 +243,7 @@ struct StreamTileArgs {
   int n_qh, group;
   int Wk, Wv;
   float scale_log2;
-  int size;
+  int mask, size;
 };
 
 // element offset of 16-byte piece pc of key r in the [64][D] image (16 pieces: an XOR with the row; 8: with its pair)
@@ -265,20 +271,21 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
   const int g = blockIdx.x / per, qh = g * a.group + (blockIdx.x - g * per) * HPW + wave / RT;
   const int rw = 32 * (wave % RT);  // the wave's first row
   const int hi = p0 + min(n, ROWS) - 1;
-  const int lo0 = a.size && p0 - a.size + 1 > 0 ? p0 - a.size + 1 : 0;
-  const int first = lo0 >> 6, last = hi >> 6;
+  const int first = first_key(p0, a.mask, a.size) >> 6, last = hi >> 6;
   // the wave's rows: 16 qb + c16; rows beyond n repeat the last one and are not stored
   bf16x8_t qf[2][NK];
-  int prow[2];
+  int prow[2], lrow[2];  // position and first visible key of the lane's rows
 #pragma unroll
   for (int qb = 0; qb < 2; ++qb) {
     const int r = min(rw + 16 * qb + c16, n - 1);
     prow[qb] = p0 + r;
+    lrow[qb] = first_key(p0 + r, a.mask, a.size);
 #pragma unroll
     for (int ks = 0; ks < NK; ++ks)
       qf[qb][ks] = frag16(a.q + (int64_t)(row0 + r) * a.q_stride + (int64_t)qh * D + 32 * ks + 8 * g4);
   }
   const int wlo = p0 + min(rw, n - 1), whi = p0 + min(rw + 31, n - 1);  // first and last row position of the wave
+  const int wfirst = first_key(wlo, a.mask, a.size), wlast = first_key(whi, a.mask, a.size);
   const bool upper = tid >= 256;
   const int ht = tid & 255;
   const bf16_t* kl = a.kc + (int64_t)g * D + (int64_t)(ht / KCH) * a.Wk + 8 * (ht % KCH);
@@ -326,7 +333,7 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
       if (t + 1 < last) fetch(t + 2);
     }
     const int kt = t << 6;
-    if (rw >= n || kt > whi || (a.size && kt + 63 < wlo - a.size + 1)) continue;  // nothing the wave's rows see
+    if (rw >= n || kt > whi || kt + 63 < wfirst) continue;  // nothing the wave's rows see
     const bf16_t *K = Ks[cur], *V = Vt[cur];
     f32x4 S[2][4];
 #pragma unroll
@@ -339,15 +346,15 @@ __global__ void __launch_bounds__(512, 2) stream_prefill_kernel(StreamTileArgs a
         S[1][kb] = mma(kf, qf[1][ks], S[1][kb]);
       }
     }
-    if (kt + 63 > wlo || (a.size && kt < whi - a.size + 1)) {  // some key is not seen by some row
+    if (kt + 63 > wlo || kt < wlast) {  // some key is not seen by some row
 #pragma unroll
       for (int qb = 0; qb < 2; ++qb)
 #pragma unroll
         for (int kb = 0; kb < 4; ++kb)
 #pragma unroll
           for (int r = 0; r < 4; ++r) {
-            const int dist = prow[qb] - (kt + 16 * kb + 4 * g4 + r);
-            if (dist < 0 || (a.size && dist >= a.size)) S[qb][kb][r] = -INFINITY;
+            const int j = kt + 16 * kb + 4 * g4 + r;
+            if (j > prow[qb] || j < lrow[qb]) S[qb][kb][r] = -INFINITY;
           }
     }
     bf16x8_t P[2][2], Pl[2][2];  // weights (FINE: hi and lo)
@@ -435,7 +442,7 @@ extern "C" {
 // 1 when the prompt kernel takes these heads: one map, an even number of heads per key/value head
 int dxm_stream_prefill_ok(int d, int dv, int maps, int group, int bs, int mask) {
   return ((d == 128 && dv == 128) || (d == 64 && dv == 64)) && maps == 1 && group % 2 == 0 && bs >= 64 &&
-         (bs & (bs - 1)) == 0 && (mask == 0 || mask == 1);
+         (bs & (bs - 1)) == 0 && mask >= 0 && mask <= 2;
 }
 
 int dxm_stream_prefill(void* out, const void* q, int64_t q_stride, const void* kc, const void* vc, const int64_t* pos,
@@ -451,7 +458,7 @@ int dxm_stream_prefill(void* out, const void* q, int64_t q_stride, const void* k
     return 4;
   StreamTileArgs a{(bf16_t*)out, (const bf16_t*)q, q_stride, (const bf16_t*)kc, (const bf16_t*)vc, pos, seq, bt, bt_stride,
                    __builtin_ctz((unsigned)bs), tiles, 1, n_qh, group, Wk, Wv, scale * 1.4426950408889634f,
-                   mask ? size : 0};
+                   mask, size};
 #define STREAM_PREFILL(D, HPW)                                  \
   if (fine) launch_stream_prefill<D, HPW, true>(a, n_tiles, st); \
   else launch_stream_prefill<D, HPW, false>(a, n_tiles, st);
@@ -467,7 +474,7 @@ int dxm_stream_prefill(void* out, const void* q, int64_t q_stride, const void* k
 // 1 when the decode kernel takes these heads: widths it is instantiated for, pages of whole 64-key tiles
 int dxm_stream_decode_ok(int d, int dv, int group, int bs, int mask) {
   return ((d == 128 && dv == 128) || (d == 64 && dv == 64)) && group >= 1 && group <= 16 && bs >= 64 &&
-         (bs & (bs - 1)) == 0 && (mask == 0 || mask == 1);
+         (bs & (bs - 1)) == 0 && mask >= 0 && mask <= 2;
 }
 
 int dxm_stream_decode(float* ws, const void* q, int64_t q_stride, const void* kc, const void* vc, const int64_t* pos,
@@ -479,7 +486,7 @@ int dxm_stream_decode(float* ws, const void* q, int64_t q_stride, const void* kc
   if ((mask && size < 1) || parts < 1 || parts > 65535 || !(scale > 0.f)) return 3;
   if (!ws || Wk % 8 || Wv % 8 || q_stride % 8 || (uintptr_t)q % 16 || (uintptr_t)kc % 16 || (uintptr_t)vc % 16) return 4;
   StreamArgs a{(const bf16_t*)q, q_stride, (const bf16_t*)kc, (const bf16_t*)vc, ws, pos, seq, bt, bt_stride,
-               __builtin_ctz((unsigned)bs), n_qh, maps, group, Wk, Wv, scale * 1.4426950408889634f, mask ? size : 0, parts};
+               __builtin_ctz((unsigned)bs), n_qh, maps, group, Wk, Wv, scale * 1.4426950408889634f, mask, size, parts};
   const dim3 grid(n_qh / group, rows, parts);
   if (d == 128) hipLaunchKernelGGL((stream_decode_kernel<128, 128>), grid, dim3(64), 0, st, a);
   else hipLaunchKernelGGL((stream_decode_kernel<64, 64>), grid, dim3(64), 0, st, a);

@@ -147,21 +147,37 @@ __global__ void __launch_bounds__(kThreads) stream_step_kernel(float* __restrict
 }
 
 // X[t, s, :] = table[ids[t], :] * scale (+ ptab[pos[t], :], a learned vector per position)
-// for every stream s (fp32 streams; product and sum are fp32)
+// for every stream s (fp32 streams; product and sum are fp32); with nw [W] the row is then
+// divided by its root mean square (eps inside the root) and multiplied by nw
 template <typename T>
 __global__ void __launch_bounds__(kThreads) embed_streams_kernel(float* __restrict__ X, const T* __restrict__ table,
                                                                  const int64_t* __restrict__ ids, int S, int W,
                                                                  int64_t vocab, const T* __restrict__ ptab,
                                                                  const int64_t* __restrict__ pos, int64_t n_pos,
-                                                                 float scale) {
+                                                                 float scale, const float* __restrict__ nw, float eps) {
+  __shared__ float red[16];
   const int64_t t = blockIdx.x;
   const int64_t id = ids[t];
   const bool ok = id >= 0 && id < vocab;
   const int64_t p = ptab ? pos[t] : -1;
   const bool pok = p >= 0 && p < n_pos;
-  for (int c = threadIdx.x; c < W; c += kThreads) {
+  auto value = [&](int c) {
     float v = ok ? ldf<T>(table, id * (int64_t)W + c) * scale : 0.f;
     if (pok) v += ldf<T>(ptab, p * (int64_t)W + c);
+    return v;
+  };
+  float r = 1.f;
+  if (nw) {
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < W; c += kThreads) {
+      const float v = value(c);
+      ss += v * v;
+    }
+    r = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
+  }
+  for (int c = threadIdx.x; c < W; c += kThreads) {
+    float v = value(c);
+    if (nw) v *= r * nw[c];
     for (int s = 0; s < S; ++s) X[(t * S + s) * (int64_t)W + c] = v;
   }
 }
@@ -183,17 +199,37 @@ __global__ void __launch_bounds__(kThreads) gather_rows_kernel(T* __restrict__ o
 //     norm 2 (layer):  out = (x - mean) / sqrt(mean((x - mean)^2) + eps) * nw + nb
 // The row stays in registers between the passes (W <= kThreads * V * kResChunks)
 // or is re-read from x by the thread that wrote it.
+// EXT (further addends, all optional; ResExt below): a second normed addend d,
+// an fp32 addend e, a constant row `bias`, the weighted sum of a mixture of
+// experts, and a list of rows: then row r of out is the result for row rows[r],
+// and x itself is left as it was.
 constexpr int kResChunks = 8;
-template <typename T, int V>
+template <typename T> struct ResExt {
+  const T* d;         // + d / sqrt(mean(d^2) + eps) * dw
+  int64_t d_stride;
+  const float* dw;
+  const float* e;     // + e, [rows, W] fp32
+  const float* bias;  // + bias, [W]
+  // + sum_k mw[row, k] * src_k: my[row * top + k] (expert outputs in slot order), or the row of mh
+  // where the choice midx[row, k] is no expert (>= experts: an identity output)
+  const T* my;
+  const float* mw;
+  const int* midx;
+  int experts, top;
+  const T* mh;
+  int64_t mh_stride;
+  const int64_t* rows;
+};
+template <typename T, int V, bool EXT>
 __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     float* __restrict__ X, const T* __restrict__ a, int64_t a_stride, const T* __restrict__ b, int64_t b_stride,
     const T* __restrict__ c, int64_t c_stride, const float* __restrict__ cw, const T* __restrict__ cg,
     int64_t cg_stride, const float* __restrict__ cgb, float eps, int norm, const float* __restrict__ nw,
-    const float* __restrict__ nb, T* __restrict__ out, T* __restrict__ xc, int W) {
+    const float* __restrict__ nb, T* __restrict__ out, T* __restrict__ xc, int W, ResExt<T> g) {
   __shared__ float red[16];
-  const int64_t row = blockIdx.x;
+  const int64_t row = EXT && g.rows ? g.rows[blockIdx.x] : (int64_t)blockIdx.x, orow = blockIdx.x;
   float* x = X + row * (int64_t)W;
-  float rc = 0.f;
+  float rc = 0.f, rd = 0.f;
   // the addend c at columns e .. e + V - 1, gated by sigmoid(cg + cgb) when a gate is given
   auto load_c = [&](int e, float* v) {
     ldv<T, V>(c + row * c_stride + e, v);
@@ -205,88 +241,127 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
       for (int i = 0; i < V; ++i) v[i] *= 1.f / (1.f + expf(-(gt[i] + (cgb ? gb[i] : 0.f))));
     }
   };
-  // (gated) addend: its chunks stay in registers between the mean square and the sum
-  float cv[kResChunks][V];
-  if (c) {
+  auto load_d = [&](int e, float* v) { ldv<T, V>(g.d + row * g.d_stride + e, v); };
+  // root mean square of an addend; its chunks stay in registers between the mean square and the sum
+  auto inv_rms = [&](auto&& load, float (*keep)[V]) {
     float ss = 0.f;
 #pragma unroll
     for (int k = 0; k < kResChunks; ++k) {
       const int e = (threadIdx.x + k * kThreads) * V;
       if (e < W) {
-        load_c(e, cv[k]);
+        load(e, keep[k]);
 #pragma unroll
-        for (int i = 0; i < V; ++i) ss += cv[k][i] * cv[k][i];
+        for (int i = 0; i < V; ++i) ss += keep[k][i] * keep[k][i];
       }
     }
     for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
       float v[V];
-      load_c(e, v);
+      load(e, v);
 #pragma unroll
       for (int i = 0; i < V; ++i) ss += v[i] * v[i];
     }
-    rc = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
+    const float r = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
     __syncthreads();
+    return r;
+  };
+  float cv[kResChunks][V], dv[EXT ? kResChunks : 1][V];
+  if (c) rc = inv_rms(load_c, cv);
+  if constexpr (EXT) {
+    if (g.d) rd = inv_rms(load_d, dv);
   }
+  // everything added at columns e .. e + V - 1; ct, dt: the values of c and d there
+  auto add = [&](int e, float* v, const float* ct, const float* dt) {
+    float t[V], w[V];
+    if (a) {
+      ldv<T, V>(a + row * a_stride + e, t);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += t[i];
+    }
+    if (b) {
+      ldv<T, V>(b + row * b_stride + e, t);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += t[i];
+    }
+    if (c) {
+      ldv<float, V>(cw + e, w);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += ct[i] * rc * w[i];
+    }
+    if constexpr (EXT) {
+      if (g.d) {
+        ldv<float, V>(g.dw + e, w);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] += dt[i] * rd * w[i];
+      }
+      if (g.bias) {
+        ldv<float, V>(g.bias + e, w);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] += w[i];
+      }
+      if (g.my) {
+        float m[V];
+#pragma unroll
+        for (int i = 0; i < V; ++i) m[i] = 0.f;
+        for (int k = 0; k < g.top; ++k) {
+          const int64_t s = row * g.top + k;
+          const float wk = g.mw[s];
+          ldv<T, V>((g.midx && g.midx[s] >= g.experts ? g.mh + row * g.mh_stride : g.my + s * (int64_t)W) + e, t);
+#pragma unroll
+          for (int i = 0; i < V; ++i) m[i] += wk * t[i];
+        }
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] += m[i];
+      }
+      if (g.e) {
+        ldv<float, V>(g.e + row * (int64_t)W + e, w);
+#pragma unroll
+        for (int i = 0; i < V; ++i) v[i] += w[i];
+      }
+    }
+  };
+  bool touch = a || b || c;
+  if constexpr (EXT) touch = !g.rows && (touch || g.d || g.e || g.bias || g.my);
+  // a wide row's tail: x and its addends from memory
+  auto wide = [&](int e, float* v) {
+    float ct[V], dt[V];
+    ldv<float, V>(x + e, v);
+    if (c) load_c(e, ct);
+    if constexpr (EXT) {
+      if (g.d) load_d(e, dt);
+    }
+    add(e, v, ct, dt);
+  };
   const bool keep = W <= kThreads * V * kResChunks;
   float r[kResChunks][V];
   float sum = 0.f;
-  const bool touch = a || b || c;
 #pragma unroll
   for (int k = 0; k < kResChunks; ++k) {
     const int e = (threadIdx.x + k * kThreads) * V;
     if (e < W) {
       ldv<float, V>(x + e, r[k]);
-      float t[V];
-      if (a) {
-        ldv<T, V>(a + row * a_stride + e, t);
-#pragma unroll
-        for (int i = 0; i < V; ++i) r[k][i] += t[i];
-      }
-      if (b) {
-        ldv<T, V>(b + row * b_stride + e, t);
-#pragma unroll
-        for (int i = 0; i < V; ++i) r[k][i] += t[i];
-      }
-      if (c) {
-        float w[V];
-        ldv<float, V>(cw + e, w);
-#pragma unroll
-        for (int i = 0; i < V; ++i) r[k][i] += cv[k][i] * rc * w[i];
-      }
+      add(e, r[k], cv[k], dv[EXT ? k : 0]);
       if (touch) stv<float, V>(x + e, r[k]);
-      if (xc) stv<T, V>(xc + row * (int64_t)W + e, r[k]);
+      if (xc) stv<T, V>(xc + orow * (int64_t)W + e, r[k]);
 #pragma unroll
       for (int i = 0; i < V; ++i) sum += r[k][i];
     }
   }
   if (!keep) {  // wide rows: the same arithmetic, chunk by chunk through x
     for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
-      float v[V], t[V];
-      ldv<float, V>(x + e, v);
-      if (a) {
-        ldv<T, V>(a + row * a_stride + e, t);
-#pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += t[i];
-      }
-      if (b) {
-        ldv<T, V>(b + row * b_stride + e, t);
-#pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += t[i];
-      }
-      if (c) {
-        float w[V];
-        load_c(e, t);
-        ldv<float, V>(cw + e, w);
-#pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += t[i] * rc * w[i];
-      }
+      float v[V];
+      wide(e, v);
       if (touch) stv<float, V>(x + e, v);
-      if (xc) stv<T, V>(xc + row * (int64_t)W + e, v);
+      if (xc) stv<T, V>(xc + orow * (int64_t)W + e, v);
 #pragma unroll
       for (int i = 0; i < V; ++i) sum += v[i];
     }
   }
   if (!norm) return;
+  // a wide row's tail once more: as this thread wrote it, or (x left as it was) summed again
+  auto again = [&](int e, float* v) {
+    if (touch || !EXT || !g.rows) ldv<float, V>(x + e, v);
+    else wide(e, v);
+  };
   float mean = 0.f;
   if (norm == 2) {
     mean = block_reduce_sum(sum, red) / (float)W;
@@ -304,7 +379,7 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
   if (!keep) {
     for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
       float v[V];
-      ldv<float, V>(x + e, v);
+      again(e, v);
 #pragma unroll
       for (int i = 0; i < V; ++i) ss += (v[i] - mean) * (v[i] - mean);
     }
@@ -319,18 +394,18 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
       if (norm == 2) ldv<float, V>(nb + e, bb);
 #pragma unroll
       for (int i = 0; i < V; ++i) o[i] = (r[k][i] - mean) * rs * w[i] + (norm == 2 ? bb[i] : 0.f);
-      stv<T, V>(out + row * (int64_t)W + e, o);
+      stv<T, V>(out + orow * (int64_t)W + e, o);
     }
   }
   if (!keep) {
     for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
       float v[V], w[V], bb[V], o[V];
-      ldv<float, V>(x + e, v);
+      again(e, v);
       ldv<float, V>(nw + e, w);
       if (norm == 2) ldv<float, V>(nb + e, bb);
 #pragma unroll
       for (int i = 0; i < V; ++i) o[i] = (v[i] - mean) * rs * w[i] + (norm == 2 ? bb[i] : 0.f);
-      stv<T, V>(out + row * (int64_t)W + e, o);
+      stv<T, V>(out + orow * (int64_t)W + e, o);
     }
   }
 }
@@ -462,19 +537,34 @@ __device__ __forceinline__ float act_fn(float z, int act) {
   return 0.5f * z * (1.f + tanhf(c * (z + 0.044715f * z * z * z)));
 }
 
-// out [rows, F] = act(gate) * up  (up null: act(gate)); gate and up are column
-// sections of wider rows (a gated feed-forward's [gate | up], an output gate
-// that is part of a fused projection)
+// out [rows, F] = act(gate + gate_b) * (up + up_b) * row_scale[row] * post  (up null: act(gate) alone); gate and
+// up are column sections of wider rows (a gated feed-forward's [gate | up], an output gate that is part of a
+// fused projection).  u_dv > 0: up is head-major, column c of row r at up[(c / u_dv) * u_head + r * u_stride + c % u_dv].
 template <typename T, int V>
 __global__ void __launch_bounds__(kThreads) act_mul_kernel(T* __restrict__ out, const T* __restrict__ gate,
                                                            int64_t g_stride, const T* __restrict__ up,
                                                            int64_t u_stride, int F, int64_t out_stride, int act,
-                                                           float limit, float alpha, float post) {
+                                                           float limit, float alpha, float post,
+                                                           const float* __restrict__ gate_b,
+                                                           const float* __restrict__ up_b,
+                                                           const float* __restrict__ row_scale, int u_dv,
+                                                           int64_t u_head) {
   const int64_t r = blockIdx.y;
+  if (row_scale) post *= row_scale[r];
   for (int c = (blockIdx.x * kThreads + threadIdx.x) * V; c < F; c += gridDim.x * kThreads * V) {
-    float g[V], u[V], o[V];
+    float g[V], u[V], o[V], t[V];
     ldv<T, V>(gate + r * g_stride + c, g);
-    if (up) ldv<T, V>(up + r * u_stride + c, u);
+    if (up) ldv<T, V>(up + r * u_stride + (u_dv ? c / u_dv * u_head + c % u_dv : (int64_t)c), u);
+    if (gate_b) {
+      ldv<float, V>(gate_b + c, t);
+#pragma unroll
+      for (int e = 0; e < V; ++e) g[e] += t[e];
+    }
+    if (up && up_b) {
+      ldv<float, V>(up_b + c, t);
+#pragma unroll
+      for (int e = 0; e < V; ++e) u[e] += t[e];
+    }
 #pragma unroll
     for (int e = 0; e < V; ++e) {
       if (act == 6) {  // clamped gated unit: g sigmoid(alpha g) (u + 1), g <= limit, |u| <= limit
@@ -628,11 +718,12 @@ int dxm_stream_step(float* X, const void* y, int64_t y_stride, const float* mix,
 }
 
 int dxm_embed_streams(float* X, const void* table, const int64_t* ids, int rows, int S, int W, int64_t vocab,
-                      const void* ptab, const int64_t* pos, int64_t n_pos, float scale, int f32, hipStream_t st) {
+                      const void* ptab, const int64_t* pos, int64_t n_pos, float scale, const float* nw, float eps, int f32,
+                      hipStream_t st) {
   if (rows <= 0) return 0;
   if (ptab && !pos) return 1;
   DISPATCH_T(f32, hipLaunchKernelGGL(embed_streams_kernel<T>, dim3(rows), dim3(kThreads), 0, st, X, (const T*)table,
-                                     ids, S, W, vocab, (const T*)ptab, pos, n_pos, scale));
+                                     ids, S, W, vocab, (const T*)ptab, pos, n_pos, scale, nw, eps));
   DX_CHECK_LAUNCH();
   return 0;
 }
@@ -648,55 +739,59 @@ int dxm_gather_rows(void* out, const void* table, const int64_t* ids, int rows, 
 
 int dxm_residual_step(float* X, const void* a, int64_t a_stride, const void* b, int64_t b_stride, const void* c,
                       int64_t c_stride, const float* cw, const void* cg, int64_t cg_stride, const float* cgb, float eps,
-                      int norm, const float* nw, const float* nb, void* out, void* xc, int rows, int W, int f32,
-                      hipStream_t st) {
+                      int norm, const float* nw, const float* nb, void* out, void* xc, int rows, int W, const void* d,
+                      int64_t d_stride, const float* dw, const float* e, const float* bias, const void* my,
+                      const float* mw, const int* midx, int experts, int top, const void* mh, int64_t mh_stride,
+                      const int64_t* pick, int f32, hipStream_t st) {
   if (rows <= 0) return 0;
   if (W < 1 || norm < 0 || norm > 2) return 1;
-  if ((c && !cw) || (norm && (!nw || !out)) || (norm == 2 && !nb) || (cg && !c)) return 2;
+  if ((c && !cw) || (norm && (!nw || !out)) || (norm == 2 && !nb) || (cg && !c) || (d && !dw)) return 2;
+  if (my && (!mw || top < 1 || (midx && !mh))) return 3;
   const int esz = f32 ? 4 : 2;
   auto al = [&](const void* p, int by) { return (uintptr_t)p % by == 0; };
   const bool vec = W % 4 == 0 && a_stride % 4 == 0 && b_stride % 4 == 0 && c_stride % 4 == 0 && cg_stride % 4 == 0 &&
-                   al(X, 16) && al(a, 4 * esz) && al(b, 4 * esz) && al(c, 4 * esz) && al(cg, 4 * esz) && al(cgb, 16) &&
-                   al(cw, 16) && al(nw, 16) && al(nb, 16) &&
-                   al(out, 4 * esz) && al(xc, 4 * esz);
-  if (vec) {
-    DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, 4>), dim3(rows), dim3(kThreads), 0, st, X, (const T*)a,
-                                       a_stride, (const T*)b, b_stride, (const T*)c, c_stride, cw, (const T*)cg, cg_stride, cgb, eps,
-                                       norm, nw, nb,
-                                       (T*)out, (T*)xc, W));
-  } else {
-    DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, 1>), dim3(rows), dim3(kThreads), 0, st, X, (const T*)a,
-                                       a_stride, (const T*)b, b_stride, (const T*)c, c_stride, cw, (const T*)cg, cg_stride, cgb, eps,
-                                       norm, nw, nb,
-                                       (T*)out, (T*)xc, W));
-  }
+                   d_stride % 4 == 0 && mh_stride % 4 == 0 && al(X, 16) && al(a, 4 * esz) && al(b, 4 * esz) &&
+                   al(c, 4 * esz) && al(cg, 4 * esz) && al(cgb, 16) && al(cw, 16) && al(nw, 16) && al(nb, 16) &&
+                   al(out, 4 * esz) && al(xc, 4 * esz) && al(d, 4 * esz) && al(dw, 16) && al(e, 16) && al(bias, 16) &&
+                   al(my, 4 * esz) && al(mh, 4 * esz);
+  const bool ext = d || e || bias || my || pick;
+#define RES(V, EXT)                                                                                                     \
+  DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, V, EXT>), dim3(rows), dim3(kThreads), 0, st, X,           \
+                                     (const T*)a, a_stride, (const T*)b, b_stride, (const T*)c, c_stride, cw,           \
+                                     (const T*)cg, cg_stride, cgb, eps, norm, nw, nb, (T*)out, (T*)xc, W,               \
+                                     (ResExt<T>{(const T*)d, d_stride, dw, e, bias, (const T*)my, mw, midx, experts,    \
+                                                top, (const T*)mh, mh_stride, pick})))
+  if (vec && ext) { RES(4, true) }
+  else if (vec) { RES(4, false) }
+  else if (ext) { RES(1, true) }
+  else { RES(1, false) }
+#undef RES
   DX_CHECK_LAUNCH();
   return 0;
 }
 
 int dxm_act_mul(void* out, const void* gate, int64_t g_stride, const void* up, int64_t u_stride, int rows, int F,
-                int64_t out_stride, int act, float limit, float alpha, float post, int f32, hipStream_t st) {
+                int64_t out_stride, int act, float limit, float alpha, float post, const float* gate_b,
+                const float* up_b, const float* row_scale, int u_dv, int64_t u_head, int f32, hipStream_t st) {
   if (rows <= 0 || F <= 0) return 0;
   if (act < 0 || act > 6 || (act == 6 && (!up || !(limit > 0.f)))) return 1;
+  if (u_dv < 0 || (u_dv && (!up || F % u_dv))) return 2;
   const int esz = f32 ? 4 : 2;
-  const bool vec = F % 4 == 0 && g_stride % 4 == 0 && u_stride % 4 == 0 && out_stride % 4 == 0 &&
-                   (uintptr_t)gate % (4 * esz) == 0 && (uintptr_t)up % (4 * esz) == 0 &&
-                   (uintptr_t)out % (4 * esz) == 0;
+  const bool vec = F % 4 == 0 && g_stride % 4 == 0 && u_stride % 4 == 0 && out_stride % 4 == 0 && u_dv % 4 == 0 &&
+                   u_head % 4 == 0 && (uintptr_t)gate % (4 * esz) == 0 && (uintptr_t)up % (4 * esz) == 0 &&
+                   (uintptr_t)out % (4 * esz) == 0 && (uintptr_t)gate_b % 16 == 0 && (uintptr_t)up_b % 16 == 0;
   const int per = kThreads * (vec ? 4 : 1);
   const int gx = (F + per - 1) / per;
   for (int r0 = 0; r0 < rows; r0 += 65535) {
     const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
-    if (vec) {
-      DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, 4>), dim3(gx, nr), dim3(kThreads), 0, st,
-                                         (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,
-                                         up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act,
-                                         limit, alpha, post));
-    } else {
-      DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, 1>), dim3(gx, nr), dim3(kThreads), 0, st,
-                                         (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,
-                                         up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act,
-                                         limit, alpha, post));
-    }
+#define ACT_MUL(V)                                                                                                     \
+  DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, V>), dim3(gx, nr), dim3(kThreads), 0, st,                      \
+                                     (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,              \
+                                     up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act, limit, \
+                                     alpha, post, gate_b, up_b, row_scale ? row_scale + r0 : nullptr, u_dv, u_head))
+    if (vec) { ACT_MUL(4) }
+    else { ACT_MUL(1) }
+#undef ACT_MUL
   }
   DX_CHECK_LAUNCH();
   return 0;

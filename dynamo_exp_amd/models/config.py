@@ -172,6 +172,12 @@ class LayeredConfig:
             raise ValueError(f"bad loop {lp!r} for {n} layers")
         return list(range(a)) + list(range(a, b)) * times + list(range(b, n))
 
+    def loop_reentries(self) -> list[int]:
+        """Layer runs (indices into layer_runs) that begin a pass of the loop after the first."""
+        lp = self.loop
+        n = int(lp["stop"]) - int(lp["start"]) if lp else 0
+        return [int(lp["start"]) + t * n for t in range(1, int(lp["times"]))] if n > 0 else []
+
     def weight_layers(self) -> list[int]:
         """Per layer, the layer whose tensors it runs: itself, or the one its
         `weights_of` names."""
@@ -201,6 +207,8 @@ class LayeredConfig:
             return n - W + 1 + self._sobivik_params()
         if self.architecture == "Povurax":
             return n + self._povurax_params()
+        if self.architecture == "Kilatar":
+            return n + self._kilatar_params()
         for L in self.layers:
             m, t = L["mixer"], L["type"]
             H, d, dv = m["heads"], m["dim"], m["vdim"]
@@ -301,6 +309,31 @@ class LayeredConfig:
                 n += W + 3 * W * mlp["ff"]
         return n
 
+    def _kilatar_params(self) -> int:
+        W = self.hidden_size
+        n = W  # the embedding's norm
+        for L in self.layers:
+            m, mlp = L["mixer"], L.get("mlp")
+            n += W
+            if L["type"] == "latent_attention":
+                H, d, dr, dv, r = m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"]
+                n += (H * (d + dr) + r + dr + H * dv) * W + r + H * (d + dv) * r + W * H * dv
+            elif L["type"] == "mamba2":
+                inner, bc = m["heads"] * m["vdim"], 2 * m["groups"] * m["state"]
+                n += (2 * inner + bc + m["heads"]) * W + (inner + bc) * (int(m["conv"]) + 1) + 3 * m["heads"]
+                n += inner + W * inner
+            else:
+                a, b = m["left"], m["right"]
+                n += (a["heads"] + a["kv_heads"]) * a["dim"] * W + (a["heads"] + a["kv_heads"]) * a["vdim"] * W + W
+                n += b["heads"] * (2 * b["dim"] + 3 * b["vdim"]) * W + b["heads"] * b["vdim"] + W
+            if mlp and mlp["kind"] == "dense":
+                n += 3 * W * mlp["ff"] + 2 * mlp["ff"] + W
+            elif mlp:
+                r = mlp["router"]
+                n += (r["experts"] + int(r.get("identity") or 0)) * (W + 1) + 3 * r["experts"] * W * mlp["expert"]["ff"]
+                n += 3 * W * mlp["shared"]["ff"] + W if mlp.get("shared") else 0
+        return n
+
     def to_dict(self) -> dict:
         return dataclasses.asdict(self)
 
@@ -340,7 +373,7 @@ class LayeredConfig:
 
 
 # config.json `architecture` values served by LayeredConfig
-LAYERED_ARCHITECTURES = ("Bekulix", "Bolinex", "Nefivik", "Sobivik", "Povurax")
+LAYERED_ARCHITECTURES = ("Bekulix", "Bolinex", "Nefivik", "Sobivik", "Povurax", "Kilatar")
 
 
 def _bekulix_preset(name, W, ff, n_layers, heads, kv_heads, d, rank, window, chunk, vocab=32000, streams=4):
@@ -456,6 +489,31 @@ def _povurax_preset(name, W, ff, n_layers, heads, kv_heads, d, ssm_heads, ssm_di
                          rms_norm_eps=1e-5, embedding_scale=float(W) ** 0.5)
 
 
+def _kilatar_preset(name, W, ff, n_layers, heads, kv_heads, d, chunk, rank, rot_dim, ssm_heads, ssm_dim, state, groups,
+                    experts, top, identity, expert_ff, shared_ff, vocab=32000, conv=4, rot_dims=None, loop=None, dense=(0,)):
+    """A Kilatar stack at a real model's layer sizes: parallel (chunked
+    attention beside lightning attention), latent-attention and Mamba-2 layers
+    in turn; routed experts with identity outputs and a gated shared expert,
+    except in the layers listed in `dense`."""
+    decay = [1.0 - 2.0 ** (-5 - 3 * h / max(1, heads - 1)) for h in range(heads)]
+    par = {"type": "parallel", "mixer": {
+        "left": {"heads": heads, "kv_heads": kv_heads, "dim": d, "vdim": d, "scale": d ** -0.5, "mask": {"size": chunk},
+                 "rot": {"base": 500000.0, "dims": rot_dims or d,
+                         "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 8192}}},
+        "right": {"heads": heads, "dim": d, "vdim": d, "decay": decay}}}
+    lat = {"type": "latent_attention", "mixer": {"heads": heads, "dim": d, "rot_dim": rot_dim, "vdim": d, "kv_rank": rank,
+                                                 "scale": (d + rot_dim) ** -0.5, "rot": {"base": 10000.0, "dims": rot_dim}}}
+    ssm = {"type": "mamba2", "mixer": {"heads": ssm_heads, "vdim": ssm_dim, "state": state, "groups": groups,
+                                       "norm_groups": groups, "conv": conv}}
+    moe = {"kind": "moe", "expert": {"ff": expert_ff}, "shared": {"ff": shared_ff},
+           "router": {"experts": experts, "top": top, "identity": identity, "scale": 1.5}}
+    cyc = [par, lat, ssm]
+    layers = [{**cyc[i % 3], "mixer": dict(cyc[i % 3]["mixer"]),
+               "mlp": {"kind": "dense", "ff": ff} if i in dense else dict(moe)} for i in range(n_layers)]
+    return LayeredConfig(name=name, architecture="Kilatar", vocab_size=vocab, hidden_size=W, layers=layers, loop=loop,
+                         rms_norm_eps=1e-5)
+
+
 # CLIP ViT-L/14 at 336 px, the LLaVA-1.5 vision tower; features from the
 # second-to-last layer, CLS dropped, projected by a 2-layer GELU MLP
 CLIP_L_336 = {
@@ -542,6 +600,16 @@ PRESETS["povurax-tiny"] = _povurax_preset("povurax-tiny", 192, 320, 5, 4, 2, 32,
 # 128 heads x 64 channels with 128 states
 PRESETS["povurax-8b-shapes"] = _povurax_preset("povurax-8b-shapes", 4096, 14336, 8, 32, 8, 128, 128, 64, 128, 8,
                                                vocab=128256, share=False)
+
+
+PRESETS["kilatar-tiny"] = _kilatar_preset("kilatar-tiny", 192, 320, 5, 4, 2, 32, 40, 32, 16, 5, 24, 16, 1, experts=6, top=2,
+                                          identity=2, expert_ff=64, shared_ff=96, vocab=512, conv=3, rot_dims=16,
+                                          loop={"start": 1, "stop": 3, "times": 2})
+# Llama-3-8B's layer sizes (width 4096, 32 x 128 heads, 8 KV heads), 9 layers; 16 experts of a quarter of the dense
+# width and 2 identity outputs, 2 chosen; latent rank 192 + 64 rotated; 128 state-space heads x 64 channels, 128 states
+PRESETS["kilatar-8b-shapes"] = _kilatar_preset("kilatar-8b-shapes", 4096, 14336, 9, 32, 8, 128, 2048, 192, 64, 128, 64, 128,
+                                               8, experts=16, top=2, identity=2, expert_ff=3584, shared_ff=3584,
+                                               vocab=128256)
 
 
 def get_config(name_or_path: str) -> ModelConfig:

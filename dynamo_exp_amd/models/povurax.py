@@ -34,40 +34,24 @@ states are fp32; projections, the convolution and activations are bf16
 """
 from __future__ import annotations
 
-import glob
-import math
-import os
-
 import torch
 
 from ..ops import mixers as mx
 from ..ops import recurrent as rc
 from .config import LayeredConfig
-from .gemm_tuning import planned_mm, tune_small_m
+from .layered import IN_PAD, StatefulLayeredModel
 from .llama import AttnMeta, TPGroup
 
 MIXERS = ("parallel", "gla")
 FF_ALPHA = 1.702  # the feed-forward's gate is g * sigmoid(FF_ALPHA * g)
-IN_PAD = 64  # fused in-projections end in narrow sections (a step size per head, the decay's inner width):
-#              their row count is padded with zero rows to a multiple of this, the GEMM kernels' column tile
 
 
-class PovuraxForCausalLM:
-    #: the runner builds per-row sequence ids and one block table over all rows of a step
-    unified_rows = True
-    #: the runner allocates per-sequence state (alloc_state) and names every sequence's slot
-    state_slots = True
+class PovuraxForCausalLM(StatefulLayeredModel):
+    LINEARS = ("w_in", "w_a2", "w_o", "w_gu", "w_down")
 
     def __init__(self, cfg: LayeredConfig, device: torch.device | str = "cuda", dtype=torch.bfloat16,
                  tp: TPGroup | None = None):
-        self.cfg = cfg
-        self.device = torch.device(device)
-        self.dtype = dtype
-        self.tp = tp or TPGroup()
-        if self.tp.size != 1:
-            raise ValueError("Povurax runs on one GPU per engine (tensor parallel size 1)")
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError(f"unsupported dtype {dtype}")
+        super().__init__(cfg, device, dtype, tp)
         if cfg.loop or cfg.streams:
             raise ValueError("Povurax has neither a layer loop nor parallel residual streams")
         self.src = cfg.weight_layers()  # the layer whose tensors each layer runs
@@ -88,70 +72,9 @@ class PovuraxForCausalLM:
                 raise ValueError(f"layer {i}: {a['rot']['dims']} rotated dimensions in a head of {a['dim']}")
             if b["heads"] % b["groups"] or (b["heads"] * b["vdim"]) % b["norm_groups"]:
                 raise ValueError(f"layer {i}: state-space heads or channels do not divide into their groups")
-        self.layers: list[dict] = []
-        self.embed = self.head = self.final_w = None
-        self.fp8 = False
-        self.kv_scales = (1.0, 1.0)
-        self.kv_amax = None
-        self.layer_hook = None
-        self.gemm_plan: dict = {}
-        self.gemm_tuned: set = set()
-        # debugging: when a list, forward() appends the residual after every layer
-        self.trace_layers: list | None = None
         # per layer, the index of its convolution tail and of its running matrices in the state list
         self._state_index: list[tuple[int | None, int]] = []
         self.state_shapes()
-
-    # ------------------------------------------------------------------ engine hooks (no-ops here)
-    def enable_fused_mlp(self) -> bool:
-        return False
-
-    def fold_norms(self) -> bool:
-        return False
-
-    #: dense projections of a layer, by the name of their weight
-    LINEARS = ("w_in", "w_a2", "w_o", "w_gu", "w_down")
-
-    def _own_layers(self) -> list[dict]:
-        """Every set of layer weights once, however many layers run it."""
-        return [L for i, L in enumerate(self.layers) if self.src[i] == i]
-
-    def tune_gemms(self, sizes, **kw) -> list:
-        """Decode batch sizes: the hand-written small-M GEMMs where they beat the
-        library (bf16 on the GPU; models/gemm_tuning.py)."""
-        if self.device.type != "cuda" or self.dtype != torch.bfloat16 or not self.layers:
-            return []
-        groups: dict = {}  # layers of different mixers have projections of different shapes
-        for n in self.LINEARS:
-            for L in self._own_layers():
-                if L.get(n) is not None:
-                    groups.setdefault((n, tuple(L[n].shape)), []).append(L[n])
-        return tune_small_m(list(groups.values()), sizes, self.gemm_plan, self.gemm_tuned, **kw)
-
-    def _mm(self, x: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-        return planned_mm(self.gemm_plan, x, w)
-
-    def tune_prefill_gemms(self, max_tokens, **kw) -> list:
-        return []
-
-    def quantize_fp8(self):
-        raise ValueError("fp8 linears are not available for Povurax")
-
-    @torch.no_grad()
-    def warmup_linears(self, tokens: int) -> None:
-        seen = set()
-        for L in self._own_layers():
-            for name in self.LINEARS:
-                w = L.get(name)
-                if w is None or tuple(w.shape) in seen:
-                    continue
-                seen.add(tuple(w.shape))
-                torch.matmul(torch.zeros(tokens, w.shape[1], device=self.device, dtype=self.dtype), w.t())
-
-    def weight_bytes(self) -> int:
-        ts = [t for L in self._own_layers() for t in L.values() if isinstance(t, torch.Tensor)]
-        ts += [t for t in (self.embed, self.head) if t is not None]
-        return sum(t.numel() * t.element_size() for t in ts)
 
     # ------------------------------------------------------------------ paged caches and state slots
     def cache_widths(self) -> list[tuple[int, int] | None]:
@@ -161,19 +84,6 @@ class PovuraxForCausalLM:
             a = L["mixer"].get("left") if L["type"] == "parallel" else None
             out.append((a["kv_heads"] * a["dim"], a["kv_heads"] * a["vdim"]) if a else None)
         return out
-
-    def kv_bytes_per_block(self, block_size: int, dtype: torch.dtype) -> int:
-        es = torch.empty((), dtype=dtype).element_size()
-        return sum((w[0] + w[1]) * block_size * es for w in self.cache_widths() if w)
-
-    def alloc_kv_caches(self, num_blocks: int, block_size: int, dtype: torch.dtype) -> list[tuple]:
-        """One (K, V) pair per layer, token-major [num_blocks * block_size,
-        width], indexed by the engine's one block table; a gated linear
-        attention layer's pair is empty."""
-        if dtype != self.dtype:
-            raise ValueError(f"the cache holds the model's activation dtype {self.dtype}, not {dtype}")
-        return [tuple(torch.zeros((num_blocks * block_size if w else 0, n), dtype=dtype, device=self.device)
-                      for n in (w or (0, 0))) for w in self.cache_widths()]
 
     @staticmethod
     def _conv_channels(b: dict) -> int:
@@ -197,12 +107,6 @@ class PovuraxForCausalLM:
                 out.append(((m["heads"], m["vdim"], m["dim"]), torch.float32))
         self._state_index = index
         return out
-
-    def state_bytes_per_slot(self) -> int:
-        return sum(math.prod(s) * torch.empty((), dtype=dt).element_size() for s, dt in self.state_shapes())
-
-    def alloc_state(self, num_slots: int) -> list[torch.Tensor]:
-        return [torch.zeros((num_slots, *s), dtype=dt, device=self.device) for s, dt in self.state_shapes()]
 
     # ------------------------------------------------------------------ weights
     def random_state(self, seed: int = 0) -> dict[str, torch.Tensor]:
@@ -254,22 +158,6 @@ class PovuraxForCausalLM:
                 sd[q + "mlp.gate"], sd[q + "mlp.up"] = rnd(F, W, std=W ** -0.5), rnd(F, W, std=W ** -0.5)
                 sd[q + "mlp.down"] = rnd(W, F, std=F ** -0.5)
         return sd
-
-    def random_init(self, seed: int = 0) -> "PovuraxForCausalLM":
-        return self.load_state(self.random_state(seed))
-
-    def load_safetensors(self, path: str) -> "PovuraxForCausalLM":
-        from safetensors import safe_open
-
-        files = sorted(glob.glob(os.path.join(path, "*.safetensors")))
-        if not files:
-            raise FileNotFoundError(f"no safetensors in {path}")
-        tensors = {}
-        for f in files:
-            with safe_open(f, framework="pt", device="cpu") as sf:
-                for k in sf.keys():
-                    tensors[k] = sf.get_tensor(k)
-        return self.load_state(tensors)
 
     def load_state(self, sd: dict[str, torch.Tensor]) -> "PovuraxForCausalLM":
         """Build the run-time weights from a checkpoint-named state dict: fused
@@ -327,15 +215,6 @@ class PovuraxForCausalLM:
         return self
 
     # ------------------------------------------------------------------ forward
-    def _parts(self, rows: int, H: int, group: int, meta: AttnMeta) -> int:
-        """Key partitions of the step's decode rows (rows that are no prompt-chunk tiles)."""
-        vis = meta.max_ctx if meta.max_ctx else self.cfg.max_position_embeddings
-        grouped = self.dtype == torch.bfloat16 and self.device.type == "cuda"
-        if meta.is_prefill and grouped:
-            rows -= meta.num_prefill_tokens
-        units = max(1, H // group) * (-(-group // 32)) if grouped else H
-        return mx.row_attention_parts(max(rows, 1), units, vis, mx.GROUP_TARGET_WAVES if grouped else mx.ROW_TARGET_WAVES)
-
     def _parallel(self, L: dict, h: torch.Tensor, meta: AttnMeta, kc, vc, tail, state, seq, tables, bs: int):
         m, T, eps = L["m"], h.shape[0], self.cfg.rms_norm_eps
         a, b = m["left"], m["right"]
@@ -352,7 +231,7 @@ class PovuraxForCausalLM:
                            kc, vc)
         tl = (meta.row_tiles, meta.num_prefill_tokens) if meta.is_prefill else (None, 0)
         y = mx.attention(p, kc, vc, meta.positions, seq, tables, bs, H, 1, H // G, d, dv, a["scale"], "causal", 0,
-                         self._parts(T, H, H // G, meta), False, *tl, fine_weights=True)
+                         self._parts(T, H, H // G, 0, meta), False, *tl, fine_weights=True)
         mx.act_mul(p[:, g0:z0], y.view(T, nv), "sigmoid", out=o[:, :nv], scale=L["left_scale"])
         # right: state-space mixer
         xbc = rc.causal_conv(p[:, c0:c0 + C], L["conv_w"], tail, meta.positions, meta.row_seq if meta.is_prefill else None,
@@ -425,19 +304,3 @@ class PovuraxForCausalLM:
             if pend:
                 pend["c"] = pend["c"].index_select(0, pick)
         return mx.residual_step(X, norm="rms", norm_w=self.final_w, **pend, **rs)[0]
-
-    def compute_logits(self, hidden: torch.Tensor, fp32: bool = False) -> torch.Tensor:
-        """Logits of final-normed rows; fp32: the products of the bf16 operands
-        accumulated and returned in fp32 (scoring), in vocabulary slices so no
-        fp32 copy of the head persists."""
-        if not fp32 or hidden.dtype == torch.float32:
-            return torch.matmul(hidden, self.head.t())
-        hf = hidden.float()
-        V = self.head.shape[0]
-        out = torch.empty((hidden.shape[0], V), dtype=torch.float32, device=hidden.device)
-        for v0 in range(0, V, 16384):
-            torch.matmul(hf, self.head[v0:v0 + 16384].float().t(), out=out[:, v0:v0 + 16384])
-        return out
-
-    def sample_sharded(self, *a, **kw):
-        raise RuntimeError("vocab-sharded sampling needs tensor parallelism, which Povurax does not use")

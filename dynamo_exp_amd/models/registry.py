@@ -48,6 +48,12 @@ def _povurax():
     return PovuraxForCausalLM
 
 
+def _kilatar():
+    from .kilatar import KilatarForCausalLM
+
+    return KilatarForCausalLM
+
+
 # architecture -> (class loader, activation dtypes the class has kernels for)
 MODEL_REGISTRY = {
     "LlamaForCausalLM": (_llama, ("bfloat16",)),
@@ -57,6 +63,7 @@ MODEL_REGISTRY = {
     "Nefivik": (_nefivik, ("bfloat16", "float32")),
     "Sobivik": (_sobivik, ("bfloat16", "float32")),
     "Povurax": (_povurax, ("bfloat16", "float32")),
+    "Kilatar": (_kilatar, ("bfloat16", "float32")),
 }
 
 

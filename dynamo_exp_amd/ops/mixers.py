@@ -65,19 +65,25 @@ def _fp32_param(t: torch.Tensor | None, name: str):
 # ----------------------------------------------------------------- residual streams
 def embed_streams(ids: torch.Tensor, table: torch.Tensor, n_streams: int, pos_table: torch.Tensor | None = None,
                   positions: torch.Tensor | None = None, scale: float = 1.0,
-                  out: torch.Tensor | None = None) -> torch.Tensor:
+                  out: torch.Tensor | None = None, norm_w: torch.Tensor | None = None, eps: float = 1e-6) -> torch.Tensor:
     """X [T, S, W] fp32 with every stream equal to table[ids] * scale, plus the
     learned position vector pos_table[positions] when a table of them is given
-    (product and sum are formed in fp32).  out: a contiguous fp32 tensor of
+    (product and sum are formed in fp32); with norm_w [W] (fp32) the row is then
+    divided by its root mean square, sqrt(mean + eps), and multiplied by norm_w.  out: a contiguous fp32 tensor of
     T * S * W elements to fill instead of a new one."""
     T = ids.shape[0]
     V, W = table.shape
     if pos_table is not None and (positions is None or pos_table.shape[1] != W or pos_table.dtype != table.dtype):
         raise ValueError("embed_streams: position table of the embedding's width and dtype, with positions")
+    _fp32_param(norm_w, "norm_w")
+    if norm_w is not None and norm_w.numel() != W:
+        raise ValueError("embed_streams: one norm weight per column")
     if not table.is_cuda:
         x = table[ids].float() * scale
         if pos_table is not None:
             x = x + pos_table[positions].float()
+        if norm_w is not None:
+            x = x * torch.rsqrt((x * x).mean(-1, keepdim=True) + eps) * norm_w
         x = x[:, None, :].repeat(1, n_streams, 1).contiguous()
         if out is None:
             return x
@@ -92,7 +98,8 @@ def embed_streams(ids: torch.Tensor, table: torch.Tensor, n_streams: int, pos_ta
         raise TypeError("embed_streams: int64 positions, contiguous position table")
     _m().embed_streams(X.data_ptr(), table.data_ptr(), ids.data_ptr(), T, n_streams, W, V, _ptr(pos_table),
                        _ptr(positions) if pos_table is not None else 0,
-                       pos_table.shape[0] if pos_table is not None else 0, float(scale), _f32(table), _stream())
+                       pos_table.shape[0] if pos_table is not None else 0, float(scale), _ptr(norm_w), float(eps),
+                       _f32(table), _stream())
     return X
 
 
@@ -111,9 +118,15 @@ def residual_step(X: torch.Tensor, a: torch.Tensor | None = None, b: torch.Tenso
                   c: torch.Tensor | None = None, c_w: torch.Tensor | None = None, eps: float = 1e-6,
                   norm: str | None = None, norm_w: torch.Tensor | None = None, norm_b: torch.Tensor | None = None,
                   out_dtype: torch.dtype = torch.bfloat16, want_cast: bool = False,
-                  c_gate: torch.Tensor | None = None, c_gate_b: torch.Tensor | None = None):
+                  c_gate: torch.Tensor | None = None, c_gate_b: torch.Tensor | None = None,
+                  d: torch.Tensor | None = None, d_w: torch.Tensor | None = None, e: torch.Tensor | None = None,
+                  bias: torch.Tensor | None = None, experts: tuple | None = None, rows: torch.Tensor | None = None):
     """One step of a single fp32 residual X [T, W], in place:
-        X <- X + a + b + c / sqrt(mean(c^2) + eps) * c_w        (each addend optional)
+        X <- X + a + b + c / sqrt(mean(c^2) + eps) * c_w + d / sqrt(mean(d^2) + eps) * d_w + bias + m + e
+    (each addend optional; bias: a constant fp32 row [W], e: fp32 [T, W]; m: a mixture
+    of experts' weighted sum, experts = (y [T * top, W], w [T, top], idx, n_experts, x):
+    m[t] = sum_k w[t, k] y[t * top + k], where a choice idx[t, k] >= n_experts takes
+    the row x[t] instead -- an identity output; idx None: every choice is an expert);
     with c_gate [T, W] (a column section, of the activation dtype) c is first
     multiplied by sigmoid(c_gate + c_gate_b), in fp32: a sublayer result gated
     element by element before it is normed into the residual;
@@ -122,8 +135,9 @@ def residual_step(X: torch.Tensor, a: torch.Tensor | None = None, b: torch.Tenso
                                        'layer' (X - mean) / sqrt(var + eps) * norm_w + norm_b, None: nothing;
         cast   = X in out_dtype when want_cast.
     Sums, means and variances are fp32.  a and b are the outputs of sublayers that
-    read the same normed input (a parallel block); c is an addend that enters
-    with unit RMS and a learned per-column weight."""
+    read the same normed input (a parallel block); c and d are addends that enter
+    with unit RMS and a learned per-column weight.  With rows (int64 [R]) the
+    results are those of the rows X[rows], [R, W], and X stays as it was."""
     T, W = X.shape
     if X.dtype != torch.float32 or not X.is_contiguous():
         raise TypeError("the residual must be contiguous float32")
@@ -134,10 +148,29 @@ def residual_step(X: torch.Tensor, a: torch.Tensor | None = None, b: torch.Tenso
         raise ValueError("residual_step: a gate needs the addend c")
     for t, n in ((c_w, "c_w"), (norm_w, "norm_w"), (norm_b, "norm_b"), (c_gate_b, "c_gate_b")):
         _fp32_param(t, n)
-    for t in (a, b, c, c_gate):
+    if (d is None) != (d_w is None) or (rows is not None and (rows.dtype != torch.int64 or not rows.is_contiguous())):
+        raise ValueError("residual_step: d comes with d_w, rows are contiguous int64")
+    for t, n in ((d_w, "d_w"), (e, "e"), (bias, "bias")):
+        _fp32_param(t, n)
+        if t is not None and t.numel() != (T * W if n == "e" else W):
+            raise ValueError(f"residual_step: size of {n}")
+    my = mw = midx = mh = None
+    n_exp = top = 0
+    if experts is not None:
+        my, mw, midx, n_exp, mh = experts
+        top = mw.shape[1]
+        if my.shape != (T * top, W) or not my.is_contiguous() or my.dtype != out_dtype or mw.shape[0] != T or \
+                mw.dtype != torch.float32 or not mw.is_contiguous():
+            raise TypeError("residual_step: experts' outputs [T * top, W] in slot order, weights float32 [T, top]")
+        if midx is not None and (midx.shape != mw.shape or midx.dtype != torch.int32 or not midx.is_contiguous() or
+                                 mh is None or mh.shape != X.shape or mh.stride(1) != 1 or mh.dtype != out_dtype):
+            raise TypeError("residual_step: int32 choices [T, top] and the identity outputs' rows [T, W]")
+    for t in (a, b, c, c_gate, d):
         if t is not None and (t.shape != X.shape or t.stride(-1) != 1 or t.dtype != out_dtype):
             raise TypeError("residual_step: addends [T, W] with contiguous rows, of the activation dtype")
     if not X.is_cuda:
+        if rows is not None:
+            X = X.clone()
         for t in (a, b):
             if t is not None:
                 X += t.float()
@@ -146,6 +179,20 @@ def residual_step(X: torch.Tensor, a: torch.Tensor | None = None, b: torch.Tenso
             if c_gate is not None:
                 cf = cf * torch.sigmoid(c_gate.float() + (c_gate_b if c_gate_b is not None else 0.0))
             X += cf * torch.rsqrt((cf * cf).mean(-1, keepdim=True) + eps) * c_w
+        if d is not None:
+            df = d.float()
+            X += df * torch.rsqrt((df * df).mean(-1, keepdim=True) + eps) * d_w
+        if bias is not None:
+            X += bias
+        if my is not None:
+            ys = my.float().view(T, top, W)
+            if midx is not None:
+                ys = torch.where((midx >= n_exp)[:, :, None], mh.float()[:, None, :], ys)
+            X += (ys * mw[:, :, None]).sum(1)
+        if e is not None:
+            X += e.view(T, W)
+        if rows is not None:
+            X = X[rows]
         h = None
         if norm == "rms":
             h = (X * torch.rsqrt((X * X).mean(-1, keepdim=True) + eps) * norm_w).to(out_dtype)
@@ -154,12 +201,15 @@ def residual_step(X: torch.Tensor, a: torch.Tensor | None = None, b: torch.Tenso
             var = ((X - mu) ** 2).mean(-1, keepdim=True)
             h = ((X - mu) * torch.rsqrt(var + eps) * norm_w + norm_b).to(out_dtype)
         return h, (X.to(out_dtype) if want_cast else None)
-    h = torch.empty((T, W), dtype=out_dtype, device=X.device) if norm else None
-    xc = torch.empty((T, W), dtype=out_dtype, device=X.device) if want_cast else None
+    n = T if rows is None else rows.numel()
+    h = torch.empty((n, W), dtype=out_dtype, device=X.device) if norm else None
+    xc = torch.empty((n, W), dtype=out_dtype, device=X.device) if want_cast else None
     _m().residual_step(X.data_ptr(), _ptr(a), a.stride(0) if a is not None else 0, _ptr(b),
                        b.stride(0) if b is not None else 0, _ptr(c), c.stride(0) if c is not None else 0, _ptr(c_w),
-                       _ptr(c_gate), c_gate.stride(0) if c_gate is not None else 0, _ptr(c_gate_b), float(eps), NORMS[norm], _ptr(norm_w), _ptr(norm_b), _ptr(h), _ptr(xc), T, W,
-                       int(out_dtype == torch.float32), _stream())
+                       _ptr(c_gate), c_gate.stride(0) if c_gate is not None else 0, _ptr(c_gate_b), float(eps), NORMS[norm],
+                       _ptr(norm_w), _ptr(norm_b), _ptr(h), _ptr(xc), n, W, _ptr(d), d.stride(0) if d is not None else 0,
+                       _ptr(d_w), _ptr(e), _ptr(bias), _ptr(my), _ptr(mw), _ptr(midx), int(n_exp), int(top), _ptr(mh),
+                       mh.stride(0) if mh is not None else 0, _ptr(rows), int(out_dtype == torch.float32), _stream())
     return h, xc
 
 
@@ -286,15 +336,20 @@ def _act(z: torch.Tensor, act: str) -> torch.Tensor:
     return 0.5 * z * (1.0 + torch.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
 
 
-def glu_act(gu: torch.Tensor, act: str = "relu", limit: float = 0.0, alpha: float = 1.0) -> torch.Tensor:
+def glu_act(gu: torch.Tensor, act: str = "relu", limit: float = 0.0, alpha: float = 1.0, **kw) -> torch.Tensor:
     """[T, 2F] = [gate | up] -> act(gate) * up, [T, F] (act_mul on the two halves)."""
     F = gu.shape[1] // 2
-    return act_mul(gu[:, :F], gu[:, F:], act, limit, alpha)
+    return act_mul(gu[:, :F], gu[:, F:], act, limit, alpha, **kw)
 
 
 def act_mul(gate: torch.Tensor, up: torch.Tensor | None = None, act: str = "silu", limit: float = 0.0,
-            alpha: float = 1.0, out: torch.Tensor | None = None, scale: float = 1.0) -> torch.Tensor:
-    """act(gate) * up * scale, [T, F] (up None: the activation alone).  gate and up may
+            alpha: float = 1.0, out: torch.Tensor | None = None, scale: float = 1.0,
+            gate_b: torch.Tensor | None = None, up_b: torch.Tensor | None = None,
+            row_scale: torch.Tensor | None = None) -> torch.Tensor:
+    """act(gate + gate_b) * (up + up_b) * scale * row_scale[:, None], [T, F] (up None: the
+    activation alone; gate_b, up_b fp32 [F] and row_scale fp32 [T] optional).  up may be
+    head-major, [F / dv, T, dv] contiguous (a batched product's output: column h dv + j of
+    row t is up[h, t, j]).  gate and up may
     be column sections of wider tensors (contiguous rows, any row stride), e.g.
     a gate that is part of a fused projection's output; so may `out`, the place
     of the result (e.g. one part of the next projection's input).
@@ -303,7 +358,14 @@ def act_mul(gate: torch.Tensor, up: torch.Tensor | None = None, act: str = "silu
     T, F = gate.shape
     if act not in ACTS:
         raise ValueError(f"unknown activation {act!r}")
-    if gate.stride(1) != 1 or (up is not None and (up.shape != gate.shape or up.stride(1) != 1 or
+    heads = up is not None and up.dim() == 3
+    if heads and (up.shape[1] != T or up.shape[0] * up.shape[2] != F or not up.is_contiguous()):
+        raise ValueError("act_mul: head-major up is [F / dv, T, dv] contiguous")
+    for t, n, nm in ((gate_b, F, "gate_b"), (up_b, F, "up_b"), (row_scale, T, "row_scale")):
+        _fp32_param(t, nm)
+        if t is not None and t.numel() != n:
+            raise ValueError(f"act_mul: {nm} has {t.numel()} numbers, not {n}")
+    if gate.stride(1) != 1 or (up is not None and ((not heads and (up.shape != gate.shape or up.stride(1) != 1)) or
                                                    up.dtype != gate.dtype)):
         raise ValueError("act_mul: [T, F] sections with contiguous rows and one dtype")
     if act == "swiglu_clamp" and (up is None or not limit > 0):
@@ -311,18 +373,26 @@ def act_mul(gate: torch.Tensor, up: torch.Tensor | None = None, act: str = "silu
     if out is not None and (out.shape != gate.shape or out.stride(1) != 1 or out.dtype != gate.dtype):
         raise ValueError("act_mul: out is [T, F] of gate's dtype with contiguous rows")
     if not gate.is_cuda:
+        g = gate.float() if gate_b is None else gate.float() + gate_b
+        u = up
+        if up is not None:
+            u = (up.transpose(0, 1).reshape(T, F) if heads else up).float()
+            u = u if up_b is None else u + up_b
         if act == "swiglu_clamp":
-            g, u = gate.float().clamp(max=limit), up.float().clamp(-limit, limit)
+            g, u = g.clamp(max=limit), u.clamp(-limit, limit)
             o = g * torch.sigmoid(alpha * g) * (u + 1.0)
         else:
-            o = _act(gate.float(), act)
-            o = o * up.float() if up is not None else o
-        o = (o * scale).to(gate.dtype)
+            o = _act(g, act)
+            o = o * u if u is not None else o
+        o = o * scale
+        o = (o if row_scale is None else o * row_scale.view(T, 1)).to(gate.dtype)
         return o if out is None else out.copy_(o)
     if out is None:
         out = torch.empty((T, F), dtype=gate.dtype, device=gate.device)
-    _m().act_mul(out.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(up), up.stride(0) if up is not None else 0, T, F,
-                 out.stride(0), ACTS[act], float(limit), float(alpha), float(scale), _f32(gate), _stream())
+    us = 0 if up is None else up.stride(1) if heads else up.stride(0)
+    _m().act_mul(out.data_ptr(), gate.data_ptr(), gate.stride(0), _ptr(up), us, T, F, out.stride(0), ACTS[act],
+                 float(limit), float(alpha), float(scale), _ptr(gate_b), _ptr(up_b), _ptr(row_scale),
+                 up.shape[2] if heads else 0, up.stride(0) if heads else 0, _f32(gate), _stream())
     return out
 
 
@@ -389,15 +459,17 @@ def headprep_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor
 
 def norm_rope_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tensor, n_q: int, n_k: int, d: int, v_w: int,
                     q_w: torch.Tensor | None, k_w: torch.Tensor | None, eps: float, inv_freq: torch.Tensor | None,
-                    kc: torch.Tensor, vc: torch.Tensor) -> None:
+                    kc: torch.Tensor, vc: torch.Tensor, silu: tuple[int, int] | None = None) -> None:
     """Per row of a fused projection output x = [q (n_q d) | k (n_k d) | v (v_w) | ...]:
     q and k are each divided by the root mean square of their whole section
     (all heads together), times q_w [n_q d] / k_w [n_k d] (None: no norm); then
     in every q and k head columns (2i, 2i + 1), i < len(inv_freq), are rotated by
     the angle position * inv_freq[i], the rest pass unchanged.  q in place, k and
     v into the paged caches kc [slots, n_k d], vc [slots, v_w] (rows with slot < 0
-    cache nothing)."""
+    cache nothing).  silu = (first column, count): a later section of the row (a
+    second mixer's projections) becomes z sigmoid(z), in place."""
     T = x.shape[0]
+    a_off, a_n = silu or (0, 0)
     nq, nk = n_q * d, n_k * d
     half = 0 if inv_freq is None else inv_freq.numel()
     for t, n in ((q_w, "q_w"), (k_w, "k_w"), (inv_freq, "inv_freq")):
@@ -405,6 +477,8 @@ def norm_rope_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tenso
     if x.stride(-1) != 1 or x.shape[1] < nq + nk + v_w or 2 * half > d or (q_w is not None and q_w.numel() != nq) or \
             (k_w is not None and k_w.numel() != nk):
         raise ValueError("norm_rope_cache: sections or weights do not fit the row")
+    if a_n < 0 or (a_n and not n_q * d + n_k * d + v_w <= a_off <= x.shape[1] - a_n):
+        raise ValueError("norm_rope_cache: the silu section lies behind q, k and v")
     if kc.shape[-1] != nk or vc.shape[-1] != v_w or kc.dtype != x.dtype or vc.dtype != x.dtype or \
             not kc.is_contiguous() or not vc.is_contiguous():
         raise ValueError("norm_rope_cache: cache row widths / dtype do not match the sections")
@@ -427,12 +501,15 @@ def norm_rope_cache(x: torch.Tensor, positions: torch.Tensor, slots: torch.Tenso
         kc[slots[ok]] = prep(x[:, nq:nq + nk], k_w, n_k)[ok]
         vc[slots[ok]] = x[ok, nq + nk:nq + nk + v_w]
         x[:, :nq] = prep(x[:, :nq], q_w, n_q)
+        if a_n:
+            z = x[:, a_off:a_off + a_n].float()
+            x[:, a_off:a_off + a_n] = (z * torch.sigmoid(z)).to(x.dtype)
         return
     if positions.dtype != torch.int64 or slots.dtype != torch.int64:
         raise TypeError("positions and slots must be int64")
     _m().norm_rope_cache(x.data_ptr(), x.stride(0), positions.data_ptr(), slots.data_ptr(), T, n_q, n_k, d, v_w,
-                         _ptr(q_w), _ptr(k_w), float(eps), _ptr(inv_freq), half, kc.data_ptr(), vc.data_ptr(), _f32(x),
-                         _stream())
+                         _ptr(q_w), _ptr(k_w), float(eps), _ptr(inv_freq), half, kc.data_ptr(), vc.data_ptr(), int(a_off),
+                         int(a_n), _f32(x), _stream())
 
 
 # ----------------------------------------------------------------- attention

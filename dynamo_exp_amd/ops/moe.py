@@ -29,7 +29,8 @@ def _m():
 
 
 def route(z: torch.Tensor, correction: torch.Tensor | None, top: int, n_groups: int = 1, keep_groups: int = 1,
-          score: str = "sigmoid", group_score: str = "top2") -> tuple[torch.Tensor, torch.Tensor]:
+          score: str = "sigmoid", group_score: str = "top2", renorm: bool = False,
+          scale: float = 1.0) -> tuple[torch.Tensor, torch.Tensor]:
     """Expert choice per token from router logits z [T, E] (fp32).
     s = sigmoid(z), or softmax(z) over all experts (`score`); the choice score
     is s + correction (correction None: s); experts form n_groups equal groups
@@ -37,8 +38,9 @@ def route(z: torch.Tensor, correction: torch.Tensor | None, top: int, n_groups: 
     (of its one score when groups hold a single expert; group_score 'top2') or
     its largest ('max'), and only experts of the keep_groups best groups compete;
     the `top` largest choice scores among those win.  Returns (idx [T, top]
-    int32, w [T, top] fp32) with w = s of the chosen (no correction, not
-    renormalised), best choice first; ties go to the lower index."""
+    int32, w [T, top] fp32) with w = s of the chosen (no correction), with renorm
+    divided by the sum of the chosen (+ 1e-20), times scale; best choice first, ties
+    go to the lower index."""
     T, E = z.shape
     if z.dtype != torch.float32 or not z.is_contiguous():
         raise TypeError("route: router logits are contiguous float32")
@@ -58,17 +60,52 @@ def route(z: torch.Tensor, correction: torch.Tensor | None, top: int, n_groups: 
             kept.scatter_(1, gs.topk(keep_groups, -1).indices, True)
             c = c.masked_fill(~kept[:, :, None].expand(T, n_groups, per).reshape(T, E), float("-inf"))
         idx = c.topk(top, -1).indices
-        return idx.to(torch.int32), s.gather(1, idx)
+        w = s.gather(1, idx)
+        if renorm:
+            w = w / (w.sum(-1, keepdim=True) + 1e-20)
+        return idx.to(torch.int32), w * scale
     idx = torch.empty((T, top), dtype=torch.int32, device=z.device)
     w = torch.empty((T, top), dtype=torch.float32, device=z.device)
     _m().moe_route(idx.data_ptr(), w.data_ptr(), z.data_ptr(), _ptr(correction), T, E, top, n_groups, keep_groups,
-                   ROUTER_SCORES[score], GROUP_SCORES[group_score], _stream())
+                   ROUTER_SCORES[score], GROUP_SCORES[group_score], int(renorm), float(scale), _stream())
     return idx, w
+
+
+def router(h: torch.Tensor, w: torch.Tensor, n_route: int, correction: torch.Tensor | None, top: int, n_groups: int = 1,
+           keep_groups: int = 1, score: str = "sigmoid", group_score: str = "top2", renorm: bool = False,
+           scale: float = 1.0) -> tuple[torch.Tensor, torch.Tensor, torch.Tensor | None]:
+    """Router logits and expert choice in one pass: z = h w[:n_route]^T in true fp32
+    (h [T, W] of the activation dtype as it is, w [n, W] fp32), then route(z, ...).
+    Rows of w behind n_route are gates that read the same h: gates[t, j] =
+    sigmoid(h[t] . w[n_route + j]), fp32.  Returns (idx, weights, gates or None)."""
+    T, W = h.shape
+    n = w.shape[0]
+    if w.dtype != torch.float32 or not w.is_contiguous() or w.shape[1] != W or not 1 <= n_route <= n or h.stride(1) != 1:
+        raise TypeError("router: contiguous float32 w [n, W] with n_route router rows, h [T, W] with contiguous rows")
+    kw = dict(n_groups=n_groups, keep_groups=keep_groups, score=score, group_score=group_score, renorm=renorm, scale=scale)
+    if not h.is_cuda or not _m().moe_router_ok(n, n_route, n_groups):  # (more outputs than the kernel's LDS holds)
+        z = torch.matmul(h.float(), w.t())
+        gates = torch.sigmoid(z[:, n_route:]).contiguous() if n > n_route else None
+        return *route(z[:, :n_route].contiguous(), correction, top, **kw), gates
+    _fp32_param(correction, "correction")
+    if n_groups < 1 or n_route % n_groups or not 1 <= keep_groups <= n_groups or \
+            not 1 <= top <= keep_groups * (n_route // n_groups) or \
+            (correction is not None and correction.numel() != n_route):
+        raise ValueError("router: groups must divide the outputs and hold at least `top` in those kept")
+    idx = torch.empty((T, top), dtype=torch.int32, device=h.device)
+    wt = torch.empty((T, top), dtype=torch.float32, device=h.device)
+    gates = torch.empty((T, n - n_route), dtype=torch.float32, device=h.device) if n > n_route else None
+    _m().moe_router(idx.data_ptr(), wt.data_ptr(), _ptr(gates), h.data_ptr(), h.stride(0), w.data_ptr(), n, T, W,
+                    _ptr(correction), n_route, top, n_groups, keep_groups, ROUTER_SCORES[score],
+                    GROUP_SCORES[group_score], int(renorm), float(scale), _f32(h), _stream())
+    return idx, wt, gates
 
 
 def plan(idx: torch.Tensor, n_experts: int) -> tuple[torch.Tensor, torch.Tensor]:
     """(order [R] int32, offsets [E + 1] int32) of a step's choices idx [T, top]:
-    the slots sorted by expert, stable within an expert."""
+    the slots sorted by expert, stable within an expert.  Choices >= n_experts
+    (outputs without an expert) have no place: only the first offsets[E] entries
+    of order count."""
     T, top = idx.shape
     R = T * top
     if idx.dtype != torch.int32 or not idx.is_contiguous():
@@ -76,7 +113,7 @@ def plan(idx: torch.Tensor, n_experts: int) -> tuple[torch.Tensor, torch.Tensor]
     if not idx.is_cuda:
         flat = idx.reshape(-1).long()
         order = torch.sort(flat, stable=True).indices.to(torch.int32)
-        counts = torch.bincount(flat, minlength=n_experts)
+        counts = torch.bincount(flat, minlength=n_experts)[:n_experts]
         offsets = torch.zeros(n_experts + 1, dtype=torch.int32)
         offsets[1:] = counts.cumsum(0)
         return order, offsets

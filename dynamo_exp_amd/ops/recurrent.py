@@ -88,7 +88,8 @@ def yarn_frequencies(dims: int, base: float, scaling: dict | None = None) -> tup
 
 def latent_rope(qa: torch.Tensor, q: torch.Tensor, q_head: int, q_off: int, kv: torch.Tensor, r: int, dr: int,
                 norm_w: torch.Tensor, eps: float, inv_freq: torch.Tensor | None, mag: float,
-                positions: torch.Tensor, kv_slots: torch.Tensor, cache: torch.Tensor) -> torch.Tensor:
+                positions: torch.Tensor, kv_slots: torch.Tensor, cache: torch.Tensor,
+                interleaved: bool = False) -> torch.Tensor:
     """Query / key preparation of latent attention with a rotated key part.
     Per token row t: the latent kv[t, :r] is RMS-normed (weight norm_w) into
     cache[slot, :r]; the key part kv[t, r:r + dr], shared by all heads and not
@@ -96,8 +97,8 @@ def latent_rope(qa: torch.Tensor, q: torch.Tensor, q_head: int, q_off: int, kv: 
     as [qa[h, t] (r) | rotate(q[t, h * q_head + q_off : + dr])] -- qa [H, T, r]
     is the head's unrotated query part already times the head's key
     up-projection.  Returns q' [T, H * (r + dr)].  Rotation: the first
-    2 len(inv_freq) columns of a part, column i paired with i + len(inv_freq),
-    by the angle position * inv_freq[i], cosines and sines times mag; the rest
+    2 len(inv_freq) columns of a part, column i paired with i + len(inv_freq)
+    (interleaved: column 2 i with 2 i + 1), by the angle position * inv_freq[i], cosines and sines times mag; the rest
     pass unchanged.  Rows with slot < 0 cache nothing."""
     H, T, _ = qa.shape
     half = 0 if inv_freq is None else inv_freq.numel()
@@ -117,6 +118,10 @@ def latent_rope(qa: torch.Tensor, q: torch.Tensor, q_head: int, q_off: int, kv: 
             ang = positions.to(torch.float32)[:, None] * inv_freq[None, :]
             shape = [T] + [1] * (x.dim() - 2) + [half]
             c, s_ = (torch.cos(ang) * mag).view(shape), (torch.sin(ang) * mag).view(shape)
+            if interleaved:
+                a_, b_ = x[..., 0:2 * half:2], x[..., 1:2 * half:2]
+                y = torch.stack([a_ * c - b_ * s_, b_ * c + a_ * s_], -1).flatten(-2)
+                return torch.cat([y, x[..., 2 * half:]], -1)
             a_, b_ = x[..., :half], x[..., half:2 * half]
             return torch.cat([a_ * c - b_ * s_, b_ * c + a_ * s_, x[..., 2 * half:]], -1)
 
@@ -134,7 +139,8 @@ def latent_rope(qa: torch.Tensor, q: torch.Tensor, q_head: int, q_off: int, kv: 
     out = torch.empty((T, H * Wc), dtype=qa.dtype, device=qa.device)
     _m().latent_rope(out.data_ptr(), qa.data_ptr(), q.data_ptr(), q.stride(0), q_head, q_off, kv.data_ptr(),
                      kv.stride(0), norm_w.data_ptr(), float(eps), _ptr(inv_freq), half, float(mag),
-                     positions.data_ptr(), kv_slots.data_ptr(), cache.data_ptr(), T, H, r, dr, _f32(qa), _stream())
+                     positions.data_ptr(), kv_slots.data_ptr(), cache.data_ptr(), T, H, r, dr, int(interleaved), _f32(qa),
+                     _stream())
     return out
 
 
