@@ -1,7 +1,7 @@
 """`bench.py --layered`: the layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik,
-Povurax) beside the closest existing model (Llama; for Nefivik also Bolinex, for
-Sobivik also Bekulix, for Povurax also Sobivik, the closest layer-listed ones) at
-equal layer sizes, random weights.
+Povurax, Kilatar) beside the closest existing model (Llama; for Nefivik also Bolinex,
+for Sobivik also Bekulix, for Povurax also Sobivik, for Kilatar also Bolinex and
+Povurax, the closest layer-listed ones) at equal layer sizes, random weights.
 `--layered-family` picks which family runs (default: Bekulix and Bolinex).
 
 Two parts, both on one GPU:
@@ -25,8 +25,8 @@ import torch
 from .. import ops
 from ..engine.engine import EngineConfig, LLMEngine
 from ..engine.request import SamplingParams
-from ..models.config import (ModelConfig, _bekulix_preset, _bolinex_preset, _nefivik_preset, _povurax_preset,
-                             _sobivik_preset)
+from ..models.config import (ModelConfig, _bekulix_preset, _bolinex_preset, _kilatar_preset, _nefivik_preset,
+                             _povurax_preset, _sobivik_preset)
 from ..ops import mixers as mx
 from ..ops import moe
 from ..ops import recurrent as rc
@@ -79,6 +79,16 @@ def _povurax_config(s: dict):
     dense feed-forwards, no layer sharing another's weights."""
     return _povurax_preset(f"povurax {s['W']}", s["W"], s["ff"], s["layers"], s["H"], s["G"], s["d"], 2 * s["W"] // 64, 64,
                            128, 8, vocab=s["vocab"], share=False, gla_ff=True)
+
+
+def _kilatar_config(s: dict):
+    """Kilatar at the size's layer shapes: parallel layers (attention in chunks of 2048 beside lightning
+    attention of the same heads), latent attention (rank 192 + 64 rotated columns) and Mamba-2 (twice the
+    width, 64 channels and 128 states a head, 8 groups) in turn; the first feed-forward dense, the others
+    8 experts of a quarter of the dense width and 2 identity outputs (two chosen) plus a gated shared one."""
+    return _kilatar_preset(f"kilatar {s['W']}", s["W"], s["ff"], s["layers"], s["H"], s["G"], s["d"], 2048, 192, 64,
+                           2 * s["W"] // 64, 64, 128, 8, experts=8, top=2, identity=2, expert_ff=s["ff"] // 4,
+                           shared_ff=s["ff"] // 4, vocab=s["vocab"])
 
 
 def _timed(fn, iters=10, warm=2) -> float:
@@ -677,6 +687,148 @@ def povurax_kernels(s: dict, L: int, B: int, T: int) -> dict:
     return res
 
 
+def kilatar_kernels(s: dict, L: int, B: int, T: int) -> dict:
+    """Kilatar's kernels alone, each beside its counterpart: chunked attention beside the same kernels with
+    a causal and a window mask; latent attention over one shared row (causal) beside Sobivik's use of it
+    (window, sink); lightning attention beside the state-space scan (4 prompts of L / 2 tokens; B decode
+    rows); rotation + cache write + silu section beside Povurax's norm + rotation + cache write; the latent
+    preparation with neighbouring pairs beside the one with halves; the router in one pass beside
+    conversion + GEMM + choice; the residual step that joins both sides, the shared expert and the routed
+    experts beside the plain one and the experts' combine; the gated units beside silu_and_mul."""
+    H, G, d, W, ff, bs = s["H"], s["G"], s["d"], s["W"], s["ff"], 64
+    dev, dt, chunk = "cuda", torch.bfloat16, 2048
+    res = {}
+
+    def put(name, us, byts=None, flops=None, **kw):
+        res[name] = {"us": round(us, 1), **kw}
+        if byts:
+            res[name]["TB/s"] = round(byts / us / 1e6, 2)
+        if flops:
+            res[name]["TFLOPs"] = round(flops / us / 1e6, 1)
+
+    print(f"[layered] kilatar kernels {W}", file=sys.stderr, flush=True)
+    # ---- attention: prompts, then decode rows
+    nb = L // bs
+    pos, j = torch.arange(L, device=dev), torch.arange(L)
+    seq = torch.zeros(L, dtype=torch.int32, device=dev)
+    bt = torch.arange(nb, dtype=torch.int32, device=dev).view(1, nb)
+    tiles = torch.tensor(mx.tile_list(0, L), dtype=torch.int32, device=dev)
+    btd = torch.randperm(B * nb, device=dev).to(torch.int32).view(B, nb)
+    posd = torch.full((B,), L - 1, device=dev)
+    for name, n_kh, dd, dv, masks in (("heads", G, d, d, (("causal", 0), ("window", chunk), ("chunk", chunk))),
+                                      ("latent", 1, 256, 192, (("causal", 0), ("window", 1024)))):
+        q, qd = torch.randn(L, H * dd, device=dev, dtype=dt), torch.randn(B, H * dd, device=dev, dtype=dt)
+        kc, kcd = (torch.randn(n * bs, n_kh * dd, device=dev, dtype=dt) for n in (nb, B * nb))
+        vc, vcd = (kc, kcd) if name == "latent" else (torch.randn_like(kc), torch.randn_like(kcd))
+        for mask, size in masks:
+            n_vis = j - mx.first_visible(j, mask, size) + 1
+            sink = dict(sink=torch.randn(H, device=dev)) if name == "latent" and size else {}
+            us = _timed(lambda: mx.attention(q, kc, vc, pos, seq, bt, bs, H, 1, H // n_kh, dd, dv, dd ** -0.5, mask, size, 1,
+                                             False, tiles, L, **sink))
+            put(f"{name}_prefill_{mask}{size or ''}", us, None, 2.0 * (dd + dv) * H * float(n_vis.sum()))
+            vis = int(n_vis[-1])
+            parts = mx.row_attention_parts(B, n_kh * -(-(H // n_kh) // 32), vis, mx.GROUP_TARGET_WAVES)
+            us = _timed(lambda: mx.attention(qd, kcd, vcd, posd, None, btd, bs, H, 1, H // n_kh, dd, dv, dd ** -0.5, mask, size,
+                                             parts, **sink))
+            put(f"{name}_decode_{mask}{size or ''}", us, B * vis * n_kh * dd * (2 if name == "latent" else 4), parts=parts)
+        del q, qd, kc, kcd, vc, vcd
+    # ---- scans
+    P, N, Gs = 64, 128, 8
+    Hs = 2 * W // P
+    inner, C, n = Hs * P, Hs * P + 2 * Gs * N, H * d
+    for tag, n_seq, rows in (("prefill", 4, L // 2), ("decode", B, 1)):
+        Tn = n_seq * rows
+        p0 = (torch.arange(rows, device=dev) + 1).repeat(n_seq)
+        step = (p0, torch.arange(0, Tn + 1, rows, dtype=torch.int32, device=dev) if rows > 1 else None,
+                torch.arange(n_seq, dtype=torch.int32, device=dev))
+
+        def scan(name, fn, heads, dk, dv, io):
+            st = n_seq * heads * dk * dv * 4 * 2  # state read and written
+            us = _timed(fn)
+            put(f"{name}_{tag}", us, io + st, 2.0 * 2 * Tn * heads * dk * dv, tok_per_s=round(Tn / us * 1e6),
+                state_TBs=round(st / us / 1e6, 2))
+
+        p = torch.randn(Tn, 4 * n, device=dev, dtype=dt)
+        dec = torch.full((H,), 0.97, device=dev)
+        state = torch.zeros(n_seq, H, d, d, device=dev)
+        scan("lightning", lambda: rc.retention(p[:, :n], p[:, n:2 * n], p[:, 2 * n:3 * n], dec, 1.0, state, *step, H, d, d),
+             H, d, d, Tn * n * (3 * 2 + 4))
+        x, u = torch.randn(Tn, C, device=dev, dtype=dt) * 0.5, torch.randn(Tn, Hs, device=dev, dtype=dt) - 2
+        rate, D, ub = torch.ones(Hs, device=dev), torch.ones(Hs, device=dev), torch.zeros(Hs, device=dev)
+        st2 = torch.zeros(n_seq, Hs, P, N, device=dev)
+        scan("ssd", lambda: rc.ssd(x[:, :inner], x[:, inner:inner + Gs * N], x[:, inner + Gs * N:], u, ub, rate, D, st2,
+                                   *step, Hs, Gs, N, P), Hs, N, P, Tn * (C * 2 + Hs * 2 + inner * 4))
+        o, hw = torch.randn(Tn, n, device=dev), torch.ones(n, device=dev)
+        for name, heads in (("head_norm_gate_all_heads", 1), ("head_norm_gate_per_head", H)):
+            put(f"{name}_{tag}", _timed(lambda: rc.head_norm_gate(o, heads, hw, p[:, 3 * n:], 1e-5, dt)), Tn * n * (4 + 2 + 2))
+        del p, x, u, o, state, st2
+    # ---- preparation + cache write
+    nbt = T // bs + 1
+    posT = torch.arange(T, device=dev)
+    kc, vc = (torch.zeros(nbt * bs, G * d, device=dev, dtype=dt) for _ in range(2))
+    qkv = torch.randn(T, (H + 2 * G) * d + 3 * n, device=dev, dtype=dt)
+    qn, kn = torch.ones(H * d, device=dev), torch.ones(G * d, device=dev)
+    inv = rc.rotary_frequencies(d, 500000.0).to(dev)
+    io, act = T * d * 2 * (2 * H + 4 * G), ((H + 2 * G) * d, 3 * n)
+    put("rope_cache_silu_section", _timed(lambda: mx.norm_rope_cache(qkv, posT, posT, H, G, d, G * d, None, None, 0.0, inv, kc,
+                                                                     vc, silu=act)), io + T * 3 * n * 2 * 2)
+    put("povurax_norm_rope_cache", _timed(lambda: mx.norm_rope_cache(qkv, posT, posT, H, G, d, G * d, qn, kn, 1e-5, inv, kc,
+                                                                     vc)), io)
+    r, dr = 192, 64
+    qa, qp = torch.randn(H, T, r, device=dev, dtype=dt), torch.randn(T, H * (d + dr), device=dev, dtype=dt)
+    kv, cn = torch.randn(T, r + dr, device=dev, dtype=dt), torch.ones(r, device=dev)
+    cache = torch.zeros(nbt * bs, r + dr, device=dev, dtype=dt)
+    fr = rc.rotary_frequencies(dr, 10000.0).to(dev)
+    for name, il in (("latent_rope_pairs", True), ("sobivik_latent_rope_halves", False)):
+        put(name, _timed(lambda: rc.latent_rope(qa, qp, d + dr, d, kv, r, dr, cn, 1e-5, fr, 1.0, posT, posT, cache,
+                                                interleaved=il)), T * 2 * (2 * H * (r + dr) + 2 * (r + dr)))
+    del qkv, qa, qp
+    # ---- gated units
+    g, a, ah = (torch.randn(*sh, device=dev, dtype=dt) for sh in ((T, n), (T, n), (H, T, d)))
+    put("output_gate_head_major", _timed(lambda: mx.act_mul(g, ah, "sigmoid")), T * n * 6)
+    put("output_gate_rows", _timed(lambda: mx.act_mul(g, a, "sigmoid")), T * n * 6)
+    gu, bias = torch.randn(T, 2 * ff, device=dev, dtype=dt), torch.randn(ff, device=dev)
+    put("glu_gelu_bias", _timed(lambda: mx.glu_act(gu, "gelu_tanh", gate_b=bias, up_b=bias)), T * ff * 2 * 3)
+    put("llama_silu_and_mul", _timed(lambda: ops.silu_and_mul(gu)), T * ff * 2 * 3)
+    del gu
+    # ---- routed feed-forward and residual: prompts, then decode rows
+    E, ident, top, fe = 8, 2, 2, ff // 4
+    rw, corr = torch.randn(E + ident + 1, W, device=dev) * W ** -0.5, torch.zeros(E + ident, device=dev)
+    wgu = torch.randn(E, 2 * fe, W, device=dev, dtype=dt) * W ** -0.5
+    wgl = moe.interleave_glu(wgu) if fe % moe.GLU_BLOCK == 0 and moe.tile_gemm_ok(wgu[0][:1], wgu) else wgu
+    wdn = torch.randn(E, W, fe, device=dev, dtype=dt) * fe ** -0.5
+    nw = torch.ones(W, device=dev)
+    for tag, rows in (("prefill", T), ("decode", B)):
+        h = torch.randn(rows, W, device=dev, dtype=dt)
+        kw = dict(score="softmax", renorm=True, scale=1.5)
+        put(f"router_{tag}", _timed(lambda: moe.router(h, rw, E + ident, corr, top, **kw)),
+            rows * W * 2 + rw.numel() * 4)
+        put(f"router_by_gemm_{tag}", _timed(lambda: moe.route(torch.matmul(h.float(), rw.t())[:, :E + ident].contiguous(), corr,
+                                                              top, **kw)), rows * W * 2 + rw.numel() * 4)
+        idx, wt, _ = moe.router(h, rw, E + ident, corr, top, **kw)
+        put(f"plan_{tag}", _timed(lambda: moe.plan(idx, E)))
+        order, offsets = moe.plan(idx, E)
+        real, used = float(offsets[-1]), int((offsets[1:] > offsets[:-1]).sum())  # slots with an expert, experts in use
+        put(f"grouped_gemm_gate_up_{tag}", _timed(lambda: moe.grouped_gemm(h, wgl, order, offsets, top, True, False,
+                                                                           glu=wgl is not wgu)),
+            used * 2 * fe * W * 2 if tag == "decode" else None, 2.0 * real * W * 2 * fe)
+        act = torch.randn(rows * top, fe, device=dev, dtype=dt)
+        put(f"grouped_gemm_down_{tag}", _timed(lambda: moe.grouped_gemm(act, wdn, order, offsets, top, False, True)),
+            used * fe * W * 2 if tag == "decode" else None, 2.0 * real * W * fe)
+        y, X = torch.randn(rows * top, W, device=dev, dtype=dt), torch.randn(rows, W, device=dev)
+        a, c, b = (torch.randn(rows, W, device=dev, dtype=dt) for _ in range(3))
+        ex = (y, wt, idx, E, h)
+        fin = dict(eps=1e-5, norm="rms", norm_w=nw, out_dtype=dt)
+        put(f"residual_step_two_sides_shared_experts_{tag}",
+            _timed(lambda: mx.residual_step(X, b=b, c=a, c_w=nw, d=c, d_w=nw, experts=ex, **fin)),
+            rows * W * (4 + 4 + 2 * 3 + 2 * top + 2))
+        put(f"residual_step_addend_experts_{tag}", _timed(lambda: mx.residual_step(X, a=a, experts=ex, **fin)),
+            rows * W * (4 + 4 + 2 + 2 * top + 2))
+        put(f"residual_step_two_addends_{tag}", _timed(lambda: mx.residual_step(X, a, b, **fin)), rows * W * (4 + 4 + 2 + 2 + 2))
+        put(f"moe_combine_{tag}", _timed(lambda: moe.combine(y, wt, b)), rows * W * 2 * (top + 2))
+    return res
+
+
 def run_layered_compare(args, dev) -> dict:
     isl, osl = min(args.isl, 2048), min(args.osl, 64)
     fam = getattr(args, "layered_family", "all")
@@ -698,18 +850,24 @@ def run_layered_compare(args, dev) -> dict:
             row["povurax_kernels"] = povurax_kernels(s, 4096, 64, 8192)
             row["sobivik"] = engine_throughput(_sobivik_config(s), dev, isl, osl, 4, 64, args.seed)
             row["params"] = {c.name: c.num_params() for c in (_povurax_config(s), _sobivik_config(s))}
+        if fam == "kilatar":
+            row["kilatar"] = engine_throughput(_kilatar_config(s), dev, isl, osl, 4, 64, args.seed)
+            row["kilatar_kernels"] = kilatar_kernels(s, 4096, 64, 8192)
+            row["bolinex"] = engine_throughput(_bolinex_config(s), dev, isl, osl, 4, 64, args.seed)
+            row["povurax"] = engine_throughput(_povurax_config(s), dev, isl, osl, 4, 64, args.seed)
+            row["params"] = {c.name: c.num_params() for c in (_kilatar_config(s), _bolinex_config(s), _povurax_config(s))}
         if fam == "nefivik":
             row["nefivik"] = engine_throughput(_nefivik_config(s), dev, isl, osl, 4, 64, args.seed)
             row["nefivik_kernels"] = nefivik_kernels(s, 4096, 64, 8192)
             row["bolinex"] = engine_throughput(_bolinex_config(s), dev, isl, osl, 4, 64, args.seed)
         row["llama"] = engine_throughput(lla, dev, isl, osl, 4, 64, args.seed)
-        if fam in ("nefivik", "sobivik"):
+        if fam in ("nefivik", "sobivik", "kilatar"):
             sizes[name] = row
             continue
         row["attention_kernels"] = attention_kernels(s, 4096, 64)
         if fam in ("all", "bekulix"):
             row["rowwise_kernels"] = rowwise_kernels(s, 8192)
         sizes[name] = row
-    return {"metric": "layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik, Povurax) beside Llama at equal layer sizes: "
+    return {"metric": "layer-listed models (Bekulix, Bolinex, Nefivik, Sobivik, Povurax, Kilatar) beside Llama at equal layer sizes: "
                       "engine prefill / decode tokens/s and kernels alone", "unit": "tokens/s", "n_gpus": 1, "dtype": "bf16",
             "family": fam, "data": "synthetic (random-token prompts, random-init weights)", "sizes": sizes}
