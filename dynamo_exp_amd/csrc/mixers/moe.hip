@@ -132,6 +132,83 @@ __global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __rest
   route_token(g, z + tc * g.E, c, c + g.E, on, idx + tc * g.top, w + tc * g.top, lane);
 }
 
+// The same result for few tokens: a workgroup per token, its row in registers as far as it fits; 4 waves share
+// the width, outputs are summed 8 at a time.  V elements per access.
+template <typename T, int V>
+__global__ void __launch_bounds__(256) moe_router_rows_kernel(int* __restrict__ idx, float* __restrict__ wgt,
+                                                              float* __restrict__ gates, const T* __restrict__ h,
+                                                              int64_t hs, const float* __restrict__ w, int n_out, int W,
+                                                              RouteArgs g) {
+  constexpr int kKeep = 4;
+  extern __shared__ float rsm[];
+  float* part = rsm;             // [4 waves][n_out]
+  float* z = part + 4 * n_out;   // [n_out]
+  float* scratch = z + n_out;    // [4][E + n_groups]
+  const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
+  const int64_t t = blockIdx.x;
+  const T* hp = h + t * hs;
+  auto load_h = [&](int e, float* x) {
+    if constexpr (V == 1) {
+      if constexpr (sizeof(T) == 2) x[0] = bf16_to_f32(hp[e]); else x[0] = hp[e];
+    } else if constexpr (sizeof(T) == 2) {
+      const uint2 q = *reinterpret_cast<const uint2*>(hp + e);
+      x[0] = bf16lo(q.x), x[1] = bf16hi(q.x), x[2] = bf16lo(q.y), x[3] = bf16hi(q.y);
+    } else {
+      const f32x4 q = *reinterpret_cast<const f32x4*>(hp + e);
+      x[0] = q[0], x[1] = q[1], x[2] = q[2], x[3] = q[3];
+    }
+  };
+  float x[kKeep][V];
+#pragma unroll
+  for (int k = 0; k < kKeep; ++k) {
+    const int e = (tid + 256 * k) * V;
+#pragma unroll
+    for (int i = 0; i < V; ++i) x[k][i] = 0.f;
+    if (e < W) load_h(e, x[k]);
+  }
+  for (int o0 = 0; o0 < n_out; o0 += 8) {
+    float acc[8];
+#pragma unroll
+    for (int j = 0; j < 8; ++j) acc[j] = 0.f;
+    auto dot = [&](int e, const float* xv) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) {
+        if (o0 + j >= n_out) break;
+        const float* wp = w + (int64_t)(o0 + j) * W + e;
+        if constexpr (V == 1) {
+          acc[j] += xv[0] * wp[0];
+        } else {
+          const f32x4 q = *reinterpret_cast<const f32x4*>(wp);
+#pragma unroll
+          for (int i = 0; i < V; ++i) acc[j] += xv[i] * q[i];
+        }
+      }
+    };
+#pragma unroll
+    for (int k = 0; k < kKeep; ++k) {
+      const int e = (tid + 256 * k) * V;
+      if (e < W) dot(e, x[k]);
+    }
+    for (int e = (tid + 256 * kKeep) * V; e < W; e += 256 * V) {
+      float t4[V];
+      load_h(e, t4);
+      dot(e, t4);
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float s = wave_reduce_sum(acc[j]);
+      if (lane == 0 && o0 + j < n_out) part[wv * n_out + o0 + j] = s;
+    }
+  }
+  __syncthreads();
+  for (int o = tid; o < n_out; o += 256) z[o] = part[o] + part[n_out + o] + part[2 * n_out + o] + part[3 * n_out + o];
+  __syncthreads();
+  for (int j = tid; j < n_out - g.E; j += 256) gates[t * (n_out - g.E) + j] = 1.f / (1.f + expf(-z[g.E + j]));
+  // (every wave takes part in the choice's barriers; wave 0 writes it)
+  float* c = scratch + wv * (g.E + g.n_groups);
+  route_token(g, z, c, c + g.E, wv == 0, idx + t * g.top, wgt + t * g.top, lane);
+}
+
 // order [R]: slots sorted by expert, stable; offsets [E + 1].  One workgroup:
 // counts by LDS atomics (the counts do not depend on their order), a serial
 // scan over the experts, then every wave places the slots of its experts in
@@ -494,6 +571,21 @@ int dxm_moe_router(int* idx, float* w, float* gates, const void* h, int64_t h_st
   if (const int bad = route_args_bad(g)) return bad;
   if (!dxm_moe_router_ok(n_out, E, n_groups) || W < 1) return 2;
   if (!idx || !w || !h || !rw || (n_out > E && !gates)) return 5;
+  const int esz = f32 ? 4 : 2;
+  if (T <= 256) {
+    const size_t lds = (5 * (size_t)n_out + 4 * (size_t)(E + n_groups)) * sizeof(float);
+    const bool vec = W % 4 == 0 && h_stride % 4 == 0 && (uintptr_t)h % (4 * esz) == 0 && (uintptr_t)rw % 16 == 0;
+#define ROUTER_ROWS(TY, V)                                                                                            \
+  hipLaunchKernelGGL((moe_router_rows_kernel<TY, V>), dim3(T), dim3(256), lds, st, idx, w, gates, (const TY*)h, h_stride, \
+                     rw, n_out, W, g);
+    if (f32 && vec) { ROUTER_ROWS(float, 4) }
+    else if (f32) { ROUTER_ROWS(float, 1) }
+    else if (vec) { ROUTER_ROWS(bf16_t, 4) }
+    else { ROUTER_ROWS(bf16_t, 1) }
+#undef ROUTER_ROWS
+    DX_CHECK_LAUNCH();
+    return 0;
+  }
   const dim3 grid((unsigned)((T + 15) / 16));
   // few tokens: more waves share the width
   const bool many = T <= 1024 && router_lds(16, n_out, E, n_groups) <= 60 * 1024;

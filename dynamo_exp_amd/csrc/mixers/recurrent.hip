@@ -733,8 +733,10 @@ void launch_head_norm_vec(void* out, const float* o, const float* w, const void*
 // out = y silu(z), divided by the root mean square of its group (n equal groups of the row, eps inside the
 // root), times w: the gate enters in front of the norm.  One workgroup per (row, group); a thread keeps its
 // elements (V neighbours at a time, up to kGnKeep times) in registers between the mean square and the result.
+// GATE 1, 2: the gate enters behind the norm instead (sigmoid(z) or silu(z); no z: none), for head norms whose
+// heads are wider than a wave's registers.
 constexpr int kGnKeep = 4;
-template <typename T, int V, int NT>
+template <typename T, int V, int NT, int GATE>
 __global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out, int64_t os,
                                                              const float* __restrict__ y, const T* __restrict__ z,
                                                              int64_t zs, const float* __restrict__ w, int n_groups,
@@ -745,17 +747,19 @@ __global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out
   const float* yp = y + row * (int64_t)n_groups * n + c0;
   const T* zp = z + row * zs + c0;
   auto load = [&](int e, float* x) {
-    float a[V], b[V];
     if constexpr (V == 1) {
-      a[0] = yp[e];
-      b[0] = ldf<T>(zp, e);
+      x[0] = yp[e];
     } else {
 #pragma unroll
-      for (int i = 0; i < V; i += 4) VecIO<float, 4>::ld(yp + e + i, a + i);
-      VecIO<T, V>::ld(zp + e, b);
+      for (int i = 0; i < V; i += 4) VecIO<float, 4>::ld(yp + e + i, x + i);
     }
+    if constexpr (GATE == 0) {
+      float b[V];
+      if constexpr (V == 1) b[0] = ldf<T>(zp, e);
+      else VecIO<T, V>::ld(zp + e, b);
 #pragma unroll
-    for (int i = 0; i < V; ++i) x[i] = a[i] * b[i] * fast_sigmoid(b[i]);
+      for (int i = 0; i < V; ++i) x[i] *= b[i] * fast_sigmoid(b[i]);
+    }
   };
   float x[kGnKeep][V], ss = 0.f;
 #pragma unroll
@@ -777,7 +781,16 @@ __global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out
   auto put = [&](int e, const float* xv) {
     float o[V];
 #pragma unroll
-    for (int i = 0; i < V; ++i) o[i] = xv[i] * inv * w[c0 + e + i];
+    for (int i = 0; i < V; ++i) o[i] = xv[i] * inv * (w ? w[c0 + e + i] : 1.f);
+    if constexpr (GATE != 0) {
+      if (z) {
+        float b[V];
+        if constexpr (V == 1) b[0] = ldf<T>(zp, e);
+        else VecIO<T, V>::ld(zp + e, b);
+#pragma unroll
+        for (int i = 0; i < V; ++i) o[i] *= GATE == 2 ? b[i] * fast_sigmoid(b[i]) : fast_sigmoid(b[i]);
+      }
+    }
     if constexpr (V == 1) stf<T>(out, row * os + c0 + e, o[0]);
     else VecIO<T, V>::st(out + row * os + c0 + e, o);
   };
@@ -791,15 +804,15 @@ __global__ void __launch_bounds__(NT) gate_group_norm_kernel(T* __restrict__ out
   }
 }
 
-template <typename T, int V>
+template <typename T, int V, int GATE = 0>
 void launch_gate_group_norm(void* out, int64_t os, const float* y, const void* z, int64_t zs, const float* w, int rows,
                             int n_groups, int n, float eps, hipStream_t st) {
   const dim3 grid((unsigned)((int64_t)rows * n_groups));
   if (n > 64 * V)
-    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 256>), grid, dim3(256), 0, st, (T*)out, os, y, (const T*)z, zs, w,
+    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 256, GATE>), grid, dim3(256), 0, st, (T*)out, os, y, (const T*)z, zs, w,
                        n_groups, n, eps);
   else
-    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 64>), grid, dim3(64), 0, st, (T*)out, os, y, (const T*)z, zs, w,
+    hipLaunchKernelGGL((gate_group_norm_kernel<T, V, 64, GATE>), grid, dim3(64), 0, st, (T*)out, os, y, (const T*)z, zs, w,
                        n_groups, n, eps);
 }
 
@@ -910,6 +923,17 @@ int dxm_head_norm_gate(void* out, const float* o, const float* w, const void* ga
       else if (dv <= 128) launch_head_norm_vec<T, 32>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
       else launch_head_norm_vec<T, 64>(out, o, w, gate, gs, n_vec, H, dv, eps, gate_act, st);
     });
+    DX_CHECK_LAUNCH();
+    return 0;
+  }
+  const int V = f32 ? 4 : 8;
+  if (dv > 512 && dv % V == 0 && gs % V == 0 && (uintptr_t)o % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+      (uintptr_t)gate % 16 == 0) {  // a workgroup per head
+    const int64_t os = (int64_t)H * dv;
+    if (f32 && gate_act) launch_gate_group_norm<float, 4, 2>(out, os, o, gate, gs, w, rows, H, dv, eps, st);
+    else if (f32) launch_gate_group_norm<float, 4, 1>(out, os, o, gate, gs, w, rows, H, dv, eps, st);
+    else if (gate_act) launch_gate_group_norm<bf16_t, 8, 2>(out, os, o, gate, gs, w, rows, H, dv, eps, st);
+    else launch_gate_group_norm<bf16_t, 8, 1>(out, os, o, gate, gs, w, rows, H, dv, eps, st);
     DX_CHECK_LAUNCH();
     return 0;
   }

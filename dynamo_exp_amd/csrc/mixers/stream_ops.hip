@@ -149,7 +149,8 @@ __global__ void __launch_bounds__(kThreads) stream_step_kernel(float* __restrict
 // X[t, s, :] = table[ids[t], :] * scale (+ ptab[pos[t], :], a learned vector per position)
 // for every stream s (fp32 streams; product and sum are fp32); with nw [W] the row is then
 // divided by its root mean square (eps inside the root) and multiplied by nw
-template <typename T>
+constexpr int kResChunks = 8;
+template <typename T, int V>
 __global__ void __launch_bounds__(kThreads) embed_streams_kernel(float* __restrict__ X, const T* __restrict__ table,
                                                                  const int64_t* __restrict__ ids, int S, int W,
                                                                  int64_t vocab, const T* __restrict__ ptab,
@@ -161,24 +162,58 @@ __global__ void __launch_bounds__(kThreads) embed_streams_kernel(float* __restri
   const bool ok = id >= 0 && id < vocab;
   const int64_t p = ptab ? pos[t] : -1;
   const bool pok = p >= 0 && p < n_pos;
-  auto value = [&](int c) {
-    float v = ok ? ldf<T>(table, id * (int64_t)W + c) * scale : 0.f;
-    if (pok) v += ldf<T>(ptab, p * (int64_t)W + c);
-    return v;
+  auto value = [&](int c, float* v) {
+    if (ok) ldv<T, V>(table + id * (int64_t)W + c, v);
+#pragma unroll
+    for (int i = 0; i < V; ++i) v[i] = ok ? v[i] * scale : 0.f;
+    if (pok) {
+      float q[V];
+      ldv<T, V>(ptab + p * (int64_t)W + c, q);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += q[i];
+    }
   };
   float r = 1.f;
+  float v[kResChunks][V];  // the row, as far as it fits
+#pragma unroll
+  for (int k = 0; k < kResChunks; ++k) {
+    const int c = (threadIdx.x + k * kThreads) * V;
+    if (c < W) value(c, v[k]);
+  }
   if (nw) {
     float ss = 0.f;
-    for (int c = threadIdx.x; c < W; c += kThreads) {
-      const float v = value(c);
-      ss += v * v;
+#pragma unroll
+    for (int k = 0; k < kResChunks; ++k)
+      if ((int)(threadIdx.x + k * kThreads) * V < W) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) ss += v[k][i] * v[k][i];
+      }
+    for (int c = (threadIdx.x + kResChunks * kThreads) * V; c < W; c += kThreads * V) {
+      float u[V];
+      value(c, u);
+#pragma unroll
+      for (int i = 0; i < V; ++i) ss += u[i] * u[i];
     }
     r = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
   }
-  for (int c = threadIdx.x; c < W; c += kThreads) {
-    float v = value(c);
-    if (nw) v *= r * nw[c];
-    for (int s = 0; s < S; ++s) X[(t * S + s) * (int64_t)W + c] = v;
+  auto put = [&](int c, float* u) {
+    if (nw) {
+      float w[V];
+      ldv<float, V>(nw + c, w);
+#pragma unroll
+      for (int i = 0; i < V; ++i) u[i] *= r * w[i];
+    }
+    for (int s = 0; s < S; ++s) stv<float, V>(X + (t * S + s) * (int64_t)W + c, u);
+  };
+#pragma unroll
+  for (int k = 0; k < kResChunks; ++k) {
+    const int c = (threadIdx.x + k * kThreads) * V;
+    if (c < W) put(c, v[k]);
+  }
+  for (int c = (threadIdx.x + kResChunks * kThreads) * V; c < W; c += kThreads * V) {
+    float u[V];
+    value(c, u);
+    put(c, u);
   }
 }
 
@@ -203,7 +238,6 @@ __global__ void __launch_bounds__(kThreads) gather_rows_kernel(T* __restrict__ o
 // an fp32 addend e, a constant row `bias`, the weighted sum of a mixture of
 // experts, and a list of rows: then row r of out is the result for row rows[r],
 // and x itself is left as it was.
-constexpr int kResChunks = 8;
 template <typename T> struct ResExt {
   const T* d;         // + d / sqrt(mean(d^2) + eps) * dw
   int64_t d_stride;
@@ -220,16 +254,25 @@ template <typename T> struct ResExt {
   int64_t mh_stride;
   const int64_t* rows;
 };
-template <typename T, int V, bool EXT>
+// sum over the workgroup (4 waves); every call of a kernel has an area `red` of its own: one barrier
+__device__ __forceinline__ float sum_all(float v, float* red) {
+  v = wave_reduce_sum(v);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+  __syncthreads();
+  return red[0] + red[1] + red[2] + red[3];
+}
+
+// KC: chunks of a row in registers.  All loads of the row are issued before the first sum over the workgroup.
+template <typename T, int V, bool EXT, int KC>
 __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     float* __restrict__ X, const T* __restrict__ a, int64_t a_stride, const T* __restrict__ b, int64_t b_stride,
     const T* __restrict__ c, int64_t c_stride, const float* __restrict__ cw, const T* __restrict__ cg,
     int64_t cg_stride, const float* __restrict__ cgb, float eps, int norm, const float* __restrict__ nw,
     const float* __restrict__ nb, T* __restrict__ out, T* __restrict__ xc, int W, ResExt<T> g) {
-  __shared__ float red[16];
+  static_assert(kThreads == 256, "sum_all adds four waves");
+  __shared__ float red[4][4];
   const int64_t row = EXT && g.rows ? g.rows[blockIdx.x] : (int64_t)blockIdx.x, orow = blockIdx.x;
   float* x = X + row * (int64_t)W;
-  float rc = 0.f, rd = 0.f;
   // the addend c at columns e .. e + V - 1, gated by sigmoid(cg + cgb) when a gate is given
   auto load_c = [&](int e, float* v) {
     ldv<T, V>(c + row * c_stride + e, v);
@@ -242,36 +285,10 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     }
   };
   auto load_d = [&](int e, float* v) { ldv<T, V>(g.d + row * g.d_stride + e, v); };
-  // root mean square of an addend; its chunks stay in registers between the mean square and the sum
-  auto inv_rms = [&](auto&& load, float (*keep)[V]) {
-    float ss = 0.f;
-#pragma unroll
-    for (int k = 0; k < kResChunks; ++k) {
-      const int e = (threadIdx.x + k * kThreads) * V;
-      if (e < W) {
-        load(e, keep[k]);
-#pragma unroll
-        for (int i = 0; i < V; ++i) ss += keep[k][i] * keep[k][i];
-      }
-    }
-    for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
-      float v[V];
-      load(e, v);
-#pragma unroll
-      for (int i = 0; i < V; ++i) ss += v[i] * v[i];
-    }
-    const float r = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
-    __syncthreads();
-    return r;
-  };
-  float cv[kResChunks][V], dv[EXT ? kResChunks : 1][V];
-  if (c) rc = inv_rms(load_c, cv);
-  if constexpr (EXT) {
-    if (g.d) rd = inv_rms(load_d, dv);
-  }
-  // everything added at columns e .. e + V - 1; ct, dt: the values of c and d there
-  auto add = [&](int e, float* v, const float* ct, const float* dt) {
-    float t[V], w[V];
+  // x and everything added to it as it is
+  auto load_x = [&](int e, float* v) {
+    float t[V];
+    ldv<float, V>(x + e, v);
     if (a) {
       ldv<T, V>(a + row * a_stride + e, t);
 #pragma unroll
@@ -282,21 +299,11 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
 #pragma unroll
       for (int i = 0; i < V; ++i) v[i] += t[i];
     }
-    if (c) {
-      ldv<float, V>(cw + e, w);
-#pragma unroll
-      for (int i = 0; i < V; ++i) v[i] += ct[i] * rc * w[i];
-    }
     if constexpr (EXT) {
-      if (g.d) {
-        ldv<float, V>(g.dw + e, w);
-#pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += dt[i] * rd * w[i];
-      }
       if (g.bias) {
-        ldv<float, V>(g.bias + e, w);
+        ldv<float, V>(g.bias + e, t);
 #pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += w[i];
+        for (int i = 0; i < V; ++i) v[i] += t[i];
       }
       if (g.my) {
         float m[V];
@@ -313,32 +320,89 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
         for (int i = 0; i < V; ++i) v[i] += m[i];
       }
       if (g.e) {
-        ldv<float, V>(g.e + row * (int64_t)W + e, w);
+        ldv<float, V>(g.e + row * (int64_t)W + e, t);
 #pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += w[i];
+        for (int i = 0; i < V; ++i) v[i] += t[i];
       }
     }
   };
-  bool touch = a || b || c;
-  if constexpr (EXT) touch = !g.rows && (touch || g.d || g.e || g.bias || g.my);
+  const bool has_d = EXT && g.d;
+  float r[KC][V], cv[KC][V], dv[EXT ? KC : 1][V], cs = 0.f, ds = 0.f;
+#pragma unroll
+  for (int k = 0; k < KC; ++k) {
+    const int e = (threadIdx.x + k * kThreads) * V;
+    if (e < W) {
+      if (c) load_c(e, cv[k]);
+      if constexpr (EXT) {
+        if (has_d) load_d(e, dv[k]);
+      }
+      load_x(e, r[k]);
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < KC; ++k) {
+    const int e = (threadIdx.x + k * kThreads) * V;
+    if (e < W) {
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        if (c) cs += cv[k][i] * cv[k][i];
+        if constexpr (EXT) {
+          if (has_d) ds += dv[k][i] * dv[k][i];
+        }
+      }
+    }
+  }
+  const int tail = (threadIdx.x + KC * kThreads) * V;  // wide rows: columns from here on are read when they are needed
+  for (int e = tail; e < W; e += kThreads * V) {
+    float v[V];
+    if (c) {
+      load_c(e, v);
+#pragma unroll
+      for (int i = 0; i < V; ++i) cs += v[i] * v[i];
+    }
+    if (has_d) {
+      load_d(e, v);
+#pragma unroll
+      for (int i = 0; i < V; ++i) ds += v[i] * v[i];
+    }
+  }
+  float rc = 0.f, rd = 0.f;
+  if (has_d) {
+    ds = wave_reduce_sum(ds);
+    if ((threadIdx.x & 63) == 0) red[1][threadIdx.x >> 6] = ds;
+  }
+  if (c) rc = rsqrtf(sum_all(cs, red[0]) / (float)W + eps);
+  else if (has_d) __syncthreads();
+  if (has_d) rd = rsqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)W + eps);
+  // the normed addends at columns e .. e + V - 1; ct, dt: the values of c and d there
+  auto add = [&](int e, float* v, const float* ct, const float* dt) {
+    float w[V];
+    if (c) {
+      ldv<float, V>(cw + e, w);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += ct[i] * rc * w[i];
+    }
+    if (has_d) {
+      ldv<float, V>(g.dw + e, w);
+#pragma unroll
+      for (int i = 0; i < V; ++i) v[i] += dt[i] * rd * w[i];
+    }
+  };
   // a wide row's tail: x and its addends from memory
   auto wide = [&](int e, float* v) {
     float ct[V], dt[V];
-    ldv<float, V>(x + e, v);
+    load_x(e, v);
     if (c) load_c(e, ct);
-    if constexpr (EXT) {
-      if (g.d) load_d(e, dt);
-    }
+    if (has_d) load_d(e, dt);
     add(e, v, ct, dt);
   };
-  const bool keep = W <= kThreads * V * kResChunks;
-  float r[kResChunks][V];
+  bool touch = a || b || c;
+  if constexpr (EXT) touch = !g.rows && (touch || g.d || g.e || g.bias || g.my);
   float sum = 0.f;
 #pragma unroll
-  for (int k = 0; k < kResChunks; ++k) {
+  for (int k = 0; k < KC; ++k) {
     const int e = (threadIdx.x + k * kThreads) * V;
     if (e < W) {
-      ldv<float, V>(x + e, r[k]);
       add(e, r[k], cv[k], dv[EXT ? k : 0]);
       if (touch) stv<float, V>(x + e, r[k]);
       if (xc) stv<T, V>(xc + orow * (int64_t)W + e, r[k]);
@@ -346,15 +410,13 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
       for (int i = 0; i < V; ++i) sum += r[k][i];
     }
   }
-  if (!keep) {  // wide rows: the same arithmetic, chunk by chunk through x
-    for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
-      float v[V];
-      wide(e, v);
-      if (touch) stv<float, V>(x + e, v);
-      if (xc) stv<T, V>(xc + orow * (int64_t)W + e, v);
+  for (int e = tail; e < W; e += kThreads * V) {
+    float v[V];
+    wide(e, v);
+    if (touch) stv<float, V>(x + e, v);
+    if (xc) stv<T, V>(xc + orow * (int64_t)W + e, v);
 #pragma unroll
-      for (int i = 0; i < V; ++i) sum += v[i];
-    }
+    for (int i = 0; i < V; ++i) sum += v[i];
   }
   if (!norm) return;
   // a wide row's tail once more: as this thread wrote it, or (x left as it was) summed again
@@ -363,50 +425,40 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     else wide(e, v);
   };
   float mean = 0.f;
-  if (norm == 2) {
-    mean = block_reduce_sum(sum, red) / (float)W;
-    __syncthreads();
-  }
+  if (norm == 2) mean = sum_all(sum, red[2]) / (float)W;
   float ss = 0.f;
 #pragma unroll
-  for (int k = 0; k < kResChunks; ++k) {
+  for (int k = 0; k < KC; ++k) {
     const int e = (threadIdx.x + k * kThreads) * V;
     if (e < W) {
 #pragma unroll
       for (int i = 0; i < V; ++i) ss += (r[k][i] - mean) * (r[k][i] - mean);
     }
   }
-  if (!keep) {
-    for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
-      float v[V];
-      again(e, v);
+  for (int e = tail; e < W; e += kThreads * V) {
+    float v[V];
+    again(e, v);
 #pragma unroll
-      for (int i = 0; i < V; ++i) ss += (v[i] - mean) * (v[i] - mean);
-    }
+    for (int i = 0; i < V; ++i) ss += (v[i] - mean) * (v[i] - mean);
   }
-  const float rs = rsqrtf(block_reduce_sum(ss, red) / (float)W + eps);
+  const float rs = rsqrtf(sum_all(ss, red[3]) / (float)W + eps);
+  auto put = [&](int e, const float* v) {
+    float w[V], bb[V], o[V];
+    ldv<float, V>(nw + e, w);
+    if (norm == 2) ldv<float, V>(nb + e, bb);
 #pragma unroll
-  for (int k = 0; k < kResChunks; ++k) {
+    for (int i = 0; i < V; ++i) o[i] = (v[i] - mean) * rs * w[i] + (norm == 2 ? bb[i] : 0.f);
+    stv<T, V>(out + orow * (int64_t)W + e, o);
+  };
+#pragma unroll
+  for (int k = 0; k < KC; ++k) {
     const int e = (threadIdx.x + k * kThreads) * V;
-    if (e < W) {
-      float w[V], bb[V], o[V];
-      ldv<float, V>(nw + e, w);
-      if (norm == 2) ldv<float, V>(nb + e, bb);
-#pragma unroll
-      for (int i = 0; i < V; ++i) o[i] = (r[k][i] - mean) * rs * w[i] + (norm == 2 ? bb[i] : 0.f);
-      stv<T, V>(out + orow * (int64_t)W + e, o);
-    }
+    if (e < W) put(e, r[k]);
   }
-  if (!keep) {
-    for (int e = (threadIdx.x + kResChunks * kThreads) * V; e < W; e += kThreads * V) {
-      float v[V], w[V], bb[V], o[V];
-      again(e, v);
-      ldv<float, V>(nw + e, w);
-      if (norm == 2) ldv<float, V>(nb + e, bb);
-#pragma unroll
-      for (int i = 0; i < V; ++i) o[i] = (v[i] - mean) * rs * w[i] + (norm == 2 ? bb[i] : 0.f);
-      stv<T, V>(out + orow * (int64_t)W + e, o);
-    }
+  for (int e = tail; e < W; e += kThreads * V) {
+    float v[V];
+    again(e, v);
+    put(e, v);
   }
 }
 
@@ -533,8 +585,8 @@ __device__ __forceinline__ float act_fn(float z, int act) {
     const float r = fmaxf(z, 0.f);
     return r * r;
   }
-  const float c = 0.7978845608028654f;          // gelu, tanh form
-  return 0.5f * z * (1.f + tanhf(c * (z + 0.044715f * z * z * z)));
+  // gelu, tanh form: 0.5 (1 + tanh u) = 1 / (1 + e^(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
+  return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
 }
 
 // out [rows, F] = act(gate + gate_b) * (up + up_b) * row_scale[row] * post  (up null: act(gate) alone); gate and
@@ -722,8 +774,15 @@ int dxm_embed_streams(float* X, const void* table, const int64_t* ids, int rows,
                       hipStream_t st) {
   if (rows <= 0) return 0;
   if (ptab && !pos) return 1;
-  DISPATCH_T(f32, hipLaunchKernelGGL(embed_streams_kernel<T>, dim3(rows), dim3(kThreads), 0, st, X, (const T*)table,
-                                     ids, S, W, vocab, (const T*)ptab, pos, n_pos, scale, nw, eps));
+  const int by = f32 ? 16 : 8;
+  const bool vec = W % 4 == 0 && (uintptr_t)X % 16 == 0 && (uintptr_t)table % by == 0 && (uintptr_t)ptab % by == 0 &&
+                   (uintptr_t)nw % 16 == 0;
+#define EMBED(V)                                                                                                         \
+  DISPATCH_T(f32, hipLaunchKernelGGL((embed_streams_kernel<T, V>), dim3(rows), dim3(kThreads), 0, st, X, (const T*)table, \
+                                     ids, S, W, vocab, (const T*)ptab, pos, n_pos, scale, nw, eps))
+  if (vec) { EMBED(4) }
+  else { EMBED(1) }
+#undef EMBED
   DX_CHECK_LAUNCH();
   return 0;
 }
@@ -755,16 +814,19 @@ int dxm_residual_step(float* X, const void* a, int64_t a_stride, const void* b, 
                    al(out, 4 * esz) && al(xc, 4 * esz) && al(d, 4 * esz) && al(dw, 16) && al(e, 16) && al(bias, 16) &&
                    al(my, 4 * esz) && al(mh, 4 * esz);
   const bool ext = d || e || bias || my || pick;
-#define RES(V, EXT)                                                                                                     \
-  DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, V, EXT>), dim3(rows), dim3(kThreads), 0, st, X,           \
+#define RES(V, EXT, KC)                                                                                                 \
+  DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, V, EXT, KC>), dim3(rows), dim3(kThreads), 0, st, X,           \
                                      (const T*)a, a_stride, (const T*)b, b_stride, (const T*)c, c_stride, cw,           \
                                      (const T*)cg, cg_stride, cgb, eps, norm, nw, nb, (T*)out, (T*)xc, W,               \
                                      (ResExt<T>{(const T*)d, d_stride, dw, e, bias, (const T*)my, mw, midx, experts,    \
                                                 top, (const T*)mh, mh_stride, pick})))
-  if (vec && ext) { RES(4, true) }
-  else if (vec) { RES(4, false) }
-  else if (ext) { RES(1, true) }
-  else { RES(1, false) }
+  const bool narrow = W <= 4 * kThreads * 4;  // four chunks hold the row: fewer registers, more workgroups per CU
+  if (vec && ext && narrow) { RES(4, true, 4) }
+  else if (vec && ext) { RES(4, true, 8) }
+  else if (vec && narrow) { RES(4, false, 4) }
+  else if (vec) { RES(4, false, 8) }
+  else if (ext) { RES(1, true, 8) }
+  else { RES(1, false, 8) }
 #undef RES
   DX_CHECK_LAUNCH();
   return 0;

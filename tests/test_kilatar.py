@@ -231,10 +231,10 @@ def test_residual_step_addends_alone(device, dtype, W):
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("W,E,top,identity,gates", [(72, 5, 2, 2, 1), (33, 1, 1, 0, 0), (21, 3, 4, 3, 1), (256, 30, 8, 2, 2),
                                                     (130, 64, 6, 5, 1), (8, 700, 3, 1, 1)])
-@pytest.mark.parametrize("T", [1, 17, 1100])
+@pytest.mark.parametrize("T", [1, 17, 300, 1100])
 def test_router_alone(device, dtype, W, E, top, identity, gates, T):
     """Logits in fp32, softmax over all outputs, choice with the correction, weights without it, divided by their
-    sum, scaled; gates of the same pass; token counts on both of the kernel's shapes."""
+    sum, scaled; gates of the same pass; token counts on all of the kernels' shapes."""
     torch.manual_seed(W + E)
     n, dt = E + identity, DT[dtype]
     h, w, corr = torch.randn(T, W).to(dt), torch.randn(n + gates, W) * W ** -0.5 * 2, torch.randn(n) * 0.2
@@ -437,7 +437,7 @@ def test_lightning_scan_alone(device, dtype, H, dk, dv):
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
-@pytest.mark.parametrize("H,dv", [(3, 14), (1, 1), (5, 64), (32, 128), (7, 9)])
+@pytest.mark.parametrize("H,dv", [(3, 14), (1, 1), (5, 64), (32, 128), (7, 9), (72, 128), (27, 19)])
 def test_norm_over_all_heads_and_gate_alone(device, dtype, H, dv):
     torch.manual_seed(dv)
     T, eps, dt = 5, 1e-3, DT[dtype]
