@@ -61,6 +61,9 @@ int dxm_moe_router(int*, float*, float*, const void*, int64_t, const float*, int
 int dxm_moe_plan(int*, int*, const int*, int, int, hipStream_t);
 int dxm_grouped_gemm(void*, const void*, int64_t, const void*, const int*, const int*, int, int, int, int, int, int,
                      int, int, hipStream_t);
+int dxm_stream_grouped_ok(int, int);
+int dxm_stream_grouped_gemm(void*, const void*, int64_t, const void*, const int*, const int*, int, int, int, int, int,
+                            int, int, int, hipStream_t);
 int dxm_moe_combine(void*, const void*, const float*, const void*, int64_t, int, int, int, int, hipStream_t);
 int dxm_diff_combine(void*, const float*, int64_t, int, float, float, float, const void*, int64_t, int, int,
                      hipStream_t);
@@ -227,6 +230,13 @@ PYBIND11_MODULE(_C_mixers, m) {
     check(dxm_grouped_gemm(P(out), P(a), as, P(w), reinterpret_cast<const int*>(order),
                            reinterpret_cast<const int*>(offsets), R, E, N, K, top, gather, scatter, f32, S(st)),
           "grouped_gemm");
+  });
+  m.def("stream_grouped_ok", &dxm_stream_grouped_ok);
+  m.def("stream_grouped_gemm", [](u out, u a, int64_t as, u w, u order, u offsets, int R, int E, int N, int K, int top,
+                                  int gather, int scatter, int glu, u st) {
+    check(dxm_stream_grouped_gemm(P(out), P(a), as, P(w), reinterpret_cast<const int*>(order),
+                                  reinterpret_cast<const int*>(offsets), R, E, N, K, top, gather, scatter, glu, S(st)),
+          "stream_grouped_gemm");
   });
   m.def("moe_combine", [](u out, u y, u w, u shared, int64_t ss, int T, int top, int W, int f32, u st) {
     check(dxm_moe_combine(P(out), P(y), F(w), P(shared), ss, T, top, W, f32, S(st)), "moe_combine");

@@ -21,6 +21,10 @@ from .mixers import _f32, _fp32_param, _ptr, _stream
 
 ROUTER_SCORES = {"sigmoid": 0, "softmax": 1}
 GROUP_SCORES = {"top2": 0, "max": 1}
+# weight-streaming grouped GEMM: up to this many rows per expert on average, and where the 256-tile kernel's
+# grid (one workgroup per expert and 256 columns) would leave a good part of the chip idle
+STREAM_ROWS = 24
+STREAM_TILES = 192
 GLU_BLOCK = 32  # rows per gate / up block of weights interleaved for the fused SwiGLU epilogue
 
 
@@ -125,12 +129,23 @@ def plan(idx: torch.Tensor, n_experts: int) -> tuple[torch.Tensor, torch.Tensor]
 
 def tile_gemm_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
     """Whether the 256 x 256-tile matrix-core GEMM (csrc/kernels/gemm256.hip, grouped
-    mode) takes a [rows, K] against w [E, N, K]; the 64 x 64-tile kernel of
-    csrc/mixers/moe.hip takes everything else."""
+    mode) takes a [rows, K] against w [E, N, K] (few rows: stream_gemm_ok); the
+    64 x 64-tile kernel of csrc/mixers/moe.hip takes everything else."""
     E, N, K = w.shape
     return (a.is_cuda and a.dtype == torch.bfloat16 and N % 256 == 0 and K % 128 == 0 and a.stride(0) % 8 == 0
             and a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and N * K < 2 ** 31
             and a.shape[0] * a.stride(0) < 2 ** 31)
+
+
+def stream_gemm_ok(a: torch.Tensor, w: torch.Tensor, R: int) -> bool:
+    """Whether the weight-streaming kernel (csrc/mixers/grouped_stream.hip) takes
+    R rows against w [E, N, K]: few rows per expert, whole pieces, and too few
+    256-column tiles for the tile kernel to fill the chip."""
+    E, N, K = w.shape
+    if tile_gemm_ok(a, w) and E * (N // 256) >= STREAM_TILES:
+        return False
+    return (a.is_cuda and a.dtype == torch.bfloat16 and R <= STREAM_ROWS * E and a.stride(0) % 8 == 0 and
+            a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and bool(_m().stream_grouped_ok(N, K)))
 
 
 def interleave_glu(w: torch.Tensor) -> torch.Tensor:
@@ -177,6 +192,10 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, order: torch.Tensor, offsets:
     if glu and not tile_gemm_ok(a, w):
         raise ValueError("grouped_gemm: the fused SwiGLU epilogue needs tile_gemm_ok operands")
     out = torch.empty((R, N // 2 if glu else N), dtype=a.dtype, device=a.device)
+    if stream_gemm_ok(a, w, R):
+        _m().stream_grouped_gemm(out.data_ptr(), a.data_ptr(), a.stride(0), w.data_ptr(), order.data_ptr(),
+                                 offsets.data_ptr(), R, E, N, K, top, int(gather), int(scatter), int(glu), _stream())
+        return out
     if tile_gemm_ok(a, w):
         _native.kernels().gemm256_grouped(out.data_ptr(), out.stride(0), a.data_ptr(), a.stride(0), a.shape[0],
                                           w.data_ptr(), order.data_ptr(), offsets.data_ptr(), R, E, N, K, top,

@@ -315,6 +315,41 @@ def test_routed_experts_alone(device, dtype, T, E, top, identity, W, ff, shared)
         assert torch.allclose(got.cpu().double(), ws, **tol(dtype, 1e-4, 4e-2))
 
 
+@pytest.mark.gpu
+@pytest.mark.parametrize("counts,K,N", [((0, 1, 16, 17, 5), 64, 32), ((3, 0, 2), 320, 96), ((40, 65, 2, 0, 31), 128, 192),
+                                        ((130, 1, 64, 33, 12, 90), 704, 64), ((7,), 4096, 256)])
+def test_few_rows_per_expert_stream_the_weights(monkeypatch, counts, K, N):
+    """The weight-streaming grouped GEMM (bf16, few rows per expert): experts without rows, with one, and with more
+    than one pass holds; widths that leave some of the waves without a piece; gathered rows in, scattered rows
+    out; the SwiGLU epilogue; choices without an expert among the slots."""
+    torch.manual_seed(K)
+    monkeypatch.setattr(moe, "STREAM_ROWS", 1 << 20)
+    monkeypatch.setattr(moe, "STREAM_TILES", 1 << 20)
+    E, top = len(counts), 2
+    flat = torch.cat([torch.full((c,), e) for e, c in enumerate(counts)] + [torch.full((4 + sum(counts) % 2,), E)])
+    idx = flat[torch.randperm(flat.numel())].view(-1, top).to(torch.int32)
+    T = idx.shape[0]
+    order, offsets = moe.plan(idx.cuda(), E)
+    n, o = int(offsets[-1]), order.cpu().long()
+    assert n == sum(counts) and offsets.cpu().tolist() == [0] + torch.tensor(counts).cumsum(0).tolist()
+    e_of = idx.reshape(-1).long()[o[:n]]
+    a, w = torch.randn(T, K).bfloat16(), (torch.randn(E, N, K) * K ** -0.5).bfloat16()
+    ac, wc = a.cuda(), w.cuda()
+    assert moe.stream_gemm_ok(ac, wc, T * top)
+    want = torch.stack([w[e].double() @ a[s // top].double() for e, s in zip(e_of.tolist(), o[:n].tolist())])
+    got = moe.grouped_gemm(ac, wc, order, offsets, top, gather=True, scatter=False)[:n].cpu().double()
+    assert float((got - want).abs().max()) < 3e-2
+    b = torch.randn(T * top, K + 8).bfloat16()[:, :K]
+    want = torch.stack([w[e].double() @ b[r].double() for r, e in enumerate(e_of.tolist())])
+    got = moe.grouped_gemm(b.cuda(), wc, order, offsets, top, gather=False, scatter=True).cpu().double()
+    assert float((got[o[:n]] - want).abs().max()) < 3e-2
+    if N % 256 == 0 and K % 128 == 0:
+        want = torch.stack([w[e].double() @ a[s // top].double() for e, s in zip(e_of.tolist(), o[:n].tolist())])
+        got = moe.grouped_gemm(ac, moe.interleave_glu(wc), order, offsets, top, gather=True, scatter=False, glu=True)
+        want = O.silu(want[:, :N // 2]) * want[:, N // 2:]
+        assert float((got[:n].cpu().double() - want).abs().max()) < 3e-2
+
+
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("F,dv", [(24, 8), (21, 7), (1028, 4), (30, 10)])
 def test_gated_units_alone(device, dtype, F, dv):
