@@ -84,6 +84,11 @@ int dxm_stream_prefill(void*, const void*, int64_t, const void*, const void*, co
 int dxm_stream_decode_ok(int, int, int, int, int);
 int dxm_stream_decode(float*, const void*, int64_t, const void*, const void*, const int64_t*, const int*, const int*, int,
                       int, int, int, int, int, int, int, int, int, float, int, int, int, hipStream_t);
+int dxm_latent_attention_ok(int, int, int, int, int, int, int);
+int dxm_latent_prefill(void*, const void*, int64_t, const void*, int, const int64_t*, const int*, const int*, int, int,
+                       const int*, int, int, int, int, float, int, int, const float*, hipStream_t);
+int dxm_latent_decode(float*, const void*, int64_t, const void*, int, const int64_t*, const int*, const int*, int, int, int,
+                      int, int, int, float, int, int, int, hipStream_t);
 int dxm_merge_parts(void*, const float*, int64_t, int, int, int, const void*, int64_t, int, int, const float*, int,
                     hipStream_t);
 }
@@ -266,6 +271,13 @@ PYBIND11_MODULE(_C_mixers, m) {
                                reinterpret_cast<const int*>(tiles), n_tiles, n_qh, group, d, dv, Wk, Wv, scale, mask, size,
                                fine, S(st)),
             "stream_prefill");
+    // one row that is key and value of all heads: the latent kernel
+    else if (cap == 0.f && !r1 && !wfn && !hbias && !gate && !keep && !out_f32 && !fine && kc == vc && Wk == Wv &&
+             qs % 8 == 0 && Wk % 8 == 0 && (q | kc) % 16 == 0 && dxm_latent_attention_ok(d, dv, n_qh, maps, group, bs, 1))
+      check(dxm_latent_prefill(P(out), P(q), qs, P(kc), Wk, reinterpret_cast<const int64_t*>(pos),
+                               reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs,
+                               reinterpret_cast<const int*>(tiles), n_tiles, n_qh, d, dv, scale, mask, size, F(sink), S(st)),
+            "latent_prefill");
     else
       check(dxm_tile_attention(P(out), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
                              reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs,
@@ -284,6 +296,12 @@ PYBIND11_MODULE(_C_mixers, m) {
                               reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs, rows, n_qh,
                               maps, group, d, dv, Wk, Wv, scale, mask, size, parts, S(st)),
             "stream_decode");
+    else if (cap == 0.f && !r1 && !wfn && !hbias && !keep && kc == vc && Wk == Wv && qs % 8 == 0 && Wk % 8 == 0 &&
+             (q | kc) % 16 == 0 && dxm_latent_attention_ok(d, dv, n_qh, maps, group, bs, 0))
+      check(dxm_latent_decode(F(ws), P(q), qs, P(kc), Wk, reinterpret_cast<const int64_t*>(pos),
+                              reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs, rows, n_qh, d, dv,
+                              scale, mask, size, parts, S(st)),
+            "latent_decode");
     else
       check(dxm_group_decode(F(ws), P(q), qs, P(kc), P(vc), reinterpret_cast<const int64_t*>(pos),
                            reinterpret_cast<const int*>(seq), reinterpret_cast<const int*>(bt), bts, bs, rows, n_qh,
