@@ -727,7 +727,8 @@ def kilatar_kernels(s: dict, L: int, B: int, T: int) -> dict:
                                              False, tiles, L, **sink))
             put(f"{name}_prefill_{mask}{size or ''}", us, None, 2.0 * (dd + dv) * H * float(n_vis.sum()))
             vis = int(n_vis[-1])
-            parts = mx.row_attention_parts(B, n_kh * -(-(H // n_kh) // 32), vis, mx.GROUP_TARGET_WAVES)
+            parts = mx.row_attention_parts(B, n_kh * -(-(H // n_kh) // 32), vis,
+                                           mx.LATENT_TARGET_GROUPS if name == "latent" else mx.GROUP_TARGET_WAVES)
             us = _timed(lambda: mx.attention(qd, kcd, vcd, posd, None, btd, bs, H, 1, H // n_kh, dd, dv, dd ** -0.5, mask, size,
                                              parts, **sink))
             put(f"{name}_decode_{mask}{size or ''}", us, B * vis * n_kh * dd * (2 if name == "latent" else 4), parts=parts)

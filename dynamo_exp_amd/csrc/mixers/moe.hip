@@ -132,18 +132,18 @@ __global__ void __launch_bounds__(64 * kRouteWaves) moe_route_kernel(int* __rest
   route_token(g, z + tc * g.E, c, c + g.E, on, idx + tc * g.top, w + tc * g.top, lane);
 }
 
-// The same result for few tokens: a workgroup per token, its row in registers as far as it fits; 4 waves share
-// the width, outputs are summed 8 at a time.  V elements per access.
-template <typename T, int V>
-__global__ void __launch_bounds__(256) moe_router_rows_kernel(int* __restrict__ idx, float* __restrict__ wgt,
-                                                              float* __restrict__ gates, const T* __restrict__ h,
-                                                              int64_t hs, const float* __restrict__ w, int n_out, int W,
-                                                              RouteArgs g) {
-  constexpr int kKeep = 4;
+// The same result for few tokens: a workgroup per token whose waves share the width, kOut outputs at a time --
+// wide rows get many waves, so that a thread has one piece of the row and all its loads are in flight together.
+template <typename T, int V, int NW>
+__global__ void __launch_bounds__(64 * NW) moe_router_rows_kernel(int* __restrict__ idx, float* __restrict__ wgt,
+                                                                  float* __restrict__ gates, const T* __restrict__ h,
+                                                                  int64_t hs, const float* __restrict__ w, int n_out, int W,
+                                                                  RouteArgs g) {
+  constexpr int kOut = 12;
   extern __shared__ float rsm[];
-  float* part = rsm;             // [4 waves][n_out]
-  float* z = part + 4 * n_out;   // [n_out]
-  float* scratch = z + n_out;    // [4][E + n_groups]
+  float* part = rsm;              // [NW waves][n_out]
+  float* z = part + NW * n_out;   // [n_out]
+  float* scratch = z + n_out;     // [NW][E + n_groups]
   const int tid = threadIdx.x, lane = tid & 63, wv = tid >> 6;
   const int64_t t = blockIdx.x;
   const T* hp = h + t * hs;
@@ -158,52 +158,44 @@ __global__ void __launch_bounds__(256) moe_router_rows_kernel(int* __restrict__ 
       x[0] = q[0], x[1] = q[1], x[2] = q[2], x[3] = q[3];
     }
   };
-  float x[kKeep][V];
+  for (int o0 = 0; o0 < n_out; o0 += kOut) {
+    float acc[kOut];
 #pragma unroll
-  for (int k = 0; k < kKeep; ++k) {
-    const int e = (tid + 256 * k) * V;
+    for (int j = 0; j < kOut; ++j) acc[j] = 0.f;
+    for (int e = tid * V; e < W; e += 64 * NW * V) {
+      float x[V];
+      load_h(e, x);
+      float q[kOut][V];
 #pragma unroll
-    for (int i = 0; i < V; ++i) x[k][i] = 0.f;
-    if (e < W) load_h(e, x[k]);
-  }
-  for (int o0 = 0; o0 < n_out; o0 += 8) {
-    float acc[8];
-#pragma unroll
-    for (int j = 0; j < 8; ++j) acc[j] = 0.f;
-    auto dot = [&](int e, const float* xv) {
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        if (o0 + j >= n_out) break;
-        const float* wp = w + (int64_t)(o0 + j) * W + e;
+      for (int j = 0; j < kOut; ++j) {
+        const float* wp = w + (int64_t)min(o0 + j, n_out - 1) * W + e;  // (past the last: not used)
         if constexpr (V == 1) {
-          acc[j] += xv[0] * wp[0];
+          q[j][0] = wp[0];
         } else {
-          const f32x4 q = *reinterpret_cast<const f32x4*>(wp);
-#pragma unroll
-          for (int i = 0; i < V; ++i) acc[j] += xv[i] * q[i];
+          const f32x4 u = *reinterpret_cast<const f32x4*>(wp);
+          q[j][0] = u[0], q[j][1] = u[1], q[j][2] = u[2], q[j][3] = u[3];
         }
       }
-    };
 #pragma unroll
-    for (int k = 0; k < kKeep; ++k) {
-      const int e = (tid + 256 * k) * V;
-      if (e < W) dot(e, x[k]);
-    }
-    for (int e = (tid + 256 * kKeep) * V; e < W; e += 256 * V) {
-      float t4[V];
-      load_h(e, t4);
-      dot(e, t4);
+      for (int j = 0; j < kOut; ++j)
+#pragma unroll
+        for (int i = 0; i < V; ++i) acc[j] += x[i] * q[j][i];
     }
 #pragma unroll
-    for (int j = 0; j < 8; ++j) {
+    for (int j = 0; j < kOut; ++j) {
       const float s = wave_reduce_sum(acc[j]);
       if (lane == 0 && o0 + j < n_out) part[wv * n_out + o0 + j] = s;
     }
   }
   __syncthreads();
-  for (int o = tid; o < n_out; o += 256) z[o] = part[o] + part[n_out + o] + part[2 * n_out + o] + part[3 * n_out + o];
+  for (int o = tid; o < n_out; o += 64 * NW) {
+    float s = 0.f;
+#pragma unroll
+    for (int k = 0; k < NW; ++k) s += part[k * n_out + o];
+    z[o] = s;
+  }
   __syncthreads();
-  for (int j = tid; j < n_out - g.E; j += 256) gates[t * (n_out - g.E) + j] = 1.f / (1.f + expf(-z[g.E + j]));
+  for (int j = tid; j < n_out - g.E; j += 64 * NW) gates[t * (n_out - g.E) + j] = 1.f / (1.f + expf(-z[g.E + j]));
   // (every wave takes part in the choice's barriers; wave 0 writes it)
   float* c = scratch + wv * (g.E + g.n_groups);
   route_token(g, z, c, c + g.E, wv == 0, idx + t * g.top, wgt + t * g.top, lane);
@@ -573,15 +565,18 @@ int dxm_moe_router(int* idx, float* w, float* gates, const void* h, int64_t h_st
   if (!idx || !w || !h || !rw || (n_out > E && !gates)) return 5;
   const int esz = f32 ? 4 : 2;
   if (T <= 256) {
-    const size_t lds = (5 * (size_t)n_out + 4 * (size_t)(E + n_groups)) * sizeof(float);
     const bool vec = W % 4 == 0 && h_stride % 4 == 0 && (uintptr_t)h % (4 * esz) == 0 && (uintptr_t)rw % 16 == 0;
-#define ROUTER_ROWS(TY, V)                                                                                            \
-  hipLaunchKernelGGL((moe_router_rows_kernel<TY, V>), dim3(T), dim3(256), lds, st, idx, w, gates, (const TY*)h, h_stride, \
-                     rw, n_out, W, g);
-    if (f32 && vec) { ROUTER_ROWS(float, 4) }
-    else if (f32) { ROUTER_ROWS(float, 1) }
-    else if (vec) { ROUTER_ROWS(bf16_t, 4) }
-    else { ROUTER_ROWS(bf16_t, 1) }
+    auto lds = [&](int nw) { return ((nw + 1) * (size_t)n_out + nw * (size_t)(E + n_groups)) * sizeof(float); };
+    const bool wide = vec && W >= 2048 && lds(16) <= 60 * 1024;
+#define ROUTER_ROWS(TY, V, NW)                                                                                        \
+  hipLaunchKernelGGL((moe_router_rows_kernel<TY, V, NW>), dim3(T), dim3(64 * NW), lds(NW), st, idx, w, gates,          \
+                     (const TY*)h, h_stride, rw, n_out, W, g);
+    if (f32 && wide) { ROUTER_ROWS(float, 4, 16) }
+    else if (f32 && vec) { ROUTER_ROWS(float, 4, 4) }
+    else if (f32) { ROUTER_ROWS(float, 1, 4) }
+    else if (wide) { ROUTER_ROWS(bf16_t, 4, 16) }
+    else if (vec) { ROUTER_ROWS(bf16_t, 4, 4) }
+    else { ROUTER_ROWS(bf16_t, 1, 4) }
 #undef ROUTER_ROWS
     DX_CHECK_LAUNCH();
     return 0;

@@ -262,8 +262,10 @@ __device__ __forceinline__ float sum_all(float v, float* red) {
   return red[0] + red[1] + red[2] + red[3];
 }
 
-// KC: chunks of a row in registers.  All loads of the row are issued before the first sum over the workgroup.
-template <typename T, int V, bool EXT, int KC>
+// KC: chunks of a row in registers.  F: which addends there are (bits below), or kAny: asked of the pointers.  With
+// known addends nothing stands between the loads of a row: all of them are issued before the first is used.
+constexpr int kHasA = 1, kHasB = 2, kHasC = 4, kHasD = 8, kHasBias = 16, kHasExperts = 32, kAny = -1;
+template <typename T, int V, bool EXT, int KC, int F>
 __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     float* __restrict__ X, const T* __restrict__ a, int64_t a_stride, const T* __restrict__ b, int64_t b_stride,
     const T* __restrict__ c, int64_t c_stride, const float* __restrict__ cw, const T* __restrict__ cg,
@@ -273,10 +275,14 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
   __shared__ float red[4][4];
   const int64_t row = EXT && g.rows ? g.rows[blockIdx.x] : (int64_t)blockIdx.x, orow = blockIdx.x;
   float* x = X + row * (int64_t)W;
+  const bool has_a = F == kAny ? a != nullptr : F & kHasA, has_b = F == kAny ? b != nullptr : F & kHasB,
+             has_c = F == kAny ? c != nullptr : F & kHasC, has_d = EXT && (F == kAny ? g.d != nullptr : F & kHasD),
+             has_bias = EXT && (F == kAny ? g.bias != nullptr : F & kHasBias),
+             has_my = EXT && (F == kAny ? g.my != nullptr : F & kHasExperts), has_e = EXT && F == kAny && g.e;
   // the addend c at columns e .. e + V - 1, gated by sigmoid(cg + cgb) when a gate is given
   auto load_c = [&](int e, float* v) {
     ldv<T, V>(c + row * c_stride + e, v);
-    if (cg) {
+    if (F == kAny && cg) {
       float gt[V], gb[V];
       ldv<T, V>(cg + row * cg_stride + e, gt);
       if (cgb) ldv<float, V>(cgb + e, gb);
@@ -285,59 +291,119 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     }
   };
   auto load_d = [&](int e, float* v) { ldv<T, V>(g.d + row * g.d_stride + e, v); };
+  // the experts' weighted sum, two choices at a time
+  auto load_experts = [&](int e, float* m) {
+#pragma unroll
+    for (int i = 0; i < V; ++i) m[i] = 0.f;
+    for (int k = 0; k < g.top; k += 2) {
+      const int64_t s0 = row * g.top + k, s1 = k + 1 < g.top ? s0 + 1 : s0;
+      const float w0 = g.mw[s0], w1 = k + 1 < g.top ? g.mw[s1] : 0.f;
+      const T* ident = g.mh + row * g.mh_stride;
+      float t0[V], t1[V];
+      ldv<T, V>((g.midx && g.midx[s0] >= g.experts ? ident : g.my + s0 * (int64_t)W) + e, t0);
+      ldv<T, V>((g.midx && g.midx[s1] >= g.experts ? ident : g.my + s1 * (int64_t)W) + e, t1);
+#pragma unroll
+      for (int i = 0; i < V; ++i) m[i] += w0 * t0[i];
+      if (k + 1 < g.top) {
+#pragma unroll
+        for (int i = 0; i < V; ++i) m[i] += w1 * t1[i];
+      }
+    }
+  };
   // x and everything added to it as it is
   auto load_x = [&](int e, float* v) {
     float t[V];
     ldv<float, V>(x + e, v);
-    if (a) {
+    if (has_a) {
       ldv<T, V>(a + row * a_stride + e, t);
 #pragma unroll
       for (int i = 0; i < V; ++i) v[i] += t[i];
     }
-    if (b) {
+    if (has_b) {
       ldv<T, V>(b + row * b_stride + e, t);
 #pragma unroll
       for (int i = 0; i < V; ++i) v[i] += t[i];
     }
     if constexpr (EXT) {
-      if (g.bias) {
+      if (has_bias) {
         ldv<float, V>(g.bias + e, t);
 #pragma unroll
         for (int i = 0; i < V; ++i) v[i] += t[i];
       }
-      if (g.my) {
-        float m[V];
+      if (has_my) {
+        load_experts(e, t);
 #pragma unroll
-        for (int i = 0; i < V; ++i) m[i] = 0.f;
-        for (int k = 0; k < g.top; ++k) {
-          const int64_t s = row * g.top + k;
-          const float wk = g.mw[s];
-          ldv<T, V>((g.midx && g.midx[s] >= g.experts ? g.mh + row * g.mh_stride : g.my + s * (int64_t)W) + e, t);
-#pragma unroll
-          for (int i = 0; i < V; ++i) m[i] += wk * t[i];
-        }
-#pragma unroll
-        for (int i = 0; i < V; ++i) v[i] += m[i];
+        for (int i = 0; i < V; ++i) v[i] += t[i];
       }
-      if (g.e) {
+      if (has_e) {
         ldv<float, V>(g.e + row * (int64_t)W + e, t);
 #pragma unroll
         for (int i = 0; i < V; ++i) v[i] += t[i];
       }
     }
   };
-  const bool has_d = EXT && g.d;
   float r[KC][V], cv[KC][V], dv[EXT ? KC : 1][V], cs = 0.f, ds = 0.f;
+  if constexpr (F == kAny) {
 #pragma unroll
-  for (int k = 0; k < KC; ++k) {
-    const int e = (threadIdx.x + k * kThreads) * V;
-    if (e < W) {
-      if (c) load_c(e, cv[k]);
-      if constexpr (EXT) {
-        if (has_d) load_d(e, dv[k]);
+    for (int k = 0; k < KC; ++k) {
+      const int e = (threadIdx.x + k * kThreads) * V;
+      if (e < W) {
+        if (has_c) load_c(e, cv[k]);
+        if constexpr (EXT) {
+          if (has_d) load_d(e, dv[k]);
+        }
+        load_x(e, r[k]);
       }
-      load_x(e, r[k]);
     }
+  } else {  // columns past the row: the last ones again (nothing of them is used)
+    float y[(F & kHasExperts) ? KC : 1][V], av[(F & kHasA) ? KC : 1][V], bv[(F & kHasB) ? KC : 1][V],
+        cb[(F & kHasBias) ? KC : 1][V];
+#pragma unroll
+    for (int k = 0; k < KC; ++k) {
+      const int e = min((int)(threadIdx.x + k * kThreads) * V, W - V);
+      ldv<float, V>(x + e, r[k]);
+      if constexpr ((F & kHasC) != 0) load_c(e, cv[k]);
+      if constexpr ((F & kHasD) != 0) load_d(e, dv[k]);
+      if constexpr ((F & kHasA) != 0) ldv<T, V>(a + row * a_stride + e, av[k]);
+      if constexpr ((F & kHasB) != 0) ldv<T, V>(b + row * b_stride + e, bv[k]);
+      if constexpr ((F & kHasBias) != 0) ldv<float, V>(g.bias + e, cb[k]);
+    }
+    if constexpr ((F & kHasExperts) != 0) {
+#pragma unroll
+      for (int k = 0; k < KC; ++k)
+#pragma unroll
+        for (int i = 0; i < V; ++i) y[k][i] = 0.f;
+      for (int c0 = 0; c0 < g.top; c0 += 2) {  // two choices at a time over all chunks
+        const int64_t s0 = row * g.top + c0, s1 = c0 + 1 < g.top ? s0 + 1 : s0;
+        const float w0 = g.mw[s0], w1 = c0 + 1 < g.top ? g.mw[s1] : 0.f;
+        const T* ident = g.mh + row * g.mh_stride;
+        const bool i0 = g.midx && g.midx[s0] >= g.experts, i1 = g.midx && g.midx[s1] >= g.experts;
+        const T *p0 = i0 ? ident : g.my + s0 * (int64_t)W, *p1 = i1 ? ident : g.my + s1 * (int64_t)W;
+        float t0[KC][V], t1[KC][V];
+#pragma unroll
+        for (int k = 0; k < KC; ++k) {
+          const int e = min((int)(threadIdx.x + k * kThreads) * V, W - V);
+          ldv<T, V>(p0 + e, t0[k]);
+          ldv<T, V>(p1 + e, t1[k]);
+        }
+#pragma unroll
+        for (int k = 0; k < KC; ++k)
+#pragma unroll
+          for (int i = 0; i < V; ++i) {
+            y[k][i] += w0 * t0[k][i];
+            if (c0 + 1 < g.top) y[k][i] += w1 * t1[k][i];
+          }
+      }
+    }
+#pragma unroll
+    for (int k = 0; k < KC; ++k)
+#pragma unroll
+      for (int i = 0; i < V; ++i) {
+        if constexpr ((F & kHasA) != 0) r[k][i] += av[k][i];
+        if constexpr ((F & kHasB) != 0) r[k][i] += bv[k][i];
+        if constexpr ((F & kHasBias) != 0) r[k][i] += cb[k][i];
+        if constexpr ((F & kHasExperts) != 0) r[k][i] += y[k][i];
+      }
   }
 #pragma unroll
   for (int k = 0; k < KC; ++k) {
@@ -345,7 +411,7 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     if (e < W) {
 #pragma unroll
       for (int i = 0; i < V; ++i) {
-        if (c) cs += cv[k][i] * cv[k][i];
+        if (has_c) cs += cv[k][i] * cv[k][i];
         if constexpr (EXT) {
           if (has_d) ds += dv[k][i] * dv[k][i];
         }
@@ -355,7 +421,7 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
   const int tail = (threadIdx.x + KC * kThreads) * V;  // wide rows: columns from here on are read when they are needed
   for (int e = tail; e < W; e += kThreads * V) {
     float v[V];
-    if (c) {
+    if (has_c) {
       load_c(e, v);
 #pragma unroll
       for (int i = 0; i < V; ++i) cs += v[i] * v[i];
@@ -371,13 +437,13 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
     ds = wave_reduce_sum(ds);
     if ((threadIdx.x & 63) == 0) red[1][threadIdx.x >> 6] = ds;
   }
-  if (c) rc = rsqrtf(sum_all(cs, red[0]) / (float)W + eps);
+  if (has_c) rc = rsqrtf(sum_all(cs, red[0]) / (float)W + eps);
   else if (has_d) __syncthreads();
   if (has_d) rd = rsqrtf((red[1][0] + red[1][1] + red[1][2] + red[1][3]) / (float)W + eps);
   // the normed addends at columns e .. e + V - 1; ct, dt: the values of c and d there
   auto add = [&](int e, float* v, const float* ct, const float* dt) {
     float w[V];
-    if (c) {
+    if (has_c) {
       ldv<float, V>(cw + e, w);
 #pragma unroll
       for (int i = 0; i < V; ++i) v[i] += ct[i] * rc * w[i];
@@ -392,12 +458,12 @@ __global__ void __launch_bounds__(kThreads) residual_step_kernel(
   auto wide = [&](int e, float* v) {
     float ct[V], dt[V];
     load_x(e, v);
-    if (c) load_c(e, ct);
+    if (has_c) load_c(e, ct);
     if (has_d) load_d(e, dt);
     add(e, v, ct, dt);
   };
-  bool touch = a || b || c;
-  if constexpr (EXT) touch = !g.rows && (touch || g.d || g.e || g.bias || g.my);
+  bool touch = has_a || has_b || has_c;
+  if constexpr (EXT) touch = !g.rows && (touch || has_d || has_e || has_bias || has_my);
   float sum = 0.f;
 #pragma unroll
   for (int k = 0; k < KC; ++k) {
@@ -814,19 +880,36 @@ int dxm_residual_step(float* X, const void* a, int64_t a_stride, const void* b, 
                    al(out, 4 * esz) && al(xc, 4 * esz) && al(d, 4 * esz) && al(dw, 16) && al(e, 16) && al(bias, 16) &&
                    al(my, 4 * esz) && al(mh, 4 * esz);
   const bool ext = d || e || bias || my || pick;
-#define RES(V, EXT, KC)                                                                                                 \
-  DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, V, EXT, KC>), dim3(rows), dim3(kThreads), 0, st, X,           \
+#define RES(V, EXT, KC, F)                                                                                              \
+  DISPATCH_T(f32, hipLaunchKernelGGL((residual_step_kernel<T, V, EXT, KC, F>), dim3(rows), dim3(kThreads), 0, st, X,           \
                                      (const T*)a, a_stride, (const T*)b, b_stride, (const T*)c, c_stride, cw,           \
                                      (const T*)cg, cg_stride, cgb, eps, norm, nw, nb, (T*)out, (T*)xc, W,               \
                                      (ResExt<T>{(const T*)d, d_stride, dw, e, bias, (const T*)my, mw, midx, experts,    \
                                                 top, (const T*)mh, mh_stride, pick})))
   const bool narrow = W <= 4 * kThreads * 4;  // four chunks hold the row: fewer registers, more workgroups per CU
-  if (vec && ext && narrow) { RES(4, true, 4) }
-  else if (vec && ext) { RES(4, true, 8) }
-  else if (vec && narrow) { RES(4, false, 4) }
-  else if (vec) { RES(4, false, 8) }
-  else if (ext) { RES(1, true, 8) }
-  else { RES(1, false, 8) }
+  // the steps of parallel layers with known addends (a re-entering addend or a list of rows: any)
+  const int f = e || pick || cg || W < 4 * kThreads ? kAny
+                : (a ? kHasA : 0) | (b ? kHasB : 0) | (c ? kHasC : 0) | (d ? kHasD : 0) | (bias ? kHasBias : 0) |
+                      (my ? kHasExperts : 0);
+#define RES_KNOWN(F) \
+  if (f == (F)) {    \
+    if (narrow) { RES(4, true, 4, F) } else { RES(4, true, 8, F) } \
+    DX_CHECK_LAUNCH(); \
+    return 0;        \
+  }
+  if (vec && ext) {
+    RES_KNOWN(kHasB | kHasC | kHasD | kHasExperts)
+    RES_KNOWN(kHasA | kHasExperts)
+    RES_KNOWN(kHasB | kHasC | kHasD | kHasBias)
+    RES_KNOWN(kHasA | kHasBias)
+  }
+#undef RES_KNOWN
+  if (vec && ext && narrow) { RES(4, true, 4, kAny) }
+  else if (vec && ext) { RES(4, true, 8, kAny) }
+  else if (vec && narrow) { RES(4, false, 4, kAny) }
+  else if (vec) { RES(4, false, 8, kAny) }
+  else if (ext) { RES(1, true, 8, kAny) }
+  else { RES(1, false, 8, kAny) }
 #undef RES
   DX_CHECK_LAUNCH();
   return 0;

@@ -288,7 +288,7 @@ class KilatarForCausalLM(StatefulLayeredModel):
                             meta.positions, meta.slot_mapping, cache, interleaved=True)
         tl = (meta.row_tiles, meta.num_prefill_tokens) if meta.is_prefill else (None, 0)
         a = mx.attention(ql, cache, cache, meta.positions, seq, tables, meta.block_size, H, 1, H, r + dr, r, m["scale"],
-                         "causal", 0, self._parts(T, H, H, 0, meta, 16 if 2 * r + dr > 256 else 32), False, *tl)
+                         "causal", 0, self._parts(T, H, H, 0, meta, latent=True), False, *tl)
         up = torch.bmm(a.view(T, H, r).transpose(0, 1), L["uv"])  # [H, T, dv]
         g0 = nq + r + dr
         mx.act_mul(p[:, g0:g0 + H * dv], up, "sigmoid", out=o)

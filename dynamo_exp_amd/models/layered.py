@@ -155,11 +155,11 @@ class StatefulLayeredModel:
         return self.load_state(tensors)
 
     # ------------------------------------------------------------------ forward
-    def _parts(self, rows: int, n_qh: int, group: int, visible: int, meta: AttnMeta, per_wave: int = 32) -> int:
+    def _parts(self, rows: int, n_qh: int, group: int, visible: int, meta: AttnMeta, latent: bool = False) -> int:
         """Key partitions of the step's decode rows (rows that are no prompt-chunk
         tiles): n_qh query heads, `group` per key/value head; visible: the most
-        keys a row sees (0: its whole context); per_wave: query heads of a group
-        that one wave of the decode kernel takes."""
+        keys a row sees (0: its whole context); latent: one shared row that is key
+        and value (a workgroup per 32 heads instead of a wave)."""
         from ..ops import mixers as mx
 
         vis = meta.max_ctx if meta.max_ctx else self.cfg.max_position_embeddings
@@ -168,8 +168,9 @@ class StatefulLayeredModel:
         grouped = self.dtype == torch.bfloat16 and self.device.type == "cuda"
         if meta.is_prefill and grouped:
             rows -= meta.num_prefill_tokens
-        units = n_qh if not grouped else max(1, n_qh // group) * (-(-group // per_wave))
-        return mx.row_attention_parts(max(rows, 1), units, vis, mx.GROUP_TARGET_WAVES if grouped else mx.ROW_TARGET_WAVES)
+        units = n_qh if not grouped else max(1, n_qh // group) * (-(-group // 32))
+        target = mx.ROW_TARGET_WAVES if not grouped else mx.LATENT_TARGET_GROUPS if latent else mx.GROUP_TARGET_WAVES
+        return mx.row_attention_parts(max(rows, 1), units, vis, target)
 
     def compute_logits(self, hidden: torch.Tensor, fp32: bool = False) -> torch.Tensor:
         """Logits of final-normed rows; fp32: the products of the bf16 operands

@@ -35,6 +35,8 @@ ROW_MIN_PART = 128
 # grouped decode kernel: one wave per workgroup, four workgroups resident per CU (LDS), so
 # about 1024 waves fill the chip once; more parts only add merge work
 GROUP_TARGET_WAVES = 1024
+# latent decode kernel: two workgroups of four waves per CU (LDS)
+LATENT_TARGET_GROUPS = 512
 
 
 def _m():

@@ -21,8 +21,8 @@ from .mixers import _f32, _fp32_param, _ptr, _stream
 
 ROUTER_SCORES = {"sigmoid": 0, "softmax": 1}
 GROUP_SCORES = {"top2": 0, "max": 1}
-# weight-streaming grouped GEMM: up to this many rows per expert on average, and where the 256-tile kernel's
-# grid (one workgroup per expert and 256 columns) would leave a good part of the chip idle
+# weight-streaming grouped GEMM: up to this many rows per expert on average where the 256-tile kernel's grid (one
+# workgroup per expert and 256 columns) would leave a good part of the chip idle, half as many elsewhere
 STREAM_ROWS = 24
 STREAM_TILES = 192
 GLU_BLOCK = 32  # rows per gate / up block of weights interleaved for the fused SwiGLU epilogue
@@ -139,12 +139,10 @@ def tile_gemm_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
 
 def stream_gemm_ok(a: torch.Tensor, w: torch.Tensor, R: int) -> bool:
     """Whether the weight-streaming kernel (csrc/mixers/grouped_stream.hip) takes
-    R rows against w [E, N, K]: few rows per expert, whole pieces, and too few
-    256-column tiles for the tile kernel to fill the chip."""
+    R rows against w [E, N, K]: few rows per expert, whole pieces."""
     E, N, K = w.shape
-    if tile_gemm_ok(a, w) and E * (N // 256) >= STREAM_TILES:
-        return False
-    return (a.is_cuda and a.dtype == torch.bfloat16 and R <= STREAM_ROWS * E and a.stride(0) % 8 == 0 and
+    most = STREAM_ROWS if not tile_gemm_ok(a, w) or E * (N // 256) < STREAM_TILES else STREAM_ROWS // 2
+    return (a.is_cuda and a.dtype == torch.bfloat16 and R <= most * E and a.stride(0) % 8 == 0 and
             a.data_ptr() % 16 == 0 and w.data_ptr() % 16 == 0 and bool(_m().stream_grouped_ok(N, K)))
 
 

@@ -230,7 +230,7 @@ def test_residual_step_addends_alone(device, dtype, W):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("W,E,top,identity,gates", [(72, 5, 2, 2, 1), (33, 1, 1, 0, 0), (21, 3, 4, 3, 1), (256, 30, 8, 2, 2),
-                                                    (130, 64, 6, 5, 1), (8, 700, 3, 1, 1)])
+                                                    (130, 64, 6, 5, 1), (8, 700, 3, 1, 1), (2056, 9, 2, 2, 1)])
 @pytest.mark.parametrize("T", [1, 17, 300, 1100])
 def test_router_alone(device, dtype, W, E, top, identity, gates, T):
     """Logits in fp32, softmax over all outputs, choice with the correction, weights without it, divided by their
