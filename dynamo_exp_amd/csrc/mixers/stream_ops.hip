@@ -652,7 +652,7 @@ __device__ __forceinline__ float act_fn(float z, int act) {
     return r * r;
   }
   // gelu, tanh form: 0.5 (1 + tanh u) = 1 / (1 + e^(-2 u)), u = sqrt(2 / pi) (z + 0.044715 z^3)
-  return z / (1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
+  return z * __builtin_amdgcn_rcpf(1.f + __expf(-1.5957691216057308f * (z + 0.044715f * z * z * z)));
 }
 
 // out [rows, F] = act(gate + gate_b) * (up + up_b) * row_scale[row] * post  (up null: act(gate) alone); gate and
