@@ -658,7 +658,8 @@ __device__ __forceinline__ float act_fn(float z, int act) {
 // out [rows, F] = act(gate + gate_b) * (up + up_b) * row_scale[row] * post  (up null: act(gate) alone); gate and
 // up are column sections of wider rows (a gated feed-forward's [gate | up], an output gate that is part of a
 // fused projection).  u_dv > 0: up is head-major, column c of row r at up[(c / u_dv) * u_head + r * u_stride + c % u_dv].
-template <typename T, int V>
+// ROWS: rows per workgroup (with biases, so that they are read once for several rows).
+template <typename T, int V, int ROWS>
 __global__ void __launch_bounds__(kThreads) act_mul_kernel(T* __restrict__ out, const T* __restrict__ gate,
                                                            int64_t g_stride, const T* __restrict__ up,
                                                            int64_t u_stride, int F, int64_t out_stride, int act,
@@ -666,34 +667,32 @@ __global__ void __launch_bounds__(kThreads) act_mul_kernel(T* __restrict__ out, 
                                                            const float* __restrict__ gate_b,
                                                            const float* __restrict__ up_b,
                                                            const float* __restrict__ row_scale, int u_dv,
-                                                           int64_t u_head) {
-  const int64_t r = blockIdx.y;
-  if (row_scale) post *= row_scale[r];
+                                                           int64_t u_head, int rows) {
+  const int r0 = blockIdx.y * ROWS, n = ROWS == 1 ? 1 : min(ROWS, rows - r0);
   for (int c = (blockIdx.x * kThreads + threadIdx.x) * V; c < F; c += gridDim.x * kThreads * V) {
-    float g[V], u[V], o[V], t[V];
-    ldv<T, V>(gate + r * g_stride + c, g);
-    if (up) ldv<T, V>(up + r * u_stride + (u_dv ? c / u_dv * u_head + c % u_dv : (int64_t)c), u);
-    if (gate_b) {
-      ldv<float, V>(gate_b + c, t);
+    float gb[V], ub[V];  // biases serve all rows of the workgroup
+    if (gate_b) ldv<float, V>(gate_b + c, gb);
+    if (up_b) ldv<float, V>(up_b + c, ub);
+    for (int i = 0; i < n; ++i) {
+      const int64_t r = r0 + i;
+      float g[V], u[V], o[V];
+      ldv<T, V>(gate + r * g_stride + c, g);
+      if (up) ldv<T, V>(up + r * u_stride + (u_dv ? c / u_dv * u_head + c % u_dv : (int64_t)c), u);
+      const float scale = row_scale ? post * row_scale[r] : post;
 #pragma unroll
-      for (int e = 0; e < V; ++e) g[e] += t[e];
-    }
-    if (up && up_b) {
-      ldv<float, V>(up_b + c, t);
-#pragma unroll
-      for (int e = 0; e < V; ++e) u[e] += t[e];
-    }
-#pragma unroll
-    for (int e = 0; e < V; ++e) {
-      if (act == 6) {  // clamped gated unit: g sigmoid(alpha g) (u + 1), g <= limit, |u| <= limit
-        const float gc = fminf(g[e], limit), uc = fminf(fmaxf(u[e], -limit), limit);
-        o[e] = gc / (1.f + __expf(-alpha * gc)) * (uc + 1.f);
-      } else {
-        o[e] = act_fn(g[e], act) * (up ? u[e] : 1.f);
+      for (int e = 0; e < V; ++e) {
+        if (gate_b) g[e] += gb[e];
+        if (up && up_b) u[e] += ub[e];
+        if (act == 6) {  // clamped gated unit: g sigmoid(alpha g) (u + 1), g <= limit, |u| <= limit
+          const float gc = fminf(g[e], limit), uc = fminf(fmaxf(u[e], -limit), limit);
+          o[e] = gc / (1.f + __expf(-alpha * gc)) * (uc + 1.f);
+        } else {
+          o[e] = act_fn(g[e], act) * (up ? u[e] : 1.f);
+        }
+        o[e] *= scale;
       }
-      o[e] *= post;
+      stv<T, V>(out + r * out_stride + c, o);
     }
-    stv<T, V>(out + r * out_stride + c, o);
   }
 }
 
@@ -927,15 +926,20 @@ int dxm_act_mul(void* out, const void* gate, int64_t g_stride, const void* up, i
                    (uintptr_t)out % (4 * esz) == 0 && (uintptr_t)gate_b % 16 == 0 && (uintptr_t)up_b % 16 == 0;
   const int per = kThreads * (vec ? 4 : 1);
   const int gx = (F + per - 1) / per;
-  for (int r0 = 0; r0 < rows; r0 += 65535) {
-    const int nr = rows - r0 < 65535 ? rows - r0 : 65535;
-#define ACT_MUL(V)                                                                                                     \
-  DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, V>), dim3(gx, nr), dim3(kThreads), 0, st,                      \
+  constexpr int kRowsPer = 8;
+  const bool many = (gate_b || up_b) && rows >= 2048;
+  const int rows_per = many ? kRowsPer : 1;
+  for (int r0 = 0; r0 < rows; r0 += 65535 * rows_per) {
+    const int nr = rows - r0 < 65535 * rows_per ? rows - r0 : 65535 * rows_per, gy = (nr + rows_per - 1) / rows_per;
+#define ACT_MUL(V, ROWS)                                                                                               \
+  DISPATCH_T(f32, hipLaunchKernelGGL((act_mul_kernel<T, V, ROWS>), dim3(gx, gy), dim3(kThreads), 0, st,                \
                                      (T*)out + r0 * out_stride, (const T*)gate + r0 * g_stride, g_stride,              \
                                      up ? (const T*)up + r0 * u_stride : nullptr, u_stride, F, out_stride, act, limit, \
-                                     alpha, post, gate_b, up_b, row_scale ? row_scale + r0 : nullptr, u_dv, u_head))
-    if (vec) { ACT_MUL(4) }
-    else { ACT_MUL(1) }
+                                     alpha, post, gate_b, up_b, row_scale ? row_scale + r0 : nullptr, u_dv, u_head, nr))
+    if (vec && many) { ACT_MUL(4, kRowsPer) }
+    else if (vec) { ACT_MUL(4, 1) }
+    else if (many) { ACT_MUL(1, kRowsPer) }
+    else { ACT_MUL(1, 1) }
 #undef ACT_MUL
   }
   DX_CHECK_LAUNCH();

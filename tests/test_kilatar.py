@@ -361,6 +361,13 @@ def test_gated_units_alone(device, dtype, F, dv):
     got = mx.glu_act(dev(gu), "gelu_tanh", gate_b=dev(gb), up_b=dev(ub), row_scale=dev(rs))
     g, u = gu[:, :F].double() + gb.double(), gu[:, F:].double() + ub.double()
     assert torch.allclose(got.cpu().double(), O.gelu_tanh(g) * u * rs.double()[:, None], **tol(dtype, 2e-5, 2e-2))
+    if F == 24:  # many rows: a workgroup takes several
+        gu = (torch.randn(2051, 2 * F) * 2).to(dt)
+        got = mx.glu_act(dev(gu), "gelu_tanh", gate_b=dev(gb), up_b=dev(ub), row_scale=dev(rs.repeat(411)[:2051].contiguous()))
+        g, u = gu[:, :F].double() + gb.double(), gu[:, F:].double() + ub.double()
+        want = O.gelu_tanh(g) * u * rs.repeat(411)[:2051].double()[:, None]
+        assert torch.allclose(got.cpu().double(), want, **tol(dtype, 2e-5, 2e-2))
+        gu = gu[:T]
     H = F // dv
     up = torch.randn(H, T, dv).to(dt)
     out = torch.full((T, F + 4), 9.0, device=device, dtype=dt)
