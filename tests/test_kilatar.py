@@ -378,16 +378,16 @@ def test_gated_units_alone(device, dtype, F, dv):
 
 def test_scaled_frequencies():
     """All three bands of the scaling, their edges, and none."""
-    for dims, base, sc in ((32, 500000.0, {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 512}), (8, 100.0, SCALING),
+    for dims, base, sc in ((40, 200000.0, {"factor": 6.0, "low": 1.0, "high": 5.0, "original": 700}), (8, 100.0, SCALING),
                            (2, 10.0, None), (64, 1e4, {"factor": 2.0, "low": 2.0, "high": 3.0, "original": 100})):
         rot = {"dims": dims, "base": base, **({"scaling": sc} if sc else {})}
         want = torch.tensor(O.frequencies(rot), dtype=torch.float64)
         assert torch.allclose(rc.rotary_frequencies(dims, base, sc).double(), want, rtol=1e-6)
-    f = torch.tensor(O.frequencies({"dims": 32, "base": 500000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0,
-                                                                               "original": 512}}))
-    plain = torch.tensor(O.frequencies({"dims": 32, "base": 500000.0}))
-    assert float((f / plain).max()) == 1.0 and abs(float((f / plain).min()) - 0.125) < 1e-6
-    assert bool(((f / plain > 0.13) & (f / plain < 0.99)).any())
+    f = torch.tensor(O.frequencies({"dims": 40, "base": 200000.0, "scaling": {"factor": 6.0, "low": 1.0, "high": 5.0,
+                                                                               "original": 700}}))
+    plain = torch.tensor(O.frequencies({"dims": 40, "base": 200000.0}))
+    assert float((f / plain).max()) == 1.0 and abs(float((f / plain).min()) - 1 / 6) < 1e-6
+    assert bool(((f / plain > 0.17) & (f / plain < 0.99)).any())
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
